@@ -2,8 +2,9 @@
 
     PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace
 
-The .so lands at substratus_amd/_C*.so (git-ignored; it travels to the GPU box
-with the gpurun snapshot).
+The libraries land at substratus_amd/_C*.so and substratus_amd/_hybrid*.so
+(git-ignored). SUB_EXT names the extensions to build, with commas between them;
+default all.
 """
 
 import os
@@ -16,12 +17,36 @@ from torch.utils.cpp_extension import BuildExtension, CUDAExtension  # noqa: E40
 
 ROOT = os.path.dirname(os.path.abspath(__file__))
 HIP_DIR = os.path.join(ROOT, "substratus_amd", "ops", "hip")
+HYBRID_DIR = os.path.join(HIP_DIR, "hybrid")
 
 # Hand-written kernel sources only. torch's CUDAExtension hipify pass emits
 # *_hip.hip/*_hip.cpp siblings into the build dir; exclude any that leak
 # in-tree so the generated copies can never shadow the originals.
-sources = [os.path.join(HIP_DIR, f) for f in sorted(os.listdir(HIP_DIR))
-           if f.endswith(".hip") and not f.endswith("_hip.hip")]
+def hip_sources(folder):
+    return [os.path.join(folder, f) for f in sorted(os.listdir(folder))
+            if f.endswith(".hip") and not f.endswith("_hip.hip")]
+
+
+def extension(name, sources):
+    return CUDAExtension(
+        name=f"substratus_amd.{name}", sources=sources,
+        extra_compile_args={
+            "cxx": ["-O3", "-std=c++17"],
+            # packed-FP32 VALU forms stay off: some of them have given
+            # wrong results on this hardware
+            "nvcc": ["-O3", "-std=c++17", "-Xclang", "-target-feature",
+                     "-Xclang", "-packed-fp32-ops"],
+        })
+
+
+# _C: the kernels of the uniform transformer families, sampling, training.
+# _hybrid: the kernels of models whose layers differ (models/hybrid.py).
+extensions = {
+    "_C": hip_sources(HIP_DIR),
+    "_hybrid": hip_sources(HYBRID_DIR) + [
+        os.path.join(HIP_DIR, "activation.hip")],
+}
+wanted = os.environ.get("SUB_EXT", ",".join(extensions)).split(",")
 
 setup(
     name="substratus_amd",
@@ -36,18 +61,6 @@ setup(
         "sub = substratus_amd.cli.main:main",
         "nbwatch = substratus_amd.containertools.nbwatch:watch",
     ]},
-    ext_modules=[
-        CUDAExtension(
-            name="substratus_amd._C",
-            sources=sources,
-            extra_compile_args={
-                "cxx": ["-O3", "-std=c++17"],
-                # packed-FP32 VALU forms stay off: some of them have given
-                # wrong results on this hardware
-                "nvcc": ["-O3", "-std=c++17", "-Xclang", "-target-feature",
-                         "-Xclang", "-packed-fp32-ops"],
-            },
-        )
-    ],
+    ext_modules=[extension(n, extensions[n]) for n in wanted],
     cmdclass={"build_ext": BuildExtension},
 )

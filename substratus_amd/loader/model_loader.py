@@ -93,12 +93,11 @@ def _try_hub_download(name: str, files_filter: str, out: str) -> bool:
 
 def _write_random_init(name: str, out: str, params: dict) -> None:
     from safetensors.torch import save_file
-    from ..models.config import get_config
-    from ..models.model import CausalLM
+    from ..models import build_model, get_config
     cfg = get_config(name)
     dtype = torch.bfloat16 if params.get("dtype", "bf16") == "bf16" \
         else torch.float32
-    model = CausalLM(cfg, device="meta", dtype=dtype)
+    model = build_model(cfg, device="meta", dtype=dtype)
     model = model.to_empty(device="cpu")
     model.init_random(seed=int(params.get("seed", 0)))
     tensors = {k: v.detach().contiguous()

@@ -1,2 +1,10 @@
 from .config import ModelConfig, get_config, register
+from . import kakovik as _kakovik  # registers the architecture and its models
+from .hybrid import HybridLM
 from .model import CausalLM
+
+
+def build_model(cfg: ModelConfig, device=None, dtype=None):
+    """The model class a config calls for, with uninitialised weights."""
+    cls = HybridLM if cfg.layers else CausalLM
+    return cls(cfg, device=device, dtype=dtype)

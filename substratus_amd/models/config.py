@@ -8,14 +8,18 @@ examples/llama2-70b/server.yaml). We implement those model families natively.
 
 from __future__ import annotations
 
+import json
+import os
 from dataclasses import dataclass, field
-from typing import Optional
+from typing import Callable, Optional
+
+from .layers import LayerSpec
 
 
 @dataclass
 class ModelConfig:
     name: str
-    family: str  # "llama" | "falcon" | "opt"
+    family: str  # "llama" | "falcon" | "opt" | "kakovik"
     hidden_size: int
     intermediate_size: int
     num_layers: int
@@ -36,9 +40,14 @@ class ModelConfig:
     # opt-style: learned positional embeddings + LayerNorm + gelu
     learned_pos_emb: bool = False
     activation: str = "silu"  # "silu" (gated) | "gelu"
+    # models of unlike layers (models/hybrid.py): one spec per layer; the
+    # uniform fields above then only size things for reports
+    layers: tuple[LayerSpec, ...] = ()
+    norm_offset: float = 0.0  # 1: norm weights are stored around zero
+    logit_scale: float = 1.0
 
     def __post_init__(self) -> None:
-        if self.head_dim == 0:
+        if self.head_dim == 0 and self.num_heads:
             self.head_dim = self.hidden_size // self.num_heads
 
     @property
@@ -47,6 +56,9 @@ class ModelConfig:
 
     def param_count(self) -> int:
         h, f, L, v = self.hidden_size, self.intermediate_size, self.num_layers, self.vocab_size
+        if self.layers:
+            return 2 * v * h + sum(s.mixer.params(h) + 3 * h * s.ff
+                                   for s in self.layers)
         qkv = h * (self.num_heads + 2 * self.num_kv_heads) * self.head_dim
         o = self.num_heads * self.head_dim * h
         if self.activation == "silu":
@@ -65,7 +77,45 @@ def register(cfg: ModelConfig) -> ModelConfig:
     return cfg
 
 
+# Model folders whose config.json spells out an architecture instead of naming
+# a registered model: "architecture" -> parser(document, tensor shapes, name).
+_ARCHITECTURES: dict[str, Callable[[dict, dict, str], ModelConfig]] = {}
+
+
+def register_architecture(name: str):
+    def add(parser):
+        _ARCHITECTURES[name] = parser
+        return parser
+    return add
+
+
+def tensor_shapes(path: str) -> dict[str, tuple[int, ...]]:
+    """Names and shapes of a safetensors file, from its header only."""
+    with open(path, "rb") as f:
+        header = json.loads(f.read(int.from_bytes(f.read(8), "little")))
+    return {k: tuple(v["shape"]) for k, v in header.items()
+            if k != "__metadata__"}
+
+
+def load_config(model_dir: str) -> ModelConfig:
+    """The config of a model folder (config.json, model.safetensors)."""
+    with open(os.path.join(model_dir, "config.json")) as f:
+        doc = json.load(f)
+    if "architecture" not in doc:
+        return get_config(doc["model"])
+    if doc["architecture"] not in _ARCHITECTURES:
+        raise KeyError(f"unknown architecture {doc['architecture']!r}; known: "
+                       f"{sorted(_ARCHITECTURES)}")
+    weights = os.path.join(model_dir, "model.safetensors")
+    shapes = tensor_shapes(weights) if os.path.exists(weights) else {}
+    name = os.path.basename(os.path.abspath(model_dir))
+    return _ARCHITECTURES[doc["architecture"]](doc, shapes, name)
+
+
 def get_config(name: str) -> ModelConfig:
+    """A registered model by name, or a model folder by path."""
+    if os.path.isfile(os.path.join(name, "config.json")):
+        return load_config(name)
     key = name.lower().split("/")[-1]
     if key in _REGISTRY:
         return _REGISTRY[key]

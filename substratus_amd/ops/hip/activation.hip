@@ -70,6 +70,32 @@ void launch_silu_mul(bf16_t* out, const bf16_t* x, long rows, int f,
       out, x, rows, f);
 }
 
+// Any width, float or bf16: the 32-bit path, and widths the vector kernel
+// does not take.
+template <class T, int BLOCK>
+__global__ void silu_mul_any_kernel(T* __restrict__ out,
+                                    const T* __restrict__ x, int f) {
+  const long row = blockIdx.x;
+  for (int i = blockIdx.y * BLOCK + threadIdx.x; i < f;
+       i += gridDim.y * BLOCK) {
+    const float g = (float)x[row * 2L * f + i];
+    const float u = (float)x[row * 2L * f + f + i];
+    out[row * (long)f + i] = (T)(g / (1.f + expf(-g)) * u);
+  }
+}
+
+void launch_silu_mul_any(float* out, const float* x, long rows, int f,
+                         hipStream_t stream) {
+  silu_mul_any_kernel<float, 256><<<dim3(rows, 4), dim3(256), 0, stream>>>(
+      out, x, f);
+}
+
+void launch_silu_mul_any(bf16_t* out, const bf16_t* x, long rows, int f,
+                         hipStream_t stream) {
+  silu_mul_any_kernel<bf16_t, 256><<<dim3(rows, 4), dim3(256), 0, stream>>>(
+      out, x, f);
+}
+
 void launch_gelu(bf16_t* out, const bf16_t* x, long n, hipStream_t stream) {
   constexpr int BLOCK = 256;
   long n8 = n / 8;

@@ -31,6 +31,7 @@ void launch_attn_prefill_probe(int, bf16_t*, const bf16_t*, const bf16_t*, const
 void launch_mfma_probe(float*, const bf16_t*, const bf16_t*, hipStream_t);
 void launch_mfma32_probe(float*, const bf16_t*, const bf16_t*, hipStream_t);
 void launch_softmax_sample(long*, const bf16_t*, const float*, const int*, const float*, const float*, int, int, hipStream_t);
+void launch_softmax_sample(long*, const float*, const float*, const int*, const float*, const float*, int, int, hipStream_t);
 void launch_cross_entropy(float*, bf16_t*, const bf16_t*, const long*, long, int, long, float, hipStream_t);
 void launch_adamw(bf16_t*, const bf16_t*, float*, float*, long, float, float, float, float, float, int, float, hipStream_t);
 void launch_adamw_f32(float*, const float*, float*, float*, long, float, float, float, float, float, int, float, hipStream_t);
@@ -421,15 +422,24 @@ torch::Tensor mfma_probe(torch::Tensor a, torch::Tensor b) {
 void softmax_sample(torch::Tensor out, torch::Tensor logits,
                     torch::Tensor temperature, torch::Tensor top_k,
                     torch::Tensor top_p, torch::Tensor uniform) {
-  check_bf16(logits, "logits");
   TORCH_CHECK(out.scalar_type() == torch::kLong, "out must be int64");
   int bsz = logits.size(0), vocab = logits.size(1);
-  TORCH_CHECK((size_t)vocab * 2 <= 160 * 1024 - 4096,
+  TORCH_CHECK((size_t)vocab * logits.element_size() <= 160 * 1024 - 4096,
               "vocab too large for LDS staging: ", vocab);
-  launch_softmax_sample(out.data_ptr<long>(), bfc(logits),
-                        temperature.data_ptr<float>(), top_k.data_ptr<int>(),
-                        top_p.data_ptr<float>(), uniform.data_ptr<float>(),
-                        bsz, vocab, stream());
+  auto go = [&](auto* data) {
+    launch_softmax_sample(out.data_ptr<long>(), data,
+                          temperature.data_ptr<float>(),
+                          top_k.data_ptr<int>(), top_p.data_ptr<float>(),
+                          uniform.data_ptr<float>(), bsz, vocab, stream());
+  };
+  if (logits.scalar_type() == torch::kFloat) {   // models served in 32 bits
+    TORCH_CHECK(logits.is_cuda() && logits.is_contiguous(),
+                "logits must be contiguous on GPU");
+    go(static_cast<const float*>(logits.data_ptr<float>()));
+  } else {
+    check_bf16(logits, "logits");
+    go(bfc(logits));
+  }
   post_launch_check("softmax_sample");
 }
 

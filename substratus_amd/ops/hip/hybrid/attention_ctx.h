@@ -1,0 +1,35 @@
+// Arguments shared by the cache-reading attention kernels.
+#pragma once
+
+#include "typed.h"
+
+template <class T>
+struct AttnCtx {
+  T* out;                  // [rows, heads * vdim]
+  const T* q;              // row r, head h at q + r * q_ld + h * dim
+  const T* gate;           // row r, head h at gate + r * g_ld + h, or null
+  const T* kc;             // [blocks, kv_heads, block_size, dim]
+  const T* vc;             // [blocks, kv_heads, block_size, vdim]
+  const float* bias;       // [heads, nbias] by distance, or null
+  const int* positions;    // [rows]
+  const int* seq_start;    // [entries + 1] row offsets, or null: one row each
+  const int* block_table;  // [entries, max_blocks]
+  long q_ld, g_ld;
+  int heads, kv_heads, dim, vdim, nbias, chunk, max_blocks, block_size;
+  float scale;
+};
+
+constexpr float LOG2E = 1.44269504088896340736f;
+
+template <class T>
+void launch_attn_ctx_any(const AttnCtx<T>&, int entries, int max_len,
+                         hipStream_t);
+
+bool attn_ctx_decode_supported(int dim, int vdim, int block_size);
+int attn_ctx_decode_splits(int entries, int heads, int kv_heads, int span);
+void launch_attn_ctx_decode(const AttnCtx<bf16_t>&, int entries, int splits,
+                            float* part_o, float* part_ml, hipStream_t);
+
+bool attn_ctx_prefill_supported(int dim, int vdim, int block_size);
+void launch_attn_ctx_prefill(const AttnCtx<bf16_t>&, int entries, int max_len,
+                             hipStream_t);

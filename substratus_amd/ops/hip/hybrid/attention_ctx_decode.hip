@@ -1,0 +1,265 @@
+// Single-token attention over the paged bf16 cache with a distance bias, a
+// chunk mask, unequal key and value head sizes and a gated output (the
+// formulas are in attention_ctx.hip). HBM-bound: every K and V row is read
+// once per group of GQ query heads.
+//
+// One page of 16 keys is a wave's unit of work. Scores: 4 lanes per key, each
+// with every fourth 16-byte piece of the row. Values: CL lanes across the
+// columns (8 each), 64/CL rows side by side. The next page's K, V and bias
+// are in flight while the current page is computed. Four waves take pages in
+// turn and merge through LDS; `splits` workgroups share one long context and
+// a second kernel merges those.
+#include "attention_ctx.h"
+
+namespace {
+
+constexpr int NW = 4;         // waves per workgroup
+constexpr int PAGE = 16;
+constexpr float NEG = -1e30f; // "no key yet": finite, so differences are too
+
+template <int DCH, int CL, int GQ>
+__global__ __launch_bounds__(NW * WAVE)
+void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
+                            float* __restrict__ part_o,
+                            float* __restrict__ part_ml) {
+  constexpr int RPI = WAVE / CL;          // V rows per instruction
+  constexpr int NV = PAGE / RPI;          // V instructions per page
+  __shared__ float s_q[GQ][DCH * 32];
+  __shared__ float s_o[NW][GQ][CL * 8];
+  __shared__ float s_ml[NW][GQ][2];
+  const int b = blockIdx.x, kvh = blockIdx.y;
+  const int split = blockIdx.z % splits;
+  const int per = a.heads / a.kv_heads;
+  const int g0 = blockIdx.z / splits * GQ;
+  const int h0 = kvh * per + g0;
+  const int nh = min(GQ, per - g0);
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  const int pos = a.positions[b];
+  const int lo = a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
+  const int* bt = a.block_table + (long)b * a.max_blocks;
+
+  for (int i = threadIdx.x; i < GQ * DCH * 32; i += NW * WAVE) {
+    const int g = i / (DCH * 32), d = i % (DCH * 32);
+    s_q[g][d] = g < nh && d < a.dim
+        ? bf2f(a.q[(long)b * a.q_ld + (long)(h0 + g) * a.dim + d]) *
+              (a.scale * LOG2E)
+        : 0.f;
+  }
+  __syncthreads();
+
+  const int key = lane >> 2, sub = lane & 3;
+  const int col = lane % CL, rg = lane / CL;
+  const int kch = a.dim / 8, vch = a.vdim / 8;
+  const int first = lo / PAGE + split * NW + wave, last = pos / PAGE;
+  const int stride = splits * NW;
+
+  uint4v kr[DCH], vr[NV];
+  float br[GQ];
+  auto load = [&](int pg) {
+    const long page = (long)bt[pg] * a.kv_heads + kvh;
+    const bf16_t* kp = a.kc + (page * PAGE + key) * a.dim;
+    const bf16_t* vp = a.vc + page * PAGE * a.vdim;
+    #pragma unroll
+    for (int i = 0; i < DCH; ++i)
+      kr[i] = sub + 4 * i < kch ? nt_load_u4(kp + (sub + 4 * i) * 8)
+                                : (uint4v){0, 0, 0, 0};
+    #pragma unroll
+    for (int i = 0; i < NV; ++i)
+      vr[i] = col < vch
+          ? nt_load_u4(vp + (long)(rg + RPI * i) * a.vdim + col * 8)
+          : (uint4v){0, 0, 0, 0};
+    #pragma unroll
+    for (int g = 0; g < GQ; ++g) {
+      const int n = min(max(pos - (pg * PAGE + key), 0), a.nbias - 1);
+      br[g] = a.bias != nullptr && g < nh
+          ? a.bias[(long)(h0 + g) * a.nbias + n] * LOG2E : 0.f;
+    }
+  };
+
+  float m[GQ], l[GQ], acc[GQ][8];
+  #pragma unroll
+  for (int g = 0; g < GQ; ++g) {
+    m[g] = NEG; l[g] = 0.f;
+    #pragma unroll
+    for (int j = 0; j < 8; ++j) acc[g][j] = 0.f;
+  }
+  if (first <= last) load(first);
+  for (int pg = first; pg <= last; pg += stride) {
+    uint4v kn[DCH], vn[NV];
+    float bn[GQ];
+    #pragma unroll
+    for (int i = 0; i < DCH; ++i) kn[i] = kr[i];
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) vn[i] = vr[i];
+    #pragma unroll
+    for (int g = 0; g < GQ; ++g) bn[g] = br[g];
+    if (pg + stride <= last) load(pg + stride);
+
+    float s[GQ];
+    #pragma unroll
+    for (int g = 0; g < GQ; ++g) s[g] = 0.f;
+    #pragma unroll
+    for (int i = 0; i < DCH; ++i) {
+      float kf[8];
+      #pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float2 t = unpack_bf16x2(kn[i][j]);
+        kf[2 * j] = t.x; kf[2 * j + 1] = t.y;
+      }
+      #pragma unroll
+      for (int g = 0; g < GQ; ++g) {
+        const float4* qp =
+            reinterpret_cast<const float4*>(&s_q[g][(sub + 4 * i) * 8]);
+        const float4 q0 = qp[0], q1 = qp[1];
+        s[g] += kf[0] * q0.x + kf[1] * q0.y + kf[2] * q0.z + kf[3] * q0.w +
+                kf[4] * q1.x + kf[5] * q1.y + kf[6] * q1.z + kf[7] * q1.w;
+      }
+    }
+    const int kpos = pg * PAGE + key;
+    const bool live = kpos >= lo && kpos <= pos;
+    #pragma unroll
+    for (int g = 0; g < GQ; ++g) {
+      s[g] += __shfl_xor(s[g], 1, WAVE);
+      s[g] += __shfl_xor(s[g], 2, WAVE);
+      s[g] = live ? s[g] + bn[g] : NEG;
+      float mx = s[g];
+      #pragma unroll
+      for (int off = 4; off < WAVE; off <<= 1)
+        mx = fmaxf(mx, __shfl_xor(mx, off, WAVE));
+      if (mx > m[g]) {                     // uniform over the wave
+        const float keep = __builtin_amdgcn_exp2f(m[g] - mx);
+        l[g] *= keep;
+        #pragma unroll
+        for (int j = 0; j < 8; ++j) acc[g][j] *= keep;
+        m[g] = mx;
+      }
+      s[g] = live ? __builtin_amdgcn_exp2f(s[g] - m[g]) : 0.f;
+      l[g] += s[g];                        // lanes hold 4 copies of each key
+    }
+    #pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      float vf[8];
+      #pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float2 t = unpack_bf16x2(vn[i][j]);
+        vf[2 * j] = t.x; vf[2 * j + 1] = t.y;
+      }
+      #pragma unroll
+      for (int g = 0; g < GQ; ++g) {
+        const float p = __shfl(s[g], (rg + RPI * i) * 4, WAVE);
+        #pragma unroll
+        for (int j = 0; j < 8; ++j) acc[g][j] += p * vf[j];
+      }
+    }
+  }
+
+  #pragma unroll
+  for (int g = 0; g < GQ; ++g) {
+    #pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      #pragma unroll
+      for (int off = CL; off < WAVE; off <<= 1)
+        acc[g][j] += __shfl_xor(acc[g][j], off, WAVE);
+      if (rg == 0) s_o[wave][g][col * 8 + j] = acc[g][j];
+    }
+    const float lt = wave_sum(l[g]) * 0.25f;
+    if (lane == 0) { s_ml[wave][g][0] = m[g]; s_ml[wave][g][1] = lt; }
+  }
+  __syncthreads();
+
+  for (int i = threadIdx.x; i < nh * a.vdim; i += NW * WAVE) {
+    const int g = i / a.vdim, c = i % a.vdim, h = h0 + g;
+    float M = s_ml[0][g][0];
+    #pragma unroll
+    for (int w = 1; w < NW; ++w) M = fmaxf(M, s_ml[w][g][0]);
+    float L = 0.f, o = 0.f;
+    #pragma unroll
+    for (int w = 0; w < NW; ++w) {
+      const float f = __builtin_amdgcn_exp2f(s_ml[w][g][0] - M);
+      L += s_ml[w][g][1] * f;
+      o += s_o[w][g][c] * f;
+    }
+    if (splits == 1) {
+      float f = 1.f / L;
+      if (a.gate != nullptr)
+        f *= sigmoid_f(bf2f(a.gate[(long)b * a.g_ld + h]));
+      a.out[((long)b * a.heads + h) * a.vdim + c] = f2bf(o * f);
+    } else {
+      const long at = ((long)b * a.heads + h) * splits + split;
+      part_o[at * a.vdim + c] = o;
+      if (c == 0) { part_ml[at * 2] = M; part_ml[at * 2 + 1] = L; }
+    }
+  }
+}
+
+__global__ __launch_bounds__(WAVE)
+void attn_ctx_merge_kernel(AttnCtx<bf16_t> a, int splits,
+                           const float* __restrict__ part_o,
+                           const float* __restrict__ part_ml) {
+  const int h = blockIdx.x;
+  const long b = blockIdx.y, at = (b * a.heads + h) * splits;
+  float M = NEG, L = 0.f;
+  for (int s = 0; s < splits; ++s) M = fmaxf(M, part_ml[(at + s) * 2]);
+  for (int s = 0; s < splits; ++s)
+    L += part_ml[(at + s) * 2 + 1] *
+         __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
+  float f = 1.f / L;
+  if (a.gate != nullptr) f *= sigmoid_f(bf2f(a.gate[b * a.g_ld + h]));
+  for (int c = threadIdx.x; c < a.vdim; c += WAVE) {
+    float o = 0.f;
+    for (int s = 0; s < splits; ++s)
+      o += part_o[(at + s) * a.vdim + c] *
+           __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
+    a.out[(b * a.heads + h) * a.vdim + c] = f2bf(o * f);
+  }
+}
+
+constexpr int pick_gq(int per) { return per >= 4 ? 4 : per >= 2 ? 2 : 1; }
+
+}  // namespace
+
+bool attn_ctx_decode_supported(int dim, int vdim, int block_size) {
+  return dim % 8 == 0 && vdim % 8 == 0 && dim <= 256 && vdim <= 256 &&
+         block_size == PAGE;
+}
+
+// Workgroups that share one context: enough to fill 256 CUs four deep, but
+// at least two pages for every wave. `span`: most keys a token can see.
+int attn_ctx_decode_splits(int entries, int heads, int kv_heads, int span) {
+  const int per = heads / kv_heads, gq = pick_gq(per);
+  const long groups = (long)entries * kv_heads * ((per + gq - 1) / gq);
+  const int pages = (span + PAGE - 1) / PAGE;
+  int s = 1;
+  while (s < 32 && groups * s < 1024 && pages >= s * 2 * NW * 2) s *= 2;
+  return s;
+}
+
+void launch_attn_ctx_decode(const AttnCtx<bf16_t>& a, int entries, int splits,
+                            float* part_o, float* part_ml,
+                            hipStream_t stream) {
+  const int per = a.heads / a.kv_heads, gq = pick_gq(per);
+  const dim3 grid(entries, a.kv_heads, (per + gq - 1) / gq * splits);
+  auto go = [&](auto dch, auto cl, auto g) {
+    attn_ctx_decode_kernel<decltype(dch)::value, decltype(cl)::value,
+                           decltype(g)::value>
+        <<<grid, dim3(NW * WAVE), 0, stream>>>(a, splits, part_o, part_ml);
+  };
+  using std::integral_constant;
+  auto by_g = [&](auto dch, auto cl) {
+    if (gq == 1) go(dch, cl, integral_constant<int, 1>{});
+    else if (gq == 2) go(dch, cl, integral_constant<int, 2>{});
+    else go(dch, cl, integral_constant<int, 4>{});
+  };
+  auto by_cl = [&](auto dch) {
+    if (a.vdim <= 64) by_g(dch, integral_constant<int, 8>{});
+    else if (a.vdim <= 128) by_g(dch, integral_constant<int, 16>{});
+    else by_g(dch, integral_constant<int, 32>{});
+  };
+  if (a.dim <= 64) by_cl(integral_constant<int, 2>{});
+  else if (a.dim <= 96) by_cl(integral_constant<int, 3>{});
+  else if (a.dim <= 128) by_cl(integral_constant<int, 4>{});
+  else by_cl(integral_constant<int, 8>{});
+  if (splits > 1)
+    attn_ctx_merge_kernel<<<dim3(a.heads, entries), dim3(WAVE), 0, stream>>>(
+        a, splits, part_o, part_ml);
+}

@@ -1,0 +1,326 @@
+// Python bindings of the hybrid-model kernels (substratus_amd._hybrid): norms
+// of a 32-bit residual, cache-reading attention, gated linear attention.
+// Every op takes float or bf16 activations. Shapes are checked here; kernels
+// are thin and trusting.
+#include <torch/extension.h>
+#include <ATen/cuda/CUDAContext.h>
+
+#include "attention_ctx.h"
+#include "gla.h"
+
+template <class T>
+void launch_stream_norm(T*, float*, const T*, const float*, const float*, long, int, float, float, float, hipStream_t);
+template <class T>
+void launch_embed_norm(T*, float*, const T*, const int*, const float*, long, int, int, float, float, hipStream_t);
+int stream_norm_max_width(int width);
+template <class T>
+void launch_qkv_prepare(T*, long, int, int, int, const float*, const float*, float, const T*, long, const float*, T*, T*, const int*, long, int, int, hipStream_t);
+void launch_silu_mul(bf16_t*, const bf16_t*, long, int, hipStream_t);
+void launch_silu_mul_any(float*, const float*, long, int, hipStream_t);
+void launch_silu_mul_any(bf16_t*, const bf16_t*, long, int, hipStream_t);
+
+namespace {
+
+using torch::Tensor;
+using OptTensor = std::optional<Tensor>;
+
+hipStream_t stream() { return at::cuda::getCurrentCUDAStream().stream(); }
+
+template <class T> struct Scalar;
+template <> struct Scalar<float> { static constexpr auto type = torch::kFloat32; };
+template <> struct Scalar<bf16_t> { static constexpr auto type = torch::kBFloat16; };
+
+void check(const Tensor& t, torch::ScalarType type, const char* name,
+           bool contiguous = true) {
+  TORCH_CHECK(t.is_cuda(), name, " must be on the GPU");
+  TORCH_CHECK(t.scalar_type() == type, name, " must be ", type, ", is ",
+              t.scalar_type());
+  TORCH_CHECK(!contiguous || t.is_contiguous(), name, " must be contiguous");
+}
+
+template <class T>
+T* ptr(const Tensor& t) { return reinterpret_cast<T*>(t.data_ptr()); }
+template <class T>
+T* ptr(const OptTensor& t) { return t ? ptr<T>(*t) : nullptr; }
+
+// [rows, n] view whose rows are `stride(0)` apart
+void check_rows(const Tensor& t, torch::ScalarType type, const char* name) {
+  check(t, type, name, false);
+  TORCH_CHECK(t.dim() == 2 && (t.stride(1) == 1 || t.size(1) == 1), name,
+              " must be [rows, n] with contiguous rows");
+}
+
+void post(const char* op) {
+  const hipError_t e = hipGetLastError();
+  TORCH_CHECK(e == hipSuccess, op, ": launch failed: ", hipGetErrorString(e));
+}
+
+template <class F>
+void by_type(const Tensor& t, F f) {
+  if (t.scalar_type() == torch::kBFloat16) f(bf16_t{});
+  else if (t.scalar_type() == torch::kFloat32) f(float{});
+  else TORCH_CHECK(false, "activations must be float32 or bfloat16");
+}
+
+void stream_norm(Tensor y, Tensor x, Tensor delta, Tensor w_post, Tensor w_pre,
+                 double off, double eps, double out_scale) {
+  const int width = x.size(-1);
+  const long rows = x.numel() / width;
+  check(x, torch::kFloat32, "x");
+  check(w_post, torch::kFloat32, "w_post");
+  check(w_pre, torch::kFloat32, "w_pre");
+  TORCH_CHECK(width <= stream_norm_max_width(width), "row too wide");
+  TORCH_CHECK(y.numel() == x.numel() && delta.numel() == x.numel() &&
+              w_post.numel() == width && w_pre.numel() == width,
+              "stream_norm: shapes differ");
+  if (rows == 0) return;
+  by_type(y, [&](auto tag) {
+    using T = decltype(tag);
+    check(y, Scalar<T>::type, "y");
+    check(delta, Scalar<T>::type, "delta");
+    launch_stream_norm<T>(ptr<T>(y), ptr<float>(x), ptr<T>(delta),
+                          ptr<float>(w_post), ptr<float>(w_pre), rows, width,
+                          off, eps, out_scale, stream());
+  });
+  post("stream_norm");
+}
+
+void embed_norm(Tensor y, Tensor x, Tensor table, Tensor tokens, Tensor w_pre,
+                double off, double eps) {
+  const int width = table.size(1);
+  const long rows = tokens.numel();
+  check(x, torch::kFloat32, "x");
+  check(tokens, torch::kInt32, "tokens");
+  check(w_pre, torch::kFloat32, "w_pre");
+  TORCH_CHECK(width <= stream_norm_max_width(width), "row too wide");
+  TORCH_CHECK(y.numel() == rows * width && x.numel() == rows * width &&
+              w_pre.numel() == width, "embed_norm: shapes differ");
+  if (rows == 0) return;
+  by_type(y, [&](auto tag) {
+    using T = decltype(tag);
+    check(y, Scalar<T>::type, "y");
+    check(table, Scalar<T>::type, "table");
+    launch_embed_norm<T>(ptr<T>(y), ptr<float>(x), ptr<T>(table),
+                         ptr<int>(tokens), ptr<float>(w_pre), rows, width,
+                         table.size(0), off, eps, stream());
+  });
+  post("embed_norm");
+}
+
+// buf [rows, >= nq + nk + nv]; kc [blocks, kv_heads, block, dim]
+void qkv_prepare(Tensor buf, int64_t nq, OptTensor qw, OptTensor kw,
+                 double eps, OptTensor v_first, OptTensor lam, Tensor kc,
+                 Tensor vc, Tensor slots) {
+  const int kv = kc.size(1), nk = kv * kc.size(3), nv = kv * vc.size(3);
+  const long rows = buf.size(0);
+  check(slots, torch::kInt32, "slots");
+  TORCH_CHECK(slots.numel() == rows, "one slot per row");
+  TORCH_CHECK(buf.size(1) >= nq + nk + nv, "buf too narrow");
+  TORCH_CHECK(kc.size(0) == vc.size(0) && kc.size(1) == vc.size(1) &&
+              kc.size(2) == vc.size(2), "caches differ");
+  TORCH_CHECK(qw.has_value() == kw.has_value(), "norm both or neither");
+  if (qw) {
+    check(*qw, torch::kFloat32, "qw");
+    check(*kw, torch::kFloat32, "kw");
+    TORCH_CHECK(qw->numel() == nq && kw->numel() == nk, "norm weight sizes");
+  }
+  if (v_first) {
+    TORCH_CHECK(lam.has_value() && lam->numel() == 1, "v_first needs lam");
+    check(*lam, torch::kFloat32, "lam");
+    TORCH_CHECK(v_first->size(0) == rows && v_first->size(1) == nv,
+                "v_first must be [rows, nv]");
+  }
+  if (rows == 0) return;
+  by_type(buf, [&](auto tag) {
+    using T = decltype(tag);
+    check_rows(buf, Scalar<T>::type, "buf");
+    check(kc, Scalar<T>::type, "kc");
+    check(vc, Scalar<T>::type, "vc");
+    if (v_first) check_rows(*v_first, Scalar<T>::type, "v_first");
+    launch_qkv_prepare<T>(ptr<T>(buf), buf.stride(0), nq, nk, nv,
+                          ptr<float>(qw), ptr<float>(kw), eps,
+                          ptr<T>(v_first), v_first ? v_first->stride(0) : 0,
+                          ptr<float>(lam), ptr<T>(kc), ptr<T>(vc),
+                          ptr<int>(slots), rows, kv, kc.size(2), stream());
+  });
+  post("qkv_prepare");
+}
+
+// One entry per row (seq_start absent) or portions of up to max_len rows.
+// `rows` are those of q; span: most keys a row can see; any: take the
+// untiled kernel.
+void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
+              OptTensor bias, Tensor positions, OptTensor seq_start,
+              Tensor block_table, double scale, int64_t chunk,
+              int64_t max_len, int64_t span, bool any) {
+  const int kv = kc.size(1), dim = kc.size(3), vdim = vc.size(3);
+  const long rows = q.size(0);
+  TORCH_CHECK(q.size(1) % dim == 0, "q is not heads * dim wide");
+  const int heads = q.size(1) / dim;
+  TORCH_CHECK(heads % kv == 0, "query heads must divide by kv heads");
+  TORCH_CHECK(vdim <= 512, "value size over 512");
+  TORCH_CHECK(vc.size(0) == kc.size(0) && vc.size(1) == kv &&
+              vc.size(2) == kc.size(2), "caches differ");
+  TORCH_CHECK(out.size(0) == rows && out.size(1) == heads * vdim,
+              "out must be [rows, heads * vdim]");
+  check(positions, torch::kInt32, "positions");
+  check(block_table, torch::kInt32, "block_table");
+  TORCH_CHECK(positions.numel() == rows, "one position per row");
+  const int entries = block_table.size(0);
+  if (seq_start) {
+    check(*seq_start, torch::kInt32, "seq_start");
+    TORCH_CHECK(seq_start->numel() == entries + 1, "entries differ");
+  } else {
+    TORCH_CHECK(rows == entries, "one row per entry");
+  }
+  if (bias) {
+    check(*bias, torch::kFloat32, "bias");
+    TORCH_CHECK(bias->dim() == 2 && bias->size(0) == heads, "bias heads");
+  }
+  if (rows == 0) return;
+  by_type(q, [&](auto tag) {
+    using T = decltype(tag);
+    check_rows(q, Scalar<T>::type, "q");
+    check(out, Scalar<T>::type, "out");
+    check(kc, Scalar<T>::type, "kc");
+    check(vc, Scalar<T>::type, "vc");
+    if (gate) {
+      check_rows(*gate, Scalar<T>::type, "gate");
+      TORCH_CHECK(gate->size(0) == rows && gate->size(1) == heads,
+                  "gate must be [rows, heads]");
+    }
+    AttnCtx<T> a{};
+    a.out = ptr<T>(out); a.q = ptr<T>(q); a.gate = ptr<T>(gate);
+    a.kc = ptr<T>(kc); a.vc = ptr<T>(vc); a.bias = ptr<float>(bias);
+    a.positions = ptr<int>(positions); a.seq_start = ptr<int>(seq_start);
+    a.block_table = ptr<int>(block_table);
+    a.q_ld = q.stride(0); a.g_ld = gate ? gate->stride(0) : 0;
+    a.heads = heads; a.kv_heads = kv; a.dim = dim; a.vdim = vdim;
+    a.nbias = bias ? bias->size(1) : 1; a.chunk = chunk;
+    a.max_blocks = block_table.size(1); a.block_size = kc.size(2);
+    a.scale = scale;
+    if constexpr (std::is_same_v<T, bf16_t>) {
+      // the tiled kernels read q rows in 16-byte pieces
+      const bool aligned = a.q_ld % 8 == 0 &&
+          reinterpret_cast<uintptr_t>(a.q) % 16 == 0;
+      if (!any && seq_start && aligned &&
+          attn_ctx_prefill_supported(dim, vdim, a.block_size)) {
+        launch_attn_ctx_prefill(a, entries, max_len, stream());
+        return;
+      }
+      if (!any && !seq_start &&
+          attn_ctx_decode_supported(dim, vdim, a.block_size)) {
+        const int splits =
+            attn_ctx_decode_splits(entries, heads, kv, span);
+        Tensor po, pml;
+        if (splits > 1) {
+          const auto opt = out.options().dtype(torch::kFloat32);
+          po = torch::empty({rows, heads, splits, vdim}, opt);
+          pml = torch::empty({rows, heads, splits, 2}, opt);
+        }
+        launch_attn_ctx_decode(a, entries, splits,
+                               splits > 1 ? ptr<float>(po) : nullptr,
+                               splits > 1 ? ptr<float>(pml) : nullptr,
+                               stream());
+        return;
+      }
+    }
+    launch_attn_ctx_any<T>(a, entries, seq_start ? max_len : 1, stream());
+  });
+  post("attn_ctx");
+}
+
+// x [rows, >= q | k | v | g | A1 h]; state [slots, heads, dim, vdim]
+void gla(Tensor out, Tensor x, Tensor a2, Tensor a2b, Tensor norm,
+         Tensor state, Tensor state_slots, Tensor positions,
+         OptTensor seq_start, double inv_tau, double eps, int64_t max_len,
+         bool recurrent) {
+  const int heads = state.size(1), dim = state.size(2), vdim = state.size(3);
+  const int rank = a2.size(1);
+  const long rows = x.size(0);
+  check(a2, torch::kFloat32, "a2");
+  check(a2b, torch::kFloat32, "a2b");
+  check(norm, torch::kFloat32, "norm");
+  check(state, torch::kFloat32, "state");
+  check(state_slots, torch::kInt32, "state_slots");
+  check(positions, torch::kInt32, "positions");
+  const int entries = state_slots.numel();
+  if (seq_start) {
+    check(*seq_start, torch::kInt32, "seq_start");
+    TORCH_CHECK(seq_start->numel() == entries + 1, "entries differ");
+  } else {
+    TORCH_CHECK(rows == entries, "one row per entry");
+  }
+  TORCH_CHECK(a2.size(0) == heads * dim && a2b.numel() == heads * dim &&
+              norm.numel() == vdim && positions.numel() == rows,
+              "gla: shapes differ");
+  TORCH_CHECK(x.size(1) >= 2 * heads * (dim + vdim) + rank, "x too narrow");
+  TORCH_CHECK(dim <= 2048 && vdim <= 2048, "head size over 2048");
+  TORCH_CHECK(out.size(0) == rows && out.size(1) == heads * vdim,
+              "out must be [rows, heads * vdim]");
+  if (rows == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    check_rows(x, Scalar<T>::type, "x");
+    check(out, Scalar<T>::type, "out");
+    Gla<T> a{};
+    a.out = ptr<T>(out); a.x = ptr<T>(x); a.ld = x.stride(0);
+    a.k_off = heads * dim; a.v_off = 2 * heads * dim;
+    a.g_off = a.v_off + heads * vdim; a.a_off = a.g_off + heads * vdim;
+    a.a2 = ptr<float>(a2); a.a2b = ptr<float>(a2b);
+    a.norm = ptr<float>(norm); a.state = ptr<float>(state);
+    a.state_slots = ptr<int>(state_slots);
+    a.positions = ptr<int>(positions); a.seq_start = ptr<int>(seq_start);
+    a.heads = heads; a.dim = dim; a.vdim = vdim; a.rank = rank;
+    a.qscale = 1.f / std::sqrt((float)dim); a.inv_tau = inv_tau; a.eps = eps;
+    if constexpr (std::is_same_v<T, bf16_t>) {
+      if (seq_start && !recurrent && gla_chunk_supported(dim, vdim, rank)) {
+        const int nseg = gla_chunk_segments(entries, heads, max_len);
+        Tensor ws, wd;
+        if (nseg > 1) {
+          const auto opt = state.options();
+          ws = torch::empty({entries, nseg, heads, dim, vdim}, opt);
+          wd = torch::empty({entries, nseg, heads, dim}, opt);
+        }
+        launch_gla_chunk(a, entries, max_len, nseg,
+                         nseg > 1 ? ptr<float>(ws) : nullptr,
+                         nseg > 1 ? ptr<float>(wd) : nullptr, stream());
+        return;
+      }
+    }
+    launch_gla_recurrent<T>(a, entries, stream());
+  });
+  post("gla");
+}
+
+void silu_mul(Tensor out, Tensor x) {
+  const int f = out.size(-1);
+  TORCH_CHECK(x.size(-1) == 2 * f && x.numel() == 2 * out.numel(),
+              "x must be twice as wide as out");
+  const long rows = out.numel() / f;
+  if (rows == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    check(x, Scalar<T>::type, "x");
+    check(out, Scalar<T>::type, "out");
+    if constexpr (std::is_same_v<T, bf16_t>) {
+      if (f % 8 == 0) {
+        launch_silu_mul(ptr<T>(out), ptr<T>(x), rows, f, stream());
+        return;
+      }
+    }
+    launch_silu_mul_any(ptr<T>(out), ptr<T>(x), rows, f, stream());
+  });
+  post("silu_mul");
+}
+
+}  // namespace
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("stream_norm", &stream_norm);
+  m.def("embed_norm", &embed_norm);
+  m.def("qkv_prepare", &qkv_prepare);
+  m.def("attn_ctx", &attn_ctx);
+  m.def("gla", &gla);
+  m.def("silu_mul", &silu_mul);
+}

@@ -1,0 +1,139 @@
+// Norms of a 32-bit residual stream, fused with what surrounds them.
+//
+//   stream_norm   x += rms(delta) * (off + w_post);  y = rms(x) * (off + w_pre)
+//   embed_norm    x  = table[token];                 y = rms(x) * (off + w_pre)
+//
+// with rms(z) = z / sqrt(mean(z^2) + eps). A block that norms both before and
+// after its sublayer needs exactly one of these between two matrix products:
+// the row of delta and the row of x are read once and stay in registers for
+// both reductions. `off` is 1 for weights stored around zero, else 0;
+// out_scale multiplies y (a logit scale folds in here, in 32 bits).
+#include "typed.h"
+
+template <class T, int VEC, int BLOCK, bool EMBED>
+__global__ __launch_bounds__(BLOCK)
+void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
+                        const T* __restrict__ delta,     // [rows, width]
+                        const T* __restrict__ table,     // [vocab, width]
+                        const int* __restrict__ tokens,  // [rows]
+                        const float* __restrict__ w_post,
+                        const float* __restrict__ w_pre, int width, int vocab,
+                        float off, float eps, float out_scale) {
+  constexpr int RCAP = 8;   // vectors per thread; the launcher checks the row
+  __shared__ float scratch[2][BLOCK / WAVE];
+  const long row = blockIdx.x;
+  const int nvec = width / VEC;
+  float* xr = x + row * width;
+  float xk[RCAP][VEC];
+  const float inv_n = 1.f / (float)width;
+
+  if constexpr (EMBED) {
+    const int tok = min(max(tokens[row], 0), vocab - 1);
+    const T* src = table + (long)tok * width;
+    #pragma unroll
+    for (int kk = 0; kk < RCAP; ++kk) {
+      const int i = threadIdx.x + kk * BLOCK;
+      if (i >= nvec) break;
+      ldv<VEC>(src + i * VEC, xk[kk]);
+    }
+  } else {
+    float dk[RCAP][VEC];
+    float ss = 0.f;
+    const T* dr = delta + row * width;
+    #pragma unroll
+    for (int kk = 0; kk < RCAP; ++kk) {
+      const int i = threadIdx.x + kk * BLOCK;
+      if (i >= nvec) break;
+      ldv<VEC>(dr + i * VEC, dk[kk]);
+      ldv<VEC>(xr + i * VEC, xk[kk]);
+      #pragma unroll
+      for (int j = 0; j < VEC; ++j) ss += dk[kk][j] * dk[kk][j];
+    }
+    ss = block_sum<BLOCK / WAVE>(ss, scratch[0]);
+    const float inv = 1.f / sqrtf(ss * inv_n + eps);
+    #pragma unroll
+    for (int kk = 0; kk < RCAP; ++kk) {
+      const int i = threadIdx.x + kk * BLOCK;
+      if (i >= nvec) break;
+      float w[VEC];
+      ldv<VEC>(w_post + i * VEC, w);
+      #pragma unroll
+      for (int j = 0; j < VEC; ++j)
+        xk[kk][j] += dk[kk][j] * inv * (off + w[j]);
+    }
+  }
+
+  float ss = 0.f;
+  #pragma unroll
+  for (int kk = 0; kk < RCAP; ++kk) {
+    const int i = threadIdx.x + kk * BLOCK;
+    if (i >= nvec) break;
+    stv<VEC>(xr + i * VEC, xk[kk]);
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) ss += xk[kk][j] * xk[kk][j];
+  }
+  ss = block_sum<BLOCK / WAVE>(ss, scratch[1]);
+  const float inv = out_scale / sqrtf(ss * inv_n + eps);
+  T* yr = y + row * width;
+  #pragma unroll
+  for (int kk = 0; kk < RCAP; ++kk) {
+    const int i = threadIdx.x + kk * BLOCK;
+    if (i >= nvec) break;
+    float w[VEC], o[VEC];
+    ldv<VEC>(w_pre + i * VEC, w);
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) o[j] = xk[kk][j] * inv * (off + w[j]);
+    stv<VEC>(yr + i * VEC, o);
+  }
+}
+
+int stream_norm_max_width(int width) {
+  return 1024 * 8 * (width % 4 == 0 ? 4 : 1);
+}
+
+template <class T, bool EMBED>
+static void launch(T* y, float* x, const T* delta, const T* table,
+                   const int* tokens, const float* w_post, const float* w_pre,
+                   long rows, int width, int vocab, float off, float eps,
+                   float out_scale, hipStream_t stream) {
+  auto go = [&](auto vec, auto block) {
+    constexpr int V = decltype(vec)::value, B = decltype(block)::value;
+    stream_norm_kernel<T, V, B, EMBED><<<dim3(rows), dim3(B), 0, stream>>>(
+        y, x, delta, table, tokens, w_post, w_pre, width, vocab, off, eps,
+        out_scale);
+  };
+  using std::integral_constant;
+  auto by_block = [&](auto vec) {
+    const int nvec = width / decltype(vec)::value;
+    if (nvec <= 128) go(vec, integral_constant<int, 64>{});
+    else if (nvec <= 256 * 8) go(vec, integral_constant<int, 256>{});
+    else go(vec, integral_constant<int, 1024>{});
+  };
+  if (width % 4 == 0) by_block(integral_constant<int, 4>{});
+  else by_block(integral_constant<int, 1>{});
+}
+
+template <class T>
+void launch_stream_norm(T* y, float* x, const T* delta, const float* w_post,
+                        const float* w_pre, long rows, int width, float off,
+                        float eps, float out_scale, hipStream_t stream) {
+  launch<T, false>(y, x, delta, nullptr, nullptr, w_post, w_pre, rows, width,
+                   0, off, eps, out_scale, stream);
+}
+
+template <class T>
+void launch_embed_norm(T* y, float* x, const T* table, const int* tokens,
+                       const float* w_pre, long rows, int width, int vocab,
+                       float off, float eps, hipStream_t stream) {
+  launch<T, true>(y, x, nullptr, table, tokens, nullptr, w_pre, rows, width,
+                  vocab, off, eps, 1.f, stream);
+}
+
+template void launch_stream_norm<float>(float*, float*, const float*,
+    const float*, const float*, long, int, float, float, float, hipStream_t);
+template void launch_stream_norm<bf16_t>(bf16_t*, float*, const bf16_t*,
+    const float*, const float*, long, int, float, float, float, hipStream_t);
+template void launch_embed_norm<float>(float*, float*, const float*,
+    const int*, const float*, long, int, int, float, float, hipStream_t);
+template void launch_embed_norm<bf16_t>(bf16_t*, float*, const bf16_t*,
+    const int*, const float*, long, int, int, float, float, hipStream_t);

@@ -1,0 +1,74 @@
+// Loads and stores of float and bf16 activations as float, one or VEC at a
+// time; the hybrid kernels are templates over the activation type.
+#pragma once
+
+#include "../common.h"
+
+DEV_INLINE float ld1(const float* p) { return *p; }
+DEV_INLINE float ld1(const bf16_t* p) { return bf2f(*p); }
+DEV_INLINE void st1(float* p, float v) { *p = v; }
+DEV_INLINE void st1(bf16_t* p, float v) { *p = f2bf(v); }
+
+template <int VEC>
+DEV_INLINE void ldv(const float* p, float* f) {
+  if constexpr (VEC == 4) {
+    const float4 u = *reinterpret_cast<const float4*>(p);
+    f[0] = u.x; f[1] = u.y; f[2] = u.z; f[3] = u.w;
+  } else {
+    #pragma unroll
+    for (int i = 0; i < VEC; ++i) f[i] = p[i];
+  }
+}
+
+template <int VEC>
+DEV_INLINE void ldv(const bf16_t* p, float* f) {
+  if constexpr (VEC == 4) {
+    const uint2 u = *reinterpret_cast<const uint2*>(p);
+    const float2 a = unpack_bf16x2(u.x), b = unpack_bf16x2(u.y);
+    f[0] = a.x; f[1] = a.y; f[2] = b.x; f[3] = b.y;
+  } else {
+    #pragma unroll
+    for (int i = 0; i < VEC; ++i) f[i] = bf2f(p[i]);
+  }
+}
+
+template <int VEC>
+DEV_INLINE void stv(float* p, const float* f) {
+  if constexpr (VEC == 4) {
+    *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+  } else {
+    #pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = f[i];
+  }
+}
+
+template <int VEC>
+DEV_INLINE void stv(bf16_t* p, const float* f) {
+  if constexpr (VEC == 4) {
+    *reinterpret_cast<uint2*>(p) =
+        make_uint2(pack_bf16x2(f[0], f[1]), pack_bf16x2(f[2], f[3]));
+  } else {
+    #pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = f2bf(f[i]);
+  }
+}
+
+DEV_INLINE float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+
+// ln(sigmoid(z)) without overflow at either end
+DEV_INLINE float log_sigmoid_f(float z) {
+  return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+}
+
+// One request's place in the batch, for kernels over single tokens and over
+// portions of prompts alike: rows [row0, row0 + n) of the packed activations.
+struct Entry {
+  int row0, n;
+};
+
+// seq_start null: entry e is the single row e.
+DEV_INLINE Entry entry_of(const int* seq_start, int e) {
+  if (seq_start == nullptr) return {e, 1};
+  const int a = seq_start[e];
+  return {a, seq_start[e + 1] - a};
+}

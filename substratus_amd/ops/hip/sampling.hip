@@ -12,12 +12,16 @@
 #define SBLOCK 256
 #define SNW (SBLOCK / WAVE)
 
-// LDS budget: V bf16 values (<= 65536 -> 128 KiB) + scratch.
-extern __shared__ unsigned short s_vals[];  // [V] bf16 bits (scaled logits)
+// LDS budget: V values (bf16: <= 65536 -> 128 KiB) + scratch.
+extern __shared__ unsigned char s_raw[];  // [V] logits as they came
 
+DEV_INLINE float val(const bf16_t& v) { return bf2f(v); }
+DEV_INLINE float val(const float& v) { return v; }
+
+template <class T>
 __global__ __launch_bounds__(SBLOCK)
 void softmax_sample_kernel(long* __restrict__ out,          // [B]
-                           const bf16_t* __restrict__ logits,  // [B, V]
+                           const T* __restrict__ logits,  // [B, V]
                            const float* __restrict__ temperature,
                            const int* __restrict__ top_k,
                            const float* __restrict__ top_p,
@@ -26,7 +30,8 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
   __shared__ float s_bcast;
   __shared__ int s_tok;
   const int b = blockIdx.x;
-  const bf16_t* row = logits + (long)b * vocab;
+  T* s_vals = reinterpret_cast<T*>(s_raw);
+  const T* row = logits + (long)b * vocab;
   const float temp = temperature[b];
   const int tid = threadIdx.x;
 
@@ -35,7 +40,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
     float best = -INFINITY;
     int besti = 0;
     for (int i = tid; i < vocab; i += SBLOCK) {
-      float v = bf2f(row[i]);
+      float v = val(row[i]);
       if (v > best || (v == best && i < besti)) { best = v; besti = i; }
     }
     // wave reduce (value, index) preferring smaller index on ties
@@ -59,15 +64,14 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
     return;
   }
 
-  // ---- stage the ORIGINAL bf16 bits into LDS + row max ----------------
+  // ---- stage the ORIGINAL logits into LDS + row max -------------------
   // (temperature is applied in fp32 at every read: staging pre-scaled bf16
   // would re-quantize x/T and shift CDF boundaries vs the fp32 reference)
   const float inv_t = 1.f / temp;
   float mx = -INFINITY;
   for (int i = tid; i < vocab; i += SBLOCK) {
-    bf16_t h = row[i];
-    s_vals[i] = *reinterpret_cast<unsigned short*>(&h);
-    mx = fmaxf(mx, bf2f(h) * inv_t);
+    s_vals[i] = row[i];
+    mx = fmaxf(mx, val(s_vals[i]) * inv_t);
   }
   __syncthreads();
   float m = block_max<SNW>(mx, scratch);
@@ -82,8 +86,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
       float mid = 0.5f * (lo + hi);
       int cnt = 0;
       for (int i = tid; i < vocab; i += SBLOCK) {
-        bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-        if (bf2f(h) * inv_t >= mid) ++cnt;
+        if (val(s_vals[i]) * inv_t >= mid) ++cnt;
       }
       __syncthreads();
       int total = (int)block_sum<SNW>((float)cnt, scratch);
@@ -98,8 +101,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
   // ---- exp-sum over kept values ---------------------------------------
   float zs = 0.f;
   for (int i = tid; i < vocab; i += SBLOCK) {
-    bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-    float v = bf2f(h) * inv_t;
+    float v = val(s_vals[i]) * inv_t;
     if (v >= thresh) zs += __expf(v - m);
   }
   __syncthreads();
@@ -114,8 +116,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
       float mid = 0.5f * (lo + hi);
       float ms = 0.f;
       for (int i = tid; i < vocab; i += SBLOCK) {
-        bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-        float v = bf2f(h) * inv_t;
+        float v = val(s_vals[i]) * inv_t;
         if (v >= mid && v >= thresh) ms += __expf(v - m);
       }
       __syncthreads();
@@ -127,8 +128,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
     // recompute z over the kept set
     float zs2 = 0.f;
     for (int i = tid; i < vocab; i += SBLOCK) {
-      bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-      float v = bf2f(h) * inv_t;
+      float v = val(s_vals[i]) * inv_t;
       if (v >= thresh) zs2 += __expf(v - m);
     }
     __syncthreads();
@@ -143,8 +143,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
   const int beg = tid * chunk, end = min(beg + chunk, vocab);
   float csum = 0.f;
   for (int i = beg; i < end; ++i) {
-    bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-    float v = bf2f(h) * inv_t;
+    float v = val(s_vals[i]) * inv_t;
     if (v >= thresh) csum += __expf(v - m);
   }
   // exclusive prefix over the 256 per-thread sums (via LDS, simple scan)
@@ -162,8 +161,7 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
     float acc = pre[tid];
     int sel = -1;
     for (int i = beg; i < end; ++i) {
-      bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-      float v = bf2f(h) * inv_t;
+      float v = val(s_vals[i]) * inv_t;
       if (v >= thresh) {
         acc += __expf(v - m);
         if (acc > r) { sel = i; break; }
@@ -177,26 +175,39 @@ void softmax_sample_kernel(long* __restrict__ out,          // [B]
     if (sel < 0) {
       // numerical edge (r ~ z): fall back to the last kept token
       for (int i = vocab - 1; i >= 0; --i) {
-        bf16_t h; *reinterpret_cast<unsigned short*>(&h) = s_vals[i];
-        if (bf2f(h) * inv_t >= thresh) { sel = i; break; }
+        if (val(s_vals[i]) * inv_t >= thresh) { sel = i; break; }
       }
     }
     out[b] = sel < 0 ? 0 : sel;
   }
 }
 
+template <class T>
+static void launch(long* out, const T* logits, const float* temperature,
+                   const int* top_k, const float* top_p, const float* uniform,
+                   int bsz, int vocab, hipStream_t stream) {
+  size_t lds = (size_t)vocab * sizeof(T);
+  static size_t max_opted = 0;
+  if (lds > 65536 && lds > max_opted) {  // opt in to >64 KiB dynamic LDS
+    (void)hipFuncSetAttribute(
+        reinterpret_cast<const void*>(&softmax_sample_kernel<T>),
+        hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    max_opted = lds;
+  }
+  softmax_sample_kernel<T><<<dim3(bsz), dim3(SBLOCK), lds, stream>>>(
+      out, logits, temperature, top_k, top_p, uniform, vocab);
+}
+
 void launch_softmax_sample(long* out, const bf16_t* logits,
                            const float* temperature, const int* top_k,
                            const float* top_p, const float* uniform, int bsz,
                            int vocab, hipStream_t stream) {
-  size_t lds = (size_t)vocab * sizeof(unsigned short);
-  static size_t max_opted = 0;
-  if (lds > 65536 && lds > max_opted) {  // opt in to >64 KiB dynamic LDS
-    (void)hipFuncSetAttribute(
-        reinterpret_cast<const void*>(&softmax_sample_kernel),
-        hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    max_opted = lds;
-  }
-  softmax_sample_kernel<<<dim3(bsz), dim3(SBLOCK), lds, stream>>>(
-      out, logits, temperature, top_k, top_p, uniform, vocab);
+  launch(out, logits, temperature, top_k, top_p, uniform, bsz, vocab, stream);
+}
+
+void launch_softmax_sample(long* out, const float* logits,
+                           const float* temperature, const int* top_k,
+                           const float* top_p, const float* uniform, int bsz,
+                           int vocab, hipStream_t stream) {
+  launch(out, logits, temperature, top_k, top_p, uniform, bsz, vocab, stream);
 }

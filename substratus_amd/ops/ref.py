@@ -232,3 +232,92 @@ def adamw_step(param: torch.Tensor, grad: torch.Tensor, exp_avg: torch.Tensor,
     denom = (exp_avg_sq / bc2).sqrt().add_(eps)
     pf.addcdiv_(exp_avg / bc1, denom, value=-lr)
     param.copy_(pf.to(param.dtype))
+
+
+# ---- hybrid models (ops/hybrid.py) ------------------------------------------
+
+def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
+    return x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def stream_norm(delta, x, w_post, w_pre, offset, eps, out_scale=1.0):
+    x += _rms(delta.float(), eps) * (offset + w_post)
+    return (_rms(x, eps) * ((offset + w_pre) * out_scale)).to(delta.dtype)
+
+
+def embed_norm(tokens, table, w_pre, offset, eps):
+    x = table[tokens.long()].float()
+    return x, (_rms(x, eps) * (offset + w_pre)).to(table.dtype)
+
+
+def qkv_prepare(buf, nq, q_norm, k_norm, eps, v_first, lam, k_cache, v_cache,
+                slots):
+    kv, dim, vdim = k_cache.shape[1], k_cache.shape[3], v_cache.shape[3]
+    nk, nv = kv * dim, kv * vdim
+    q, k, v = (t.float() for t in
+               buf[:, :nq + nk + nv].split([nq, nk, nv], dim=1))
+    if q_norm is not None:
+        q, k = _rms(q, eps) * q_norm, _rms(k, eps) * k_norm
+        buf[:, :nq] = q.to(buf.dtype)
+    if v_first is not None:
+        v = (1 - lam) * v + lam * v_first.float()
+    kv_append(k.view(-1, kv, dim), v.view(-1, kv, vdim), k_cache, v_cache,
+              slots)
+
+
+def _entry_rows(seq_start, rows):
+    if seq_start is None:
+        return [(i, i + 1) for i in range(rows)]
+    s = seq_start.tolist()
+    return list(zip(s[:-1], s[1:]))
+
+
+def attn_ctx(out, q, gate, k_cache, v_cache, bias, positions, seq_start,
+             block_table, scale, chunk, max_len, span, any_size):
+    kv, bs, dim = k_cache.shape[1:]
+    vdim = v_cache.shape[3]
+    for e, (a, b) in enumerate(_entry_rows(seq_start, q.shape[0])):
+        pos = positions[a:b].long()
+        n = int(pos[-1]) + 1
+        blocks = block_table[e, :(n + bs - 1) // bs].long()
+        k, v = (c[blocks].transpose(1, 2).reshape(-1, kv, c.shape[3])[:n]
+                .float() for c in (k_cache, v_cache))
+        qe = q[a:b].float().view(b - a, kv, -1, dim)
+        s = torch.einsum("ikgd,jkd->kgij", qe, k) * scale
+        dist = pos[:, None] - torch.arange(n, device=pos.device)
+        if bias is not None:
+            s = s + bias[:, dist.clamp(0, bias.shape[1] - 1)].view(
+                kv, -1, b - a, n)
+        seen = dist >= 0
+        if chunk:
+            seen &= (pos // chunk)[:, None] == torch.arange(
+                n, device=pos.device) // chunk
+        p = torch.softmax(s.masked_fill(~seen, float("-inf")), -1)
+        o = torch.einsum("kgij,jkd->ikgd", p, v).reshape(b - a, -1, vdim)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[a:b].float())[:, :, None]
+        out[a:b] = o.reshape(b - a, -1).to(out.dtype)
+
+
+def gla(out, x, a2, a2_bias, norm, state, state_slots, positions, seq_start,
+        inv_tau, eps, max_len, recurrent):
+    _, heads, dim, vdim = state.shape
+    f = x.float()
+    q, k, v, g, a1 = f[:, :2 * heads * (dim + vdim) + a2.shape[1]].split(
+        [heads * dim] * 2 + [heads * vdim] * 2 + [a2.shape[1]], dim=1)
+    alpha = torch.exp(torch.nn.functional.logsigmoid(a1 @ a2.T + a2_bias)
+                      * inv_tau).view(-1, heads, dim, 1)
+    q = q.view(-1, heads, dim, 1) * dim ** -0.5
+    k = k.view(-1, heads, dim, 1)
+    v = v.view(-1, heads, 1, vdim)
+    for e, (a, b) in enumerate(_entry_rows(seq_start, x.shape[0])):
+        slot = int(state_slots[e])
+        s = torch.zeros(heads, dim, vdim, device=x.device) \
+            if slot < 0 or int(positions[a]) == 0 else state[slot]
+        for t in range(a, b):
+            s = alpha[t] * s + k[t] * v[t]
+            o = _rms((s * q[t]).sum(1), eps) * norm
+            out[t] = (o.reshape(-1) * torch.nn.functional.silu(g[t])).to(
+                out.dtype)
+        if slot >= 0:
+            state[slot] = s

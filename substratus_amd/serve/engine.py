@@ -11,6 +11,11 @@ slots are available (prefilling them in one packed varlen batch), then runs
 one decode step for every running sequence. Preemption: when the allocator
 runs out of blocks mid-decode, the youngest sequence is evicted back to the
 wait queue (its blocks freed, prompt re-prefilled later).
+
+Models that take portions (models/hybrid.py) are scheduled by tokens instead:
+a step is one batch of single decoded tokens beside portions of prompts, up to
+prefill_chunk tokens, run by execute() on the paged cache and the recurrent
+state. When nothing is left to prefill the step is the same captured decode.
 """
 
 from __future__ import annotations
@@ -23,9 +28,10 @@ from typing import Optional
 import torch
 
 from .. import ops
+from ..models import CausalLM, HybridLM, build_model
 from ..models.config import ModelConfig, get_config
-from ..models.model import CausalLM
 from ..parallel.comm import state
+from .batch import StepBatch
 from .kv_cache import (DEFAULT_BLOCK_SIZE, BlockAllocator, OutOfBlocks,
                        PagedKVCache, SequenceState)
 
@@ -71,7 +77,7 @@ class StepOutput:
 
 class Engine:
     def __init__(self, cfg: EngineConfig, device: Optional[str] = None,
-                 model: Optional[CausalLM] = None):
+                 model: Optional[CausalLM | HybridLM] = None):
         self.cfg = cfg
         self.mcfg: ModelConfig = get_config(cfg.model)
         if device is None:
@@ -82,9 +88,12 @@ class Engine:
             load_tunables()     # pre-tuned GEMM solutions (no-op sans table)
         if model is None:
             with torch.no_grad():
-                model = CausalLM(self.mcfg, device="meta", dtype=cfg.dtype)
+                model = build_model(self.mcfg, device="meta", dtype=cfg.dtype)
                 model = model.to_empty(device=self.device)
                 model.init_random(cfg.seed)
+        if self.mcfg.layers and (cfg.quant or cfg.kv_dtype):
+            raise ValueError(f"{self.mcfg.family} models are served with "
+                             "plain weights and caches, not quantized ones")
         if cfg.quant:
             from ..models.quant import quantize_model
             from ..parallel.comm import state as _pstate
@@ -92,6 +101,7 @@ class Engine:
                 "quantized serving is single-rank for now"
             quantize_model(model, cfg.quant)
         self.model = model.eval()
+        self.takes_portions = getattr(self.model, "takes_portions", False)
         n_kv_local = self.model.n_kv_heads
         kv_dtype = cfg.dtype
         if cfg.kv_dtype == "fp8":
@@ -99,12 +109,13 @@ class Engine:
             kv_dtype = torch.float8_e4m3fn
         elif cfg.kv_dtype is not None:
             raise ValueError(f"unknown kv_dtype {cfg.kv_dtype!r}")
-        kv_bytes_per_el = 1 if kv_dtype == torch.float8_e4m3fn else 2
+        kv_bytes_per_el = kv_dtype.itemsize
         if cfg.kv_blocks is not None:
             num_blocks = cfg.kv_blocks
         elif self.device.type == "cuda":
             free, _total = torch.cuda.mem_get_info(self.device)
             budget = int(free * cfg.gpu_mem_fraction)
+            budget -= PagedKVCache.state_bytes(self.mcfg, cfg.max_batch)
             num_blocks = PagedKVCache.blocks_for_memory(
                 self.mcfg, n_kv_local, budget, cfg.block_size,
                 dtype_bytes=kv_bytes_per_el)
@@ -128,7 +139,7 @@ class Engine:
                 (cfg.max_seq_len + cfg.block_size - 1) // cfg.block_size)
         self.kv = PagedKVCache(self.mcfg, n_kv_local, num_blocks,
                                cfg.block_size, device=self.device,
-                               dtype=kv_dtype)
+                               dtype=kv_dtype, state_slots=cfg.max_batch)
         self.max_blocks_per_seq = (cfg.max_seq_len + cfg.block_size - 1) // cfg.block_size
         self._next_id = itertools.count()
         self.waiting: list[SequenceState] = []
@@ -167,7 +178,7 @@ class Engine:
         while self.waiting and len(self.running) + len(admitted) < self.cfg.max_batch:
             seq = self.waiting[0]
             nblk = seq.needed_blocks(self.cfg.block_size, extra_tokens=1)
-            if admitted and seq.length > budget:
+            if admitted and seq.length > budget and not self.takes_portions:
                 # budget gates only the 2nd+ admission: a prompt longer than
                 # prefill_chunk must still go through alone or it would
                 # never be admitted (livelock)
@@ -184,7 +195,7 @@ class Engine:
                 continue
             if self.kv.allocator.free_count < nblk + 2 * len(self.running):
                 break  # keep headroom for running seqs to grow
-            seq.blocks = self.kv.allocator.alloc(nblk)
+            self.kv.reserve(seq, seq.length + 1)
             admitted.append(self.waiting.pop(0))
             budget -= seq.length
         return admitted
@@ -192,12 +203,71 @@ class Engine:
     def _preempt_youngest(self) -> None:
         assert self.running, "out of KV blocks with nothing to preempt"
         seq = self.running.pop()  # youngest = most recently admitted
-        self.kv.allocator.free(seq.blocks)
-        seq.blocks = []
+        self.kv.release(seq)
         # keep generated tokens: readmission re-prefills the whole token list
         # (prompt + generated so far). num_prompt stays at the true prompt
         # length so the max_new_tokens budget is not reset by preemption.
         self.waiting.insert(0, seq)
+
+    # -------------------------------------------------------------- portions
+    def execute(self, entries: list[tuple[SequenceState, int, list[int]]]
+                ) -> torch.Tensor:
+        """Run the next n tokens of every (sequence, n, wanted offsets) as one
+        batch, from the cache and state that earlier steps left; their room
+        must be reserved. Returns the wanted logits, entries in order."""
+        batch = StepBatch.build(
+            [(s.tokens[s.num_computed:s.num_computed + n], s.num_computed,
+              s.blocks, s.state_slot, want) for s, n, want in entries],
+            self.cfg.block_size, self.device)
+        with torch.no_grad():
+            logits = self.model.forward_step(batch, self.kv.layers)
+        for s, n, _ in entries:
+            s.num_computed += n
+        return logits
+
+    def _plan(self) -> list[tuple[SequenceState, int, list[int]]]:
+        """This step's tokens: one for every sequence that decodes, the rest
+        of the prefill_chunk tokens to prompts in order of admission."""
+        budget = self.cfg.prefill_chunk - sum(
+            s.length - s.num_computed == 1 for s in self.running)
+        plan = []
+        for s in self.running:
+            left = s.length - s.num_computed
+            n = left if left == 1 else min(left, budget)
+            if n <= 0:
+                continue
+            if left > 1:
+                budget -= n
+            plan.append((s, n, [n - 1] if n == left else []))
+        if not plan:    # a chunk smaller than the batch still moves on
+            s = self.running[0]
+            plan.append((s, 1, []))
+        return plan
+
+    def _step_portions(self) -> list[StepOutput]:
+        out: list[StepOutput] = []
+        self.running.extend(self._try_admit(out))
+        while self.running:
+            plan = self._plan()
+            try:
+                for s, n, _ in plan:
+                    self.kv.reserve(s, s.num_computed + n)
+            except OutOfBlocks:
+                self._preempt_youngest()
+                continue
+            if all(s.length - s.num_computed == 1 for s in self.running):
+                res = self._decode()
+            else:
+                if self.graph_runner is not None:
+                    self.graph_runner.invalidate()
+                logits = self.execute(plan)
+                done = [s for s, _, want in plan if want]
+                res = self._emit(done, logits) if done else []
+            out.extend(res)
+            self._retire(self.running, res)
+            self.steps += 1
+            break
+        return out
 
     # --------------------------------------------------------------- prefill
     def _prefill(self, seqs: list[SequenceState]) -> list[StepOutput]:
@@ -236,8 +306,12 @@ class Engine:
         (not the engine's CPU generator)."""
         from .kv_cache import OutOfBlocks
         from .graph_runner import GraphDecodeRunner
-        if self.graph_runner is None:
-            self.graph_runner = GraphDecodeRunner(self)
+        try:
+            if self.graph_runner is None:
+                self.graph_runner = GraphDecodeRunner(self)
+        except OutOfBlocks:     # no page left for padded lanes
+            self._preempt_youngest()
+            return self._decode() if self.running else []
         runner = self.graph_runner
         ids = [s.seq_id for s in self.running]
         try:
@@ -251,6 +325,7 @@ class Engine:
         out = []
         for seq, tok in zip(self.running, toks):
             self.tokens_generated += 1
+            seq.num_computed = seq.length - 1
             done = (seq.num_generated >= seq.max_new_tokens or
                     (seq.eos_token >= 0 and tok == seq.eos_token) or
                     seq.length >= self.cfg.max_seq_len)
@@ -275,6 +350,8 @@ class Engine:
                 except OutOfBlocks:
                     self._preempt_youngest()
                     return self._decode() if self.running else []
+        if self.takes_portions:
+            return self._emit(seqs, self.execute([(s, 1, [0]) for s in seqs]))
         tokens = torch.tensor([s.tokens[-1] for s in seqs], dtype=torch.int64,
                               device=dev)
         positions = torch.tensor([s.length - 1 for s in seqs],
@@ -320,7 +397,10 @@ class Engine:
 
     # ----------------------------------------------------------------- step
     def step(self) -> list[StepOutput]:
-        """One engine iteration: admit+prefill, then decode everyone running."""
+        """One engine iteration: admit+prefill, then decode everyone running
+        (for models that take portions: both as one batch)."""
+        if self.takes_portions:
+            return self._step_portions()
         out: list[StepOutput] = []
         admitted = self._try_admit(out)
         if admitted:
@@ -352,15 +432,11 @@ class Engine:
         for i, s in enumerate(self.waiting):
             if s.seq_id == seq_id:
                 del self.waiting[i]
-                if s.blocks:        # waiting seqs hold none today (fresh
-                    self.kv.allocator.free(s.blocks)   # and preempted both
-                    s.blocks = []                      # freed) — stay safe
+                self.kv.release(s)   # waiting seqs hold nothing — stay safe
                 return True
         for s in self.running:
             if s.seq_id == seq_id:
-                if s.blocks:
-                    self.kv.allocator.free(s.blocks)
-                    s.blocks = []
+                self.kv.release(s)
                 self.running = [r for r in self.running
                                 if r.seq_id != seq_id]
                 return True
@@ -372,9 +448,7 @@ class Engine:
         followers can apply it independently and stay lockstep."""
         self.waiting.clear()
         for s in self.running:
-            if s.blocks:
-                self.kv.allocator.free(s.blocks)
-                s.blocks = []
+            self.kv.release(s)
         self.running.clear()
         if self.graph_runner is not None:
             self.graph_runner.invalidate()
@@ -384,6 +458,5 @@ class Engine:
         if not finished:
             return
         for seq in [s for s in pool if s.seq_id in finished and s.blocks]:
-            self.kv.allocator.free(seq.blocks)
-            seq.blocks = []
+            self.kv.release(seq)
         self.running = [s for s in self.running if s.seq_id not in finished]

@@ -58,6 +58,8 @@ class GraphDecodeRunner:
         self.seq_lens = torch.ones(B, dtype=torch.int32, device=dev)
         self.slots = torch.zeros(B, dtype=torch.int32, device=dev)
         self.block_table = torch.zeros(B, maxb, dtype=torch.int32, device=dev)
+        # recurrent state: -1 on padded lanes, which then touch none
+        self.state_slots = torch.full((B,), -1, dtype=torch.int32, device=dev)
         self.temp = torch.zeros(B, dtype=torch.float32, device=dev)
         self.top_k = torch.zeros(B, dtype=torch.int32, device=dev)
         self.top_p = torch.ones(B, dtype=torch.float32, device=dev)
@@ -104,6 +106,8 @@ class GraphDecodeRunner:
         self.seq_lens[:b] = torch.tensor(lens, dtype=torch.int32)
         self.slots[:b] = torch.tensor(slots, dtype=torch.int32)
         self.block_table[:b] = bt.to(self.device)
+        self.state_slots[:b] = torch.tensor(
+            [s.state_slot for s in seqs] + [-1] * (b - n), dtype=torch.int32)
         self.temp[:b] = torch.tensor(
             [s.temperature for s in seqs] + [0.0] * (b - n))
         self.top_k[:b] = torch.tensor(
@@ -115,9 +119,10 @@ class GraphDecodeRunner:
     # ------------------------------------------------------------- capture
     def _decode_gen(self, lo: int, hi: int):
         sl = slice(lo, hi)
+        state = (self.state_slots[sl],) if self.eng.takes_portions else ()
         return self.model.decode_ops(
             self.tokens[sl], self.positions[sl], self.eng.kv.layers,
-            self.slots[sl], self.block_table[sl], self.seq_lens[sl])
+            self.slots[sl], self.block_table[sl], self.seq_lens[sl], *state)
 
     def _step_body(self, b: int) -> None:
         # Op-skewed dual-stream decode: split the batch in half and
@@ -192,7 +197,10 @@ class GraphDecodeRunner:
         # and restore the small state. The scribbled KV positions are always
         # rewritten by rope_kv_append before attention ever reads them (a
         # position's KV is written in the same step that first includes it),
-        # so the cache needs no restore.
+        # so the cache needs no restore. Recurrent state is not rewritten: the
+        # warmup runs with every lane padded, which leaves the slots alone.
+        slots = self.state_slots.clone()
+        self.state_slots.fill_(-1)
         saved = [t.clone() for t in (self.tokens, self.positions,
                                      self.seq_lens, self.slots)]
         s = torch.cuda.Stream()
@@ -219,6 +227,7 @@ class GraphDecodeRunner:
         for dst, src in zip((self.tokens, self.positions, self.seq_lens,
                              self.slots), saved):
             dst.copy_(src)
+        self.state_slots.copy_(slots)
         torch.cuda.synchronize()
         self.graphs[b] = g
         return g

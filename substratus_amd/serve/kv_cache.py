@@ -4,6 +4,10 @@ Layout per layer: k_cache/v_cache of shape [num_blocks, n_kv_heads, block_size,
 head_dim] — one block's K rows for one head are a contiguous
 block_size × head_dim panel (16×128 bf16 = 4 KiB), the unit the decode
 attention kernel streams through LDS/registers with wide coalesced loads.
+
+Models of unlike layers (ModelConfig.layers) keep per layer what its mixer
+asks for: pages with its own head sizes, or a 32-bit recurrent state for each
+of `state_slots` requests. A layer's entry in `layers` is (k, v) or (state,).
 """
 
 from __future__ import annotations
@@ -39,31 +43,104 @@ class BlockAllocator:
         self._free.extend(blocks)
 
 
+class OutOfSlots(RuntimeError):
+    pass
+
+
+class SlotAllocator:
+    """State slots, one per live request. A slot holds whatever its last
+    owner left: kernels start from zero at a request's position 0."""
+
+    def __init__(self, num_slots: int):
+        self.num_slots = num_slots
+        self._free = list(range(num_slots - 1, -1, -1))
+
+    @property
+    def free_count(self) -> int:
+        return len(self._free)
+
+    def alloc(self) -> int:
+        if not self._free:
+            raise OutOfSlots(f"all {self.num_slots} state slots are taken")
+        return self._free.pop()
+
+    def free(self, slot: int) -> None:
+        self._free.append(slot)
+
+
 class PagedKVCache:
-    """Per-rank paged KV cache for every layer of one model."""
+    """Per-rank cache and state manager for every layer of one model."""
 
     def __init__(self, cfg: ModelConfig, n_kv_heads_local: int, num_blocks: int,
                  block_size: int = DEFAULT_BLOCK_SIZE, device="cpu",
-                 dtype=torch.bfloat16):
+                 dtype=torch.bfloat16, state_slots: int = 0):
         self.cfg = cfg
         self.block_size = block_size
         self.num_blocks = num_blocks
-        self.layers: list[tuple[torch.Tensor, torch.Tensor]] = []
-        for _ in range(cfg.num_layers):
+        self.layers: list[tuple[torch.Tensor, ...]] = []
+        self.slots = SlotAllocator(
+            state_slots if any(s.mixer.state_bytes() for s in cfg.layers)
+            else 0)
+        for spec in cfg.layers:
+            m = spec.mixer
+            if m.state_bytes():
+                self.layers.append((torch.zeros(
+                    state_slots, m.heads, m.dim, m.vdim, device=device,
+                    dtype=torch.float32),))
+            else:
+                self.layers.append(tuple(
+                    torch.zeros(num_blocks, m.kv_heads, block_size, d,
+                                device=device, dtype=dtype)
+                    for d in (m.dim, m.vdim)))
+        for _ in range(0 if cfg.layers else cfg.num_layers):
             k = torch.zeros(num_blocks, n_kv_heads_local, block_size,
                             cfg.head_dim, device=device, dtype=dtype)
             v = torch.zeros_like(k)
             self.layers.append((k, v))
         self.allocator = BlockAllocator(num_blocks)
 
+    def reserve(self, seq: "SequenceState", tokens: int) -> None:
+        """Pages for the sequence's first `tokens` tokens and, if the model
+        has recurrent layers, a state slot; all of it or OutOfBlocks /
+        OutOfSlots and nothing."""
+        need = (tokens + self.block_size - 1) // self.block_size
+        need -= len(seq.blocks)
+        if need > self.allocator.free_count:
+            raise OutOfBlocks(f"need {need} KV blocks, "
+                              f"{self.allocator.free_count} free")
+        if seq.state_slot < 0 and self.slots.num_slots:
+            seq.state_slot = self.slots.alloc()
+        if need > 0:
+            seq.blocks.extend(self.allocator.alloc(need))
+
+    def release(self, seq: "SequenceState") -> None:
+        """Give back everything the sequence holds; what it had computed is
+        lost with it."""
+        if seq.blocks:
+            self.allocator.free(seq.blocks)
+            seq.blocks = []
+        if seq.state_slot >= 0:
+            self.slots.free(seq.state_slot)
+            seq.state_slot = -1
+        seq.num_computed = 0
+
+    @staticmethod
+    def state_bytes(cfg: ModelConfig, state_slots: int) -> int:
+        return state_slots * sum(s.mixer.state_bytes() for s in cfg.layers)
+
     @staticmethod
     def blocks_for_memory(cfg: ModelConfig, n_kv_heads_local: int,
                           bytes_budget: int,
                           block_size: int = DEFAULT_BLOCK_SIZE,
                           dtype_bytes: int = 2) -> int:
-        per_block = (2 * cfg.num_layers * n_kv_heads_local * block_size *
-                     cfg.head_dim * dtype_bytes)
-        return max(bytes_budget // per_block, 1)
+        if cfg.layers:
+            per_block = block_size * sum(s.mixer.kv_bytes(dtype_bytes)
+                                         for s in cfg.layers)
+        else:
+            per_block = (2 * cfg.num_layers * n_kv_heads_local * block_size *
+                         cfg.head_dim * dtype_bytes)
+        # no attention layer: pages are numbers in a block table only
+        return max(bytes_budget // max(per_block, 1), 1)
 
 
 @dataclass(slots=True)
@@ -80,6 +157,8 @@ class SequenceState:
     batch_slot: int = -1            # position in the decode batch
     finished: bool = False
     eos_token: int = -1
+    state_slot: int = -1            # recurrent state, -1: holds none
+    num_computed: int = 0           # tokens already in the cache and state
 
     @property
     def length(self) -> int:

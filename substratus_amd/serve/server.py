@@ -49,7 +49,9 @@ def resolve_model_name(params: dict, model_dir: str | None = None) -> str:
     cfg_path = os.path.join(model_dir, "config.json")
     if os.path.exists(cfg_path):
         with open(cfg_path) as f:
-            return json.load(f)["model"]
+            doc = json.load(f)
+        # a folder that spells its architecture out is its own model name
+        return model_dir if "architecture" in doc else doc["model"]
     return params.get("name", params.get("model", "llama2-7b"))
 
 
@@ -222,7 +224,7 @@ def create_app(engine: Optional[Engine] = None,
     app.state.worker = worker
     app.state.engine = engine
     vocab = engine.mcfg.vocab_size
-    model_id = engine.cfg.model
+    model_id = engine.mcfg.name
     # real tokenizer.json from the artifacts when present (loader exports
     # one), byte-level fallback otherwise
     tok_obj = tokenizer_mod.load(os.environ.get("MODEL_DIR",
@@ -511,38 +513,9 @@ def _find_gguf(model_dir: str | None = None) -> Optional[str]:
 def _maybe_load_weights(engine: Engine,
                         model_dir: str | None = None) -> None:
     model_dir = model_dir or os.environ.get("MODEL_DIR", "/content/model")
-    path = os.path.join(model_dir, "model.safetensors")
-    if not os.path.exists(path):
-        # search newest checkpoint (trainer artifacts layout)
-        if os.path.isdir(model_dir):
-            ckpts = sorted((d for d in os.listdir(model_dir)
-                            if d.startswith("checkpoint-")),
-                           key=lambda d: int(d.split("-")[1]))
-            if ckpts:
-                path = os.path.join(model_dir, ckpts[-1], "model.safetensors")
-    if os.path.exists(path):
-        from safetensors.torch import load_file
-        from ..models.hf_compat import (hf_falcon_to_native,
-                                        hf_llama_to_native,
-                                        hf_opt_to_native,
-                                        is_hf_falcon_state_dict,
-                                        is_hf_llama_state_dict,
-                                        is_hf_opt_state_dict)
-        from ..parallel.comm import state as pstate
-        sd = load_file(path)
-        if is_hf_llama_state_dict(sd):
-            # HF-layout checkpoint (meta-llama/Llama-2-* naming)
-            sd = hf_llama_to_native(sd, engine.mcfg)
-        elif is_hf_falcon_state_dict(sd):
-            sd = hf_falcon_to_native(sd, engine.mcfg)
-        elif is_hf_opt_state_dict(sd):
-            sd = hf_opt_to_native(sd, engine.mcfg)
-        st = pstate()
-        if st.tp_size > 1:
-            from ..models.sharding import shard_state_dict
-            sd = shard_state_dict(sd, engine.mcfg, st.tp_rank, st.tp_size)
-        engine.model.load_state_dict(
-            {k: v.to(engine.device, engine.cfg.dtype) for k, v in sd.items()})
+    from ..models.weights import load_weights
+    load_weights(engine.model, engine.mcfg, model_dir, engine.device,
+                 engine.cfg.dtype)
 
 
 def main() -> None:

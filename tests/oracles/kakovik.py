@@ -33,18 +33,13 @@ def silu(z):
 def distance_bucket(n, rows, furthest):
     """Row of the relative-distance table for distance n: one row per distance
     over the first half, then rows at equal steps of ln n up to `furthest`.
-
-    Row half+k starts at the smallest n with n/half >= (furthest/half)^(k/rest);
-    compared as integers, so that no logarithm is rounded at a row's start.
+    (The small number keeps a distance exactly at a row's start in that row.)
     """
     half = rows // 2
     if n < half:
         return n
-    rest = rows - half
-    k = 0
-    while k < rest and n ** rest * half ** (k + 1) >= furthest ** (k + 1) * half ** rest:
-        k += 1
-    return min(rows - 1, half + k)
+    steps = math.log(n / half) / math.log(furthest / half) * (rows - half)
+    return min(rows - 1, half + math.floor(steps + 1e-9))
 
 
 def distance_bias(rel, n_max, furthest):
