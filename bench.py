@@ -34,7 +34,9 @@ def parse_args():
     p.add_argument("--gpus", type=int, default=1)
     p.add_argument("--steps", type=int, default=64)
     p.add_argument("--warmup", type=int, default=16)
-    p.add_argument("--mode", choices=["serve", "train"], default="serve")
+    p.add_argument("--mode", choices=["serve", "train", "hybrid"], default="serve",
+                   help="hybrid: prefill and decode of hybrid-layer models "
+                        "beside the uniform model of equal size")
     p.add_argument("--model", default=None, help="override model config")
     p.add_argument("--batch", type=int, default=512)
     p.add_argument("--prompt-len", type=int, default=512)
@@ -143,7 +145,7 @@ def bench_serve(args) -> None:
     t_pref = time.time()
     t_first = None
     stuck = 0
-    while eng.waiting:
+    while eng.prefilling():
         n_wait = len(eng.waiting)
         outs = eng.step()
         # a too-small KV pool can preempt-admit-preempt forever: fail
@@ -234,10 +236,102 @@ def bench_train(args) -> None:
     run_train_bench(args)
 
 
+# hybrid-layer model, the uniform model of equal width, depth and feed-forward,
+# and (batch, prompt length) points
+HYBRID_PAIRS = [
+    ("kakovik-1b", "llama-1b", [(8, 512), (64, 512), (256, 512), (16, 3072)]),
+    ("kakovik-7b", "llama2-7b", [(8, 512), (64, 512), (256, 512),
+                                 (16, 3072)]),
+]
+HYBRID_TINY = [("kakovik-tiny", "llama-tiny", [(2, 24)])]
+
+
+def bench_hybrid(args) -> None:
+    """Prefill and decode tokens/s on one device, random weights: every model
+    of a pair at the same points. The first prefill of a point warms up."""
+    from substratus_amd.serve.engine import Engine, EngineConfig
+    on_gpu = torch.cuda.is_available()
+    device = "cuda:0" if on_gpu else "cpu"
+    pairs = HYBRID_PAIRS if on_gpu else HYBRID_TINY
+    if args.model:
+        pairs = [p for p in HYBRID_PAIRS + HYBRID_TINY if args.model in p[:2]]
+
+    def sync():
+        if on_gpu:
+            torch.cuda.synchronize()
+
+    def point(eng, batch, prompt_len):
+        g = torch.Generator().manual_seed(7)
+        for attempt in range(2):
+            for _ in range(batch):
+                eng.add_request(
+                    torch.randint(0, eng.mcfg.vocab_size, (prompt_len,),
+                                  generator=g).tolist(),
+                    max_new_tokens=args.warmup + args.steps + 32)
+            sync()
+            t0 = time.time()
+            while eng.prefilling():
+                eng.step()
+            sync()
+            prefill = time.time() - t0
+            if attempt == 0:
+                eng.abort_all()
+        for _ in range(args.warmup):
+            eng.decode_only_step()
+        sync()
+        t0 = time.time()
+        for _ in range(args.steps):
+            eng.decode_only_step()
+        sync()
+        decode = time.time() - t0
+        assert len(eng.running) == batch
+        eng.abort_all()
+        return batch * prompt_len / prefill, batch * args.steps / decode
+
+    rows = []
+    for pair in pairs:
+        for model in pair[:2]:
+            points = pair[2]
+            max_seq = max(p for _, p in points) + args.warmup + args.steps + 64
+            blocks = max(b * ((p + args.warmup + args.steps + 64) // 16 + 1)
+                         for b, p in points)
+            # prefill_chunk bounds a step's prompt tokens for both
+            eng = Engine(EngineConfig(
+                model=model, dtype=torch.bfloat16 if on_gpu else torch.float32,
+                max_batch=max(b for b, _ in points), max_seq_len=max_seq,
+                kv_blocks=blocks + 1, prefill_chunk=16384), device=device)
+            for batch, prompt_len in points:
+                pre, dec = point(eng, batch, prompt_len)
+                rows.append({"model": model, "batch": batch,
+                             "prompt_len": prompt_len,
+                             "prefill_tokens_per_s": round(pre),
+                             "decode_tokens_per_s": round(dec),
+                             "decode_ms_per_step": round(batch / dec * 1e3,
+                                                         3)})
+                log(f"[bench] {rows[-1]}")
+            del eng
+            if on_gpu:
+                torch.cuda.empty_cache()
+    best = max((r for r in rows if r["model"] == pairs[-1][0]),
+               key=lambda r: r["decode_tokens_per_s"])
+    print(json.dumps({
+        "metric": "hybrid_decode_tokens_per_s",
+        "value": best["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+        "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": best["decode_ms_per_step"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16" if on_gpu else "fp32", "data": "synthetic",
+        "config": {"model": best["model"], "global_batch": best["batch"],
+                   "seq_len": best["prompt_len"] + args.warmup + args.steps,
+                   "parallelism": "dp1", "points": rows}}), flush=True)
+
+
 def main() -> None:
     args = parse_args()
     if args.mode == "serve":
         bench_serve(args)
+    elif args.mode == "hybrid":
+        bench_hybrid(args)
     else:
         bench_train(args)
 

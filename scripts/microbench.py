@@ -66,6 +66,137 @@ def bench_norm(B=64, h=4096):
     print(f"rms_norm_residual B={B} h={h}: {dt*1e6:.1f} us")
 
 
+HBM = 8.0e12          # bytes/s
+MFMA = 2.5e15         # dense bf16 flop/s
+
+
+def report(name, dt, nbytes, flops=0.0):
+    """Time beside the roofline: the larger of the HBM and matrix-core times
+    of the work the op cannot avoid."""
+    ideal = max(nbytes / HBM, flops / MFMA)
+    print(f"{name:58s} {dt*1e6:9.1f} us  {nbytes/dt/1e12:5.2f} TB/s "
+          f"{flops/dt/1e12:6.0f} TF/s  {100*ideal/dt:5.1f}% of roofline",
+          flush=True)
+
+
+def bench_hybrid():
+    """Kernels of hybrid-layer models beside the like kernels of the uniform
+    families, at equal sizes."""
+    from substratus_amd.ops import hybrid as hy
+    from substratus_amd.serve.batch import StepBatch
+    torch.manual_seed(0)
+    bf = dict(device="cuda", dtype=torch.bfloat16)
+
+    def batch_of(n, first, tokens):
+        need = (first + tokens + 15) // 16
+        return StepBatch.build(
+            [([1] * tokens, first, list(range(i * need, (i + 1) * need)), i,
+              []) for i in range(n)], 16, torch.device("cuda"))
+
+    for rows, w in ((64, 4096), (256, 4096), (16384, 4096)):
+        x = torch.randn(rows, w, **bf)
+        r = torch.randn(rows, w, **bf)
+        wt = torch.randn(w, **bf)
+        it = 200 if rows < 1000 else 50
+        report(f"rms_norm_residual rows={rows} w={w}",
+               timeit(lambda: ops.rms_norm_residual(x, r, wt, 1e-5), it),
+               rows * w * 8)
+        xf = torch.randn(rows, w, device="cuda")
+        w32 = torch.randn(w, device="cuda")
+        report(f"  stream_norm rows={rows} w={w}",
+               timeit(lambda: hy.stream_norm(x, xf, w32, w32, 1.0, 1e-5), it),
+               rows * w * 12)
+
+    h, d = 32, 128
+    for rows in (64, 256, 16384):
+        nb = (rows + 15) // 16
+        buf = torch.randn(rows, 3 * h * d + 32, **bf)
+        kc = torch.zeros(nb, h, 16, d, **bf)
+        vc = torch.zeros_like(kc)
+        pos = torch.arange(rows, device="cuda", dtype=torch.int32)
+        q, k, v = (buf[:, i * h * d:(i + 1) * h * d].view(rows, h, d)
+                   for i in range(3))
+        it = 200 if rows < 1000 else 50
+        report(f"rope_kv_append rows={rows} {h}x{d}",
+               timeit(lambda: ops.rope_kv_append(q, k, v, pos, kc, vc, pos,
+                                                 1e4), it),
+               rows * h * d * 2 * 7)
+        w32 = torch.ones(h * d, device="cuda")
+        vf = torch.randn(rows, h * d, **bf)
+        lam = torch.tensor(0.5, device="cuda")
+        report(f"  qkv_prepare rows={rows} {h}x{d}",
+               timeit(lambda: hy.qkv_prepare(buf, h * d, w32, w32, 1e-5, vf,
+                                             lam, kc, vc, pos), it),
+               rows * h * d * 2 * 7)
+        del buf, kc, vc, q, k, v, vf
+
+    bias = torch.randn(h, 4096, device="cuda")
+    for b, ctx, hq, hkv in ((8, 512, 32, 32), (64, 512, 32, 32),
+                            (256, 512, 32, 32), (64, 2048, 32, 32),
+                            (64, 2048, 32, 8)):
+        nb = b * ctx // 16
+        kc = torch.randn(nb, hkv, 16, d, **bf)
+        vc = torch.randn_like(kc)
+        q = torch.randn(b, hq * d, **bf)
+        bt = torch.arange(nb, device="cuda", dtype=torch.int32).view(b, -1)
+        lens = torch.full((b,), ctx, device="cuda", dtype=torch.int32)
+        nbytes = 2 * b * ctx * hkv * d * 2
+        it = 100
+        report(f"paged_attn_decode b={b} ctx={ctx} {hq}/{hkv}x{d}",
+               timeit(lambda: ops.paged_attn_decode(
+                   q.view(b, hq, d), kc, vc, bt, lens, d ** -0.5), it),
+               nbytes)
+        sb = batch_of(b, ctx - 1, 1)
+        gate = torch.randn(b, hq, **bf)
+        report(f"  attn_ctx single b={b} ctx={ctx} {hq}/{hkv}x{d}",
+               timeit(lambda: hy.attn_ctx(q, gate, kc, vc, bias, sb,
+                                          d ** -0.5, 4096), it), nbytes)
+        del kc, vc
+
+    for b, s_ in ((32, 512), (8, 2048), (4, 4096)):
+        t = b * s_
+        q, k, v = (torch.randn(t, h, d, **bf) for _ in range(3))
+        ss = torch.arange(0, t + 1, s_, dtype=torch.int32, device="cuda")
+        flops = 4.0 * b * h * (s_ * (s_ + 1) / 2) * d
+        nbytes = 4 * t * h * d * 2
+        report(f"attn_v5 b={b} s={s_} {h}x{d}",
+               timeit(lambda: ops.attn_prefill(q, k, v, ss, d ** -0.5), 20),
+               nbytes, flops)
+        sb = batch_of(b, 0, s_)
+        kc = torch.randn(t // 16, h, 16, d, **bf)
+        vc = torch.randn_like(kc)
+        gate = torch.randn(t, h, **bf)
+        q2 = q.view(t, h * d)
+        report(f"  attn_ctx portions b={b} s={s_} {h}x{d}",
+               timeit(lambda: hy.attn_ctx(q2, gate, kc, vc, bias, sb,
+                                          d ** -0.5, 4096), 20),
+               nbytes, flops)
+        del q, k, v, kc, vc
+
+    gh, gd, gv, r = 16, 128, 256, 16
+    a2 = torch.randn(gh * gd, r, device="cuda") * 0.25
+    ab = torch.randn(gh * gd, device="cuda")
+    nw = torch.ones(gv, device="cuda")
+    ld = 2 * gh * (gd + gv) + r
+    for b in (8, 64, 256):
+        state = torch.zeros(b, gh, gd, gv, device="cuda")
+        x = torch.randn(b, ld, **bf)
+        sb = batch_of(b, 100, 1)
+        report(f"  gla single b={b} {gh}x{gd}x{gv}",
+               timeit(lambda: hy.gla(x, a2, ab, nw, state, sb, 16.0, 1e-5),
+                      100), state.numel() * 8 + x.numel() * 2)
+    for b, s_ in ((32, 512), (8, 2048), (1, 8192)):
+        t = b * s_
+        state = torch.zeros(b, gh, gd, gv, device="cuda")
+        x = torch.randn(t, ld, **bf)
+        sb = batch_of(b, 0, s_)
+        # two state products and, within chunks of 32, two score products
+        flops = t * gh * (4.0 * gd * gv + 32.0 * (gd + gv))
+        report(f"  gla portions b={b} s={s_} {gh}x{gd}x{gv}",
+               timeit(lambda: hy.gla(x, a2, ab, nw, state, sb, 16.0, 1e-5),
+                      20), x.numel() * 2 + t * gh * gv * 2, flops)
+
+
 def bench_sample(B=64, V=32000):
     logits = torch.randn(B, V, device="cuda").bfloat16()
     temp = torch.zeros(B, device="cuda")
@@ -295,6 +426,8 @@ if __name__ == "__main__":
         bench_prefill_ablation()
     if a.which in ("all", "rope"):
         bench_rope()
+    if a.which == "hybrid":
+        bench_hybrid()
     if a.which in ("all", "norm"):
         bench_norm()
     if a.which in ("all", "sample"):

@@ -150,6 +150,13 @@ register(ModelConfig(
     vocab_size=128256, max_position_embeddings=8192, rope_theta=500000.0,
     rms_norm_eps=1e-5))
 
+# A small llama-shaped model (random weights), the uniform counterpart of
+# kakovik-1b.
+register(ModelConfig(
+    name="llama-1b", family="llama", hidden_size=2048, intermediate_size=5632,
+    num_layers=16, num_heads=16, num_kv_heads=16, vocab_size=32000,
+    max_position_embeddings=4096, rms_norm_eps=1e-5))
+
 # A tiny llama for CPU tests and CI.
 # Tiny llama for CPU tests/CI and GPU numerics tests (head_dim=64, GQA=2).
 register(ModelConfig(

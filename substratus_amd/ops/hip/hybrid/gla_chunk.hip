@@ -40,26 +40,17 @@ namespace {
 constexpr int C = 32;               // tokens per chunk
 constexpr int MAXW = 8;             // waves per workgroup
 constexpr int MAXRANK = 64;
-constexpr float DIRECT_BELOW = -60.f;
+constexpr float DIRECT_BELOW = -86.f;      // in powers of two: e^-60
+constexpr float LOG2E = 1.44269504088896340736f;
+constexpr int BUFFER_FLAGS = 0x00020000;   // untyped, offset-checked
+constexpr int OUT_OF_RANGE = 0x7ffffff0;   // beyond any buffer's end
 
 // place of element i (of 16) so that a lane half reads 8 in a row
 DEV_INLINE int perm16(int i) {
   return (i & ~12) | (i & 4) << 1 | (i & 8) >> 1;
 }
 
-DEV_INLINE short bf_bits(float f) {
-  const bf16_t b = f2bf(f);
-  return *reinterpret_cast<const short*>(&b);
-}
-
-DEV_INLINE float bits_f(short s) {
-  return __uint_as_float((unsigned)(unsigned short)s << 16);
-}
-
-DEV_INLINE void split_bf(float f, short* hi, short* lo) {
-  *hi = bf_bits(f);
-  *lo = bf_bits(f - bits_f(*hi));
-}
+DEV_INLINE float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 
 DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
   unsigned r;
@@ -67,17 +58,20 @@ DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
   return r;
 }
 
+// two floats as bf16 high parts and low parts, each pair in one word
+DEV_INLINE void split_pair(float f0, float f1, unsigned* hi, unsigned* lo) {
+  *hi = cvt_pk_bf16(f0, f1);
+  const float2 back = unpack_bf16x2(*hi);
+  *lo = cvt_pk_bf16(f0 - back.x, f1 - back.y);
+}
+
 // 8 consecutive accumulator rows as bf16 high and low operand parts
-template <int AT>
-DEV_INLINE void split_rows(const float16v& f, short8* hi, short8* lo) {
+template <int AT, class F>
+DEV_INLINE void split_rows(const F& f, short8* hi, short8* lo) {
   unsigned h[4], l[4];
   #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const float f0 = f[AT + 2 * i], f1 = f[AT + 2 * i + 1];
-    h[i] = cvt_pk_bf16(f0, f1);
-    const float2 back = unpack_bf16x2(h[i]);
-    l[i] = cvt_pk_bf16(f0 - back.x, f1 - back.y);
-  }
+  for (int i = 0; i < 4; ++i)
+    split_pair(f[AT + 2 * i], f[AT + 2 * i + 1], &h[i], &l[i]);
   *hi = *reinterpret_cast<const short8*>(h);
   *lo = *reinterpret_cast<const short8*>(l);
 }
@@ -92,20 +86,27 @@ struct Lds {
   alignas(16) short q[2][C][DP + 8];      // [hi|lo][token][channel, permuted]
   alignas(16) short k[2][C][DP + 8];
   alignas(16) short kt[2][DP][C + 8];     // [hi|lo][channel][token, permuted]
-  float end[DP];                          // e^(b_end)
-  float total[DP];                        // b_end summed over the segment
-  float a1[C][MAXRANK + 4];
-  float ssq[MAXW][C];
+  alignas(16) float end[DP];              // e^(b_end)
+  float total[DP];                        // b_end (base 2) over the segment
+  alignas(16) float ssq[MAXW][C];
+  float score[C][C + 1];                  // [key][query] of a direct chunk
   int direct[2];
 };
 
 // OUT: write outputs and the final state; else leave the segment's own state
 // and decay in the workspace.
+//
+// Making q~, k~ and k^ is divided into tasks of 32 channels: one kind makes
+// q~, the other k~ and k^. Both begin with the channel block's decays, a
+// product of the rows' A1 h with A2 on the matrix cores whose accumulators
+// hold a channel per lane and the tokens in registers. A wave takes its tasks
+// with their rows loaded a chunk ahead.
 template <int DT, bool OUT>
 __global__ __launch_bounds__(MAXW * WAVE)
 void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
                       float* __restrict__ ws, float* __restrict__ ws_decay) {
   constexpr int DP = DT * 32;
+  constexpr int TASKS = OUT ? 2 * DT : DT;
   __shared__ Lds<DT> s;
   const int e = blockIdx.x / nseg, seg = blockIdx.x % nseg, h = blockIdx.y;
   const Entry en = entry_of(a.seq_start, e);
@@ -114,11 +115,13 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
   const int len = min(seg_len, en.n - t0);
   const bool last = t0 + seg_len >= en.n;
   const int nw = blockDim.x / WAVE, tid = threadIdx.x;
-  const int wave = tid / WAVE, lane = tid % WAVE;
+  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int lane = tid % WAVE;
   const int lo5 = lane & 31, hi = lane >> 5;
   const int col = wave * 32 + lo5;
   const bool col_ok = col < a.vdim;
   const long row0 = en.row0 + t0;
+  const int ld = (int)a.ld;
   const int slot = a.state_slots[e];
   const long hstate = (long)a.dim * a.vdim;
   float* slot_state = slot < 0 ? nullptr
@@ -126,7 +129,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
   float* seg_state =
       ws + (((long)e * nseg + seg) * a.heads + h) * hstate;
 
-  // accumulator row r of channel tile i is channel 32i + crow(r)
+  // accumulator row r of a 32-row tile
   auto crow = [&](int r) { return (r & 3) + 8 * (r >> 2) + 4 * hi; };
 
   float16v st[DT];
@@ -139,150 +142,226 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
     for (int r = 0; r < 16; ++r) {
       const int d = 32 * i + crow(r);
       st[i][r] = init != nullptr && d < a.dim && col_ok
-          ? init[(long)d * a.vdim + col] : 0.f;
+          ? init[d * a.vdim + col] : 0.f;
     }
+  const float inv_vdim = 1.f / (float)a.vdim;
   const float nweight = OUT && col_ok ? a.norm[col] : 0.f;
   if (tid < 2) s.direct[tid] = 0;
   for (int d = tid; d < DP; d += blockDim.x) s.total[d] = 0.f;
-
-  auto stage_a1 = [&](int c0) {
-    for (int i = tid; i < C * a.rank; i += blockDim.x) {
-      const int t = i / a.rank, r = i % a.rank;
-      s.a1[t][r] = c0 + t < len
-          ? bf2f(a.x[(row0 + c0 + t) * a.ld + a.a_off + r]) : 0.f;
-    }
-  };
-  stage_a1(0);
   __syncthreads();
 
-  // Logs of decays, summed along the chunk, for 16 channels at a time:
-  // lane = (channel, quarter of the tokens); f(d, tq, b[8], b_end).
-  auto decays = [&](int c0, auto f) {
-    const int dl = lane & 15, tq = lane >> 4;
-    for (int d0 = wave * 16; d0 < DP; d0 += nw * 16) {
-      const int d = d0 + dl;
-      float b[8];
-      if (d < a.dim) {
-        const int c = h * a.dim + d;
-        const float z0 = a.a2b[c];
-        #pragma unroll
-        for (int i = 0; i < 8; ++i) b[i] = z0;
-        for (int r = 0; r < a.rank; ++r) {
-          const float w = a.a2[(long)c * a.rank + r];
-          #pragma unroll
-          for (int i = 0; i < 8; ++i) b[i] += s.a1[tq * 8 + i][r] * w;
-        }
-        #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          const float z = b[i];
-          const float ls = fminf(z, 0.f) -
-                           __logf(1.f + __expf(-fabsf(z)));
-          b[i] = c0 + tq * 8 + i < len ? ls * a.inv_tau : 0.f;
-        }
-      } else {
-        #pragma unroll
-        for (int i = 0; i < 8; ++i) b[i] = 0.f;
+  // The segment's rows as a bounded buffer: rows past its end read as zero
+  // and are not written, so the last chunk needs no code of its own.
+  const auto rows_in = __builtin_amdgcn_make_buffer_rsrc(
+      const_cast<bf16_t*>(a.x) + row0 * ld, 0, len * ld * 2, BUFFER_FLAGS);
+  const int out_ld = a.heads * a.vdim;
+  const auto rows_out = __builtin_amdgcn_make_buffer_rsrc(
+      a.out + row0 * out_ld, 0, OUT ? len * out_ld * 2 : 0, BUFFER_FLAGS);
+
+  // Column `at` of the rows of tokens crow(r) of the chunk at c0. (One word
+  // per value until use: packing them would wait for the loads.)
+  auto load16 = [&](int c0, int at, unsigned* f) {
+    const int off = ((c0 + 4 * hi) * ld + at) * 2;
+    #pragma unroll
+    for (int r = 0; r < 16; ++r)
+      f[r] = __builtin_amdgcn_raw_buffer_load_b16(
+          rows_in, off + ((r & 3) + 8 * (r >> 2)) * ld * 2, 0, 0);
+  };
+  // a task's rows: q (kind 0) or k (kind 1) of channel block `tile`
+  auto load_task = [&](int c0, int task, unsigned* f) {
+    const int tile = OUT ? task >> 1 : task, kind = OUT ? task & 1 : 1;
+    load16(c0, (kind ? a.k_off : 0) + h * a.dim +
+               min(32 * tile + lo5, a.dim - 1), f);
+  };
+  auto load_a1 = [&](int c0, int r0, unsigned* f) {
+    const int off = ((c0 + lo5) * ld + a.a_off) * 2;
+    #pragma unroll
+    for (int j = 0; j < 8; ++j)
+      f[j] = __builtin_amdgcn_raw_buffer_load_b16(
+          rows_in, off + min(r0 + 8 * hi + j, a.rank - 1) * 2, 0, 0);
+  };
+  auto pack8 = [&](const unsigned* f) {
+    unsigned w[4];
+    #pragma unroll
+    for (int j = 0; j < 4; ++j) w[j] = f[2 * j] | f[2 * j + 1] << 16;
+    return *reinterpret_cast<const short8*>(w);
+  };
+  // rows of A2 for channel block `tile`, zero outside rank and head
+  auto load_a2 = [&](int tile, int r0, short8* wh, short8* wl) {
+    const int d = 32 * tile + lo5;
+    const float* w2 = a.a2 + (long)(h * a.dim + min(d, a.dim - 1)) * a.rank;
+    float w[8];
+    #pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int r = r0 + 8 * hi + j;
+      w[j] = w2[min(r, a.rank - 1)];
+      if (r >= a.rank) w[j] = 0.f;
+    }
+    split_rows<0>(w, wh, wl);
+  };
+  // Summed logs (base 2) of the decays, b[r] for token crow(r); returns their end.
+  // The first 16 inner columns come loaded.
+  auto logs = [&](int c0, int tile, const unsigned* a1, short8 wh, short8 wl,
+                  float* b) {
+    const int d = 32 * tile + lo5;
+    float16v z = {};
+    z = mma(pack8(a1), wh, z);
+    z = mma(pack8(a1), wl, z);
+    for (int r0 = 16; r0 < a.rank; r0 += 16) {
+      unsigned more[8];
+      load_a1(c0, r0, more);
+      load_a2(tile, r0, &wh, &wl);
+      z = mma(pack8(more), wh, z);
+      z = mma(pack8(more), wl, z);
+    }
+    const float zb = a.a2b[h * a.dim + min(d, a.dim - 1)];
+    const int lim = d < a.dim ? len - c0 - 4 * hi : 0;
+    float gs[4], og[4];
+    #pragma unroll
+    for (int g = 0; g < 4; ++g) {
+      #pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int r = 4 * g + j;
+        const float v = (z[r] + zb) * LOG2E;
+        const float ls = fminf(v, 0.f) -
+                         __builtin_amdgcn_logf(1.f + exp2_f(-fabsf(v)));
+        b[r] = ls * (8 * g + j < lim ? a.inv_tau : 0.f);
+        if (j > 0) b[r] += b[r - 1];
       }
+      gs[g] = b[4 * g + 3];
+      og[g] = __shfl_xor(gs[g], 32, WAVE);
+    }
+    float before = 0.f;          // over the tokens ahead of each four
+    #pragma unroll
+    for (int g = 0; g < 4; ++g) {
+      const float add = before + (hi ? og[g] : 0.f);
       #pragma unroll
-      for (int i = 1; i < 8; ++i) b[i] += b[i - 1];
-      float before = 0.f;             // sum over earlier quarters
-      const float mine = b[7];
-      #pragma unroll
-      for (int k = 1; k < 4; ++k) {
-        const float u = __shfl(mine, dl + 16 * (k - 1), WAVE);
-        if (tq >= k) before += u;
-      }
-      #pragma unroll
-      for (int i = 0; i < 8; ++i) b[i] += before;
-      const float end = __shfl(b[7], 48 + dl, WAVE);
-      f(d, tq, b, end);
+      for (int j = 0; j < 4; ++j) b[4 * g + j] += add;
+      before += gs[g] + og[g];
+    }
+    return before;
+  };
+  // s.q / s.k rows from values per token
+  auto put_rows = [&](short (*dst)[C][DP + 8], int tile, const float* f) {
+    const int at = 32 * tile + (lo5 & 16) + perm16(lo5 & 15);
+    #pragma unroll
+    for (int r = 0; r < 16; r += 2) {
+      unsigned ph, pl;
+      split_pair(f[r], f[r + 1], &ph, &pl);
+      dst[0][crow(r)][at] = (short)ph;
+      dst[0][crow(r + 1)][at] = (short)(ph >> 16);
+      dst[1][crow(r)][at] = (short)pl;
+      dst[1][crow(r + 1)][at] = (short)(pl >> 16);
     }
   };
+  auto do_task = [&](int c0, int task, const unsigned* a1, short8 wh,
+                     short8 wl, const unsigned* rows) {
+    const int tile = OUT ? task >> 1 : task, kind = OUT ? task & 1 : 1;
+    const int d = 32 * tile + lo5;
+    float b[16], f[16];
+    const float end = logs(c0, tile, a1, wh, wl, b);
+    if (kind == 0) {
+      const float scale = d < a.dim ? a.qscale : 0.f;
+      #pragma unroll
+      for (int r = 0; r < 16; ++r)
+        f[r] = __uint_as_float(rows[r] << 16) * scale * exp2_f(b[r]);
+      put_rows(s.q, tile, f);
+      return;
+    }
+    const int lim = d < a.dim ? len - c0 - 4 * hi : 0;
+    float k[16];
+    #pragma unroll
+    for (int r = 0; r < 16; ++r)
+      k[r] = (r & 3) + 8 * (r >> 2) < lim
+          ? __uint_as_float(rows[r] << 16) : 0.f;
+    #pragma unroll
+    for (int r = 0; r < 16; ++r) f[r] = k[r] * exp2_f(end - b[r]);
+    short8 kh, kl;
+    split_rows<0>(f, &kh, &kl);
+    *reinterpret_cast<short8*>(&s.kt[0][d][8 * hi]) = kh;
+    *reinterpret_cast<short8*>(&s.kt[1][d][8 * hi]) = kl;
+    split_rows<8>(f, &kh, &kl);
+    *reinterpret_cast<short8*>(&s.kt[0][d][16 + 8 * hi]) = kh;
+    *reinterpret_cast<short8*>(&s.kt[1][d][16 + 8 * hi]) = kl;
+    if (OUT) {
+      #pragma unroll
+      for (int r = 0; r < 16; ++r) f[r] = k[r] * exp2_f(-b[r]);
+      put_rows(s.k, tile, f);
+    }
+    if (hi == 0) {
+      s.end[d] = exp2_f(end);
+      if (!OUT) s.total[d] += end;
+    }
+    if (OUT && end < DIRECT_BELOW) s.direct[(c0 / C) & 1] = 1;
+  };
+
+  // the wave's first task comes loaded; its part of A2 stays for the segment
+  const int vcol = h * a.vdim + min(col, a.vdim - 1);
+  unsigned task_rows[16], vraw[16], a1[8];
+  short8 wh0 = {}, wl0 = {};
+  if (wave < TASKS) {
+    load_task(0, wave, task_rows);
+    load_a2(OUT ? wave >> 1 : wave, 0, &wh0, &wl0);
+  }
+  load_a1(0, 0, a1);
+  load16(0, a.v_off + vcol, vraw);
 
   for (int c0 = 0; c0 < len; c0 += C) {
     const int par = (c0 / C) & 1;
-    // V as the second operand of both products, straight from the rows:
-    // token order as in the accumulators
-    short8 vf[2];
-    #pragma unroll
-    for (int g = 0; g < 2; ++g)
-      #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int t = c0 + 16 * g + crow(j);
-        vf[g][j] = t < len && col_ok
-            ? *reinterpret_cast<const short*>(
-                  a.x + (row0 + t) * a.ld + a.v_off + h * a.vdim + col)
-            : (short)0;
+    #pragma unroll 1
+    for (int task = wave; task < TASKS; task += nw) {
+      short8 wh = wh0, wl = wl0;
+      if (task != wave) {
+        load_task(c0, task, task_rows);
+        load_a2(OUT ? task >> 1 : task, 0, &wh, &wl);
       }
-
-    decays(c0, [&](int d, int tq, const float* b, float end) {
-      const int c = h * a.dim + d;
-      const int dpos = (d & ~15) | perm16(d & 15);
-      short kh[8], kl[8];
-      #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const int t = tq * 8 + i;
-        const bool ok = c0 + t < len && d < a.dim;
-        const bf16_t* x = a.x + (row0 + (ok ? c0 + t : 0)) * a.ld;
-        const float k = ok ? bf2f(x[a.k_off + c]) : 0.f;
-        split_bf(k * __expf(end - b[i]), &kh[i], &kl[i]);
-        if (OUT) {
-          const float q = ok ? bf2f(x[c]) * a.qscale : 0.f;
-          short ph, pl;
-          split_bf(q * __expf(b[i]), &ph, &pl);
-          s.q[0][t][dpos] = ph;
-          s.q[1][t][dpos] = pl;
-          split_bf(k * __expf(-b[i]), &ph, &pl);
-          s.k[0][t][dpos] = ph;
-          s.k[1][t][dpos] = pl;
-        }
-      }
-      // tokens 8tq..8tq+7 of the permuted order: two runs of four
-      const int at = (tq >> 1) * 16 + (tq & 1) * 4;
-      #pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        *reinterpret_cast<short4v*>(&s.kt[0][d][at + 8 * u]) =
-            (short4v){kh[4 * u], kh[4 * u + 1], kh[4 * u + 2], kh[4 * u + 3]};
-        *reinterpret_cast<short4v*>(&s.kt[1][d][at + 8 * u]) =
-            (short4v){kl[4 * u], kl[4 * u + 1], kl[4 * u + 2], kl[4 * u + 3]};
-      }
-      if (tq == 3) {
-        s.end[d] = __expf(end);
-        if (!OUT) s.total[d] += end;
-        if (OUT && end < DIRECT_BELOW) s.direct[par] = 1;
-      }
-    });
+      do_task(c0, task, a1, wh, wl, task_rows);
+    }
+    // V as the second operand of both products: token order as in the
+    // accumulators
+    const short8 vf[2] = {pack8(vraw), pack8(vraw + 8)};
     __syncthreads();
     const bool direct = OUT && s.direct[par] != 0;    // uniform
     if (OUT && tid == 0) s.direct[par ^ 1] = 0;
 
+    if (direct) {
+      // the summed logs take the place of k~
+      float (*sb)[DP + 8] = reinterpret_cast<float (*)[DP + 8]>(s.k);
+      for (int tile = wave; tile < DT; tile += nw) {
+        float b[16];
+        short8 wh, wl;
+        load_a2(tile, 0, &wh, &wl);
+        logs(c0, tile, a1, wh, wl, b);
+        #pragma unroll
+        for (int r = 0; r < 16; ++r) sb[crow(r)][32 * tile + lo5] = b[r];
+      }
+      __syncthreads();
+      const bf16_t* x = a.x + (row0 + c0) * ld + h * a.dim;
+      for (int i = tid; i < C * C; i += blockDim.x) {
+        const int ks = i / C, qt = i % C;
+        float acc = 0.f;
+        if (ks <= qt && c0 + qt < len) {
+          for (int d = 0; d < a.dim; ++d)
+            acc += bf2f(x[qt * ld + d]) * a.qscale *
+                   bf2f(x[ks * ld + a.k_off + d]) *
+                   exp2_f(sb[qt][d] - sb[ks][d]);
+        }
+        s.score[ks][qt] = acc;
+      }
+      __syncthreads();
+    }
+
+    unsigned graw[16];
+    if (OUT) load16(c0, a.g_off + vcol, graw);
+    if (c0 + C < len) {
+      if (wave < TASKS) load_task(c0 + C, wave, task_rows);
+      load_a1(c0 + C, 0, a1);
+      load16(c0 + C, a.v_off + vcol, vraw);
+    }
+
     float16v o = {};
     if (OUT) {
       float16v at = {};             // A^T: row = key token, column = query
-      if (direct) {
-        // the summed logs take the place of k~
-        float (*sb)[DP + 8] = reinterpret_cast<float (*)[DP + 8]>(s.k);
-        decays(c0, [&](int d, int tq, const float* b, float) {
-          #pragma unroll
-          for (int i = 0; i < 8; ++i) sb[tq * 8 + i][d] = b[i];
-        });
-        __syncthreads();
-        if (c0 + lo5 < len) {
-          const bf16_t* q = a.x + (row0 + c0 + lo5) * a.ld + h * a.dim;
-          #pragma unroll
-          for (int r = 0; r < 16; ++r) {
-            const int ks = crow(r);
-            if (ks > lo5) continue;
-            const bf16_t* k =
-                a.x + (row0 + c0 + ks) * a.ld + a.k_off + h * a.dim;
-            float acc = 0.f;
-            for (int d = 0; d < a.dim; ++d)
-              acc += bf2f(q[d]) * a.qscale * bf2f(k[d]) *
-                     __expf(sb[lo5][d] - sb[ks][d]);
-            at[r] = acc;
-          }
-        }
-      }
       #pragma unroll
       for (int i = 0; i < DT; ++i) {
         #pragma unroll
@@ -296,16 +375,16 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
           o = mma(qh, sh, o);
           o = mma(qh, sl, o);
           o = mma(ql, sh, o);
-          if (!direct) {
-            const short8 kh =
-                *reinterpret_cast<const short8*>(&s.k[0][lo5][d]);
-            const short8 kl =
-                *reinterpret_cast<const short8*>(&s.k[1][lo5][d]);
-            at = mma(kh, qh, at);
-            at = mma(kh, ql, at);
-            at = mma(kl, qh, at);
-          }
+          const short8 kh = *reinterpret_cast<const short8*>(&s.k[0][lo5][d]);
+          const short8 kl = *reinterpret_cast<const short8*>(&s.k[1][lo5][d]);
+          at = mma(kh, qh, at);
+          at = mma(kh, ql, at);
+          at = mma(kl, qh, at);
         }
+      }
+      if (direct) {
+        #pragma unroll
+        for (int r = 0; r < 16; ++r) at[r] = s.score[crow(r)][lo5];
       }
       #pragma unroll
       for (int r = 0; r < 16; ++r)
@@ -322,7 +401,12 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
     #pragma unroll
     for (int i = 0; i < DT; ++i) {
       #pragma unroll
-      for (int r = 0; r < 16; ++r) st[i][r] *= s.end[32 * i + crow(r)];
+      for (int g = 0; g < 4; ++g) {
+        const float4 f = *reinterpret_cast<const float4*>(
+            &s.end[32 * i + 8 * g + 4 * hi]);
+        st[i][4 * g] *= f.x; st[i][4 * g + 1] *= f.y;
+        st[i][4 * g + 2] *= f.z; st[i][4 * g + 3] *= f.w;
+      }
       #pragma unroll
       for (int g = 0; g < 2; ++g) {
         const short8 kh = *reinterpret_cast<const short8*>(
@@ -333,14 +417,13 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
         st[i] = mma(kl, vf[g], st[i]);
       }
     }
-    if (c0 + C < len) stage_a1(c0 + C);
 
     if (OUT) {
       // sum of squares of each token over the wave's 32 columns: halve the
       // set of tokens a lane holds at every exchange
       float q[16];
       #pragma unroll
-      for (int r = 0; r < 16; ++r) q[r] = o[r] * o[r];
+      for (int r = 0; r < 16; ++r) q[r] = col_ok ? o[r] * o[r] : 0.f;
       #pragma unroll
       for (int w = 8; w >= 1; w >>= 1) {
         #pragma unroll
@@ -356,20 +439,31 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
     }
     __syncthreads();
     if (OUT) {
+      float ss[16];
+      #pragma unroll
+      for (int r = 0; r < 16; ++r) ss[r] = 0.f;
+      #pragma unroll 2
+      for (int w = 0; w < nw; ++w)
+        #pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          const float4 f = *reinterpret_cast<const float4*>(
+              &s.ssq[w][8 * g + 4 * hi]);
+          ss[4 * g] += f.x; ss[4 * g + 1] += f.y;
+          ss[4 * g + 2] += f.z; ss[4 * g + 3] += f.w;
+        }
       #pragma unroll
       for (int r = 0; r < 16; ++r) {
-        const int t = crow(r);
-        float ss = 0.f;
-        for (int w = 0; w < nw; ++w) ss += s.ssq[w][t];
-        if (c0 + t < len && col_ok) {
-          const long row = row0 + c0 + t;
-          const float g =
-              bf2f(a.x[row * a.ld + a.g_off + h * a.vdim + col]);
-          const float inv = 1.f / sqrtf(ss / (float)a.vdim + a.eps);
-          a.out[(row * a.heads + h) * a.vdim + col] =
-              f2bf(o[r] * inv * nweight * (g / (1.f + __expf(-g))));
-        }
+        const float g = __uint_as_float(graw[r] << 16);
+        o[r] *= __builtin_amdgcn_rsqf(ss[r] * inv_vdim + a.eps) * nweight *
+                g * __builtin_amdgcn_rcpf(1.f + exp2_f(-g * LOG2E));
       }
+      const int off = col_ok
+          ? ((c0 + 4 * hi) * out_ld + h * a.vdim + col) * 2 : OUT_OF_RANGE;
+      #pragma unroll
+      for (int r = 0; r < 16; ++r)
+        __builtin_amdgcn_raw_buffer_store_b16(
+            cvt_pk_bf16(o[r], o[r]), rows_out,
+            col_ok ? off + ((r & 3) + 8 * (r >> 2)) * out_ld * 2 : off, 0, 0);
       // ssq is written again only after the next chunk's barrier
     }
   }
@@ -388,7 +482,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
   if (!OUT) {
     for (int d = tid; d < a.dim; d += blockDim.x)
       ws_decay[(((long)e * nseg + seg) * a.heads + h) * a.dim + d] =
-          expf(s.total[d]);
+          exp2_f(s.total[d]);
   }
 }
 

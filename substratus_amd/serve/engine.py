@@ -171,6 +171,11 @@ class Engine:
     def has_work(self) -> bool:
         return bool(self.waiting or self.running)
 
+    def prefilling(self) -> bool:
+        """Some request has not had its whole prompt computed yet."""
+        return bool(self.waiting) or self.takes_portions and any(
+            s.length - s.num_computed > 1 for s in self.running)
+
     # ------------------------------------------------------------ scheduling
     def _try_admit(self, out: list[StepOutput]) -> list[SequenceState]:
         admitted = []
