@@ -6,8 +6,9 @@
 // One page of 16 keys is a wave's unit of work. Scores: 4 lanes per key, each
 // with every fourth 16-byte piece of the row. Values: CL lanes across the
 // columns (8 each), 64/CL rows side by side. The next page's K, V and bias
-// are in flight while the current page is computed. Four waves take pages in
-// turn and merge through LDS; `splits` workgroups share one long context and
+// are in flight while the current page is computed. Queries stay bf16 and
+// scores are sums of v_dot2_f32_bf16 (two products added to a float), so K
+// needs no unpacking. Four waves take pages in turn and merge through LDS; `splits` workgroups share one long context and
 // a second kernel merges those.
 #include "attention_ctx.h"
 
@@ -17,6 +18,14 @@ constexpr int NW = 4;         // waves per workgroup
 constexpr int PAGE = 16;
 constexpr float NEG = -1e30f; // "no key yet": finite, so differences are too
 
+typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2_t;
+
+DEV_INLINE float dot2(unsigned a, unsigned b, float c) {
+  return __builtin_amdgcn_fdot2_f32_bf16(
+      __builtin_bit_cast(bf16x2_t, a), __builtin_bit_cast(bf16x2_t, b), c,
+      false);
+}
+
 template <int DCH, int CL, int GQ>
 __global__ __launch_bounds__(NW * WAVE)
 void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
@@ -24,7 +33,7 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
                             float* __restrict__ part_ml) {
   constexpr int RPI = WAVE / CL;          // V rows per instruction
   constexpr int NV = PAGE / RPI;          // V instructions per page
-  __shared__ float s_q[GQ][DCH * 32];
+  __shared__ alignas(16) unsigned s_q[GQ][DCH * 16];
   __shared__ float s_o[NW][GQ][CL * 8];
   __shared__ float s_ml[NW][GQ][2];
   const int b = blockIdx.x, kvh = blockIdx.y;
@@ -38,12 +47,11 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   const int lo = a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
   const int* bt = a.block_table + (long)b * a.max_blocks;
 
-  for (int i = threadIdx.x; i < GQ * DCH * 32; i += NW * WAVE) {
-    const int g = i / (DCH * 32), d = i % (DCH * 32);
-    s_q[g][d] = g < nh && d < a.dim
-        ? bf2f(a.q[(long)b * a.q_ld + (long)(h0 + g) * a.dim + d]) *
-              (a.scale * LOG2E)
-        : 0.f;
+  for (int i = threadIdx.x; i < GQ * DCH * 16; i += NW * WAVE) {
+    const int g = i / (DCH * 16), d = i % (DCH * 16) * 2;
+    const unsigned short* q = reinterpret_cast<const unsigned short*>(a.q) +
+                              (long)b * a.q_ld + (long)(h0 + g) * a.dim + d;
+    s_q[g][d / 2] = g < nh && d < a.dim ? q[0] | (unsigned)q[1] << 16 : 0u;
   }
   __syncthreads();
 
@@ -52,6 +60,7 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   const int kch = a.dim / 8, vch = a.vdim / 8;
   const int first = lo / PAGE + split * NW + wave, last = pos / PAGE;
   const int stride = splits * NW;
+  const float scale2 = a.scale * LOG2E;
 
   uint4v kr[DCH], vr[NV];
   float br[GQ];
@@ -100,19 +109,14 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     for (int g = 0; g < GQ; ++g) s[g] = 0.f;
     #pragma unroll
     for (int i = 0; i < DCH; ++i) {
-      float kf[8];
-      #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float2 t = unpack_bf16x2(kn[i][j]);
-        kf[2 * j] = t.x; kf[2 * j + 1] = t.y;
-      }
       #pragma unroll
       for (int g = 0; g < GQ; ++g) {
-        const float4* qp =
-            reinterpret_cast<const float4*>(&s_q[g][(sub + 4 * i) * 8]);
-        const float4 q0 = qp[0], q1 = qp[1];
-        s[g] += kf[0] * q0.x + kf[1] * q0.y + kf[2] * q0.z + kf[3] * q0.w +
-                kf[4] * q1.x + kf[5] * q1.y + kf[6] * q1.z + kf[7] * q1.w;
+        const uint4 qp =
+            *reinterpret_cast<const uint4*>(&s_q[g][(sub + 4 * i) * 4]);
+        s[g] = dot2(kn[i][0], qp.x, s[g]);
+        s[g] = dot2(kn[i][1], qp.y, s[g]);
+        s[g] = dot2(kn[i][2], qp.z, s[g]);
+        s[g] = dot2(kn[i][3], qp.w, s[g]);
       }
     }
     const int kpos = pg * PAGE + key;
@@ -121,7 +125,7 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     for (int g = 0; g < GQ; ++g) {
       s[g] += __shfl_xor(s[g], 1, WAVE);
       s[g] += __shfl_xor(s[g], 2, WAVE);
-      s[g] = live ? s[g] + bn[g] : NEG;
+      s[g] = live ? s[g] * scale2 + bn[g] : NEG;
       float mx = s[g];
       #pragma unroll
       for (int off = 4; off < WAVE; off <<= 1)
