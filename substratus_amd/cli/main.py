@@ -10,6 +10,7 @@ Commands (reference internal/cli/*.go):
   sub get [scope]             list kinds with ready state (models, models/x)
   sub delete kind/name        delete
   sub infer                   completion request against a ready Server
+  sub generate                completion in this process, from a model folder
 
 Rendering uses rich tables/spinners instead of the reference's bubbletea TUI
 (internal/tui; same information architecture: ready checkmarks, conditions,
@@ -439,6 +440,49 @@ def infer(server: str = typer.Option(..., "--server", "-s"),
                    timeout=300)
     r.raise_for_status()
     console.print(r.json()["choices"][0]["text"])
+
+
+@app.command()
+def generate(model: str = typer.Option(..., "--model", "-m",
+                                       help="registered model name, or a "
+                                            "folder with config.json and "
+                                            "model.safetensors"),
+             prompt: str = typer.Argument("", help="prompt text"),
+             tokens: str = typer.Option("", help="prompt as token ids with "
+                                                 "commas between them; the "
+                                                 "answer is then ids, too"),
+             max_tokens: int = typer.Option(32),
+             temperature: float = typer.Option(0.0),
+             top_k: int = typer.Option(0), top_p: float = typer.Option(1.0),
+             dtype: str = typer.Option("bfloat16"),
+             device: Optional[str] = typer.Option(None)):
+    """One completion on the local engine, no platform and no server."""
+    import torch
+
+    from ..models import get_config
+    from ..models.weights import load_weights
+    from ..serve import tokenizer
+    from ..serve.engine import Engine, EngineConfig
+    tok = tokenizer.load(model if os.path.isdir(model) else None,
+                         get_config(model).vocab_size)
+    ids = [int(t) for t in tokens.split(",")] if tokens else tok.encode(prompt)
+    eng = Engine(EngineConfig(model=model, dtype=getattr(torch, dtype),
+                              max_batch=1,
+                              max_seq_len=len(ids) + max_tokens + 1),
+                 device=device)
+    if os.path.isdir(model):
+        load_weights(eng.model, eng.mcfg, model, eng.device, eng.cfg.dtype)
+    eng.add_request(ids, max_new_tokens=max_tokens, temperature=temperature,
+                    top_k=top_k, top_p=top_p,
+                    eos_token=-1 if tokens else tok.eos)
+    out: list[int] = []
+    while eng.has_work():
+        for o in eng.step():
+            if o.error:
+                console.print(f"[red]{o.error}[/red]")
+                raise typer.Exit(1)
+            out.append(o.token)
+    print(",".join(map(str, out)) if tokens else tok.decode(out))
 
 
 def main() -> None:

@@ -1,0 +1,743 @@
+"""Kakovik models through the engine against the plain float64 implementation
+in tests/oracles, on the CPU ops and on the GPU kernels."""
+
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+from oracles import kakovik as oracle
+from oracles import models
+from substratus_amd.models import get_config
+from substratus_amd.models.layers import distance_bias, distance_bucket
+from substratus_amd.models.weights import load_weights
+from substratus_amd.ops import hybrid as ops
+from substratus_amd.serve.batch import StepBatch
+from substratus_amd.serve.engine import Engine, EngineConfig
+from substratus_amd.serve.kv_cache import OutOfSlots
+from substratus_amd.serve.trace import TraceReplay
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+PLACES = [pytest.param(("cpu", "float32"), id="cpu"),
+          pytest.param(("cuda", "float32"), id="gpu-f32",
+                       marks=pytest.mark.gpu),
+          pytest.param(("cuda", "bfloat16"), id="gpu-bf16",
+                       marks=pytest.mark.gpu)]
+# of logits, root mean square, relative to the logits' own
+LIMIT = {"float32": 1e-4, "bfloat16": 0.06}
+
+
+@pytest.fixture(scope="module")
+def folder(tmp_path_factory):
+    """name -> (folder, config, weights)"""
+    made = {}
+
+    def get(name):
+        if name not in made:
+            d = str(tmp_path_factory.mktemp(name))
+            made[name] = (d, *models.write(d, name))
+        return made[name]
+    return get
+
+
+_expected = {}
+
+
+def expected(cfg, w, toks, key):
+    if key not in _expected:
+        _expected[key] = oracle.forward(cfg, w, toks)
+    return _expected[key]
+
+
+def error(got, want):
+    d = got.double() - want
+    d = d - d.mean(-1, keepdim=True)
+    return float((d.pow(2).mean(-1).sqrt() / want.std()).max())
+
+
+class Replayed:
+    """A TraceReplay with whole requests' tokens known ahead."""
+
+    def __init__(self, folder, place, max_tokens):
+        device, self.dtype = place
+        self.trace = TraceReplay(folder, self.dtype, max_tokens, device)
+        self.got, self.at = {}, {}
+
+    def step(self, parts, end=()):
+        """parts: (name, all tokens, how many of them next)"""
+        entries = []
+        for name, toks, n in parts:
+            a = self.at.get(name, 0)
+            entries.append({"id": name, "tokens": toks[a:a + n],
+                            "want": list(range(n))})
+            self.at[name] = a + n
+        logits = self.trace.step(entries, list(end))
+        for name, _, n in parts:
+            self.got.setdefault(name, []).append(logits[:n])
+            logits = logits[n:]
+        assert logits.shape[0] == 0
+
+    def check(self, name, want):
+        got = torch.cat(self.got[name])
+        assert error(got, want[:got.shape[0]]) < LIMIT[self.dtype], name
+
+
+def replay_cut(folder, place, toks, cuts):
+    r = Replayed(folder, place, (len(toks) + 63) // 64 * 64)
+    for n in cuts:
+        r.step([("a", toks, n)])
+    assert r.at["a"] == len(toks)
+    return r
+
+
+# ---- configuration and registry ---------------------------------------------
+
+def test_config_is_read_from_the_folder(folder):
+    d, doc, _ = folder("mixed")
+    cfg = get_config(d)
+    assert cfg.family == "kakovik" and cfg.num_layers == 5
+    assert (cfg.hidden_size, cfg.vocab_size) == (80, 101)
+    assert cfg.logit_scale == 0.7 and cfg.norm_offset == 1.0
+    a = cfg.layers[1].mixer
+    assert (a.heads, a.kv_heads, a.dim, a.vdim, a.chunk) == (4, 2, 32, 24, 40)
+    assert (a.bias_rows, a.bias_max, a.v_mix) == (12, 130, True)
+    assert cfg.layers[0].mixer.rank == 8 and cfg.layers[0].ff == 0
+    assert [s.ff for s in cfg.layers] == [0, 112, 72, 96, 0]
+
+
+def test_param_count_matches_the_weights(folder):
+    for name in models.CONFIGS:
+        d, _, w = folder(name)
+        big = sum(t.numel() for t in w.values() if t.dim() == 2
+                  and t.shape[0] != models.CONFIGS[name][1])
+        assert get_config(d).param_count() == big
+
+
+def test_registered_sizes():
+    for name in ("kakovik-tiny", "kakovik-1b", "kakovik-7b"):
+        cfg = get_config(name)
+        assert cfg.layers and cfg.param_count() > 0
+
+
+@pytest.mark.parametrize("change", [
+    {"architecture": "Nothing"},
+    {"layers": [{"type": "other", "mixer": {}, "mlp": None}]},
+    {"layers": [dict(models.gla(1, 8, 8, 2.0), mlp={"kind": "other"})]}])
+def test_unknown_parts_are_refused(tmp_path, change):
+    doc = dict(models.CONFIGS["mixed"][0], **change)
+    (tmp_path / "config.json").write_text(json.dumps(doc))
+    with pytest.raises((KeyError, ValueError), match="unknown"):
+        get_config(str(tmp_path))
+
+
+def test_no_quantized_weights_or_caches(folder):
+    for kw in ({"quant": "q4_0"}, {"kv_dtype": "fp8"}):
+        with pytest.raises(ValueError):
+            Engine(EngineConfig(model=folder("mixed")[0],
+                                dtype=torch.float32, kv_blocks=8,
+                                max_seq_len=64, **kw), device="cpu")
+
+
+# ---- mechanisms alone -------------------------------------------------------
+
+@pytest.mark.parametrize("rows,furthest", [(32, 240), (8, 50), (12, 130),
+                                           (7, 20), (2, 9), (16, 2000),
+                                           (32, 33), (6, 24)])
+def test_distance_buckets(rows, furthest):
+    for n in range(2 * furthest):
+        assert distance_bucket(n, rows, furthest) == \
+            oracle.distance_bucket(n, rows, furthest), n
+
+
+def test_distance_bucket_at_a_rows_start():
+    """Rows start at half * 2^k here: exactly at those distances."""
+    assert [distance_bucket(n, 8, 64) for n in
+            (3, 4, 7, 8, 15, 16, 31, 32, 63, 64, 1000)] == \
+        [3, 4, 4, 5, 5, 6, 6, 7, 7, 7, 7]
+
+
+@pytest.mark.parametrize("chunk", [0, 10, 500])
+def test_distance_bias_covers_every_distance(chunk):
+    rel = torch.randn(12, 3)
+    got = distance_bias(rel, chunk, 90)
+    reach = chunk or 300
+    want = oracle.distance_bias(rel, reach, 90)
+    n = torch.arange(reach).clamp(max=got.shape[1] - 1)
+    assert torch.equal(got[:, n], want)
+
+
+def put(t, place):
+    return t.to(place[0], getattr(torch, place[1]))
+
+
+def request_batch(place, spans):
+    """One request per (first position, tokens), on pages in falling order."""
+    entries, top = [], sum((a + n + 15) // 16 for a, n in spans)
+    pages = top
+    for i, (a, n) in enumerate(spans):
+        need = (a + n + 15) // 16
+        entries.append(([0] * n, a, list(range(top - 1, top - 1 - need, -1)),
+                        i, []))
+        top -= need
+    return StepBatch.build(entries, 16, torch.device(place[0])), pages
+
+
+def tol(place):
+    return 2e-4 if place[1] == "float32" else 2e-2
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_norms_around_the_residual(place):
+    g = torch.Generator().manual_seed(0)
+    d, x, wp, wn = (torch.randn(s, generator=g)
+                    for s in ((5, 96), (5, 96), (96,), (96,)))
+    d = put(d, place)
+    xs = x.to(place[0], copy=True)
+    y = ops.stream_norm(d, xs, wp.to(place[0]), wn.to(place[0]), 1.0, 1e-2,
+                        0.5)
+    want_x = x.double() + oracle.stream_norm(d.cpu().double(), wp, 1e-2)
+    want = oracle.stream_norm(want_x, wn, 1e-2) * 0.5
+    assert float((xs.cpu() - want_x).abs().max()) < 1e-5
+    assert xs.dtype == torch.float32
+    assert float((y.cpu().double() - want).abs().max()) < tol(place)
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_projection_norms_and_value_blend(place):
+    g = torch.Generator().manual_seed(1)
+    heads, kv, d, dv, n = 4, 2, 24, 16, 5
+    buf, first = torch.randn(n, heads * d + kv * (d + dv) + 8, generator=g), \
+        torch.randn(n, kv * dv, generator=g)
+    qw, kw = (1 + torch.randn(m * d, generator=g) for m in (heads, kv))
+    buf, first = put(buf, place), put(first, place)
+    batch, pages = request_batch(place, [(30, n)])
+    kc = torch.zeros(pages, kv, 16, d, dtype=buf.dtype, device=place[0])
+    vc = torch.zeros(pages, kv, 16, dv, dtype=buf.dtype, device=place[0])
+    ref = buf.cpu().double()
+    ops.qkv_prepare(buf, heads * d, qw.to(place[0]), kw.to(place[0]), 1e-3,
+                    first, torch.tensor(0.3, device=place[0]), kc, vc,
+                    batch.slots)
+    q, k, v = ref[:, :heads * d], ref[:, heads * d:(heads + kv) * d], \
+        ref[:, (heads + kv) * d:(heads + kv) * d + kv * dv]
+    blocks = batch.block_table[0].long()
+    rows = slice(30, 30 + n)
+
+    def cached(c):
+        return c[blocks].transpose(1, 2).reshape(-1, kv * c.shape[3])[rows] \
+            .cpu().double()
+    for got, want in (
+            (buf[:, :heads * d].cpu().double(), oracle.rms(q, 1e-3) * qw),
+            (cached(kc), oracle.rms(k, 1e-3) * kw),
+            (cached(vc), oracle.mix_values(v, first.cpu().double(), 0.3))):
+        assert float((got - want).abs().max()) < tol(place) * 2
+
+
+def standing_out(place, span, chunk, key, bias=None, dim=32, vdim=16):
+    """Attention of one request's rows over keys among which `key` stands
+    out, and values that tell positions apart: value column c of position p
+    is 1 where p % vdim == c, scaled by its page."""
+    batch, pages = request_batch(place, [span])
+    n = batch.tokens.shape[0]
+    kc = torch.zeros(pages, 1, 16, dim)
+    vc = torch.zeros(pages, 1, 16, vdim)
+    for j, page in enumerate(batch.block_table[0].tolist()):
+        for o in range(16):
+            p = 16 * j + o
+            vc[page, 0, o, p % vdim] = 1 + p // 16
+    kc[batch.block_table[0, key // 16], 0, key % 16, 0] = 30.0
+    q = torch.zeros(n, dim)
+    q[:, 0] = 1.0
+    if bias is not None:
+        bias = bias.to(place[0])
+    out = ops.attn_ctx(put(q, place), None, put(kc, place), put(vc, place),
+                       bias, batch, 1.0, chunk)
+    return out.float().cpu(), batch.positions.tolist()
+
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("chunk,key", [
+    (0, 0), (0, 15), (0, 16), (0, 17), (0, 400), (48, 0), (48, 47), (48, 48),
+    (48, 95), (48, 96), (20, 39), (20, 40), (20, 19), (64, 63), (64, 64)])
+def test_a_key_that_stands_out(place, chunk, key):
+    """Seen by its own chunk's later positions only, in prompts, in decoding,
+    at page borders and far away."""
+    vdim = 16
+    spans = [(0, 140), (key, 2), (key + 1, 3), (max(key - 2, 0), 5)] + \
+        [(p, 1) for p in {key, key + 1, 500, (key // 16 + 1) * 16} |
+         ({(key // chunk + 1) * chunk - 1, (key // chunk + 1) * chunk}
+          if chunk else set())]
+    for span in spans:
+        reach = span[0] + span[1]
+        if reach <= key:
+            continue
+        out, pos = standing_out(place, span, chunk, key, vdim=vdim)
+        for row, p in zip(out, pos):
+            seen = oracle.visible(p, key, chunk or 1 << 30)
+            at = 1.0 + key // 16
+            if seen:
+                assert abs(float(row[key % vdim]) - at) < 0.02 * at, (p, key)
+            else:
+                lo = p // chunk * chunk if chunk else 0
+                want = torch.zeros(vdim)
+                for j in range(lo, p + 1):
+                    want[j % vdim] += 1 + j // 16
+                want /= p + 1 - lo
+                assert torch.allclose(row, want, rtol=2e-2, atol=1e-2), (p,
+                                                                        key)
+
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("distance", [0, 1, 5, 31, 32, 100])
+def test_a_distance_that_stands_out(place, distance):
+    bias = torch.zeros(1, 160)
+    bias[0, distance] = 40.0
+    vdim = 16
+    for span in ((0, 140), (139, 1), (distance, 2)):
+        batch_out, pos = standing_out(place, span, 0, 0, bias, vdim=vdim)
+        for row, p in zip(batch_out, pos):
+            if p >= distance and p != distance:    # key 0 stands out itself
+                j = p - distance
+                assert abs(float(row[j % vdim]) - (1 + j // 16)) < \
+                    0.02 * (1 + j // 16) + 0.02, p
+
+
+def random_gla(place, n, heads=2, dim=24, vdim=16, rank=4, seed=3, shift=2.0):
+    g = torch.Generator().manual_seed(seed)
+    x = put(torch.randn(n, 2 * heads * (dim + vdim) + rank, generator=g),
+            place)
+    a2 = torch.randn(heads * dim, rank, generator=g).bfloat16().float()
+    a2b = torch.randn(heads * dim, generator=g) * 2 + shift
+    norm = 1 + 0.2 * torch.randn(vdim, generator=g)
+    return x, a2, a2b, norm
+
+
+def gla_oracle(x, a2, a2b, norm, tau, heads, dim, vdim, eps):
+    f = x.cpu().double()
+    q, k, v, gate, a1 = f.split([heads * dim] * 2 + [heads * vdim] * 2 +
+                                [a2.shape[1]], dim=1)
+    alpha = oracle.sigmoid(a1 @ a2.double().T + a2b) ** (1 / tau)
+    o, s = oracle.recur(q.view(-1, heads, dim) * dim ** -0.5,
+                        k.view(-1, heads, dim), v.view(-1, heads, vdim),
+                        alpha.view(-1, heads, dim))
+    o = (oracle.rms(o, eps) * norm).reshape(len(f), -1)
+    return o * oracle.silu(gate), s
+
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("cuts", [[200], [1] * 70, [33, 1, 2, 31, 32, 64, 37],
+                                  [2, 2, 2, 100]])
+@pytest.mark.parametrize("tau,shift", [(16.0, 2.0), (1.0, 0.0), (1.0, -8.0)])
+def test_recurrence_carries_its_state(place, cuts, tau, shift):
+    """However a sequence is cut; also with channels that keep nothing."""
+    heads, dim, vdim = 2, 24, 16
+    x, a2, a2b, norm = random_gla(place, sum(cuts), shift=shift)
+    small = [t.to(place[0]) for t in (a2, a2b, norm)]
+    # slot 1 of 3, left full of numbers by someone else
+    state = torch.full((3, heads, dim, vdim), 7.0, device=place[0])
+    got, at = [], 0
+    for n in cuts:
+        batch = StepBatch.build([([0] * n, at, [0] * 20, 1, [])], 16,
+                                torch.device(place[0]))
+        got.append(ops.gla(x[at:at + n], *small, state, batch, tau, 1e-5))
+        at += n
+    want, s = gla_oracle(x, a2, a2b, norm, tau, heads, dim, vdim, 1e-5)
+    err = (torch.cat(got).cpu().double() - want).abs().max() / want.abs().max()
+    assert float(err) < tol(place)
+    assert float((state[1].cpu().double() - s).abs().max()
+                 / s.abs().max()) < 2e-4      # 32-bit in every place
+    assert bool((state[0] == 7).all()) and bool((state[2] == 7).all())
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_recurrence_finds_a_far_key(place):
+    """One key written early, nothing decays, asked for 500 tokens later."""
+    heads, dim, vdim, n = 1, 32, 16, 600
+    x = torch.zeros(n, 2 * (dim + vdim) + 4)
+    x[20, dim + 5] = 1.0                                    # k
+    x[20, 2 * dim:2 * dim + vdim] = torch.arange(vdim) + 1.0  # v
+    x[520, 5] = 1.0                                         # q
+    x[:, 2 * dim + vdim:2 * dim + 2 * vdim] = 30.0          # open gate
+    x = put(x, place)
+    a2 = torch.zeros(dim, 4, device=place[0])
+    a2b = torch.full((dim,), 30.0, device=place[0])
+    norm = torch.ones(vdim, device=place[0])
+    for cuts in ([n], [19, 2, 400, 99, 1, 79], [500] + [1] * 25):
+        state = torch.zeros(1, heads, dim, vdim, device=place[0])
+        got, at = [], 0
+        for c in cuts:
+            batch = StepBatch.build([([0] * c, at, [0] * 40, 0, [])], 16,
+                                    torch.device(place[0]))
+            got.append(ops.gla(x[at:at + c], a2, a2b, norm, state, batch,
+                               16.0, 1e-9))
+            at += c
+        row = torch.cat(got)[520].float().cpu()
+        v = torch.arange(vdim) + 1.0
+        want = v / v.pow(2).mean().sqrt() * 30
+        assert torch.allclose(row, want, rtol=1e-2), cuts
+
+
+# ---- whole models -----------------------------------------------------------
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("name", list(models.CONFIGS))
+def test_whole_prompts(folder, name, place):
+    d, cfg, w = folder(name)
+    for n, seed in ((130, 1), (1, 2), (2, 3), (17, 4)):
+        toks = models.tokens(cfg, n, seed)
+        want = expected(cfg, w, toks, (name, n, seed))
+        replay_cut(d, place, toks, [n]).check("a", want)
+
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("name", list(models.CONFIGS))
+def test_token_by_token(folder, name, place):
+    """From the first token on, across page and chunk edges."""
+    d, cfg, w = folder(name)
+    toks = models.tokens(cfg, 130, 1)
+    want = expected(cfg, w, toks, (name, 130, 1))
+    replay_cut(d, place, toks, [1] * 130).check("a", want)
+
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+@pytest.mark.parametrize("size", [2, 3, 7, 16, 17, 33, 64])
+def test_portions(folder, name, size, place):
+    d, cfg, w = folder(name)
+    toks = models.tokens(cfg, 130, 1)
+    want = expected(cfg, w, toks, (name, 130, 1))
+    cuts = [size] * (110 // size)
+    cuts += [110 - sum(cuts)] if sum(cuts) < 110 else []
+    replay_cut(d, place, toks, cuts + [1] * 20).check("a", want)
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_unequal_requests_in_one_batch(folder, place):
+    """Portions beside single tokens, requests that pause, end and start, in
+    a pool that makes them use each other's pages and slots."""
+    name = "mixed"
+    d, cfg, w = folder(name)
+    toks = {k: models.tokens(cfg, n, s) for k, n, s in
+            (("a", 130, 1), ("b", 50, 5), ("c", 90, 6), ("d", 17, 4),
+             ("e", 60, 7), ("f", 40, 8))}
+    r = Replayed(d, place, 384)
+    free = r.trace.engine.kv.allocator.free_count
+
+    def step(*parts, end=()):
+        r.step([(k, toks[k], n) for k, n in parts], end)
+    step(("a", 2), ("b", 31))
+    step(("b", 1), ("a", 40), ("c", 3))
+    step(("c", 1), ("b", 1), ("a", 1), ("d", 16))
+    step(("d", 1), ("a", 50), ("b", 16), end=["d"])
+    step(("b", 1), ("a", 1), end=["b"])
+    step(("e", 60), ("c", 29), ("a", 1))
+    step(("a", 1), ("f", 2))
+    step(("f", 37), ("a", 20), ("c", 57), end=["c", "e"])
+    step(("f", 1), ("a", 13), end=["a", "f"])
+    for k in "abcdef":
+        n = len(toks[k])
+        want = expected(cfg, w, toks[k],
+                        (name, n, {"a": 1, "b": 5, "c": 6, "d": 4, "e": 7,
+                                   "f": 8}[k]))
+        r.check(k, want)
+    kv = r.trace.engine.kv
+    assert kv.allocator.free_count == free and kv.slots.free_count == 4
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_pages_and_slots_are_used_again(folder, place):
+    """One pool, one request after another in it: what the last one left
+    must not show."""
+    d, cfg, w = folder("mixed")
+    r = Replayed(d, place, 192)
+    for i, (n, seed) in enumerate([(130, 1), (17, 4), (90, 6), (130, 1),
+                                   (2, 3)]):
+        toks = models.tokens(cfg, n, seed)
+        r.step([(f"r{i}", toks, n - 1)])
+        r.step([(f"r{i}", toks, 1)], end=[f"r{i}"])
+        r.check(f"r{i}", expected(cfg, w, toks, ("mixed", n, seed)))
+
+
+def test_more_requests_than_slots_are_refused(folder):
+    d, cfg, _ = folder("mixed")
+    trace = TraceReplay(d, "float32", 320, "cpu")
+    one = [{"id": i, "tokens": [1], "want": []} for i in range(5)]
+    trace.step(one[:4], [])
+    with pytest.raises(OutOfSlots):
+        trace.step(one[4:], [])
+    trace.step([], [0])
+
+
+def test_no_room_takes_nothing(folder):
+    from substratus_amd.serve.kv_cache import OutOfBlocks, SequenceState
+    d, cfg, _ = folder("mixed")
+    trace = TraceReplay(d, "float32", 64, "cpu")
+    seq = SequenceState(0, list(range(65)), 0, 0)
+    with pytest.raises(OutOfBlocks):
+        trace.engine.kv.reserve(seq, 65)
+    assert seq.blocks == [] and seq.state_slot == -1
+    assert trace.engine.kv.slots.free_count == 4
+
+
+PLANTED = {
+    "chunk one longer": ("visible",
+                         lambda i, j, c: j <= i and i // (c + 1) == j // (c + 1)),
+    "no chunk": ("visible", lambda i, j, c: j <= i),
+    "own key unseen": ("visible", lambda i, j, c: j <= i and
+                       (i == 0 or j != i or i % c == 0) and i // c == j // c),
+    "next distance": ("distance_bucket",
+                      lambda n, r, f: min(r - 1, n + 1)),
+    "values not blended": ("mix_values", lambda v, f, lam: v),
+    "blend the other way": ("mix_values",
+                            lambda v, f, lam: lam * v + (1 - lam) * f),
+    "plain norm weights": ("stream_norm",
+                           lambda x, w, eps: oracle.rms(x, eps) * w),
+    "state lost": ("recur", lambda q, k, v, a, state=None:
+                   ((k * q).sum(-1, keepdim=True) * v, None)),
+    "no decay": ("key_decay", lambda w, p, h, tau:
+                 torch.ones(h.shape[0], w[p + "a2"].shape[0],
+                            dtype=torch.float64)),
+    "decay without its root": ("key_decay", lambda w, p, h, tau: oracle.sigmoid(
+        (h @ w[p + "a1"].T) @ w[p + "a2"].T + w[p + "a2.b"])),
+    "ungated feed-forward": ("silu", lambda z: z),
+}
+
+
+@pytest.mark.parametrize("what", list(PLANTED))
+def test_faults_would_show(folder, monkeypatch, what):
+    """A mistake planted in the oracle is far outside the limits above."""
+    d, cfg, w = folder("mixed")
+    toks = models.tokens(cfg, 130, 1)
+    r = replay_cut(d, ("cpu", "float32"), toks, [130])
+    monkeypatch.setattr(oracle, *PLANTED[what])
+    wrong = oracle.forward(cfg, w, toks)
+    assert error(torch.cat(r.got["a"]), wrong) > 3 * LIMIT["bfloat16"]
+
+
+# ---- generation -------------------------------------------------------------
+
+def engine_for(folder, place, **kw):
+    args = dict(max_batch=3, max_seq_len=192, kv_blocks=64, prefill_chunk=48)
+    args.update(kw)
+    dtype = getattr(torch, place[1])
+    eng = Engine(EngineConfig(model=folder, dtype=dtype, **args),
+                 device=place[0])
+    assert load_weights(eng.model, eng.mcfg, folder, eng.device, dtype)
+    return eng
+
+
+def generate(eng, prompts, new):
+    ids = [eng.add_request(p, max_new_tokens=n) for p, n in zip(prompts, new)]
+    out = {i: [] for i in ids}
+    for _ in range(2000):
+        if not eng.has_work():
+            break
+        for o in eng.step():
+            assert o.error is None
+            out[o.seq_id].append(o.token)
+    assert not eng.has_work()
+    return [out[i] for i in ids]
+
+
+def check_greedy(cfg, w, prompt, got, dtype):
+    """Every token is the oracle's choice for what precedes it, up to ties
+    within rounding."""
+    logits = oracle.forward(cfg, w, prompt + got)[len(prompt) - 1:-1]
+    slack = 4 * LIMIT[dtype] * float(logits.std())
+    best = logits.max(-1).values
+    mine = logits[torch.arange(len(got)), torch.tensor(got)]
+    assert bool((best - mine <= slack).all())
+    return float((logits.argmax(-1) == torch.tensor(got)).double().mean())
+
+
+@pytest.mark.parametrize("place", PLACES)
+@pytest.mark.parametrize("name", list(models.CONFIGS))
+def test_greedy_generation(folder, name, place):
+    """More requests than slots, prompts longer than a step's tokens."""
+    d, cfg, w = folder(name)
+    lens, new = (70, 5, 100, 1, 33), (30, 12, 9, 40, 1)
+    prompts = [models.tokens(cfg, n, 20 + n) for n in lens]
+    eng = engine_for(d, place)
+    got = generate(eng, prompts, new)
+    for p, g, n in zip(prompts, got, new):
+        assert len(g) == n
+        same = check_greedy(cfg, w, p, g, place[1])
+        assert same > (0.98 if place[1] == "float32" else 0.7)
+    assert eng.kv.slots.free_count == eng.kv.slots.num_slots
+    assert eng.kv.allocator.free_count >= 63     # a page for padded lanes
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_generation_with_preemption(folder, place):
+    """Too few pages for all: the youngest gives its pages and state back
+    and is computed again."""
+    d, cfg, w = folder("mixed")
+    prompts = [models.tokens(cfg, n, 40 + n) for n in (40, 45, 50)]
+    eng = engine_for(d, place, kv_blocks=13)
+    seen = []
+    whole = eng._preempt_youngest
+    eng._preempt_youngest = lambda: (seen.append(1), whole())
+    got = generate(eng, prompts, (40, 40, 40))
+    assert seen
+    for p, g in zip(prompts, got):
+        check_greedy(cfg, w, p, g, place[1])
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_long_decoding(folder, place):
+    d, cfg, w = folder("mixed")
+    prompt = models.tokens(cfg, 3, 77)
+    eng = engine_for(d, place, max_seq_len=320)
+    (got,) = generate(eng, [prompt], (250,))
+    check_greedy(cfg, w, prompt, got, place[1])
+
+
+def test_abort_gives_everything_back(folder):
+    d, cfg, _ = folder("mixed")
+    eng = engine_for(d, ("cpu", "float32"))
+    ids = [eng.add_request(models.tokens(cfg, 60, s), max_new_tokens=20)
+           for s in range(4)]
+    eng.step()
+    assert eng.abort(ids[0]) and eng.abort(ids[3])
+    eng.step()
+    eng.abort_all()
+    assert eng.kv.allocator.free_count == 64
+    assert eng.kv.slots.free_count == 3
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_captured_decode_equals_eager(folder, dtype):
+    """Replays between eager steps of joining requests, padded lanes beside
+    live ones: the same tokens as without capture."""
+    d, cfg, _ = folder("mixed")
+    prompts = [models.tokens(cfg, n, 60 + n) for n in (20, 3, 50, 31, 9, 44)]
+    new = (50, 20, 35, 8, 30, 25)
+    runs = []
+    for graphs in (False, True, True):
+        eng = engine_for(d, ("cuda", dtype), max_batch=5, use_graphs=graphs)
+        ids = [eng.add_request(p, max_new_tokens=n)
+               for p, n in zip(prompts[:3], new)]
+        out = {}
+        for step in range(200):
+            if step in (7, 8, 19):
+                k = len(ids)
+                ids.append(eng.add_request(prompts[k], max_new_tokens=new[k]))
+            for o in eng.step():
+                out.setdefault(o.seq_id, []).append(o.token)
+            if step % 5 == 0:
+                torch.cuda.synchronize()
+            if not eng.has_work():
+                break
+        assert (eng.graph_runner is not None) == graphs
+        runs.append([out[i] for i in ids])
+    assert [len(r) for r in runs[0]] == list(new)
+    assert runs[1] == runs[2]
+    same = sum(a == b for x, y in zip(runs[0], runs[1])
+               for a, b in zip(x, y)) / sum(new)
+    assert same == 1.0 if dtype == "float32" else same > 0.5
+
+
+@pytest.mark.gpu
+def test_sampling_of_float_logits():
+    from substratus_amd import ops as base
+    g = torch.Generator().manual_seed(0)
+    logits = torch.randn(6, 700, generator=g) * 3
+    args = (torch.tensor([0, 0.7, 1.0, 1.0, 1.3, 0.9]),
+            torch.tensor([0, 0, 20, 0, 5, 0], dtype=torch.int32),
+            torch.tensor([1.0, 1.0, 1.0, 0.8, 0.9, 0.5]),
+            torch.tensor([0.1, 0.3, 0.5, 0.2, 0.1, 0.4]))
+    got = base.softmax_sample(logits.cuda(), *(t.cuda() for t in args)).cpu()
+    assert got[0] == logits[0].argmax()
+    probs = torch.softmax(logits / args[0].clamp(min=1e-3)[:, None], -1)
+    for b in range(6):
+        assert probs[b, got[b]] > 0
+
+
+# ---- entry points -----------------------------------------------------------
+
+TRACE = [{"step": 0, "entries": [
+             {"id": "a", "tokens": [1, 2, 3], "want": [0, 2]},
+             {"id": "b", "tokens": [4], "want": [0]}], "end": []},
+         {"step": 1, "entries": [{"id": "a", "tokens": [5], "want": []}],
+          "end": ["b"]},
+         {"step": 2, "entries": [{"id": "c", "tokens": [4, 9], "want": [0]},
+                                 {"id": "a", "tokens": [6], "want": [0]}],
+          "end": ["a", "c"]}]
+
+
+@pytest.mark.parametrize("place", PLACES)
+def test_trace_run(folder, place, tmp_path):
+    d, cfg, w = folder("mixed")
+    r = subprocess.run(
+        [os.path.join(ROOT, "bin", "trace_run"), "--model", d, "--dtype",
+         place[1], "--out", str(tmp_path), "--max-tokens", "192", "--device",
+         place[0]], input="\n".join(map(json.dumps, TRACE)) + "\n",
+        capture_output=True, text=True, timeout=110)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [x for x in r.stdout.splitlines() if x.startswith("done")] == \
+        ["done 0", "done 1", "done 2"]
+    assert sorted(os.listdir(tmp_path)) == ["0.f32", "2.f32"]
+
+    def rows(step):
+        data = (tmp_path / f"{step}.f32").read_bytes()
+        return torch.frombuffer(bytearray(data), dtype=torch.float32).view(
+            -1, cfg["vocab"])
+    a = oracle.forward(cfg, w, [1, 2, 3, 5, 6])
+    b = oracle.forward(cfg, w, [4, 9])
+    assert error(rows(0), torch.stack([a[0], a[2], b[0]])) < LIMIT[place[1]]
+    assert error(rows(2), torch.stack([b[0], a[4]])) < LIMIT[place[1]]
+
+
+def test_trace_run_needs_known_models(tmp_path):
+    r = subprocess.run(
+        [os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path),
+         "--out", str(tmp_path), "--max-tokens", "64", "--device", "cpu"],
+        input="", capture_output=True, text=True, timeout=110)
+    assert r.returncode != 0
+
+
+def test_served_over_http(folder, monkeypatch):
+    from fastapi.testclient import TestClient
+    from substratus_amd.serve import server
+    d, cfg, w = folder("mixed")
+    monkeypatch.setenv("MODEL_DIR", d)
+    monkeypatch.setenv("PARAMS_PATH", os.path.join(d, "none.json"))
+    monkeypatch.setattr(torch.cuda, "is_available", lambda: False)
+    app = server.create_app()
+    assert app.state.engine.mcfg.family == "kakovik"
+    prompt = models.tokens(cfg, 20, 5)
+    with TestClient(app) as client:
+        r = client.post("/v1/completions", json={
+            "prompt": prompt, "max_tokens": 6, "temperature": 0.0})
+        assert r.status_code == 200
+        assert r.json()["usage"]["prompt_tokens"] == 20
+        assert client.get("/stats").json()["served_tokens_total"] >= 1
+    app.state.worker.stop()
+
+
+def test_generate_command(folder, monkeypatch):
+    from typer.testing import CliRunner
+    from substratus_amd.cli.main import app
+    d, cfg, w = folder("mixed")
+    prompt = models.tokens(cfg, 12, 9)
+    r = CliRunner().invoke(app, [
+        "generate", "--model", d, "--tokens", ",".join(map(str, prompt)),
+        "--max-tokens", "8", "--dtype", "float32", "--device", "cpu"])
+    assert r.exit_code == 0, r.output
+    got = [int(t) for t in r.output.strip().splitlines()[-1].split(",")]
+    assert check_greedy(cfg, w, prompt, got, "float32") == 1.0
+
+
+def test_loader_writes_a_registered_model(tmp_path):
+    from substratus_amd.loader import model_loader
+    d = model_loader.run(str(tmp_path), {"name": "kakovik-tiny"})
+    cfg = get_config(d)
+    assert cfg.name == "kakovik-tiny"
+    eng = Engine(EngineConfig(model=d, dtype=torch.float32, max_batch=2,
+                              max_seq_len=64, kv_blocks=8), device="cpu")
+    assert load_weights(eng.model, eng.mcfg, d, eng.device, torch.float32)
+    assert len(generate(eng, [[1, 2, 3]], [4])[0]) == 4
