@@ -52,6 +52,9 @@ def ensure_built() -> None:
                 cwd=ROOT, check=True, stdout=sys.stderr,
                 env=dict(os.environ, PYTORCH_ROCM_ARCH="gfx950",
                          SUB_EXT="_hybrid"))
+            if not built():   # imports it afresh, past the import cache
+                raise RuntimeError("built, but cannot be imported: "
+                                   "substratus_amd._hybrid")
 
 
 class TraceReplay:
