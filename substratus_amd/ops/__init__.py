@@ -221,11 +221,12 @@ def linear(x: torch.Tensor, weight: torch.Tensor,
     ceiling on this chip (~1.33-1.47 PF, guide 8-phase template) equals
     hipBLASLt's best here. The kernel stays for measurement and as the
     base for a future counted-vmcnt schedule."""
+    if (os.environ.get("SUB_MGEMM") != "1" or x.dtype != torch.bfloat16
+            or torch.is_grad_enabled() and (
+                x.requires_grad or weight.requires_grad)):
+        return torch.nn.functional.linear(x, weight, bias)
     ext = _dispatch(x)
-    if (ext is None or torch.is_grad_enabled() and (
-            x.requires_grad or weight.requires_grad)
-            or x.dtype != torch.bfloat16
-            or os.environ.get("SUB_MGEMM") != "1"):
+    if ext is None:
         return torch.nn.functional.linear(x, weight, bias)
     x2 = x.reshape(-1, x.shape[-1])
     m, k = x2.shape
