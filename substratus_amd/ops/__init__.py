@@ -217,9 +217,8 @@ def linear(x: torch.Tensor, weight: torch.Tensor,
     NOT on by default: the round-3 measurement (profiles/mgemm_r02.md)
     shows hipBLASLt's MT192/MT256 solutions at 1.3-4.1 TB/s of weight
     stream on the llama2-7b decode shapes vs our kernel's 1.0-2.25 — the
-    library already implements the deep-pipelined schedule whose measured
-    ceiling on this chip (~1.33-1.47 PF, guide 8-phase template) equals
-    hipBLASLt's best here. The kernel stays for measurement and as the
+    library's measured rates reach the ceiling measured for a deep-pipelined
+    schedule on this chip (~1.33-1.47 PF). The kernel stays for measurement and as the
     base for a future counted-vmcnt schedule."""
     if (os.environ.get("SUB_MGEMM") != "1" or x.dtype != torch.bfloat16
             or torch.is_grad_enabled() and (

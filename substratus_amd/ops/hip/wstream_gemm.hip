@@ -41,10 +41,9 @@
 //      per wave, every 16-B W fragment needs 16x16-B A-fragment LDS reads
 //      (A:W = 16:1), capping the W stream at ~LDS_BW/16 per CU. Breaking
 //      it needs A-reuse across n-tiles per wave (acc > 128 VGPRs → AGPR
-//      accumulators), lds-dma staging and counted-vmcnt phases — the
-//      library-grade schedule hipBLASLt already has (its M=256 solutions
-//      run 40-65% of the 6.3 TB/s roofline; TunableOp confirms +2% is all
-//      the library has left). hipBLASLt stays the production path; the
+//      accumulators), lds-dma staging and counted-vmcnt phases.
+//      hipBLASLt's M=256 solutions measure 40-65% of the 6.3 TB/s roofline
+//      (TunableOp finds +2% among them). hipBLASLt stays the production path; the
 //      remaining decode-GEMM headroom (~3.8 ms/step at B=256) is a
 //      known-open item, quantified in profiles/decode_step_profile_r01.txt.
 #include "common.h"
