@@ -7,6 +7,7 @@ A model is a tuple of LayerSpec; the mixer's spec type selects the mixer
 
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 from functools import lru_cache
 from typing import Union
@@ -99,7 +100,8 @@ def distance_bias(table: torch.Tensor, chunk: int,
                   furthest: int) -> torch.Tensor:
     """[rows, heads] table -> float32 [heads, n], the bias of each distance;
     column n - 1 also stands for every larger distance."""
-    n = furthest + 1 if chunk == 0 else min(chunk, furthest + 1)
+    n = math.ceil(furthest) + 1
+    n = n if chunk == 0 else min(chunk, n)
     rows = torch.tensor(_buckets(max(n, 1), table.shape[0], furthest),
                         device=table.device)
     return table.float()[rows].T.contiguous()

@@ -298,6 +298,9 @@ def _rope_train(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor,
 class CausalLM(nn.Module):
     def __init__(self, cfg: ModelConfig, device=None, dtype=torch.bfloat16):
         super().__init__()
+        if cfg.layers:
+            raise ValueError(f"{cfg.name}: models of unlike layers are built "
+                             "by models.build_model, and served only")
         self.cfg = cfg
         st = state()
         self.embed_tokens = nn.Embedding(cfg.vocab_size, cfg.hidden_size,

@@ -274,7 +274,9 @@ void gla(Tensor out, Tensor x, Tensor a2, Tensor a2b, Tensor norm,
     a.heads = heads; a.dim = dim; a.vdim = vdim; a.rank = rank;
     a.qscale = 1.f / std::sqrt((float)dim); a.inv_tau = inv_tau; a.eps = eps;
     if constexpr (std::is_same_v<T, bf16_t>) {
-      if (seq_start && !recurrent && gla_chunk_supported(dim, vdim, rank)) {
+      // the chunk kernel addresses a segment's rows with 32-bit offsets
+      if (seq_start && !recurrent && gla_chunk_supported(dim, vdim, rank) &&
+          max_len * a.ld * 2 < 0x7ffffff0 - (1 << 20)) {
         const int nseg = gla_chunk_segments(entries, heads, max_len);
         Tensor ws, wd;
         if (nseg > 1) {

@@ -50,6 +50,23 @@ def test_bench_train_schema():
     assert r["metric"] == "fine_tune_tokens_per_s"
 
 
+@pytest.mark.timeout(300)
+def test_bench_hybrid_schema():
+    out = subprocess.run(
+        [sys.executable, "bench.py", "--mode", "hybrid", "--steps", "2",
+         "--warmup", "1", "--model", "kakovik-tiny"],
+        cwd=ROOT, capture_output=True, text=True, timeout=280,
+        env=dict(os.environ, HIP_VISIBLE_DEVICES=""))
+    assert out.returncode == 0, out.stderr[-2000:]
+    r = _last_json(out.stdout)
+    assert REQUIRED <= set(r)
+    assert r["metric"] == "hybrid_decode_tokens_per_s"
+    models = {p["model"] for p in r["config"]["points"]}
+    assert models == {"kakovik-tiny", "llama-tiny"}
+    for p in r["config"]["points"]:
+        assert p["prefill_tokens_per_s"] > 0 and p["decode_tokens_per_s"] > 0
+
+
 @pytest.mark.timeout(600)
 def test_bench_torchrun_2rank_gloo():
     """The exact launch shape the driver uses for N>1 (loopback rendezvous)."""

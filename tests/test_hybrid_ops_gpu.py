@@ -72,14 +72,14 @@ def test_embed_norm(width, dtype):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("f", [320, 37, 64])
+@pytest.mark.parametrize("f", [328, 37, 64])
 def test_silu_mul(f, dtype):
     x = rand(5, 2 * f, seed=7, dtype=dtype, scale=3.0)
     close(ops.silu_mul(x.cuda()), ops.silu_mul(x), dtype)
 
 
 # heads, kv heads, dim, vdim
-SHAPES = [(4, 4, 96, 48), (4, 2, 64, 128), (6, 1, 32, 32), (8, 2, 128, 128),
+SHAPES = [(5, 5, 96, 40), (4, 2, 64, 128), (6, 1, 32, 32), (8, 2, 128, 128),
           (3, 3, 40, 24), (2, 1, 20, 12), (5, 1, 256, 256), (2, 2, 112, 160)]
 
 
@@ -161,7 +161,7 @@ def gla_inputs(shape, batch, dtype, seed, z_shift=0.0):
     return x, a2, a2b, norm, state
 
 
-GLA_SHAPES = [(6, 48, 64, 16), (2, 64, 32, 16), (3, 128, 256, 16),
+GLA_SHAPES = [(5, 48, 72, 16), (2, 64, 32, 33), (3, 128, 256, 16),
               (2, 40, 24, 8), (1, 20, 300, 5), (2, 256, 96, 16), (2, 17, 7, 3)]
 
 

@@ -134,6 +134,14 @@ def test_unknown_parts_are_refused(tmp_path, change):
         get_config(str(tmp_path))
 
 
+def test_not_a_uniform_transformer(folder):
+    from substratus_amd.models import CausalLM, HybridLM, build_model
+    cfg = get_config(folder("mixed")[0])
+    with pytest.raises(ValueError, match="build_model"):
+        CausalLM(cfg, device="meta")
+    assert isinstance(build_model(cfg, device="meta"), HybridLM)
+
+
 def test_no_quantized_weights_or_caches(folder):
     for kw in ({"quant": "q4_0"}, {"kv_dtype": "fp8"}):
         with pytest.raises(ValueError):
@@ -144,7 +152,7 @@ def test_no_quantized_weights_or_caches(folder):
 
 # ---- mechanisms alone -------------------------------------------------------
 
-@pytest.mark.parametrize("rows,furthest", [(32, 240), (8, 50), (12, 130),
+@pytest.mark.parametrize("rows,furthest", [(32, 260), (8, 50), (12, 130),
                                            (7, 20), (2, 9), (16, 2000),
                                            (32, 33), (6, 24)])
 def test_distance_buckets(rows, furthest):
