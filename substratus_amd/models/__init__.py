@@ -1,5 +1,6 @@
 from .config import ModelConfig, get_config, register
-from . import kakovik as _kakovik  # registers the architecture and its models
+from . import guronex as _guronex  # registers the architecture and its models
+from . import kakovik as _kakovik  # the same
 from .hybrid import HybridLM
 from .model import CausalLM
 

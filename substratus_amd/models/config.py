@@ -19,7 +19,7 @@ from .layers import LayerSpec
 @dataclass
 class ModelConfig:
     name: str
-    family: str  # "llama" | "falcon" | "opt" | "kakovik"
+    family: str  # "llama" | "falcon" | "opt" | "kakovik" | "guronex"
     hidden_size: int
     intermediate_size: int
     num_layers: int
@@ -44,6 +44,9 @@ class ModelConfig:
     # uniform fields above then only size things for reports
     layers: tuple[LayerSpec, ...] = ()
     norm_offset: float = 0.0  # 1: norm weights are stored around zero
+    pre_norm: bool = True     # sublayers read the normed residual, or itself
+    residual_mult: float = 1.0  # factor of what sublayers add to the residual
+    side_dim: int = 0         # per layer: size of an input for the token itself
     logit_scale: float = 1.0
 
     def __post_init__(self) -> None:
@@ -57,8 +60,9 @@ class ModelConfig:
     def param_count(self) -> int:
         h, f, L, v = self.hidden_size, self.intermediate_size, self.num_layers, self.vocab_size
         if self.layers:
-            return 2 * v * h + sum(s.mixer.params(h) + 3 * h * s.ff
-                                   for s in self.layers)
+            side = self.side_dim * len(self.layers)
+            return 2 * v * h + side * (v + 2 * h) \
+                + sum(s.params(h) for s in self.layers)
         qkv = h * (self.num_heads + 2 * self.num_kv_heads) * self.head_dim
         o = self.num_heads * self.head_dim * h
         if self.activation == "silu":

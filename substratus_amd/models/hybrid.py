@@ -1,6 +1,7 @@
-"""Decoder-only model whose layers differ: a list of mixers (attention, gated
-linear attention, ...) and optional feed-forwards around a 32-bit residual,
-each sublayer normed before and after.
+"""Decoder-only model whose layers differ: a list of mixers (attention, latent
+attention, gated linear attention, ...) and optional feed-forwards (dense or
+mixtures of experts) around a 32-bit residual, each sublayer normed before and
+after, or after only. A layer may end with an input for the token itself.
 
 The engine drives it like the uniform families (models/model.py), with one
 difference: a step is a StepBatch (serve/batch.py) of single tokens and prompt
@@ -24,7 +25,8 @@ from ..parallel.comm import state
 from ..parallel.tp import Linear
 from ..serve.batch import StepBatch
 from .config import ModelConfig
-from .layers import AttentionSpec, GLASpec, LayerSpec, distance_bias
+from .layers import (AttentionSpec, GLASpec, LatentAttentionSpec, LayerSpec,
+                     MoESpec, distance_bias)
 
 
 def _f32(*shape: int, device=None) -> nn.Parameter:
@@ -121,28 +123,118 @@ class GLAMixer(nn.Module):
         return self.w_out(o)
 
 
-MIXERS = {AttentionSpec: AttentionMixer, GLASpec: GLAMixer}
+class LatentMixer(nn.Module):
+    """Softmax attention over a paged cache of latents, the layer's own or an
+    earlier layer's; heads expand keys and values from them, or queries and
+    outputs are moved into the latent space (ops.latent_attn)."""
+
+    def __init__(self, spec: LatentAttentionSpec, width: int, eps: float,
+                 device=None, dtype=None):
+        super().__init__()
+        self.spec, self.eps = spec, eps
+        self.own = spec.kv_from is None
+        self.nq = spec.heads * (spec.dim + spec.rot_dim)
+        self.ng = spec.heads * spec.vdim if spec.out_gate else 0
+        self.w_in = Linear(width, _padded(self.nq + self.ng +
+                                          (spec.row if self.own else 0)),
+                           device=device, dtype=dtype)
+        self.w_out = Linear(spec.heads * spec.vdim, width, device=device,
+                            dtype=dtype)
+        # keys of all heads, then values of all heads
+        self.w_ukv = nn.Parameter(torch.empty(
+            spec.heads * (spec.dim + spec.vdim), spec.rank, device=device,
+            dtype=dtype))
+        if self.own:
+            self.c_norm = _f32(spec.rank, device=device)
+
+    def finish_weights(self) -> None:
+        s = self.spec
+        self._uk_t = self.w_ukv[:s.heads * s.dim].view(
+            s.heads, s.dim, s.rank).transpose(1, 2).contiguous()
+        self._turns = s.rot.turns(self.w_ukv.device)
+
+    def forward(self, y: torch.Tensor, cache: tuple, batch: StepBatch,
+                shared: dict) -> torch.Tensor:
+        buf = self.w_in(y)
+        at = self.nq + self.ng
+        ops.latent_prepare(buf, self.spec, at if self.own else -1,
+                           self.c_norm if self.own else None, self.eps,
+                           self._turns, batch.positions, cache[0],
+                           batch.slots)
+        gate = buf[:, self.nq:at] if self.ng else None
+        o = ops.latent_attn(buf[:, :self.nq], gate, cache[0], self.w_ukv,
+                            self._uk_t, batch, self.spec, shared)
+        return self.w_out(o)
+
+
+MIXERS = {AttentionSpec: AttentionMixer, GLASpec: GLAMixer,
+          LatentAttentionSpec: LatentMixer}
+
+
+class Experts(nn.Module):
+    """A mixture of experts: what every token adds is left as rows to pick
+    and weigh, which the norm that follows does on its way."""
+
+    def __init__(self, spec: MoESpec, width: int, device=None, dtype=None):
+        super().__init__()
+        self.spec = spec
+
+        def weight(*shape):
+            return nn.Parameter(torch.empty(shape, device=device,
+                                            dtype=dtype))
+        self.router = weight(spec.experts, width)
+        self.up = weight(spec.experts, spec.ff, width)
+        self.down = weight(spec.experts, width, spec.ff)
+
+    def forward(self, y: torch.Tensor) -> ops.Picked:
+        return ops.experts(y, self.router, self.up, self.down, self.spec)
+
+
+class SideInput(nn.Module):
+    """A layer's input for the token itself: a gate of the stream times the
+    token's entry in a table, projected."""
+
+    def __init__(self, dim: int, width: int, device=None, dtype=None):
+        super().__init__()
+        self.w_gate = nn.Parameter(torch.empty(dim, width, device=device,
+                                               dtype=dtype))
+        self.w_proj = Linear(dim, width, device=device, dtype=dtype)
+        self.norm = _f32(width, device=device)
+
+    def forward(self, y: torch.Tensor, tokens: torch.Tensor,
+                table: torch.Tensor, layer: int) -> torch.Tensor:
+        return self.w_proj(ops.side_gate(y, self.w_gate, tokens, table,
+                                         layer * self.w_gate.shape[0]))
 
 
 class HybridLayer(nn.Module):
-    def __init__(self, spec: LayerSpec, width: int, eps: float, device=None,
+    def __init__(self, spec: LayerSpec, cfg: ModelConfig, device=None,
                  dtype=None):
         super().__init__()
         self.spec = spec
-        self.mixer = MIXERS[type(spec.mixer)](spec.mixer, width, eps, device,
-                                              dtype)
-        self.norm1 = _f32(width, device=device)
-        self.norm1b = _f32(width, device=device)
+        width = cfg.hidden_size
+        self.mixer = MIXERS[type(spec.mixer)](spec.mixer, width,
+                                              cfg.rms_norm_eps, device, dtype)
+
+        def norm(there):
+            return _f32(width, device=device) if there else None
+        self.norm1 = norm(cfg.pre_norm)
+        self.norm1b = norm(True)
+        ff = bool(spec.ff or spec.moe)
+        self.norm2 = norm(ff and cfg.pre_norm)
+        self.norm2b = norm(ff)
         if spec.ff:
-            self.norm2 = _f32(width, device=device)
-            self.norm2b = _f32(width, device=device)
             self.w_gateup = Linear(width, 2 * spec.ff, device=device,
                                    dtype=dtype)
             self.w_down = Linear(spec.ff, width, device=device, dtype=dtype)
+        if spec.moe:
+            self.experts = Experts(spec.moe, width, device, dtype)
+        if cfg.side_dim:
+            self.side = SideInput(cfg.side_dim, width, device, dtype)
 
-    def feed_forward(self, y: torch.Tensor) -> torch.Tensor:
-        if y.shape[0] == 0:
-            return y
+    def feed_forward(self, y: torch.Tensor):
+        if self.spec.moe:
+            return self.experts(y)
         return self.w_down(ops.silu_mul(self.w_gateup(y)))
 
 
@@ -153,15 +245,19 @@ class HybridLM(nn.Module):
         super().__init__()
         if state().tp_size > 1:
             raise NotImplementedError(
-                f"{cfg.family} models are served on one GPU: their norms span "
-                "all heads of a projection, which tensor parallelism divides")
+                f"{cfg.family} models are served on one GPU: the norms and "
+                "the latents of their layers span all heads, which tensor "
+                "parallelism divides")
         self.cfg, self.eps = cfg, cfg.rms_norm_eps
         self.n_kv_heads = cfg.num_kv_heads
         self.embed = nn.Embedding(cfg.vocab_size, cfg.hidden_size,
                                   device=device, dtype=dtype)
         self.layers = nn.ModuleList(
-            HybridLayer(s, cfg.hidden_size, self.eps, device, dtype)
-            for s in cfg.layers)
+            HybridLayer(s, cfg, device, dtype) for s in cfg.layers)
+        if cfg.side_dim:
+            self.side_embed = nn.Parameter(torch.empty(
+                cfg.vocab_size, cfg.side_dim * len(cfg.layers), device=device,
+                dtype=dtype))
         self.final_norm = _f32(cfg.hidden_size, device=device)
         self.head = Linear(cfg.hidden_size, cfg.vocab_size, device=device,
                            dtype=dtype)
@@ -176,7 +272,7 @@ class HybridLM(nn.Module):
             leaf = name.rsplit(".", 1)[-1]
             if leaf in ("norm1", "norm1b", "norm2", "norm2b", "final_norm"):
                 p.fill_(neutral)
-            elif leaf in ("q_norm", "k_norm", "norm"):
+            elif leaf in ("q_norm", "k_norm", "norm", "c_norm"):
                 p.fill_(1.0)
             elif leaf == "vmix":
                 p.fill_(0.5)
@@ -201,36 +297,35 @@ class HybridLM(nn.Module):
         models/model.py decode_ops); returns the logits of batch.want, or of
         every row."""
         off, eps = self.cfg.norm_offset, self.eps
+        mult = self.cfg.residual_mult
         x, y = ops.embed_norm(batch.tokens, self.embed.weight,
                               self.layers[0].norm1, off, eps)
+        tokens = batch.tokens
         shared: dict = {}     # what a layer leaves for later layers' mixers
         for i, layer in enumerate(self.layers):
             last = i + 1 == len(self.layers)
             after = self.final_norm if last else self.layers[i + 1].norm1
             scale = self.cfg.logit_scale if last else 1.0
-            delta = layer.mixer(y, caches[i], batch, shared)
+            delta, post = layer.mixer(y, caches[i], batch, shared), \
+                layer.norm1b
             yield
-            post = layer.norm1b
-            if layer.spec.ff:
-                if last:
-                    delta, x = self._wanted(delta, x, batch)
-                y = ops.stream_norm(delta, x, post, layer.norm2, off, eps)
-                delta = layer.feed_forward(y)
-                post = layer.norm2b
+            if last and batch.want is not None:
+                # past the last mixer only rows with wanted logits go on
+                if batch.want.shape[0] == 0:
+                    return y.new_empty(0, self.cfg.vocab_size)
+                delta, x, tokens = (t[batch.want] for t in (delta, x, tokens))
+            if layer.norm2b is not None:
+                y = ops.stream_norm(delta, x, post, layer.norm2, off, eps,
+                                    mult=mult)
+                delta, post = layer.feed_forward(y), layer.norm2b
                 yield
-            elif last:
-                delta, x = self._wanted(delta, x, batch)
-            y = ops.stream_norm(delta, x, post, after, off, eps, scale)
-        if y.shape[0] == 0:
-            return y.new_empty(0, self.cfg.vocab_size)
+            if self.cfg.side_dim:
+                y = ops.stream_norm(delta, x, post, None, off, eps, mult=mult)
+                delta, post = layer.side(y, tokens, self.side_embed, i), \
+                    layer.side.norm
+                yield
+            y = ops.stream_norm(delta, x, post, after, off, eps, scale, mult)
         return self.head(y)
-
-    @staticmethod
-    def _wanted(delta, x, batch: StepBatch):
-        """Past the last mixer only rows with wanted logits go on."""
-        if batch.want is None:
-            return delta, x
-        return delta[batch.want], x[batch.want]
 
     def forward_step(self, batch: StepBatch,
                      caches: list[tuple]) -> torch.Tensor:
@@ -244,11 +339,10 @@ class HybridLM(nn.Module):
     def decode_ops(self, tokens: torch.Tensor, positions: torch.Tensor,
                    kv_caches: list[tuple], slots: torch.Tensor,
                    block_table: torch.Tensor, seq_lens: torch.Tensor,
-                   state_slots: torch.Tensor):
+                   state_slots: torch.Tensor, block_size: int):
         """One token per request, device-resident state (graph capture)."""
         n = tokens.shape[0]
-        bs = max((c[0].shape[2] for c in kv_caches if len(c) == 2), default=1)
         batch = StepBatch(tokens.int(), positions, slots, block_table,
                           state_slots, n, None, 0,
-                          block_table.shape[1] * bs)
+                          block_table.shape[1] * block_size)
         return (yield from self.step_ops(batch, kv_caches))

@@ -10,7 +10,7 @@ from __future__ import annotations
 import math
 from dataclasses import dataclass
 from functools import lru_cache
-from typing import Union
+from typing import Optional, Union
 
 import torch
 
@@ -64,9 +64,82 @@ class GLASpec:
 
 
 @dataclass(frozen=True)
+class RotarySpec:
+    """Rotation of the first `dims` elements of a vector: element i turns with
+    element i + dims / 2, at position p by p * base ** (-2 i / dims)."""
+    base: float
+    dims: int
+
+    def turns(self, device=None) -> torch.Tensor:
+        """float64 [dims / 2]: full turns per position. Whole turns drop out
+        of position * turns before anything is rounded to 32 bits."""
+        i = torch.arange(self.dims // 2, dtype=torch.float64)
+        return (self.base ** (-2.0 * i / self.dims) / (2 * math.pi)).to(device)
+
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention whose keys and values are projections of one latent vector
+    per token, beside a rotated key part that all heads share."""
+    heads: int
+    dim: int                 # unrotated query/key size of a head
+    rot_dim: int             # rotated query/key size of a head
+    vdim: int                # value size of a head
+    rank: int                # size of the latent
+    scale: float
+    rot: RotarySpec
+    kv_from: Optional[int] = None   # layer whose latents it attends to
+    out_gate: bool = False   # sigmoid gate per element on the output
+
+    @property
+    def row(self) -> int:
+        """Elements the cache holds per token: latent, rotated key part."""
+        return self.rank + self.rot_dim
+
+    def kv_bytes(self, itemsize: int) -> int:
+        return self.row * itemsize if self.kv_from is None else 0
+
+    def state_bytes(self) -> int:
+        return 0
+
+    def params(self, width: int) -> int:
+        rows = self.heads * (self.dim + self.rot_dim +
+                             self.vdim * (1 + self.out_gate)) \
+            + (self.row if self.kv_from is None else 0)
+        return width * rows + self.heads * self.rank * (self.dim + self.vdim)
+
+
+@dataclass(frozen=True)
+class MoESpec:
+    """Experts, of which a token uses the `top` best of the `keep` best
+    groups of neighbours; weights are softmax scores over all experts."""
+    experts: int
+    top: int
+    ff: int                  # inner size of one expert
+    groups: int = 1
+    keep: int = 1
+
+    def __post_init__(self) -> None:
+        if self.experts % self.groups or not 0 < self.keep <= self.groups:
+            raise ValueError(f"{self.experts} experts in {self.groups} "
+                             f"groups, {self.keep} kept")
+        if not 0 < self.top <= self.keep * (self.experts // self.groups):
+            raise ValueError(f"top {self.top} of {self.keep} groups of "
+                             f"{self.experts // self.groups} experts")
+
+    def params(self, width: int) -> int:
+        return width * self.experts * (1 + 2 * self.ff)
+
+
+@dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[AttentionSpec, GLASpec]
+    mixer: Union[AttentionSpec, GLASpec, LatentAttentionSpec]
     ff: int = 0              # inner size of the gated feed-forward, 0: none
+    moe: Optional[MoESpec] = None   # experts instead of it
+
+    def params(self, width: int) -> int:
+        return self.mixer.params(width) + 3 * width * self.ff \
+            + (self.moe.params(width) if self.moe else 0)
 
 
 def distance_bucket(n: int, rows: int, furthest: int) -> int:

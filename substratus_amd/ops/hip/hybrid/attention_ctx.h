@@ -9,17 +9,20 @@ struct AttnCtx {
   const T* q;              // row r, head h at q + r * q_ld + h * dim
   const T* gate;           // row r, head h at gate + r * g_ld + h, or null
   const T* kc;             // [blocks, kv_heads, block_size, dim]
-  const T* vc;             // [blocks, kv_heads, block_size, vdim]
+  const T* vc;             // [blocks, kv_heads, block_size, vdim], rows of
+                           // v_ld elements (values may be part of the keys)
   const float* bias;       // [heads, nbias] by distance, or null
   const int* positions;    // [rows]
   const int* seq_start;    // [entries + 1] row offsets, or null: one row each
   const int* block_table;  // [entries, max_blocks]
-  long q_ld, g_ld;
+  long q_ld, g_ld, v_ld;
   int heads, kv_heads, dim, vdim, nbias, chunk, max_blocks, block_size;
   float scale;
 };
 
 constexpr float LOG2E = 1.44269504088896340736f;
+
+constexpr int ATTN_ANY_VDIM = 1024;   // largest value size
 
 template <class T>
 void launch_attn_ctx_any(const AttnCtx<T>&, int entries, int max_len,

@@ -11,7 +11,8 @@
 // (attention_ctx_decode.hip, attention_ctx_prefill.hip) do not take.
 #include "attention_ctx.h"
 
-template <class T>
+// CMAX: value columns per lane
+template <class T, int CMAX>
 __global__ __launch_bounds__(WAVE)
 void attn_ctx_any_kernel(AttnCtx<T> a) {
   extern __shared__ float s_q[];                 // [dim] + [WAVE] weights
@@ -29,7 +30,6 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
   for (int i = lane; i < a.dim; i += WAVE) s_q[i] = ld1(q + i) * a.scale;
   __syncthreads();
 
-  constexpr int CMAX = 8;                        // columns per lane
   float acc[CMAX];
   #pragma unroll
   for (int c = 0; c < CMAX; ++c) acc[c] = 0.f;
@@ -60,7 +60,7 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
       const int kj = k0 + j;
       const long page = bt[kj / a.block_size];
       const T* v = a.vc + ((page * a.kv_heads + kvh) * a.block_size +
-                           kj % a.block_size) * a.vdim;
+                           kj % a.block_size) * a.v_ld;
       const float pj = s_p[j];
       #pragma unroll
       for (int c = 0; c < CMAX; ++c) {
@@ -83,8 +83,13 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
 template <class T>
 void launch_attn_ctx_any(const AttnCtx<T>& a, int entries, int max_len,
                          hipStream_t stream) {
-  attn_ctx_any_kernel<T><<<dim3(max_len, a.heads, entries), dim3(WAVE),
-                           (a.dim + WAVE) * sizeof(float), stream>>>(a);
+  auto go = [&](auto cmax) {
+    attn_ctx_any_kernel<T, decltype(cmax)::value>
+        <<<dim3(max_len, a.heads, entries), dim3(WAVE),
+           (a.dim + WAVE) * sizeof(float), stream>>>(a);
+  };
+  if (a.vdim <= 4 * WAVE) go(std::integral_constant<int, 4>{});
+  else go(std::integral_constant<int, ATTN_ANY_VDIM / WAVE>{});
 }
 
 template void launch_attn_ctx_any<float>(const AttnCtx<float>&, int, int,

@@ -67,7 +67,7 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   auto load = [&](int pg) {
     const long page = (long)bt[pg] * a.kv_heads + kvh;
     const bf16_t* kp = a.kc + (page * PAGE + key) * a.dim;
-    const bf16_t* vp = a.vc + page * PAGE * a.vdim;
+    const bf16_t* vp = a.vc + page * PAGE * a.v_ld;
     #pragma unroll
     for (int i = 0; i < DCH; ++i)
       kr[i] = sub + 4 * i < kch ? nt_load_u4(kp + (sub + 4 * i) * 8)
@@ -75,7 +75,7 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     #pragma unroll
     for (int i = 0; i < NV; ++i)
       vr[i] = col < vch
-          ? nt_load_u4(vp + (long)(rg + RPI * i) * a.vdim + col * 8)
+          ? nt_load_u4(vp + (long)(rg + RPI * i) * a.v_ld + col * 8)
           : (uint4v){0, 0, 0, 0};
     #pragma unroll
     for (int g = 0; g < GQ; ++g) {

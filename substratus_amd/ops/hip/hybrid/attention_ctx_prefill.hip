@@ -134,7 +134,7 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
       if (pgv[i] >= 0 && d < a.vdim)
         st_v[i] = *reinterpret_cast<const uint4*>(
             a.vc + (((long)pgv[i] * a.kv_heads + kvh) * PAGE +
-                    (st * CH + r) % PAGE) * a.vdim + d);
+                    (st * CH + r) % PAGE) * a.v_ld + d);
     }
     if (a.bias != nullptr) {
       const int n = qa0 - (st * CH + CH - 1) + tid;

@@ -7,9 +7,15 @@
 
 #include "attention_ctx.h"
 #include "gla.h"
+#include "group_gemm.h"
 
 template <class T>
-void launch_stream_norm(T*, float*, const T*, const float*, const float*, long, int, float, float, float, hipStream_t);
+void launch_stream_norm(T*, float*, const T*, const int*, const float*, int, const float*, const float*, long, int, float, float, float, float, hipStream_t);
+template <class T>
+void launch_latent_prepare(T*, long, int, int, int, int, int, const float*, float, const double*, int, const int*, T*, const int*, long, hipStream_t);
+int moe_max_experts();
+void launch_moe_select(int*, float*, const float*, int, int, int, int, int, hipStream_t);
+void launch_moe_sort(int*, int*, int*, int*, const int*, int, int, int, int, hipStream_t);
 template <class T>
 void launch_embed_norm(T*, float*, const T*, const int*, const float*, long, int, int, float, float, hipStream_t);
 int stream_norm_max_width(int width);
@@ -62,39 +68,59 @@ void by_type(const Tensor& t, F f) {
   else TORCH_CHECK(false, "activations must be float32 or bfloat16");
 }
 
-void stream_norm(Tensor y, Tensor x, Tensor delta, Tensor w_post, Tensor w_pre,
-                 double off, double eps, double out_scale) {
+// rows [pool, width], picked by at and weights [rows of x, picks], or
+// [rows of x, width] without those
+void stream_norm(Tensor y, Tensor x, Tensor rows, OptTensor at,
+                 OptTensor weights, Tensor w_post, OptTensor w_pre, double off,
+                 double eps, double out_scale, double mult) {
   const int width = x.size(-1);
-  const long rows = x.numel() / width;
+  const long n = x.numel() / width;
   check(x, torch::kFloat32, "x");
   check(w_post, torch::kFloat32, "w_post");
-  check(w_pre, torch::kFloat32, "w_pre");
   TORCH_CHECK(width <= stream_norm_max_width(width), "row too wide");
-  TORCH_CHECK(y.numel() == x.numel() && delta.numel() == x.numel() &&
-              w_post.numel() == width && w_pre.numel() == width,
-              "stream_norm: shapes differ");
-  if (rows == 0) return;
+  TORCH_CHECK(y.numel() == x.numel() && w_post.numel() == width &&
+              rows.size(-1) == width, "stream_norm: shapes differ");
+  if (w_pre) {
+    check(*w_pre, torch::kFloat32, "w_pre");
+    TORCH_CHECK(w_pre->numel() == width, "stream_norm: shapes differ");
+  }
+  TORCH_CHECK(at.has_value() == weights.has_value(), "at needs weights");
+  int picks = 0;
+  if (at) {
+    check(*at, torch::kInt32, "at");
+    check(*weights, torch::kFloat32, "weights");
+    TORCH_CHECK(at->dim() == 2 && at->size(0) == n &&
+                at->sizes() == weights->sizes(), "picks differ");
+    picks = at->size(1);
+  } else {
+    TORCH_CHECK(rows.numel() == x.numel(), "stream_norm: shapes differ");
+  }
+  if (n == 0) return;
   by_type(y, [&](auto tag) {
     using T = decltype(tag);
     check(y, Scalar<T>::type, "y");
-    check(delta, Scalar<T>::type, "delta");
-    launch_stream_norm<T>(ptr<T>(y), ptr<float>(x), ptr<T>(delta),
-                          ptr<float>(w_post), ptr<float>(w_pre), rows, width,
-                          off, eps, out_scale, stream());
+    check(rows, Scalar<T>::type, "delta");
+    launch_stream_norm<T>(ptr<T>(y), ptr<float>(x), ptr<T>(rows), ptr<int>(at),
+                          ptr<float>(weights), picks, ptr<float>(w_post),
+                          ptr<float>(w_pre), n, width, off, eps, out_scale,
+                          mult, stream());
   });
   post("stream_norm");
 }
 
-void embed_norm(Tensor y, Tensor x, Tensor table, Tensor tokens, Tensor w_pre,
-                double off, double eps) {
+void embed_norm(Tensor y, Tensor x, Tensor table, Tensor tokens,
+                OptTensor w_pre, double off, double eps) {
   const int width = table.size(1);
   const long rows = tokens.numel();
   check(x, torch::kFloat32, "x");
   check(tokens, torch::kInt32, "tokens");
-  check(w_pre, torch::kFloat32, "w_pre");
   TORCH_CHECK(width <= stream_norm_max_width(width), "row too wide");
-  TORCH_CHECK(y.numel() == rows * width && x.numel() == rows * width &&
-              w_pre.numel() == width, "embed_norm: shapes differ");
+  TORCH_CHECK(y.numel() == rows * width && x.numel() == rows * width,
+              "embed_norm: shapes differ");
+  if (w_pre) {
+    check(*w_pre, torch::kFloat32, "w_pre");
+    TORCH_CHECK(w_pre->numel() == width, "embed_norm: shapes differ");
+  }
   if (rows == 0) return;
   by_type(y, [&](auto tag) {
     using T = decltype(tag);
@@ -158,7 +184,8 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
   TORCH_CHECK(q.size(1) % dim == 0, "q is not heads * dim wide");
   const int heads = q.size(1) / dim;
   TORCH_CHECK(heads % kv == 0, "query heads must divide by kv heads");
-  TORCH_CHECK(vdim <= 512, "value size over 512");
+  TORCH_CHECK(vdim <= ATTN_ANY_VDIM, "value size over ", ATTN_ANY_VDIM);
+  TORCH_CHECK(dim <= 8192, "key size over 8192");
   TORCH_CHECK(vc.size(0) == kc.size(0) && vc.size(1) == kv &&
               vc.size(2) == kc.size(2), "caches differ");
   TORCH_CHECK(out.size(0) == rows && out.size(1) == heads * vdim,
@@ -183,7 +210,13 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     check_rows(q, Scalar<T>::type, "q");
     check(out, Scalar<T>::type, "out");
     check(kc, Scalar<T>::type, "kc");
-    check(vc, Scalar<T>::type, "vc");
+    // values may be the first columns of wider rows
+    check(vc, Scalar<T>::type, "vc", false);
+    const long v_ld = vc.stride(2);
+    TORCH_CHECK(vc.stride(3) == 1 && v_ld >= vdim &&
+                vc.stride(1) == v_ld * vc.size(2) &&
+                vc.stride(0) == vc.stride(1) * kv,
+                "vc rows must be equally far apart");
     if (gate) {
       check_rows(*gate, Scalar<T>::type, "gate");
       TORCH_CHECK(gate->size(0) == rows && gate->size(1) == heads,
@@ -194,6 +227,7 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     a.kc = ptr<T>(kc); a.vc = ptr<T>(vc); a.bias = ptr<float>(bias);
     a.positions = ptr<int>(positions); a.seq_start = ptr<int>(seq_start);
     a.block_table = ptr<int>(block_table);
+    a.v_ld = v_ld;
     a.q_ld = q.stride(0); a.g_ld = gate ? gate->stride(0) : 0;
     a.heads = heads; a.kv_heads = kv; a.dim = dim; a.vdim = vdim;
     a.nbias = bias ? bias->size(1) : 1; a.chunk = chunk;
@@ -203,6 +237,7 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
       // the tiled kernels read q rows in 16-byte pieces
       const bool aligned = a.q_ld % 8 == 0 &&
           reinterpret_cast<uintptr_t>(a.q) % 16 == 0;
+      any = any || v_ld % 8 != 0;
       if (!any && seq_start && aligned &&
           attn_ctx_prefill_supported(dim, vdim, a.block_size)) {
         launch_attn_ctx_prefill(a, entries, max_len, stream());
@@ -228,6 +263,203 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     launch_attn_ctx_any<T>(a, entries, seq_start ? max_len : 1, stream());
   });
   post("attn_ctx");
+}
+
+// buf rows [queries | ... | latent | key part], the latter from column c_at
+// on, or nowhere (-1); cache [blocks, 1, block, rank + rot_dim]
+void latent_prepare(Tensor buf, int64_t heads, int64_t dim, int64_t rot_dim,
+                    int64_t c_at, OptTensor norm, double eps, Tensor turns,
+                    Tensor positions, Tensor cache, Tensor slots) {
+  const long rows = buf.size(0);
+  const int half = turns.numel(), row = cache.size(3);
+  const int rank = row - rot_dim;
+  check(turns, torch::kFloat64, "turns");
+  check(positions, torch::kInt32, "positions");
+  check(slots, torch::kInt32, "slots");
+  TORCH_CHECK(positions.numel() == rows && slots.numel() == rows,
+              "one position and slot per row");
+  TORCH_CHECK(2 * half <= rot_dim && half <= 4096, "too many turns");
+  TORCH_CHECK(heads * (dim + rot_dim) <= buf.size(1), "buf too narrow");
+  TORCH_CHECK(rank > 0 && cache.size(1) == 1, "cache must hold latents");
+  TORCH_CHECK((c_at >= 0) == norm.has_value(), "latents need their norm");
+  if (norm) {
+    check(*norm, torch::kFloat32, "norm");
+    TORCH_CHECK(norm->numel() == rank, "norm size");
+    TORCH_CHECK(c_at + row <= buf.size(1), "buf too narrow");
+  }
+  if (rows == 0) return;
+  by_type(buf, [&](auto tag) {
+    using T = decltype(tag);
+    check_rows(buf, Scalar<T>::type, "buf");
+    check(cache, Scalar<T>::type, "cache");
+    launch_latent_prepare<T>(ptr<T>(buf), buf.stride(0), heads, dim, rot_dim,
+                             c_at, rank, ptr<float>(norm), eps,
+                             ptr<double>(turns), half, ptr<int>(positions),
+                             ptr<T>(cache), ptr<int>(slots), rows, stream());
+  });
+  post("latent_prepare");
+}
+
+template <class T, class Y>
+void group_gemm(const GroupGemm<T, Y>& a, int tile, const char* op) {
+  TORCH_CHECK(a.tiles == nullptr || group_gemm_takes(a, tile), op,
+              ": tiles of ", tile, " rows");
+  launch_group_gemm<T, Y>(a, tile, stream());
+  post(op);
+}
+
+template <class T, class Y = T>
+GroupGemm<T, Y> product(const Tensor& y, const Tensor& x, const Tensor& w) {
+  GroupGemm<T, Y> a{};
+  check_rows(x, Scalar<T>::type, "x");
+  check(y, Scalar<Y>::type, "y");
+  check(w, Scalar<T>::type, "w");
+  a.y = ptr<Y>(y); a.x = ptr<T>(x); a.w = ptr<T>(w);
+  a.y_ld = y.stride(0); a.x_ld = x.stride(0);
+  a.n = w.size(-2); a.k = w.size(-1);
+  a.groups = w.dim() == 3 ? w.size(0) : 1;
+  a.m = x.size(0);
+  a.act = Act::NONE;
+  return a;
+}
+
+// out [rows, heads, n + tail], x [rows, heads, k + tail] view, w [heads, n, k]
+void head_linear(Tensor out, Tensor x, Tensor w, OptTensor gate,
+                 int64_t tail) {
+  const long rows = x.size(0), heads = w.size(0), n = w.size(1),
+             k = w.size(2);
+  TORCH_CHECK(x.dim() == 3 && x.size(1) == heads && x.size(2) == k + tail &&
+              (x.stride(2) == 1 || x.size(2) == 1) && tail >= 0,
+              "x must be [rows, heads, k + tail]");
+  TORCH_CHECK(out.dim() == 3 && out.size(0) == rows && out.size(1) == heads &&
+              out.size(2) == n + tail, "out must be [rows, heads, n + tail]");
+  if (gate)
+    TORCH_CHECK(gate->size(0) == rows && gate->size(1) == heads * n,
+                "gate must be [rows, heads * n]");
+  if (rows == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    check(x, Scalar<T>::type, "x", false);
+    check(w, Scalar<T>::type, "w");
+    check(out, Scalar<T>::type, "out");
+    GroupGemm<T, T> a{};
+    a.y = ptr<T>(out); a.x = ptr<T>(x); a.w = ptr<T>(w);
+    a.y_ld = heads * (n + tail); a.y_gs = n + tail;
+    a.x_ld = x.stride(0); a.x_gs = x.stride(1);
+    a.m = rows; a.n = n; a.k = k; a.groups = heads; a.tail = tail;
+    a.act = Act::NONE;
+    if (gate) {
+      check_rows(*gate, Scalar<T>::type, "gate");
+      a.act = Act::GATE;
+      a.gate = ptr<T>(gate); a.gate_ld = gate->stride(0); a.gate_gs = n;
+    }
+    group_gemm(a, group_gemm_tile(rows, 1, std::is_same_v<T, bf16_t>, k, 8),
+               "head_linear");
+  });
+}
+
+// z [rows, experts] in float32
+void router_scores(Tensor z, Tensor x, Tensor w) {
+  TORCH_CHECK(x.size(1) == w.size(1) && z.size(0) == x.size(0) &&
+              z.size(1) == w.size(0), "router_scores: shapes differ");
+  if (x.size(0) == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    group_gemm(product<T, float>(z, x, w),
+               group_gemm_tile(x.size(0), 1, std::is_same_v<T, bf16_t>,
+                               w.size(1), 8), "router_scores");
+  });
+}
+
+// gelu_tanh(x w^T) * table[tokens, t_at : t_at + n]
+void side_gate(Tensor out, Tensor x, Tensor w, Tensor tokens, Tensor table,
+               int64_t t_at) {
+  check(tokens, torch::kInt32, "tokens");
+  TORCH_CHECK(x.size(1) == w.size(1) && out.size(0) == x.size(0) &&
+              out.size(1) == w.size(0) && tokens.numel() == x.size(0),
+              "side_gate: shapes differ");
+  TORCH_CHECK(t_at >= 0 && t_at + w.size(0) <= table.size(1),
+              "table too narrow");
+  if (x.size(0) == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    check(table, Scalar<T>::type, "table");
+    auto a = product<T>(out, x, w);
+    a.act = Act::SIDE;
+    a.tokens = ptr<int>(tokens); a.table = ptr<T>(table) + t_at;
+    a.t_ld = table.stride(0); a.vocab = table.size(0);
+    group_gemm(a, group_gemm_tile(x.size(0), 1, std::is_same_v<T, bf16_t>,
+                                  w.size(1), 8), "side_gate");
+  });
+}
+
+void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
+                int64_t keep) {
+  const long rows = z.size(0), experts = z.size(1), top = ids.size(1);
+  check(ids, torch::kInt32, "ids");
+  check(weights, torch::kFloat32, "weights");
+  check(z, torch::kFloat32, "z");
+  TORCH_CHECK(ids.size(0) == rows && ids.sizes() == weights.sizes(),
+              "moe_select: shapes differ");
+  TORCH_CHECK(experts <= moe_max_experts(), "too many experts");
+  TORCH_CHECK(groups > 0 && experts % groups == 0 && keep > 0 &&
+              keep <= groups && top > 0 && top <= experts / groups * keep,
+              "moe_select: cannot choose so many");
+  if (rows == 0) return;
+  launch_moe_select(ptr<int>(ids), ptr<float>(weights), ptr<float>(z), rows,
+                    experts, top, groups, keep, stream());
+  post("moe_select");
+}
+
+int64_t moe_tile(int64_t packed, int64_t experts, bool bf16, int64_t k,
+                 int64_t n) {
+  return group_gemm_tile(packed, experts, bf16, k, n);
+}
+
+// tiles: [1 + 2 * bound], of which each expert's last may be short
+void moe_sort(Tensor at, Tensor src, Tensor start, Tensor tiles, Tensor ids,
+              int64_t tile) {
+  const long n = ids.numel(), experts = start.numel() - 1;
+  for (const Tensor* t : {&at, &src, &start, &tiles, &ids})
+    check(*t, torch::kInt32, "moe_sort tensors");
+  TORCH_CHECK(at.numel() == n && src.numel() == n && tile > 0 &&
+              experts > 0 && experts <= moe_max_experts(),
+              "moe_sort: shapes differ");
+  TORCH_CHECK(tiles.numel() >= 1 + 2 * ((n + tile - 1) / tile +
+                                        std::min(experts, n)),
+              "moe_sort: room for too few tiles");
+  if (n == 0) return;
+  launch_moe_sort(ptr<int>(at), ptr<int>(src), ptr<int>(start),
+                  ptr<int>(tiles), ptr<int>(ids), n, ids.size(-1), experts,
+                  tile, stream());
+  post("moe_sort");
+}
+
+// Every packed row by its expert's matrix: out [packed, n], w [experts, n, k];
+// packed row r is row src[r] of x, or row r.
+void expert_linear(Tensor out, Tensor x, Tensor w, OptTensor src,
+                   Tensor start, Tensor tiles, int64_t tile, bool gelu) {
+  check(start, torch::kInt32, "start");
+  check(tiles, torch::kInt32, "tiles");
+  TORCH_CHECK(w.dim() == 3 && start.numel() == w.size(0) + 1 &&
+              x.size(1) == w.size(2) && out.size(1) == w.size(1),
+              "expert_linear: shapes differ");
+  if (src) {
+    check(*src, torch::kInt32, "src");
+    TORCH_CHECK(src->numel() == out.size(0), "one source per row");
+  } else {
+    TORCH_CHECK(x.size(0) == out.size(0), "expert_linear: rows differ");
+  }
+  if (out.size(0) == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    auto a = product<T>(out, x, w);
+    a.m = out.size(0);
+    a.src = ptr<int>(src); a.start = ptr<int>(start);
+    a.tiles = ptr<int>(tiles); a.max_tiles = (tiles.numel() - 1) / 2;
+    if (gelu) a.act = Act::GELU;
+    group_gemm(a, tile, "expert_linear");
+  });
 }
 
 // x [rows, >= q | k | v | g | A1 h]; state [slots, heads, dim, vdim]
@@ -325,4 +557,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_ctx", &attn_ctx);
   m.def("gla", &gla);
   m.def("silu_mul", &silu_mul);
+  m.def("latent_prepare", &latent_prepare);
+  m.def("head_linear", &head_linear);
+  m.def("router_scores", &router_scores);
+  m.def("side_gate", &side_gate);
+  m.def("moe_select", &moe_select);
+  m.def("moe_tile", &moe_tile);
+  m.def("moe_sort", &moe_sort);
+  m.def("expert_linear", &expert_linear);
 }

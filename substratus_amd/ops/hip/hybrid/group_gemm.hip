@@ -1,0 +1,212 @@
+// Grouped products (group_gemm.h), two kernels:
+//
+//   stream   bf16, few rows per group: bound by reading the weights once.
+//            Every wave takes a share of the inner dimension of a tile of
+//            BM rows and 64 columns, with both operands going from memory
+//            straight into the matrix cores' registers (a fragment is 16
+//            consecutive bytes of a row, so nothing is gained by LDS); there
+//            is no barrier until the four partial tiles are added up.
+//   any      float, and bf16 sizes whose rows are not 16-byte pieces.
+//
+// Weights are the first operand, so a lane ends up with four consecutive
+// columns of one row and stores them together.
+#include "group_gemm.h"
+
+namespace {
+
+typedef __attribute__((ext_vector_type(8))) short short8;
+typedef __attribute__((ext_vector_type(4))) float float4v;
+
+constexpr int NW = 4;          // waves: shares of the inner dimension
+constexpr int BN = 64;
+constexpr int KC = 32;         // inner step of one matrix instruction
+
+DEV_INLINE short8 frag(const bf16_t* p, bool there) {
+  return there ? *reinterpret_cast<const short8*>(p)
+               : (short8){0, 0, 0, 0, 0, 0, 0, 0};
+}
+
+template <class Y, int FM>
+__global__ __launch_bounds__(NW * WAVE)
+void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
+  constexpr int BM = FM * 16, FN = BN / 16, PAD = 4;
+  __shared__ alignas(16) float s_p[NW][BM][BN + PAD];
+  const Tile t = tile_of(a, blockIdx.y, blockIdx.z, BM);
+  if (t.r1 <= t.r0) return;
+  const int n0 = blockIdx.x * BN;
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  const int lo = lane & 15, kq = (lane >> 4) * 8;
+
+  const bf16_t* wp[FN];
+  const bf16_t* xp[FM];
+  #pragma unroll
+  for (int f = 0; f < FN; ++f)      // past the last column: computed, dropped
+    wp[f] = a.w + ((long)t.g * a.n + min(n0 + f * 16 + lo, a.n - 1)) * a.k +
+            kq;
+  #pragma unroll
+  for (int f = 0; f < FM; ++f) {
+    const int r = min(t.r0 + f * 16 + lo, t.r1 - 1);
+    xp[f] = a.x + (long)(a.src != nullptr ? a.src[r] : r) * a.x_ld +
+            t.g * a.x_gs + kq;
+  }
+  float4v acc[FN][FM];
+  #pragma unroll
+  for (int i = 0; i < FN; ++i)
+    #pragma unroll
+    for (int j = 0; j < FM; ++j) acc[i][j] = (float4v){0.f, 0.f, 0.f, 0.f};
+
+  const int chunks = (a.k + KC - 1) / KC;
+  const int c0 = chunks * wave / NW, c1 = chunks * (wave + 1) / NW;
+  auto step = [&](int c, bool whole) {
+    const int k = c * KC;
+    short8 wf[FN], xf[FM];
+    #pragma unroll
+    for (int f = 0; f < FN; ++f) wf[f] = frag(wp[f] + k, whole || k + kq < a.k);
+    #pragma unroll
+    for (int f = 0; f < FM; ++f) xf[f] = frag(xp[f] + k, whole || k + kq < a.k);
+    #pragma unroll
+    for (int i = 0; i < FN; ++i)
+      #pragma unroll
+      for (int j = 0; j < FM; ++j)
+        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j],
+                                                            acc[i][j], 0, 0, 0);
+  };
+  const int full = min(c1, a.k / KC);
+  int c = c0;
+  #pragma unroll 4
+  for (; c < full; ++c) step(c, true);
+  for (; c < c1; ++c) step(c, false);
+
+  #pragma unroll
+  for (int i = 0; i < FN; ++i)
+    #pragma unroll
+    for (int j = 0; j < FM; ++j)
+      *reinterpret_cast<float4v*>(
+          &s_p[wave][j * 16 + lo][i * 16 + (lane >> 4) * 4]) = acc[i][j];
+  __syncthreads();
+  const bool quads = a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0;
+  for (int i = threadIdx.x; i < BM * BN / 4; i += NW * WAVE) {
+    const int r = t.r0 + i / (BN / 4), c4 = i % (BN / 4) * 4, n = n0 + c4;
+    if (r >= t.r1 || n >= a.n) continue;
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+    #pragma unroll
+    for (int w = 0; w < NW; ++w) {
+      const float4v p =
+          *reinterpret_cast<const float4v*>(&s_p[w][r - t.r0][c4]);
+      #pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] += p[j];
+    }
+    #pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (n + j < a.n) v[j] = group_act(a, r, t.g, n + j, v[j]);
+    Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n;
+    if (quads) {
+      stv<4>(y, v);
+    } else {
+      #pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (n + j < a.n) st1(y + j, v[j]);
+    }
+  }
+  if (a.tail && blockIdx.x == 0) copy_tail(a, t, threadIdx.x, NW * WAVE);
+}
+
+// 32 x 32 outputs per workgroup, 2 x 2 per thread, operands through LDS.
+constexpr int AT = 32, AK = 16;
+
+template <class T, class Y>
+__global__ __launch_bounds__(256)
+void group_gemm_any_kernel(GroupGemm<T, Y> a) {
+  __shared__ float s_x[AK][AT + 1], s_w[AK][AT + 1];
+  const Tile t = tile_of(a, blockIdx.y, blockIdx.z, AT);
+  if (t.r1 <= t.r0) return;
+  const int n0 = blockIdx.x * AT;
+  const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
+  float acc[2][2] = {{0.f, 0.f}, {0.f, 0.f}};
+  for (int k0 = 0; k0 < a.k; k0 += AK) {
+    for (int i = threadIdx.x; i < AT * AK; i += 256) {
+      const int r = t.r0 + i / AK, n = n0 + i / AK, k = k0 + i % AK;
+      const bool in = k < a.k;
+      s_x[i % AK][i / AK] = in && r < t.r1
+          ? ld1(a.x + (long)(a.src != nullptr ? a.src[r] : r) * a.x_ld +
+                t.g * a.x_gs + k) : 0.f;
+      s_w[i % AK][i / AK] = in && n < a.n
+          ? ld1(a.w + ((long)t.g * a.n + n) * a.k + k) : 0.f;
+    }
+    __syncthreads();
+    #pragma unroll
+    for (int k = 0; k < AK; ++k)
+      #pragma unroll
+      for (int i = 0; i < 2; ++i)
+        #pragma unroll
+        for (int j = 0; j < 2; ++j)
+          acc[i][j] += s_x[k][ty + 16 * i] * s_w[k][tx + 16 * j];
+    __syncthreads();
+  }
+  #pragma unroll
+  for (int i = 0; i < 2; ++i)
+    #pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int r = t.r0 + ty + 16 * i, n = n0 + tx + 16 * j;
+      if (r < t.r1 && n < a.n)
+        st1(a.y + (long)r * a.y_ld + t.g * a.y_gs + n,
+            group_act(a, r, t.g, n, acc[i][j]));
+    }
+  if (a.tail && blockIdx.x == 0) copy_tail(a, t, threadIdx.x, 256);
+}
+
+// rows of both operands are whole, aligned 16-byte pieces
+template <class Y>
+bool pieces(const GroupGemm<bf16_t, Y>& a) {
+  auto ok = [](const void* p) {
+    return reinterpret_cast<uintptr_t>(p) % 16 == 0;
+  };
+  return a.k % 8 == 0 && a.x_ld % 8 == 0 && a.x_gs % 8 == 0 && ok(a.x) &&
+         ok(a.w);
+}
+
+}  // namespace
+
+int group_gemm_tile(long rows, int groups, bool bf16, int k, int n) {
+  if (!bf16 || k % 8 || n % 8) return AT;
+  const long per = rows / groups;
+  return per <= 16 ? 16 : per <= 48 ? 32 : 64;
+}
+
+template <class T, class Y>
+bool group_gemm_takes(const GroupGemm<T, Y>& a, int tile) {
+  if constexpr (std::is_same_v<T, bf16_t>)
+    if (pieces(a) && (tile == 16 || tile == 32 || tile == 64)) return true;
+  return tile == AT;
+}
+
+template <class T, class Y>
+void launch_group_gemm(const GroupGemm<T, Y>& a, int tile,
+                       hipStream_t stream) {
+  const bool packed = a.tiles != nullptr;
+  const int mt = packed ? a.max_tiles : (a.m + tile - 1) / tile;
+  const int gz = packed ? 1 : a.groups;
+  if constexpr (std::is_same_v<T, bf16_t>) {
+    if (pieces(a) && (tile == 16 || tile == 32 || tile == 64)) {
+      const dim3 grid((a.n + BN - 1) / BN, mt, gz), block(NW * WAVE);
+      if (tile == 16)
+        group_gemm_stream_kernel<Y, 1><<<grid, block, 0, stream>>>(a);
+      else if (tile == 32)
+        group_gemm_stream_kernel<Y, 2><<<grid, block, 0, stream>>>(a);
+      else
+        group_gemm_stream_kernel<Y, 4><<<grid, block, 0, stream>>>(a);
+      return;
+    }
+  }
+  const int rows = packed ? mt : (a.m + AT - 1) / AT;
+  group_gemm_any_kernel<T, Y><<<dim3((a.n + AT - 1) / AT, rows, gz), 256, 0,
+                                stream>>>(a);
+}
+
+#define INSTANTIATE(T, Y)                                                    \
+  template bool group_gemm_takes<T, Y>(const GroupGemm<T, Y>&, int);         \
+  template void launch_group_gemm<T, Y>(const GroupGemm<T, Y>&, int,         \
+                                        hipStream_t);
+INSTANTIATE(float, float)
+INSTANTIATE(bf16_t, bf16_t)
+INSTANTIATE(bf16_t, float)

@@ -1,0 +1,90 @@
+// Everything between a latent-attention layer's input projection and its
+// scores, in one pass over the projected row of each token:
+//   * the rotated part of every query head, in place,
+//   * the RMS-normed latent and the rotated key part, to the paged cache
+//     (layers that use another one's latents have neither).
+// Row layout: [queries, head by head: dim | rot_dim][...][latent | key part].
+//
+// Element i of a rotated part turns with element i + half. Angles are formed
+// as turns in 64 bits, whole turns dropped, so that positions far away are as
+// exact as near ones.
+#include "typed.h"
+
+namespace {
+
+constexpr int BLOCK = 256;
+
+template <class T>
+__global__ __launch_bounds__(BLOCK)
+void latent_prepare_kernel(T* __restrict__ buf, long ld, int heads, int dim,
+                           int rot_dim, int c_at, int rank,
+                           const float* __restrict__ norm, float eps,
+                           const double* __restrict__ turns, int half,
+                           const int* __restrict__ positions,
+                           T* __restrict__ cache, const int* __restrict__ slots) {
+  extern __shared__ float s_cs[];               // cos, sin of every pair
+  __shared__ float scratch[BLOCK / WAVE];
+  const long row = blockIdx.x;
+  T* q = buf + row * ld;
+  const double pos = positions[row];
+  for (int i = threadIdx.x; i < half; i += BLOCK) {
+    double t = pos * turns[i];
+    t -= rint(t);
+    float s, c;
+    sincospif((float)(2.0 * t), &s, &c);
+    s_cs[2 * i] = c;
+    s_cs[2 * i + 1] = s;
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < heads * half; i += BLOCK) {
+    const int h = i / half, j = i % half;
+    T* p = q + (long)h * (dim + rot_dim) + dim + j;
+    const float u = ld1(p), v = ld1(p + half);
+    const float c = s_cs[2 * j], s = s_cs[2 * j + 1];
+    st1(p, u * c - v * s);
+    st1(p + half, v * c + u * s);
+  }
+  if (c_at < 0) return;
+  const T* lat = q + c_at;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < rank; i += BLOCK) {
+    const float f = ld1(lat + i);
+    ss += f * f;
+  }
+  ss = block_sum<BLOCK / WAVE>(ss, scratch);
+  const float inv = 1.f / sqrtf(ss / (float)rank + eps);
+  T* out = cache + (long)slots[row] * (rank + rot_dim);
+  for (int i = threadIdx.x; i < rank; i += BLOCK)
+    st1(out + i, ld1(lat + i) * inv * norm[i]);
+  for (int j = threadIdx.x; j < rot_dim; j += BLOCK) {
+    const float x = ld1(lat + rank + j);
+    float y = x;
+    if (j < half)
+      y = x * s_cs[2 * j] - ld1(lat + rank + j + half) * s_cs[2 * j + 1];
+    else if (j < 2 * half)
+      y = x * s_cs[2 * (j - half)] +
+          ld1(lat + rank + j - half) * s_cs[2 * (j - half) + 1];
+    st1(out + rank + j, y);
+  }
+}
+
+}  // namespace
+
+template <class T>
+void launch_latent_prepare(T* buf, long ld, int heads, int dim, int rot_dim,
+                           int c_at, int rank, const float* norm, float eps,
+                           const double* turns, int half, const int* positions,
+                           T* cache, const int* slots, long rows,
+                           hipStream_t stream) {
+  latent_prepare_kernel<T><<<dim3(rows), dim3(BLOCK),
+                             2 * half * sizeof(float), stream>>>(
+      buf, ld, heads, dim, rot_dim, c_at, rank, norm, eps, turns, half,
+      positions, cache, slots);
+}
+
+template void launch_latent_prepare<float>(float*, long, int, int, int, int,
+    int, const float*, float, const double*, int, const int*, float*,
+    const int*, long, hipStream_t);
+template void launch_latent_prepare<bf16_t>(bf16_t*, long, int, int, int, int,
+    int, const float*, float, const double*, int, const int*, bf16_t*,
+    const int*, long, hipStream_t);

@@ -1,7 +1,11 @@
 // Norms of a 32-bit residual stream, fused with what surrounds them.
 //
-//   stream_norm   x += rms(delta) * (off + w_post);  y = rms(x) * (off + w_pre)
-//   embed_norm    x  = table[token];                 y = rms(x) * (off + w_pre)
+//   stream_norm   x += mult * rms(delta) * (off + w_post)
+//                 y  = rms(x) * (off + w_pre)
+//   embed_norm    x  = table[token];   y = rms(x) * (off + w_pre)
+//
+// Without w_pre, y is x. delta is a row per token, or the weighted sum of
+// `picks` rows of a pool (what a mixture of experts adds), formed on the way.
 //
 // with rms(z) = z / sqrt(mean(z^2) + eps). A block that norms both before and
 // after its sublayer needs exactly one of these between two matrix products:
@@ -10,15 +14,21 @@
 // out_scale multiplies y (a logit scale folds in here, in 32 bits).
 #include "typed.h"
 
-template <class T, int VEC, int BLOCK, bool EMBED>
+enum Source { EMBED, ROW, PICKED };
+
+template <class T, int VEC, int BLOCK, Source SRC>
 __global__ __launch_bounds__(BLOCK)
 void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
                         const T* __restrict__ delta,     // [rows, width]
+                        const int* __restrict__ at,      // [rows, picks]
+                        const float* __restrict__ wt,    // [rows, picks]
+                        int picks,
                         const T* __restrict__ table,     // [vocab, width]
                         const int* __restrict__ tokens,  // [rows]
                         const float* __restrict__ w_post,
                         const float* __restrict__ w_pre, int width, int vocab,
-                        float off, float eps, float out_scale) {
+                        float off, float eps, float out_scale,
+                        float mult) {
   constexpr int RCAP = 8;   // vectors per thread; the launcher checks the row
   __shared__ float scratch[2][BLOCK / WAVE];
   const long row = blockIdx.x;
@@ -27,7 +37,7 @@ void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
   float xk[RCAP][VEC];
   const float inv_n = 1.f / (float)width;
 
-  if constexpr (EMBED) {
+  if constexpr (SRC == EMBED) {
     const int tok = min(max(tokens[row], 0), vocab - 1);
     const T* src = table + (long)tok * width;
     #pragma unroll
@@ -44,13 +54,25 @@ void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
     for (int kk = 0; kk < RCAP; ++kk) {
       const int i = threadIdx.x + kk * BLOCK;
       if (i >= nvec) break;
-      ldv<VEC>(dr + i * VEC, dk[kk]);
+      if constexpr (SRC == ROW) {
+        ldv<VEC>(dr + i * VEC, dk[kk]);
+      } else {
+        #pragma unroll
+        for (int j = 0; j < VEC; ++j) dk[kk][j] = 0.f;
+        for (int p = 0; p < picks; ++p) {
+          float f[VEC];
+          ldv<VEC>(delta + (long)at[row * picks + p] * width + i * VEC, f);
+          const float w = wt[row * picks + p];
+          #pragma unroll
+          for (int j = 0; j < VEC; ++j) dk[kk][j] += w * f[j];
+        }
+      }
       ldv<VEC>(xr + i * VEC, xk[kk]);
       #pragma unroll
       for (int j = 0; j < VEC; ++j) ss += dk[kk][j] * dk[kk][j];
     }
     ss = block_sum<BLOCK / WAVE>(ss, scratch[0]);
-    const float inv = 1.f / sqrtf(ss * inv_n + eps);
+    const float inv = mult / sqrtf(ss * inv_n + eps);
     #pragma unroll
     for (int kk = 0; kk < RCAP; ++kk) {
       const int i = threadIdx.x + kk * BLOCK;
@@ -63,18 +85,20 @@ void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
     }
   }
 
+  T* yr = y + row * width;
   float ss = 0.f;
   #pragma unroll
   for (int kk = 0; kk < RCAP; ++kk) {
     const int i = threadIdx.x + kk * BLOCK;
     if (i >= nvec) break;
     stv<VEC>(xr + i * VEC, xk[kk]);
+    if (w_pre == nullptr) stv<VEC>(yr + i * VEC, xk[kk]);
     #pragma unroll
     for (int j = 0; j < VEC; ++j) ss += xk[kk][j] * xk[kk][j];
   }
+  if (w_pre == nullptr) return;
   ss = block_sum<BLOCK / WAVE>(ss, scratch[1]);
   const float inv = out_scale / sqrtf(ss * inv_n + eps);
-  T* yr = y + row * width;
   #pragma unroll
   for (int kk = 0; kk < RCAP; ++kk) {
     const int i = threadIdx.x + kk * BLOCK;
@@ -91,16 +115,17 @@ int stream_norm_max_width(int width) {
   return 1024 * 8 * (width % 4 == 0 ? 4 : 1);
 }
 
-template <class T, bool EMBED>
-static void launch(T* y, float* x, const T* delta, const T* table,
+template <class T, Source SRC>
+static void launch(T* y, float* x, const T* delta, const int* at,
+                   const float* wt, int picks, const T* table,
                    const int* tokens, const float* w_post, const float* w_pre,
                    long rows, int width, int vocab, float off, float eps,
-                   float out_scale, hipStream_t stream) {
+                   float out_scale, float mult, hipStream_t stream) {
   auto go = [&](auto vec, auto block) {
     constexpr int V = decltype(vec)::value, B = decltype(block)::value;
-    stream_norm_kernel<T, V, B, EMBED><<<dim3(rows), dim3(B), 0, stream>>>(
-        y, x, delta, table, tokens, w_post, w_pre, width, vocab, off, eps,
-        out_scale);
+    stream_norm_kernel<T, V, B, SRC><<<dim3(rows), dim3(B), 0, stream>>>(
+        y, x, delta, at, wt, picks, table, tokens, w_post, w_pre, width,
+        vocab, off, eps, out_scale, mult);
   };
   using std::integral_constant;
   auto by_block = [&](auto vec) {
@@ -113,27 +138,35 @@ static void launch(T* y, float* x, const T* delta, const T* table,
   else by_block(integral_constant<int, 1>{});
 }
 
+// at, wt null: delta is [rows, width]
 template <class T>
-void launch_stream_norm(T* y, float* x, const T* delta, const float* w_post,
+void launch_stream_norm(T* y, float* x, const T* delta, const int* at,
+                        const float* wt, int picks, const float* w_post,
                         const float* w_pre, long rows, int width, float off,
-                        float eps, float out_scale, hipStream_t stream) {
-  launch<T, false>(y, x, delta, nullptr, nullptr, w_post, w_pre, rows, width,
-                   0, off, eps, out_scale, stream);
+                        float eps, float out_scale, float mult,
+                        hipStream_t stream) {
+  if (at == nullptr)
+    launch<T, ROW>(y, x, delta, at, wt, picks, nullptr, nullptr, w_post,
+                   w_pre, rows, width, 0, off, eps, out_scale, mult, stream);
+  else
+    launch<T, PICKED>(y, x, delta, at, wt, picks, nullptr, nullptr, w_post,
+                      w_pre, rows, width, 0, off, eps, out_scale, mult,
+                      stream);
 }
 
 template <class T>
 void launch_embed_norm(T* y, float* x, const T* table, const int* tokens,
                        const float* w_pre, long rows, int width, int vocab,
                        float off, float eps, hipStream_t stream) {
-  launch<T, true>(y, x, nullptr, table, tokens, nullptr, w_pre, rows, width,
-                  vocab, off, eps, 1.f, stream);
+  launch<T, EMBED>(y, x, nullptr, nullptr, nullptr, 0, table, tokens, nullptr,
+                   w_pre, rows, width, vocab, off, eps, 1.f, 1.f, stream);
 }
 
-template void launch_stream_norm<float>(float*, float*, const float*,
-    const float*, const float*, long, int, float, float, float, hipStream_t);
-template void launch_stream_norm<bf16_t>(bf16_t*, float*, const bf16_t*,
-    const float*, const float*, long, int, float, float, float, hipStream_t);
-template void launch_embed_norm<float>(float*, float*, const float*,
-    const int*, const float*, long, int, int, float, float, hipStream_t);
-template void launch_embed_norm<bf16_t>(bf16_t*, float*, const bf16_t*,
-    const int*, const float*, long, int, int, float, float, hipStream_t);
+#define INSTANTIATE(T)                                                        \
+  template void launch_stream_norm<T>(T*, float*, const T*, const int*,       \
+      const float*, int, const float*, const float*, long, int, float, float, \
+      float, float, hipStream_t);                                             \
+  template void launch_embed_norm<T>(T*, float*, const T*, const int*,        \
+      const float*, long, int, int, float, float, hipStream_t);
+INSTANTIATE(float)
+INSTANTIATE(bf16_t)

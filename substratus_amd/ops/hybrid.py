@@ -1,7 +1,7 @@
 """Ops of models whose layers differ from one another (models/hybrid.py):
 norms around a 32-bit residual, attention that reads the paged cache for
-single tokens and prompt portions alike, gated linear attention with a
-recurrent state per request.
+single tokens and prompt portions alike, attention over a cache of latents,
+gated linear attention with a recurrent state per request, mixtures of experts.
 
 Same policy as the rest of ops: GPU tensors need the HIP extension
 (substratus_amd._hybrid), CPU tensors run the plain implementations in ref.py.
@@ -11,7 +11,7 @@ weights and recurrent state are always float32.
 
 from __future__ import annotations
 
-from typing import Optional
+from typing import NamedTuple, Optional, Union
 
 import torch
 
@@ -34,22 +34,36 @@ def _ext():
     return _EXT
 
 
-def stream_norm(delta: torch.Tensor, x: torch.Tensor, w_post: torch.Tensor,
-                w_pre: torch.Tensor, offset: float, eps: float,
-                out_scale: float = 1.0) -> torch.Tensor:
-    """x += rms(delta) * (offset + w_post) in place; returns
-    rms(x) * (offset + w_pre) * out_scale in delta's dtype."""
+class Picked(NamedTuple):
+    """Rows of a sum: token t has sum_k weights[t, k] * rows[at[t, k]]."""
+    rows: torch.Tensor       # [packed, width]
+    at: torch.Tensor         # [tokens, k] int32
+    weights: torch.Tensor    # [tokens, k] float32
+
+
+def stream_norm(delta: Union[torch.Tensor, Picked], x: torch.Tensor,
+                w_post: torch.Tensor, w_pre: Optional[torch.Tensor],
+                offset: float, eps: float, out_scale: float = 1.0,
+                mult: float = 1.0) -> torch.Tensor:
+    """x += mult * rms(delta) * (offset + w_post) in place; returns
+    rms(x) * (offset + w_pre) * out_scale in delta's dtype, or without w_pre
+    x itself."""
+    rows, at, weights = delta if isinstance(delta, Picked) \
+        else (delta, None, None)
     if not x.is_cuda:
-        return ref.stream_norm(delta, x, w_post, w_pre, offset, eps, out_scale)
-    y = torch.empty_like(delta)
-    _ext().stream_norm(y, x, delta, w_post, w_pre, offset, eps, out_scale)
+        return ref.stream_norm(rows, at, weights, x, w_post, w_pre, offset,
+                               eps, out_scale, mult)
+    y = torch.empty(x.shape, dtype=rows.dtype, device=x.device)
+    _ext().stream_norm(y, x, rows, at, weights, w_post, w_pre, offset, eps,
+                       out_scale, mult)
     return y
 
 
-def embed_norm(tokens: torch.Tensor, table: torch.Tensor, w_pre: torch.Tensor,
-               offset: float, eps: float) -> tuple[torch.Tensor, torch.Tensor]:
-    """x = table[tokens] (float32) and rms(x) * (offset + w_pre) in the
-    table's dtype; tokens int32."""
+def embed_norm(tokens: torch.Tensor, table: torch.Tensor,
+               w_pre: Optional[torch.Tensor], offset: float,
+               eps: float) -> tuple[torch.Tensor, torch.Tensor]:
+    """x = table[tokens] (float32) and rms(x) * (offset + w_pre), or without
+    w_pre x itself, in the table's dtype; tokens int32."""
     if not table.is_cuda:
         return ref.embed_norm(tokens, table, w_pre, offset, eps)
     shape = (tokens.shape[0], table.shape[1])
@@ -93,6 +107,105 @@ def attn_ctx(q: torch.Tensor, gate: Optional[torch.Tensor],
         fn(out[rows], q[rows], None if gate is None else gate[rows], k_cache,
            v_cache, bias, batch.positions[rows], seq_start,
            batch.block_table[ents], scale, chunk, max_len, span, any_size)
+    return out
+
+
+def latent_prepare(buf: torch.Tensor, spec, c_at: int,
+                   norm: Optional[torch.Tensor], eps: float,
+                   turns: torch.Tensor, positions: torch.Tensor,
+                   cache: torch.Tensor, slots: torch.Tensor) -> None:
+    """buf rows begin with queries, head by head [dim, rot_dim], and have
+    [latent, rotated key part] from column c_at on (-1: not). Rotates the
+    queries in place, writes the normed latent and the rotated key part to
+    the cache."""
+    fn = _ext().latent_prepare if buf.is_cuda else ref.latent_prepare
+    fn(buf, spec.heads, spec.dim, spec.rot_dim, c_at, norm, eps, turns,
+       positions, cache, slots)
+
+
+def head_linear(x: torch.Tensor, w: torch.Tensor,
+                gate: Optional[torch.Tensor] = None,
+                tail: int = 0) -> torch.Tensor:
+    """Per head h: x[:, h, :k] @ w[h].T, times sigmoid(gate) if there is one;
+    the `tail` elements that follow in x are appended as they are.
+
+    x [rows, heads, k + tail] may be a view of wider rows; w [heads, n, k];
+    gate [rows, heads * n]. Returns [rows, heads, n + tail]."""
+    out = x.new_empty(x.shape[0], w.shape[0], w.shape[1] + tail)
+    (_ext() if x.is_cuda else ref).head_linear(out, x, w, gate, tail)
+    return out
+
+
+def _latent_absorbed(out, q, gate, cache, w_uv, uk_t, batch, rows, ents,
+                     seq_start, max_len, spec) -> None:
+    """Queries are moved into the latent space, where all heads attend to one
+    key per token; what they find is expanded to values afterwards."""
+    n = q.shape[0]
+    qa = head_linear(q.view(n, spec.heads, spec.dim + spec.rot_dim), uk_t,
+                     tail=spec.rot_dim)
+    o = q.new_empty(n, spec.heads * spec.rank)
+    fn = _ext().attn_ctx if q.is_cuda else ref.attn_ctx
+    fn(o, qa.view(n, -1), None, cache, cache[..., :spec.rank], None,
+       batch.positions[rows], seq_start, batch.block_table[ents], spec.scale,
+       0, max_len, batch.max_context, False)
+    out[rows] = head_linear(o.view(n, spec.heads, spec.rank), w_uv,
+                            gate).view(n, -1)
+
+
+def latent_attn(q: torch.Tensor, gate: Optional[torch.Tensor],
+                cache: torch.Tensor, w_ukv: torch.Tensor, uk_t: torch.Tensor,
+                batch, spec, shared: dict) -> torch.Tensor:
+    """Latent attention of a batch's rows over the paged cache, which already
+    holds their own latents. q [rows, heads * (dim + rot_dim)] is rotated;
+    gate [rows, heads * vdim]; w_ukv has the rows that make all heads' keys,
+    then those that make their values; uk_t is the former as [heads, rank,
+    dim]."""
+    out = q.new_empty(q.shape[0], spec.heads * spec.vdim)
+    w_uv = w_ukv[spec.heads * spec.dim:].view(spec.heads, spec.vdim, spec.rank)
+    for rows, ents, seq_start, max_len in batch.parts():
+        _latent_absorbed(out, q[rows], None if gate is None else gate[rows],
+                         cache, w_uv, uk_t, batch, rows, ents, seq_start,
+                         max_len, spec)
+    return out
+
+
+def experts(y: torch.Tensor, router: torch.Tensor, up: torch.Tensor,
+            down: torch.Tensor, spec) -> Picked:
+    """A mixture of experts: y [rows, width], router [experts, width], up
+    [experts, ff, width], down [experts, width, ff]. Scores are 32-bit."""
+    rows = y.shape[0]
+    if not y.is_cuda:
+        return Picked(*ref.experts(y, router, up, down, spec.top, spec.groups,
+                                   spec.keep))
+    ext = _ext()
+    i32 = dict(dtype=torch.int32, device=y.device)
+    z = torch.empty(rows, spec.experts, dtype=torch.float32, device=y.device)
+    ext.router_scores(z, y, router)
+    ids = torch.empty(rows, spec.top, **i32)
+    weights = torch.empty(rows, spec.top, dtype=torch.float32,
+                          device=y.device)
+    ext.moe_select(ids, weights, z, spec.groups, spec.keep)
+    packed = rows * spec.top
+    tile = ext.moe_tile(packed, spec.experts, y.dtype == torch.bfloat16,
+                        y.shape[1], spec.ff)
+    at = torch.empty(rows, spec.top, **i32)
+    src = torch.empty(packed, **i32)
+    start = torch.empty(spec.experts + 1, **i32)
+    tiles = torch.empty(1 + 2 * ((packed + tile - 1) // tile +
+                                 min(spec.experts, packed)), **i32)
+    ext.moe_sort(at, src, start, tiles, ids, tile)
+    h = y.new_empty(packed, spec.ff)
+    ext.expert_linear(h, y, up, src, start, tiles, tile, True)
+    out = y.new_empty(packed, y.shape[1])
+    ext.expert_linear(out, h, down, None, start, tiles, tile, False)
+    return Picked(out, at, weights)
+
+
+def side_gate(y: torch.Tensor, w: torch.Tensor, tokens: torch.Tensor,
+              table: torch.Tensor, at: int) -> torch.Tensor:
+    """gelu_tanh(y @ w.T) * table[tokens, at : at + dim]; tokens int32."""
+    out = y.new_empty(y.shape[0], w.shape[0])
+    (_ext() if y.is_cuda else ref).side_gate(out, y, w, tokens, table, at)
     return out
 
 

@@ -240,14 +240,89 @@ def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
     return x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps)
 
 
-def stream_norm(delta, x, w_post, w_pre, offset, eps, out_scale=1.0):
-    x += _rms(delta.float(), eps) * (offset + w_post)
-    return (_rms(x, eps) * ((offset + w_pre) * out_scale)).to(delta.dtype)
+def stream_norm(rows, at, weights, x, w_post, w_pre, offset, eps,
+                out_scale=1.0, mult=1.0):
+    delta = rows.float() if at is None else \
+        (rows[at.long()].float() * weights[:, :, None]).sum(1)
+    x += mult * _rms(delta, eps) * (offset + w_post)
+    y = x if w_pre is None else _rms(x, eps) * ((offset + w_pre) * out_scale)
+    return y.to(rows.dtype, copy=True)
 
 
 def embed_norm(tokens, table, w_pre, offset, eps):
     x = table[tokens.long()].float()
-    return x, (_rms(x, eps) * (offset + w_pre)).to(table.dtype)
+    y = x if w_pre is None else _rms(x, eps) * (offset + w_pre)
+    return x, y.to(table.dtype, copy=True)
+
+
+def _rotate(x, turns, positions):
+    """x [rows, ..., n] float, its first 2 * len(turns) elements turned."""
+    half = turns.shape[0]
+    t = positions.double()[:, None] * turns
+    a = ((t - t.round()) * (2 * math.pi)).float()
+    a = a.view(-1, *[1] * (x.dim() - 2), half)
+    u, v = x[..., :half].clone(), x[..., half:2 * half].clone()
+    x[..., :half] = u * a.cos() - v * a.sin()
+    x[..., half:2 * half] = v * a.cos() + u * a.sin()
+    return x
+
+
+def latent_prepare(buf, heads, dim, rot_dim, c_at, norm, eps, turns,
+                   positions, cache, slots):
+    n = heads * (dim + rot_dim)
+    q = buf[:, :n].to(torch.float32, copy=True).view(-1, heads, dim + rot_dim)
+    _rotate(q[..., dim:], turns, positions)
+    buf[:, :n] = q.view(-1, n).to(buf.dtype)
+    if c_at < 0:
+        return
+    rank = norm.shape[0]
+    row = buf[:, c_at:c_at + rank + rot_dim].to(torch.float32, copy=True)
+    row = torch.cat([_rms(row[:, :rank], eps) * norm,
+                     _rotate(row[:, rank:], turns, positions)], 1)
+    bs = cache.shape[2]
+    cache[slots.long() // bs, 0, slots.long() % bs] = row.to(cache.dtype)
+
+
+def head_linear(out, x, w, gate, tail):
+    k = w.shape[2]
+    o = torch.matmul(x[..., :k].float().transpose(0, 1).contiguous(),
+                     w.float().transpose(1, 2).contiguous()).transpose(0, 1)
+    if gate is not None:
+        o = o * torch.sigmoid(gate.float()).view(o.shape)
+    out[..., :w.shape[1]] = o.to(out.dtype)
+    if tail:
+        out[..., w.shape[1]:] = x[..., k:k + tail]
+
+
+def moe_select(z, top, groups, keep):
+    """(ids [rows, top] int32, weights float32), best first, of scores z."""
+    s = torch.softmax(z, -1)
+    best = s.view(-1, groups, s.shape[1] // groups).amax(-1)
+    kept = torch.zeros_like(best, dtype=torch.bool).scatter_(
+        1, best.topk(keep, 1).indices, True)
+    kept = kept.repeat_interleave(s.shape[1] // groups, 1)
+    weights, ids = s.masked_fill(~kept, -1.0).topk(top, 1)
+    return ids.int(), weights
+
+
+def experts(y, router, up, down, top, groups, keep):
+    """(rows, at, weights) of the chosen experts' outputs, token by token."""
+    f = y.float()
+    ids, weights = moe_select(f @ router.float().T, top, groups, keep)
+    out = y.new_zeros(y.shape[0] * top, y.shape[1])
+    flat = ids.reshape(-1)
+    for e in flat.unique().tolist():
+        r = (flat == e).nonzero()[:, 0]
+        h = torch.nn.functional.gelu(f[r // top] @ up[e].float().T)
+        out[r] = (h.to(y.dtype).float() @ down[e].float().T).to(y.dtype)
+    at = torch.arange(flat.shape[0], dtype=torch.int32).view(-1, top)
+    return out, at.to(y.device), weights
+
+
+def side_gate(out, y, w, tokens, table, at):
+    z = torch.nn.functional.gelu(y.float() @ w.float().T, approximate="tanh")
+    e = table[tokens.long(), at:at + w.shape[0]].float()
+    out.copy_((z * e).to(out.dtype))
 
 
 def qkv_prepare(buf, nq, q_norm, k_norm, eps, v_first, lam, k_cache, v_cache,

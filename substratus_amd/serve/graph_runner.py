@@ -119,7 +119,8 @@ class GraphDecodeRunner:
     # ------------------------------------------------------------- capture
     def _decode_gen(self, lo: int, hi: int):
         sl = slice(lo, hi)
-        state = (self.state_slots[sl],) if self.eng.takes_portions else ()
+        state = (self.state_slots[sl], self.bs) \
+            if self.eng.takes_portions else ()
         return self.model.decode_ops(
             self.tokens[sl], self.positions[sl], self.eng.kv.layers,
             self.slots[sl], self.block_table[sl], self.seq_lens[sl], *state)

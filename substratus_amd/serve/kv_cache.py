@@ -6,8 +6,10 @@ block_size × head_dim panel (16×128 bf16 = 4 KiB), the unit the decode
 attention kernel streams through LDS/registers with wide coalesced loads.
 
 Models of unlike layers (ModelConfig.layers) keep per layer what its mixer
-asks for: pages with its own head sizes, or a 32-bit recurrent state for each
-of `state_slots` requests. A layer's entry in `layers` is (k, v) or (state,).
+asks for: pages with its own head sizes, pages of latents, or a 32-bit recurrent
+state for each of `state_slots` requests. A layer's entry in `layers` is (k, v),
+(latents,) or (state,). A layer that attends to another one's latents has that
+layer's very entry, and takes no memory of its own.
 """
 
 from __future__ import annotations
@@ -17,6 +19,7 @@ from dataclasses import dataclass, field
 import torch
 
 from ..models.config import ModelConfig
+from ..models.layers import LatentAttentionSpec
 
 DEFAULT_BLOCK_SIZE = 16
 
@@ -83,7 +86,14 @@ class PagedKVCache:
             else 0)
         for spec in cfg.layers:
             m = spec.mixer
-            if m.state_bytes():
+            if isinstance(m, LatentAttentionSpec):
+                # one row per token, as one key head of which the first
+                # columns are also the values
+                self.layers.append(
+                    self.layers[m.kv_from] if m.kv_from is not None else
+                    (torch.zeros(num_blocks, 1, block_size, m.row,
+                                 device=device, dtype=dtype),))
+            elif m.state_bytes():
                 self.layers.append((torch.zeros(
                     state_slots, m.heads, m.dim, m.vdim, device=device,
                     dtype=torch.float32),))
