@@ -242,8 +242,12 @@ HYBRID_PAIRS = [
     ("kakovik-1b", "llama-1b", [(8, 512), (64, 512), (256, 512), (16, 3072)]),
     ("kakovik-7b", "llama2-7b", [(8, 512), (64, 512), (256, 512),
                                  (16, 3072)]),
+    ("guronex-1b", "llama-1b", [(8, 512), (64, 512), (256, 512), (16, 3072)]),
+    ("guronex-7b", "llama2-7b", [(8, 512), (64, 512), (256, 512),
+                                 (16, 3072)]),
 ]
-HYBRID_TINY = [("kakovik-tiny", "llama-tiny", [(2, 24)])]
+HYBRID_TINY = [("kakovik-tiny", "llama-tiny", [(2, 24)]),
+               ("guronex-tiny", "llama-tiny", [(2, 24)])]
 
 
 def bench_hybrid(args) -> None:
@@ -292,6 +296,8 @@ def bench_hybrid(args) -> None:
     for pair in pairs:
         for model in pair[:2]:
             points = pair[2]
+            if any(r["model"] == model for r in rows):
+                continue        # the same uniform model, measured already
             max_seq = max(p for _, p in points) + args.warmup + args.steps + 64
             blocks = max(b * ((p + args.warmup + args.steps + 64) // 16 + 1)
                          for b, p in points)

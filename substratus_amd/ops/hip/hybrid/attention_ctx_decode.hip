@@ -264,6 +264,12 @@ void launch_attn_ctx_decode(const AttnCtx<bf16_t>& a, int entries, int splits,
   else if (a.dim <= 128) by_cl(integral_constant<int, 4>{});
   else by_cl(integral_constant<int, 8>{});
   if (splits > 1)
-    attn_ctx_merge_kernel<<<dim3(a.heads, entries), dim3(WAVE), 0, stream>>>(
-        a, splits, part_o, part_ml);
+    launch_attn_ctx_merge(a, entries, splits, part_o, part_ml, stream);
+}
+
+void launch_attn_ctx_merge(const AttnCtx<bf16_t>& a, long rows, int splits,
+                           const float* part_o, const float* part_ml,
+                           hipStream_t stream) {
+  attn_ctx_merge_kernel<<<dim3(a.heads, rows), dim3(WAVE), 0, stream>>>(
+      a, splits, part_o, part_ml);
 }

@@ -14,6 +14,8 @@
 //     step and workgroup in LDS;
 //   * the weights enter the second product as bf16 high and low parts, i.e.
 //     with 16 mantissa bits, so softmax weights keep more than bf16 carries;
+//   * keys and values may also lie unpaged, projected for this step from what
+//     the cache holds (FLAT), with a key part that all heads share;
 //   * V is staged with keys 4..7 and 8..11 of every 16 exchanged, which is
 //     the order in which the score accumulators hold them: weights need no
 //     lane exchange before the second product.
@@ -40,7 +42,7 @@ DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
 }
 
 // KK: 16-wide steps of the key size; DC: 32-wide tiles of the value size
-template <int KK, int DC, int WAVES>
+template <int KK, int DC, int WAVES, bool FLAT>
 __global__ __launch_bounds__(WAVES * WAVE)
 void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   constexpr int THREADS = WAVES * WAVE;
@@ -61,7 +63,9 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   const int q0_tile = tile * QT;
   if (q0_tile >= en.n) return;
   const int kvh = head / (a.heads / a.kv_heads);
-  const int* bt = a.block_table + (long)e * a.max_blocks;
+  const int* bt = FLAT ? nullptr : a.block_table + (long)e * a.max_blocks;
+  const long flat0 = FLAT ? a.ctx_start[e] : 0;
+  const int kd = a.dim - a.shared;               // a head's own key elements
 
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
   const int lo5 = lane & 31, hi = lane >> 5;
@@ -106,13 +110,13 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
     for (int i = 0; i < LK; ++i) {
       const int key = st * CH + (i * THREADS + tid) / (KK * 2);
       pgk[i] = st < steps && key < total && key < st * CH + CH
-          ? bt[key / PAGE] : -1;
+          ? (FLAT ? key : bt[key / PAGE]) : -1;
     }
     #pragma unroll
     for (int i = 0; i < LV; ++i) {
       const int key = st * CH + (i * THREADS + tid) / (DC * 4);
       pgv[i] = st < steps && key < total && key < st * CH + CH
-          ? bt[key / PAGE] : -1;
+          ? (FLAT ? key : bt[key / PAGE]) : -1;
     }
   };
   auto stage_load = [&](int st) {
@@ -121,7 +125,13 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
       const int f = i * THREADS + tid;
       const int r = f / (KK * 2), d = f % (KK * 2) * 8;
       st_k[i] = make_uint4(0, 0, 0, 0);
-      if (pgk[i] >= 0 && d < a.dim)
+      if constexpr (FLAT) {
+        const long at = flat0 + pgk[i];
+        if (pgk[i] >= 0 && d < a.dim)
+          st_k[i] = *reinterpret_cast<const uint4*>(
+              d < kd ? a.kc + at * a.v_ld + (long)head * kd + d
+                     : a.kr + at * a.shared + d - kd);
+      } else if (pgk[i] >= 0 && d < a.dim)
         st_k[i] = *reinterpret_cast<const uint4*>(
             a.kc + (((long)pgk[i] * a.kv_heads + kvh) * PAGE +
                     (st * CH + r) % PAGE) * a.dim + d);
@@ -131,7 +141,11 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
       const int f = i * THREADS + tid;
       const int r = f / (DC * 4), d = f % (DC * 4) * 8;
       st_v[i] = make_uint4(0, 0, 0, 0);
-      if (pgv[i] >= 0 && d < a.vdim)
+      if constexpr (FLAT) {
+        if (pgv[i] >= 0 && d < a.vdim)
+          st_v[i] = *reinterpret_cast<const uint4*>(
+              a.vc + (flat0 + pgv[i]) * a.v_ld + (long)head * a.vdim + d);
+      } else if (pgv[i] >= 0 && d < a.vdim)
         st_v[i] = *reinterpret_cast<const uint4*>(
             a.vc + (((long)pgv[i] * a.kv_heads + kvh) * PAGE +
                     (st * CH + r) % PAGE) * a.v_ld + d);
@@ -275,17 +289,26 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   if (wave_live && qpos < total) {
     const long r = en.row0 + row;
     float f = 1.f / l;
-    if (a.gate != nullptr) f *= sigmoid_f(bf2f(a.gate[r * a.g_ld + head]));
+    if (!FLAT && a.gate != nullptr)
+      f *= sigmoid_f(bf2f(a.gate[r * a.g_ld + head]));
     bf16_t* op = a.out + (r * a.heads + head) * a.vdim;
     #pragma unroll
     for (int c = 0; c < DC; ++c) {
       #pragma unroll
       for (int rr = 0; rr < 4; ++rr) {
         const int d0 = c * 32 + 8 * rr + 4 * hi;
-        if (d0 < a.vdim)
-          *reinterpret_cast<uint2*>(op + d0) = make_uint2(
-              pack_bf16x2(o_t[c][rr * 4] * f, o_t[c][rr * 4 + 1] * f),
-              pack_bf16x2(o_t[c][rr * 4 + 2] * f, o_t[c][rr * 4 + 3] * f));
+        if (d0 < a.vdim) {
+          float o[4];
+          #pragma unroll
+          for (int j = 0; j < 4; ++j) o[j] = o_t[c][rr * 4 + j] * f;
+          if (FLAT && a.gate != nullptr) {
+            float g[4];
+            ldv<4>(a.gate + r * a.g_ld + (long)head * a.vdim + d0, g);
+            #pragma unroll
+            for (int j = 0; j < 4; ++j) o[j] *= sigmoid_f(g[j]);
+          }
+          stv<4>(op + d0, o);
+        }
       }
     }
   }
@@ -302,9 +325,13 @@ void launch_attn_ctx_prefill(const AttnCtx<bf16_t>& a, int entries,
                              int max_len, hipStream_t stream) {
   auto go = [&](auto kk, auto dc, auto waves) {
     constexpr int W = decltype(waves)::value;
-    attn_ctx_prefill_kernel<decltype(kk)::value, decltype(dc)::value, W>
-        <<<dim3(entries, a.heads, (max_len + W * 32 - 1) / (W * 32)),
-           dim3(W * WAVE), 0, stream>>>(a);
+    const dim3 grid(entries, a.heads, (max_len + W * 32 - 1) / (W * 32));
+    if (a.ctx_start != nullptr)
+      attn_ctx_prefill_kernel<decltype(kk)::value, decltype(dc)::value, W,
+                              true><<<grid, dim3(W * WAVE), 0, stream>>>(a);
+    else
+      attn_ctx_prefill_kernel<decltype(kk)::value, decltype(dc)::value, W,
+                              false><<<grid, dim3(W * WAVE), 0, stream>>>(a);
   };
   using std::integral_constant;
   auto by_dc = [&](auto kk) {
@@ -318,5 +345,6 @@ void launch_attn_ctx_prefill(const AttnCtx<bf16_t>& a, int entries,
   if (a.dim <= 64) by_dc(integral_constant<int, 4>{});
   else if (a.dim <= 96) by_dc(integral_constant<int, 6>{});
   else if (a.dim <= 128) by_dc(integral_constant<int, 8>{});
+  else if (a.dim <= 192) by_dc(integral_constant<int, 12>{});
   else by_dc(integral_constant<int, 16>{});
 }

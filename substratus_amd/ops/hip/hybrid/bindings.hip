@@ -5,6 +5,8 @@
 #include <torch/extension.h>
 #include <ATen/cuda/CUDAContext.h>
 
+#include <numeric>
+
 #include "attention_ctx.h"
 #include "gla.h"
 #include "group_gemm.h"
@@ -13,6 +15,7 @@ template <class T>
 void launch_stream_norm(T*, float*, const T*, const int*, const float*, int, const float*, const float*, long, int, float, float, float, float, hipStream_t);
 template <class T>
 void launch_latent_prepare(T*, long, int, int, int, int, int, const float*, float, const double*, int, const int*, T*, const int*, long, hipStream_t);
+void launch_latent_gather(void*, void*, const void*, int, int, int, const int*, int, const int*, int, int, hipStream_t);
 int moe_max_experts();
 void launch_moe_select(int*, float*, const float*, int, int, int, int, int, hipStream_t);
 void launch_moe_sort(int*, int*, int*, int*, const int*, int, int, int, int, hipStream_t);
@@ -238,6 +241,25 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
       const bool aligned = a.q_ld % 8 == 0 &&
           reinterpret_cast<uintptr_t>(a.q) % 16 == 0;
       any = any || v_ld % 8 != 0;
+      if (!any && aligned && kv == 1 && a.kc == a.vc && v_ld == dim && !bias &&
+          !gate && chunk == 0 &&
+          attn_latent_supported(dim, vdim, a.block_size)) {
+        const int longest = seq_start ? max_len : 1;
+        const int splits = attn_latent_splits(entries, longest, heads, span);
+        Tensor po, pml;
+        if (splits > 1) {
+          const auto opt = out.options().dtype(torch::kFloat32);
+          po = torch::empty({rows, heads, splits, vdim}, opt);
+          pml = torch::empty({rows, heads, splits, 2}, opt);
+        }
+        launch_attn_latent(a, entries, longest, splits,
+                           splits > 1 ? ptr<float>(po) : nullptr,
+                           splits > 1 ? ptr<float>(pml) : nullptr, stream());
+        if (splits > 1)
+          launch_attn_ctx_merge(a, rows, splits, ptr<float>(po),
+                                ptr<float>(pml), stream());
+        return;
+      }
       if (!any && seq_start && aligned &&
           attn_ctx_prefill_supported(dim, vdim, a.block_size)) {
         launch_attn_ctx_prefill(a, entries, max_len, stream());
@@ -263,6 +285,74 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     launch_attn_ctx_any<T>(a, entries, seq_start ? max_len : 1, stream());
   });
   post("attn_ctx");
+}
+
+// Portions over keys and values that lie unpaged, ctx_start[e + 1] -
+// ctx_start[e] of them per entry: kv rows [keys of all heads | values of all
+// heads], kr rows the key part that follows every head's own. gate by column.
+void attn_flat(Tensor out, Tensor q, OptTensor gate, Tensor kv, Tensor kr,
+               Tensor positions, Tensor seq_start, Tensor ctx_start,
+               int64_t heads, int64_t vdim, double scale, int64_t max_len) {
+  using T = bf16_t;
+  const long rows = q.size(0), entries = seq_start.numel() - 1;
+  const long dim = q.size(1) / heads, shared = kr.size(1);
+  check_rows(q, Scalar<T>::type, "q");
+  check(out, Scalar<T>::type, "out");
+  check(kv, Scalar<T>::type, "kv");
+  check(kr, Scalar<T>::type, "kr");
+  check(positions, torch::kInt32, "positions");
+  check(seq_start, torch::kInt32, "seq_start");
+  check(ctx_start, torch::kInt32, "ctx_start");
+  TORCH_CHECK(q.size(1) == heads * dim && kv.size(0) == kr.size(0) &&
+              kv.size(1) == heads * (dim - shared + vdim) && shared < dim,
+              "kv must be [keys, heads * (own + vdim)]");
+  TORCH_CHECK(out.size(0) == rows && out.size(1) == heads * vdim &&
+              positions.numel() == rows && ctx_start.numel() == entries + 1,
+              "attn_flat: shapes differ");
+  AttnCtx<T> a{};
+  a.dim = dim; a.vdim = vdim; a.shared = shared;
+  TORCH_CHECK(attn_ctx_prefill_supported(dim, vdim, 16) && shared % 8 == 0 &&
+              q.stride(0) % 8 == 0 &&
+              reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0,
+              "attn_flat: sizes must be multiples of 8");
+  if (gate) {
+    check_rows(*gate, Scalar<T>::type, "gate");
+    TORCH_CHECK(gate->size(0) == rows && gate->size(1) == heads * vdim &&
+                gate->stride(0) % 4 == 0 &&
+                reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0,
+                "gate must be [rows, heads * vdim]");
+  }
+  if (rows == 0) return;
+  a.out = ptr<T>(out); a.q = ptr<T>(q); a.gate = ptr<T>(gate);
+  a.kc = ptr<T>(kv); a.vc = a.kc + heads * (dim - shared); a.kr = ptr<T>(kr);
+  a.positions = ptr<int>(positions); a.seq_start = ptr<int>(seq_start);
+  a.ctx_start = ptr<int>(ctx_start);
+  a.q_ld = q.stride(0); a.g_ld = gate ? gate->stride(0) : 0;
+  a.v_ld = kv.size(1);
+  a.heads = a.kv_heads = heads; a.nbias = 1; a.block_size = 16;
+  a.scale = scale;
+  launch_attn_ctx_prefill(a, entries, max_len, stream());
+  post("attn_flat");
+}
+
+// c [keys, rank] and kr [keys, rot] of whole contexts, entry by entry
+void latent_gather(Tensor c, Tensor kr, Tensor cache, Tensor block_table,
+                   Tensor ctx_start) {
+  check(block_table, torch::kInt32, "block_table");
+  check(ctx_start, torch::kInt32, "ctx_start");
+  check(c, cache.scalar_type(), "c");
+  check(kr, cache.scalar_type(), "kr");
+  check(cache, cache.scalar_type(), "cache");
+  const int entries = block_table.size(0);
+  TORCH_CHECK(cache.size(1) == 1 && cache.size(3) == c.size(1) + kr.size(1) &&
+              c.size(0) == kr.size(0) && ctx_start.numel() == entries + 1,
+              "latent_gather: shapes differ");
+  if (entries == 0) return;
+  launch_latent_gather(c.data_ptr(), kr.data_ptr(), cache.data_ptr(),
+                       cache.element_size(), c.size(1), kr.size(1),
+                       ptr<int>(block_table), block_table.size(1),
+                       ptr<int>(ctx_start), entries, cache.size(2), stream());
+  post("latent_gather");
 }
 
 // buf rows [queries | ... | latent | key part], the latter from column c_at
@@ -353,7 +443,7 @@ void head_linear(Tensor out, Tensor x, Tensor w, OptTensor gate,
       a.act = Act::GATE;
       a.gate = ptr<T>(gate); a.gate_ld = gate->stride(0); a.gate_gs = n;
     }
-    group_gemm(a, group_gemm_tile(rows, 1, std::is_same_v<T, bf16_t>, k, 8),
+    group_gemm(a, group_gemm_tile(rows, 1, std::is_same_v<T, bf16_t>, k),
                "head_linear");
   });
 }
@@ -366,8 +456,9 @@ void router_scores(Tensor z, Tensor x, Tensor w) {
   by_type(x, [&](auto tag) {
     using T = decltype(tag);
     group_gemm(product<T, float>(z, x, w),
-               group_gemm_tile(x.size(0), 1, std::is_same_v<T, bf16_t>,
-                               w.size(1), 8), "router_scores");
+               std::min(64, group_gemm_tile(
+                   x.size(0), 1, std::is_same_v<T, bf16_t>, w.size(1))),
+               "router_scores");
   });
 }
 
@@ -388,8 +479,9 @@ void side_gate(Tensor out, Tensor x, Tensor w, Tensor tokens, Tensor table,
     a.act = Act::SIDE;
     a.tokens = ptr<int>(tokens); a.table = ptr<T>(table) + t_at;
     a.t_ld = table.stride(0); a.vocab = table.size(0);
-    group_gemm(a, group_gemm_tile(x.size(0), 1, std::is_same_v<T, bf16_t>,
-                                  w.size(1), 8), "side_gate");
+    group_gemm(a, std::min(128, group_gemm_tile(
+                   x.size(0), 1, std::is_same_v<T, bf16_t>, w.size(1))),
+               "side_gate");
   });
 }
 
@@ -413,7 +505,7 @@ void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
 
 int64_t moe_tile(int64_t packed, int64_t experts, bool bf16, int64_t k,
                  int64_t n) {
-  return group_gemm_tile(packed, experts, bf16, k, n);
+  return group_gemm_tile(packed, experts, bf16, std::gcd(k, n));
 }
 
 // tiles: [1 + 2 * bound], of which each expert's last may be short
@@ -557,6 +649,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_ctx", &attn_ctx);
   m.def("gla", &gla);
   m.def("silu_mul", &silu_mul);
+  m.def("attn_flat", &attn_flat);
+  m.def("latent_gather", &latent_gather);
   m.def("latent_prepare", &latent_prepare);
   m.def("head_linear", &head_linear);
   m.def("router_scores", &router_scores);

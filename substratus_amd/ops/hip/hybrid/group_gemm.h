@@ -79,8 +79,9 @@ DEV_INLINE void copy_tail(const GroupGemm<T, Y>& a, Tile t, int tid,
   }
 }
 
-// Row tile that suits `rows` rows in `groups` groups.
-int group_gemm_tile(long rows, int groups, bool bf16, int k, int n);
+// Row tile that suits `rows` rows in `groups` groups, with inner sizes that
+// are multiples of `ks` (packed rows are cut once for two products).
+int group_gemm_tile(long rows, int groups, bool bf16, int ks);
 
 // Whether packed rows may come in tiles of this size.
 template <class T, class Y>
@@ -88,3 +89,8 @@ bool group_gemm_takes(const GroupGemm<T, Y>&, int tile);
 
 template <class T, class Y>
 void launch_group_gemm(const GroupGemm<T, Y>&, int tile, hipStream_t);
+
+// Tiles of 128 or 256 rows (group_gemm_tile.hip).
+template <class Y>
+void launch_group_gemm_tile(const GroupGemm<bf16_t, Y>&, int tile,
+                            hipStream_t);

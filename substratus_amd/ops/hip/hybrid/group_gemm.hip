@@ -1,4 +1,4 @@
-// Grouped products (group_gemm.h), two kernels:
+// Grouped products (group_gemm.h) of few rows per group, and of any size:
 //
 //   stream   bf16, few rows per group: bound by reading the weights once.
 //            Every wave takes a share of the inner dimension of a tile of
@@ -167,16 +167,20 @@ bool pieces(const GroupGemm<bf16_t, Y>& a) {
 
 }  // namespace
 
-int group_gemm_tile(long rows, int groups, bool bf16, int k, int n) {
-  if (!bf16 || k % 8 || n % 8) return AT;
+int group_gemm_tile(long rows, int groups, bool bf16, int ks) {
+  if (!bf16 || ks % 8) return AT;
   const long per = rows / groups;
+  if (ks % 64 == 0 && per >= 96) return per >= 768 ? 256 : 128;
   return per <= 16 ? 16 : per <= 48 ? 32 : 64;
 }
 
 template <class T, class Y>
 bool group_gemm_takes(const GroupGemm<T, Y>& a, int tile) {
-  if constexpr (std::is_same_v<T, bf16_t>)
+  if constexpr (std::is_same_v<T, bf16_t>) {
     if (pieces(a) && (tile == 16 || tile == 32 || tile == 64)) return true;
+    if (pieces(a) && (tile == 128 || tile == 256))
+      return a.k % 64 == 0 && a.tail == 0;
+  }
   return tile == AT;
 }
 
@@ -184,10 +188,15 @@ template <class T, class Y>
 void launch_group_gemm(const GroupGemm<T, Y>& a, int tile,
                        hipStream_t stream) {
   const bool packed = a.tiles != nullptr;
-  const int mt = packed ? a.max_tiles : (a.m + tile - 1) / tile;
   const int gz = packed ? 1 : a.groups;
   if constexpr (std::is_same_v<T, bf16_t>) {
-    if (pieces(a) && (tile == 16 || tile == 32 || tile == 64)) {
+    if (!packed && tile > 64 && !group_gemm_takes(a, tile)) tile = 64;
+    if (group_gemm_takes(a, tile) && pieces(a)) {
+      if (tile > 64) {
+        launch_group_gemm_tile(a, tile, stream);
+        return;
+      }
+      const int mt = packed ? a.max_tiles : (a.m + tile - 1) / tile;
       const dim3 grid((a.n + BN - 1) / BN, mt, gz), block(NW * WAVE);
       if (tile == 16)
         group_gemm_stream_kernel<Y, 1><<<grid, block, 0, stream>>>(a);
@@ -198,8 +207,8 @@ void launch_group_gemm(const GroupGemm<T, Y>& a, int tile,
       return;
     }
   }
-  const int rows = packed ? mt : (a.m + AT - 1) / AT;
-  group_gemm_any_kernel<T, Y><<<dim3((a.n + AT - 1) / AT, rows, gz), 256, 0,
+  const int mt = packed ? a.max_tiles : (a.m + AT - 1) / AT;
+  group_gemm_any_kernel<T, Y><<<dim3((a.n + AT - 1) / AT, mt, gz), 256, 0,
                                 stream>>>(a);
 }
 

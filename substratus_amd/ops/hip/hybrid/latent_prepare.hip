@@ -68,7 +68,48 @@ void latent_prepare_kernel(T* __restrict__ buf, long ld, int heads, int dim,
   }
 }
 
+// Rows of whole contexts out of the pages: latents to c, key parts to kr.
+// Sizes are in pieces of type P.
+template <class P>
+__global__ __launch_bounds__(BLOCK)
+void latent_gather_kernel(P* __restrict__ c, P* __restrict__ kr,
+                          const P* __restrict__ cache, int rank, int rot,
+                          const int* __restrict__ block_table, int max_blocks,
+                          const int* __restrict__ ctx_start, int block_size) {
+  const int e = blockIdx.y, page = blockIdx.x;
+  const int at = ctx_start[e], n = ctx_start[e + 1] - at;
+  const int rows = min(block_size, n - page * block_size);
+  if (rows <= 0) return;
+  const int row = rank + rot;
+  const long first = at + (long)page * block_size;
+  const P* src = cache + (long)block_table[(long)e * max_blocks + page] *
+                 block_size * row;
+  for (int i = threadIdx.x; i < rows * row; i += BLOCK) {
+    const long r = first + i / row;
+    const int d = i % row;
+    if (d < rank) c[r * rank + d] = src[i];
+    else kr[r * rot + d - rank] = src[i];
+  }
+}
+
 }  // namespace
+
+void launch_latent_gather(void* c, void* kr, const void* cache, int itemsize,
+                          int rank, int rot, const int* block_table,
+                          int max_blocks, const int* ctx_start, int entries,
+                          int block_size, hipStream_t stream) {
+  auto go = [&](auto piece) {
+    using P = decltype(piece);
+    const int per = sizeof(P) / itemsize;
+    latent_gather_kernel<P><<<dim3(max_blocks, entries), BLOCK, 0, stream>>>(
+        (P*)c, (P*)kr, (const P*)cache, rank / per, rot / per, block_table,
+        max_blocks, ctx_start, block_size);
+  };
+  const int bytes = 16 / itemsize;
+  if (rank % bytes == 0 && rot % bytes == 0) go(uint4{});
+  else if (itemsize == 4) go(unsigned{});
+  else go((unsigned short)0);
+}
 
 template <class T>
 void launch_latent_prepare(T* buf, long ld, int heads, int dim, int rot_dim,

@@ -15,7 +15,7 @@ from typing import NamedTuple, Optional, Union
 
 import torch
 
-from . import ref
+from . import linear, ref
 
 _EXT = None
 
@@ -125,13 +125,16 @@ def latent_prepare(buf: torch.Tensor, spec, c_at: int,
 
 def head_linear(x: torch.Tensor, w: torch.Tensor,
                 gate: Optional[torch.Tensor] = None,
-                tail: int = 0) -> torch.Tensor:
+                tail: int = 0,
+                out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per head h: x[:, h, :k] @ w[h].T, times sigmoid(gate) if there is one;
     the `tail` elements that follow in x are appended as they are.
 
     x [rows, heads, k + tail] may be a view of wider rows; w [heads, n, k];
-    gate [rows, heads * n]. Returns [rows, heads, n + tail]."""
-    out = x.new_empty(x.shape[0], w.shape[0], w.shape[1] + tail)
+    gate [rows, heads * n]. Returns [rows, heads, n + tail]; out: contiguous
+    room for it."""
+    shape = (x.shape[0], w.shape[0], w.shape[1] + tail)
+    out = x.new_empty(shape) if out is None else out.view(shape)
     (_ext() if x.is_cuda else ref).head_linear(out, x, w, gate, tail)
     return out
 
@@ -148,24 +151,71 @@ def _latent_absorbed(out, q, gate, cache, w_uv, uk_t, batch, rows, ents,
     fn(o, qa.view(n, -1), None, cache, cache[..., :spec.rank], None,
        batch.positions[rows], seq_start, batch.block_table[ents], spec.scale,
        0, max_len, batch.max_context, False)
-    out[rows] = head_linear(o.view(n, spec.heads, spec.rank), w_uv,
-                            gate).view(n, -1)
+    head_linear(o.view(n, spec.heads, spec.rank), w_uv, gate, out=out)
+
+
+def _latent_expanded(out, q, gate, cache, w_ukv, batch, rows, ents, seq_start,
+                     max_len, spec, shared) -> None:
+    """Keys and values of all heads are made for the whole contexts of the
+    batch's portions; layers on the same cache share what is read from it."""
+    held = shared.get(cache.data_ptr())
+    if held is None:
+        held = shared[cache.data_ptr()] = tuple(
+            q.new_empty(batch.total_context, n)
+            for n in (spec.rank, spec.rot_dim))
+        _ext().latent_gather(*held, cache, batch.block_table[ents],
+                             batch.ctx_start)
+    c, kr = held
+    _ext().attn_flat(out, q, gate, linear(c, w_ukv), kr,
+                     batch.positions[rows], seq_start, batch.ctx_start,
+                     spec.heads, spec.vdim, spec.scale, max_len)
+
+
+EXPAND_BYTES = 4 << 30      # most memory for keys and values of one layer
+
+
+def _expanding_pays(batch, spec, rows: int) -> bool:
+    """Fewer multiplications with keys and values made for every head than
+    with queries moved into the latent space."""
+    own = spec.rank * (spec.dim + spec.vdim)
+    if 2 * batch.total_context * spec.heads * (spec.dim + spec.vdim) \
+            > EXPAND_BYTES:
+        return False
+    return (batch.total_context - rows) * own < batch.pairs * (
+        2 * spec.rank - spec.dim - spec.vdim)
+
+
+def _flat_takes(q, gate, spec) -> bool:
+    """Sizes that attn_flat is made for; any others stay in latent space."""
+    return (q.is_cuda and q.dtype == torch.bfloat16
+            and not any(n % 8 for n in (spec.dim, spec.rot_dim, spec.vdim,
+                                        q.stride(0), q.storage_offset()))
+            and (gate is None or gate.storage_offset() % 8 == 0)
+            and spec.dim + spec.rot_dim <= 256 and spec.vdim <= 256)
 
 
 def latent_attn(q: torch.Tensor, gate: Optional[torch.Tensor],
                 cache: torch.Tensor, w_ukv: torch.Tensor, uk_t: torch.Tensor,
-                batch, spec, shared: dict) -> torch.Tensor:
+                batch, spec, shared: dict,
+                expand: Optional[bool] = None) -> torch.Tensor:
     """Latent attention of a batch's rows over the paged cache, which already
     holds their own latents. q [rows, heads * (dim + rot_dim)] is rotated;
     gate [rows, heads * vdim]; w_ukv has the rows that make all heads' keys,
     then those that make their values; uk_t is the former as [heads, rank,
-    dim]."""
+    dim]. `shared` lasts for one batch. expand: how portions are computed,
+    None: as pays."""
     out = q.new_empty(q.shape[0], spec.heads * spec.vdim)
     w_uv = w_ukv[spec.heads * spec.dim:].view(spec.heads, spec.vdim, spec.rank)
     for rows, ents, seq_start, max_len in batch.parts():
-        _latent_absorbed(out, q[rows], None if gate is None else gate[rows],
-                         cache, w_uv, uk_t, batch, rows, ents, seq_start,
-                         max_len, spec)
+        args = (out[rows], q[rows], None if gate is None else gate[rows],
+                cache)
+        where = (batch, rows, ents, seq_start, max_len, spec)
+        if seq_start is not None and _flat_takes(q, gate, spec) and (
+                _expanding_pays(batch, spec, args[1].shape[0])
+                if expand is None else expand):
+            _latent_expanded(*args, w_ukv, *where, shared)
+        else:
+            _latent_absorbed(*args, w_uv, uk_t, *where)
     return out
 
 

@@ -25,6 +25,10 @@ class StepBatch:
     max_context: int            # no row has more positions than this
     want: Optional[torch.Tensor] = None  # int64 rows whose logits are needed;
                                          # None: all
+    ctx_start: Optional[torch.Tensor] = None  # [portions + 1] int32, keys that
+                                              # the portions see, summed up
+    total_context: int = 0      # the last of those
+    pairs: int = 0              # portions' rows times the keys they see
 
     def parts(self) -> Iterator[tuple[slice, slice, Optional[torch.Tensor],
                                       int]]:
@@ -55,7 +59,7 @@ class StepBatch:
         table = np.zeros((len(entries), maxb), np.int32)
         tokens, positions, slots = (np.empty(rows, np.int32)
                                     for _ in range(3))
-        starts = [0]
+        starts, contexts, pairs = [0], [0], 0
         for at, i in enumerate(order):
             toks, first, blocks, _, _ = entries[i]
             table[at, :len(blocks)] = blocks
@@ -66,18 +70,22 @@ class StepBatch:
                 + pos % block_size
             if len(toks) > 1:
                 starts.append(starts[-1] + len(toks))
+                contexts.append(contexts[-1] + first + len(toks))
+                pairs += len(toks) * (first + len(toks))
         state = np.array([entries[i][3] for i in order], np.int32)
         want = np.array([row_of[i] + o for i, e in enumerate(entries)
                          for o in e[4]], np.int32)
         # one host-to-device copy for everything
         parts = [tokens, positions, slots, state,
-                 np.array(starts, np.int32), want, table.reshape(-1)]
+                 np.array(starts, np.int32), np.array(contexts, np.int32),
+                 want, table.reshape(-1)]
         dev = torch.from_numpy(np.concatenate(parts)).to(device)
-        tokens, positions, slots, state, starts_t, want, table = \
+        tokens, positions, slots, state, starts_t, contexts_t, want, table = \
             dev.split([len(p) for p in parts])
         portions = len(starts) > 1
         return cls(
             tokens, positions, slots, table.view(len(entries), maxb), state,
             singles, starts_t if portions else None,
             int(np.diff(starts).max()) if portions else 0,
-            maxb * block_size, want.long())
+            maxb * block_size, want.long(),
+            contexts_t if portions else None, contexts[-1], pairs)
