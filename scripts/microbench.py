@@ -197,6 +197,201 @@ def bench_hybrid():
                       20), x.numel() * 2 + t * gh * gv * 2, flops)
 
 
+def bench_latent():
+    """Kernels of latent-attention models with experts beside the like kernels
+    and products of the uniform families, at 7b sizes."""
+    from substratus_amd.models.layers import (LatentAttentionSpec, MoESpec,
+                                              RotarySpec)
+    from substratus_amd.ops import hybrid as hy
+    from substratus_amd.serve.batch import StepBatch
+    torch.manual_seed(0)
+    bf = dict(device="cuda", dtype=torch.bfloat16)
+    F = torch.nn.functional
+    h, d, r, rank, w = 32, 128, 64, 512, 4096
+    spec = LatentAttentionSpec(h, d, r, d, rank, (d + r) ** -0.5,
+                               RotarySpec(1e4, r), None, True)
+    moe = MoESpec(32, 8, 2048, 8, 4)
+
+    def batch_of(n, first, tokens):
+        need = (first + tokens + 15) // 16
+        return StepBatch.build(
+            [([1] * tokens, first, list(range(i * need, (i + 1) * need)), i,
+              []) for i in range(n)], 16, torch.device("cuda"))
+
+    for rows in (64, 256, 16384):
+        it = 100 if rows < 1000 else 20
+        x, xf = torch.randn(rows, w, **bf), torch.randn(rows, w,
+                                                        device="cuda")
+        w32 = torch.randn(w, device="cuda")
+        res, wt = torch.randn(rows, w, **bf), torch.randn(w, **bf)
+        report(f"rms_norm_residual rows={rows} w={w}",
+               timeit(lambda: ops.rms_norm_residual(x, res, wt, 1e-5), it),
+               rows * w * 8)
+        report(f"  stream_norm rows={rows} w={w}",
+               timeit(lambda: hy.stream_norm(x, xf, w32, None, 0.0, 1e-5), it),
+               rows * w * 12)
+        at = torch.randperm(rows * 8, device="cuda").int().view(rows, 8)
+        pk = hy.Picked(torch.randn(rows * 8, w, **bf), at,
+                       torch.rand(rows, 8, device="cuda"))
+        report(f"  stream_norm of 8 picks rows={rows} w={w}",
+               timeit(lambda: hy.stream_norm(pk, xf, w32, None, 0.0, 1e-5),
+                      it), rows * w * 26)
+        del pk, res
+        kc = torch.zeros((rows + 15) // 16, h, 16, d, **bf)
+        vc = torch.zeros_like(kc)
+        pos = torch.arange(rows, device="cuda", dtype=torch.int32)
+        qkv = torch.randn(rows, 3 * h * d, **bf)
+        q, k, v = (qkv[:, i * h * d:(i + 1) * h * d].view(rows, h, d)
+                   for i in range(3))
+        report(f"rope_kv_append rows={rows} {h}x{d}",
+               timeit(lambda: ops.rope_kv_append(q, k, v, pos, kc, vc, pos,
+                                                 1e4), it),
+               rows * h * d * 2 * 7)
+        buf = torch.randn(rows, h * (d + r) + h * d + rank + r, **bf)
+        cache = torch.zeros((rows + 15) // 16, 1, 16, spec.row, **bf)
+        norm, turns = torch.ones(rank, device="cuda"), spec.rot.turns("cuda")
+        report(f"  latent_prepare rows={rows}",
+               timeit(lambda: hy.latent_prepare(
+                   buf, spec, h * (2 * d + r), norm, 1e-5, turns, pos, cache,
+                   pos), it), rows * (h * r * 2 + spec.row * 2) * 2)
+        router = torch.randn(moe.experts, w, **bf) * 0.02
+        ext = hy._ext()
+        z = torch.empty(rows, moe.experts, device="cuda")
+        report(f"  router_scores rows={rows} {w}->{moe.experts}",
+               timeit(lambda: ext.router_scores(z, x, router), it),
+               rows * w * 2 + router.numel() * 2, 2.0 * rows * w * moe.experts)
+        ids = torch.empty(rows, moe.top, device="cuda", dtype=torch.int32)
+        wts = torch.empty(rows, moe.top, device="cuda")
+        report(f"  moe_select rows={rows} {moe.top}/{moe.experts}",
+               timeit(lambda: ext.moe_select(ids, wts, z, moe.groups,
+                                             moe.keep), it),
+               rows * (moe.experts + 2 * moe.top) * 4)
+        packed = rows * moe.top
+        tile = ext.moe_tile(packed, moe.experts, True, w, moe.ff)
+        i32 = dict(device="cuda", dtype=torch.int32)
+        at2, src = torch.empty(rows, moe.top, **i32), torch.empty(packed, **i32)
+        start = torch.empty(moe.experts + 1, **i32)
+        tiles = torch.empty(1 + 2 * ((packed + tile - 1) // tile + moe.experts),
+                            **i32)
+        report(f"  moe_sort packed={packed}",
+               timeit(lambda: ext.moe_sort(at2, src, start, tiles, ids, tile),
+                      it), packed * 12)
+        up = torch.randn(moe.experts, moe.ff, w, **bf) * 0.02
+        down = torch.randn(moe.experts, w, moe.ff, **bf) * 0.02
+        hid, out = torch.empty(packed, moe.ff, **bf), torch.empty(packed, w,
+                                                                  **bf)
+        ff = 11008
+        dense = torch.randn(2 * ff, w, **bf) * 0.02
+        report(f"linear rows={rows} {w}->{2 * ff}",
+               timeit(lambda: F.linear(x, dense), it),
+               dense.numel() * 2 + rows * (w + 2 * ff) * 2,
+               2.0 * rows * dense.numel())
+        dn = torch.randn(w, ff, **bf) * 0.02
+        y = torch.randn(rows, ff, **bf)
+        report(f"linear rows={rows} {ff}->{w}",
+               timeit(lambda: F.linear(y, dn), it),
+               dn.numel() * 2 + rows * (w + ff) * 2, 2.0 * rows * dn.numel())
+        live = int((start[1:] > start[:-1]).sum())
+        wb = live * moe.ff * w * 2
+        report(f"  expert_linear up packed={packed} {w}->{moe.ff} "
+               f"x{live}", timeit(lambda: ext.expert_linear(
+                   hid, x, up, src, start, tiles, tile, True), it),
+               wb + rows * w * 2 + packed * moe.ff * 2,
+               2.0 * packed * w * moe.ff)
+        report(f"  expert_linear down packed={packed} {moe.ff}->{w}",
+               timeit(lambda: ext.expert_linear(
+                   out, hid, down, None, start, tiles, tile, False), it),
+               wb + packed * (moe.ff + w) * 2, 2.0 * packed * w * moe.ff)
+        del up, down, hid, out, dense, dn, y
+        side = 256
+        wg = torch.randn(side, w, **bf) * 0.02
+        table = torch.randn(1000, side, **bf)
+        tok = torch.randint(0, 1000, (rows,), **i32)
+        report(f"linear rows={rows} {w}->{side}",
+               timeit(lambda: F.linear(x, wg), it),
+               wg.numel() * 2 + rows * (w + side) * 2,
+               2.0 * rows * wg.numel())
+        report(f"  side_gate rows={rows} {w}->{side}",
+               timeit(lambda: hy.side_gate(x, wg, tok, table, 0), it),
+               wg.numel() * 2 + rows * (w + 2 * side) * 2,
+               2.0 * rows * wg.numel())
+        if rows < 1000:
+            uk_t = torch.randn(h, rank, d, **bf)
+            uv = torch.randn(h, d, rank, **bf)
+            gate = torch.randn(rows, h * d, **bf)
+            q3 = torch.randn(rows, h, d + r, **bf)
+            o3 = torch.randn(rows, h, rank, **bf)
+            report(f"  head_linear in rows={rows} {h}x{d}->{rank}",
+                   timeit(lambda: hy.head_linear(q3, uk_t, tail=r), it),
+                   (uk_t.numel() + rows * h * (d + rank + 2 * r)) * 2)
+            report(f"  head_linear out rows={rows} {h}x{rank}->{d}",
+                   timeit(lambda: hy.head_linear(o3, uv, gate), it),
+                   (uv.numel() + rows * h * (2 * d + rank)) * 2)
+
+    for b, ctx in ((8, 512), (64, 512), (256, 512), (16, 3072), (64, 4096)):
+        sb = batch_of(b, ctx - 1, 1)
+        nb = b * ctx // 16
+        cache = torch.randn(nb, 1, 16, spec.row, **bf)
+        qa = torch.randn(b, h * spec.row, **bf)
+        kc = torch.randn(nb, h, 16, d, **bf)
+        vc = torch.randn_like(kc)
+        bt = torch.arange(nb, device="cuda", dtype=torch.int32).view(b, -1)
+        lens = torch.full((b,), ctx, device="cuda", dtype=torch.int32)
+        q = torch.randn(b, h, d, **bf)
+        report(f"paged_attn_decode b={b} ctx={ctx} {h}/{h}x{d}",
+               timeit(lambda: ops.paged_attn_decode(q, kc, vc, bt, lens,
+                                                    d ** -0.5), 50),
+               2 * b * ctx * h * d * 2)
+        del kc, vc
+        o = torch.empty(b, h * rank, **bf)
+        report(f"  attn_latent single b={b} ctx={ctx} {h}x{spec.row}",
+               timeit(lambda: hy._ext().attn_ctx(
+                   o, qa, None, cache, cache[..., :rank], None, sb.positions,
+                   None, sb.block_table, spec.scale, 0, 1, ctx, False), 50),
+               b * ctx * spec.row * 2 + b * h * (spec.row + rank) * 2,
+               2.0 * b * ctx * h * (spec.row + rank))
+
+    for b, s_ in ((32, 512), (8, 2048), (4, 4096)):
+        t = b * s_
+        q, k, v = (torch.randn(t, h, d, **bf) for _ in range(3))
+        ss = torch.arange(0, t + 1, s_, dtype=torch.int32, device="cuda")
+        report(f"attn_v5 b={b} s={s_} {h}x{d}",
+               timeit(lambda: ops.attn_prefill(q, k, v, ss, d ** -0.5), 20),
+               4 * t * h * d * 2, 4.0 * b * h * (s_ * (s_ + 1) / 2) * d)
+        del q, k, v
+        sb = batch_of(b, 0, s_)
+        q2 = torch.randn(t, h * (d + r), **bf)
+        gate = torch.randn(t, h * d, **bf)
+        kv, kr = torch.randn(t, 2 * h * d, **bf), torch.randn(t, r, **bf)
+        o = torch.empty(t, h * d, **bf)
+        flops = b * h * s_ * (s_ + 1) * (2 * d + r)
+        report(f"  attn_flat b={b} s={s_} {h}x{d}+{r}",
+               timeit(lambda: hy._ext().attn_flat(
+                   o, q2, gate, kv, kr, sb.positions, sb.seq_start,
+                   sb.ctx_start, h, d, spec.scale, s_), 20),
+               t * (h * (5 * d + r) + r) * 2, flops)
+        cache = torch.randn(t // 16, 1, 16, spec.row, **bf)
+        c = torch.empty(t, rank, **bf)
+        report(f"  latent_gather keys={t}",
+               timeit(lambda: hy._ext().latent_gather(
+                   c, kr, cache, sb.block_table, sb.ctx_start), 20),
+               t * spec.row * 4)
+        del q2, gate, kv, o, cache
+    for b, first, n in ((16, 2048, 16), (4, 4096, 64)):
+        sb = batch_of(b, first, n)
+        cache = torch.randn(b * (first + n) // 16, 1, 16, spec.row, **bf)
+        qa = torch.randn(b * n, h * spec.row, **bf)
+        o = torch.empty(b * n, h * rank, **bf)
+        report(f"  attn_latent portions b={b} {n} after {first}",
+               timeit(lambda: hy._ext().attn_ctx(
+                   o, qa, None, cache, cache[..., :rank], None, sb.positions,
+                   sb.seq_start, sb.block_table, spec.scale, 0, n, first + n,
+                   False), 20),
+               b * (first + n) * spec.row * 2 + b * n * h * 2 * (
+                   spec.row + rank),
+               2.0 * b * n * (first + n / 2) * h * (spec.row + rank))
+
+
 def bench_sample(B=64, V=32000):
     logits = torch.randn(B, V, device="cuda").bfloat16()
     temp = torch.zeros(B, device="cuda")
@@ -428,6 +623,8 @@ if __name__ == "__main__":
         bench_rope()
     if a.which == "hybrid":
         bench_hybrid()
+    if a.which == "latent":
+        bench_latent()
     if a.which in ("all", "norm"):
         bench_norm()
     if a.which in ("all", "sample"):

@@ -196,26 +196,35 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   }
 }
 
-__global__ __launch_bounds__(WAVE)
+// VEC columns per thread
+template <int VEC>
+__global__
 void attn_ctx_merge_kernel(AttnCtx<bf16_t> a, int splits,
                            const float* __restrict__ part_o,
                            const float* __restrict__ part_ml) {
   const int h = blockIdx.x;
   const long b = blockIdx.y, at = (b * a.heads + h) * splits;
-  float M = NEG, L = 0.f;
+  const int c = threadIdx.x * VEC;
+  if (c >= a.vdim) return;
+  float M = NEG;
   for (int s = 0; s < splits; ++s) M = fmaxf(M, part_ml[(at + s) * 2]);
-  for (int s = 0; s < splits; ++s)
-    L += part_ml[(at + s) * 2 + 1] *
-         __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
+  float L = 0.f, o[VEC];
+  #pragma unroll
+  for (int j = 0; j < VEC; ++j) o[j] = 0.f;
+  #pragma unroll 4
+  for (int s = 0; s < splits; ++s) {
+    const float f = __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
+    float p[VEC];
+    ldv<VEC>(part_o + (at + s) * a.vdim + c, p);
+    L += part_ml[(at + s) * 2 + 1] * f;
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) o[j] += p[j] * f;
+  }
   float f = 1.f / L;
   if (a.gate != nullptr) f *= sigmoid_f(bf2f(a.gate[b * a.g_ld + h]));
-  for (int c = threadIdx.x; c < a.vdim; c += WAVE) {
-    float o = 0.f;
-    for (int s = 0; s < splits; ++s)
-      o += part_o[(at + s) * a.vdim + c] *
-           __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
-    a.out[(b * a.heads + h) * a.vdim + c] = f2bf(o * f);
-  }
+  #pragma unroll
+  for (int j = 0; j < VEC; ++j) o[j] *= f;
+  stv<VEC>(a.out + (b * a.heads + h) * a.vdim + c, o);
 }
 
 constexpr int pick_gq(int per) { return per >= 4 ? 4 : per >= 2 ? 2 : 1; }
@@ -270,6 +279,7 @@ void launch_attn_ctx_decode(const AttnCtx<bf16_t>& a, int entries, int splits,
 void launch_attn_ctx_merge(const AttnCtx<bf16_t>& a, long rows, int splits,
                            const float* part_o, const float* part_ml,
                            hipStream_t stream) {
-  attn_ctx_merge_kernel<<<dim3(a.heads, rows), dim3(WAVE), 0, stream>>>(
-      a, splits, part_o, part_ml);
+  // value sizes of the split kernels are multiples of 8, at most 512
+  attn_ctx_merge_kernel<4><<<dim3(a.heads, rows), (a.vdim / 4 + 63) / 64 * 64,
+                             0, stream>>>(a, splits, part_o, part_ml);
 }

@@ -8,6 +8,8 @@
 
 #include "typed.h"
 
+#include <type_traits>
+
 enum class Act {
   NONE,
   GELU,      // exact gelu
@@ -48,23 +50,51 @@ DEV_INLINE Tile tile_of(const GroupGemm<T, Y>& a, int i, int g, int bm) {
   return {grp, r0, min(r0 + bm, a.start[grp + 1])};
 }
 
+// FAST: to about 1e-7 and 1e-6, for bf16 results; erf by formula 7.1.26 of
+// Abramowitz and Stegun, Handbook of Mathematical Functions.
+template <bool FAST>
 DEV_INLINE float gelu_erf_f(float v) {
-  return 0.5f * v * (1.f + erff(v * 0.70710678118654752440f));
+  const float z = v * 0.70710678118654752440f;
+  if constexpr (!FAST) return 0.5f * v * (1.f + erff(z));
+  const float x = fabsf(z);
+  const float t = __builtin_amdgcn_rcpf(1.f + 0.3275911f * x);
+  const float p = t * (0.254829592f + t * (-0.284496736f + t * (1.421413741f +
+                  t * (-1.453152027f + t * 1.061405429f))));
+  const float e = p * __expf(-x * x);            // 1 - erf(x)
+  return 0.5f * v * (z < 0.f ? e : 2.f - e);
 }
 
-template <class T, class Y>
+template <bool FAST>
+DEV_INLINE float gelu_tanh_f(float v) {
+  const float in = 0.79788456080286535588f * (v + 0.044715f * v * v * v);
+  if constexpr (!FAST) return 0.5f * v * (1.f + tanhf(in));
+  // (1 + tanh(x)) / 2 = 1 / (1 + exp(-2 x))
+  return v * __builtin_amdgcn_rcpf(1.f + __expf(-2.f * in));
+}
+
+template <Act ACT, bool FAST, class T, class Y>
 DEV_INLINE float group_act(const GroupGemm<T, Y>& a, int r, int g, int n,
                            float v) {
-  if (a.act == Act::GELU) return gelu_erf_f(v);
-  if (a.act == Act::GATE)
+  if constexpr (ACT == Act::GELU) return gelu_erf_f<FAST>(v);
+  if constexpr (ACT == Act::GATE)
     return v * sigmoid_f(ld1(a.gate + (long)r * a.gate_ld +
                              (long)g * a.gate_gs + n));
-  if (a.act == Act::SIDE) {
-    const float in = 0.79788456080286535588f * (v + 0.044715f * v * v * v);
+  if constexpr (ACT == Act::SIDE) {
     const int t = min(max(a.tokens[r], 0), a.vocab - 1);
-    return 0.5f * v * (1.f + tanhf(in)) * ld1(a.table + (long)t * a.t_ld + n);
+    return gelu_tanh_f<FAST>(v) * ld1(a.table + (long)t * a.t_ld + n);
   }
   return v;
+}
+
+// Calls f(integral_constant<Act>) with the product's.
+template <class F>
+void by_act(Act act, F f) {
+  switch (act) {
+    case Act::NONE: f(std::integral_constant<Act, Act::NONE>{}); break;
+    case Act::GELU: f(std::integral_constant<Act, Act::GELU>{}); break;
+    case Act::GATE: f(std::integral_constant<Act, Act::GATE>{}); break;
+    case Act::SIDE: f(std::integral_constant<Act, Act::SIDE>{}); break;
+  }
 }
 
 // What the blocks of a tile's first columns do on the side.

@@ -2,10 +2,11 @@
 //
 //   stream   bf16, few rows per group: bound by reading the weights once.
 //            Every wave takes a share of the inner dimension of a tile of
-//            BM rows and 64 columns, with both operands going from memory
+//            BM rows and 64 columns (4 waves, or 16 where there are few
+//            tiles), with both operands going from memory
 //            straight into the matrix cores' registers (a fragment is 16
 //            consecutive bytes of a row, so nothing is gained by LDS); there
-//            is no barrier until the four partial tiles are added up.
+//            is no barrier until the partial tiles are added up.
 //   any      float, and bf16 sizes whose rows are not 16-byte pieces.
 //
 // Weights are the first operand, so a lane ends up with four consecutive
@@ -17,16 +18,19 @@ namespace {
 typedef __attribute__((ext_vector_type(8))) short short8;
 typedef __attribute__((ext_vector_type(4))) float float4v;
 
-constexpr int NW = 4;          // waves: shares of the inner dimension
 constexpr int BN = 64;
 constexpr int KC = 32;         // inner step of one matrix instruction
 
+// ONCE: nobody reads it again
+template <bool ONCE>
 DEV_INLINE short8 frag(const bf16_t* p, bool there) {
-  return there ? *reinterpret_cast<const short8*>(p)
-               : (short8){0, 0, 0, 0, 0, 0, 0, 0};
+  if (!there) return (short8){0, 0, 0, 0, 0, 0, 0, 0};
+  if constexpr (ONCE) return __builtin_bit_cast(short8, nt_load_u4(p));
+  else return *reinterpret_cast<const short8*>(p);
 }
 
-template <class Y, int FM>
+// NW waves: shares of the inner dimension
+template <class Y, Act ACT, int FM, int NW>
 __global__ __launch_bounds__(NW * WAVE)
 void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
   constexpr int BM = FM * 16, FN = BN / 16, PAD = 4;
@@ -57,25 +61,36 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
 
   const int chunks = (a.k + KC - 1) / KC;
   const int c0 = chunks * wave / NW, c1 = chunks * (wave + 1) / NW;
-  auto step = [&](int c, bool whole) {
-    const int k = c * KC;
-    short8 wf[FN], xf[FM];
+  // U chunks at a time: their loads are in flight together
+  auto steps = [&](int c, auto u, bool whole) {
+    constexpr int U = decltype(u)::value;
+    short8 wf[U][FN], xf[U][FM];
     #pragma unroll
-    for (int f = 0; f < FN; ++f) wf[f] = frag(wp[f] + k, whole || k + kq < a.k);
-    #pragma unroll
-    for (int f = 0; f < FM; ++f) xf[f] = frag(xp[f] + k, whole || k + kq < a.k);
-    #pragma unroll
-    for (int i = 0; i < FN; ++i)
+    for (int i = 0; i < U; ++i) {
+      const int k = (c + i) * KC;
+      const bool there = whole || k + kq < a.k;
       #pragma unroll
-      for (int j = 0; j < FM; ++j)
-        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j],
-                                                            acc[i][j], 0, 0, 0);
+      for (int f = 0; f < FN; ++f) wf[i][f] = frag<true>(wp[f] + k, there);
+      #pragma unroll
+      for (int f = 0; f < FM; ++f) xf[i][f] = frag<false>(xp[f] + k, there);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+    #pragma unroll
+    for (int u = 0; u < U; ++u)
+      #pragma unroll
+      for (int i = 0; i < FN; ++i)
+        #pragma unroll
+        for (int j = 0; j < FM; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              wf[u][i], xf[u][j], acc[i][j], 0, 0, 0);
   };
+  constexpr int U = FM == 4 ? 2 : 4;
   const int full = min(c1, a.k / KC);
   int c = c0;
-  #pragma unroll 4
-  for (; c < full; ++c) step(c, true);
-  for (; c < c1; ++c) step(c, false);
+  for (; c + U <= full; c += U)
+    steps(c, std::integral_constant<int, U>{}, true);
+  for (; c < full; ++c) steps(c, std::integral_constant<int, 1>{}, true);
+  if (c < c1) steps(c, std::integral_constant<int, 1>{}, false);
 
   #pragma unroll
   for (int i = 0; i < FN; ++i)
@@ -98,7 +113,8 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
     }
     #pragma unroll
     for (int j = 0; j < 4; ++j)
-      if (n + j < a.n) v[j] = group_act(a, r, t.g, n + j, v[j]);
+      if (n + j < a.n)
+        v[j] = group_act<ACT, true>(a, r, t.g, n + j, v[j]);
     Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n;
     if (quads) {
       stv<4>(y, v);
@@ -114,7 +130,7 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
 // 32 x 32 outputs per workgroup, 2 x 2 per thread, operands through LDS.
 constexpr int AT = 32, AK = 16;
 
-template <class T, class Y>
+template <class T, class Y, Act ACT>
 __global__ __launch_bounds__(256)
 void group_gemm_any_kernel(GroupGemm<T, Y> a) {
   __shared__ float s_x[AK][AT + 1], s_w[AK][AT + 1];
@@ -150,7 +166,7 @@ void group_gemm_any_kernel(GroupGemm<T, Y> a) {
       const int r = t.r0 + ty + 16 * i, n = n0 + tx + 16 * j;
       if (r < t.r1 && n < a.n)
         st1(a.y + (long)r * a.y_ld + t.g * a.y_gs + n,
-            group_act(a, r, t.g, n, acc[i][j]));
+            group_act<ACT, false>(a, r, t.g, n, acc[i][j]));
     }
   if (a.tail && blockIdx.x == 0) copy_tail(a, t, threadIdx.x, 256);
 }
@@ -171,7 +187,7 @@ int group_gemm_tile(long rows, int groups, bool bf16, int ks) {
   if (!bf16 || ks % 8) return AT;
   const long per = rows / groups;
   if (ks % 64 == 0 && per >= 96) return per >= 768 ? 256 : 128;
-  return per <= 16 ? 16 : per <= 48 ? 32 : 64;
+  return per <= 6 ? 16 : per <= 20 ? 32 : 64;
 }
 
 template <class T, class Y>
@@ -196,20 +212,36 @@ void launch_group_gemm(const GroupGemm<T, Y>& a, int tile,
         launch_group_gemm_tile(a, tile, stream);
         return;
       }
+      const int nt = (a.n + BN - 1) / BN;
+      // smaller tiles of unpacked rows while the chip is not full
+      while (!packed && tile > 16 &&
+             (long)nt * ((a.m + tile - 1) / tile) * gz < 512) tile /= 2;
       const int mt = packed ? a.max_tiles : (a.m + tile - 1) / tile;
-      const dim3 grid((a.n + BN - 1) / BN, mt, gz), block(NW * WAVE);
-      if (tile == 16)
-        group_gemm_stream_kernel<Y, 1><<<grid, block, 0, stream>>>(a);
+      const dim3 grid(nt, mt, gz);
+      auto go = [&](auto fm, auto nw) {
+        constexpr int FM = decltype(fm)::value, NW = decltype(nw)::value;
+        by_act(a.act, [&](auto act) {
+          group_gemm_stream_kernel<Y, decltype(act)::value, FM, NW>
+              <<<grid, dim3(NW * WAVE), 0, stream>>>(a);
+        });
+      };
+      using std::integral_constant;
+      if (tile == 16 && (long)nt * mt * gz < 256 && a.k >= 1024)
+        go(integral_constant<int, 1>{}, integral_constant<int, 16>{});
+      else if (tile == 16)
+        go(integral_constant<int, 1>{}, integral_constant<int, 4>{});
       else if (tile == 32)
-        group_gemm_stream_kernel<Y, 2><<<grid, block, 0, stream>>>(a);
+        go(integral_constant<int, 2>{}, integral_constant<int, 4>{});
       else
-        group_gemm_stream_kernel<Y, 4><<<grid, block, 0, stream>>>(a);
+        go(integral_constant<int, 4>{}, integral_constant<int, 4>{});
       return;
     }
   }
   const int mt = packed ? a.max_tiles : (a.m + AT - 1) / AT;
-  group_gemm_any_kernel<T, Y><<<dim3((a.n + AT - 1) / AT, mt, gz), 256, 0,
-                                stream>>>(a);
+  by_act(a.act, [&](auto act) {
+    group_gemm_any_kernel<T, Y, decltype(act)::value>
+        <<<dim3((a.n + AT - 1) / AT, mt, gz), 256, 0, stream>>>(a);
+  });
 }
 
 #define INSTANTIATE(T, Y)                                                    \
