@@ -50,7 +50,7 @@ void launch_attn_ctx_prefill(const AttnCtx<bf16_t>&, int entries, int max_len,
 bool attn_latent_supported(int dim, int vdim, int block_size);
 int attn_latent_splits(int entries, int max_len, int heads, int span);
 void launch_attn_latent(const AttnCtx<bf16_t>&, int entries, int max_len,
-                        int splits, float* part_o, float* part_ml,
+                        int span, int splits, float* part_o, float* part_ml,
                         hipStream_t);
 void launch_attn_ctx_merge(const AttnCtx<bf16_t>&, long rows, int splits,
                            const float* part_o, const float* part_ml,

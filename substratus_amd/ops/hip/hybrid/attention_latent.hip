@@ -7,14 +7,13 @@
 // goes to LDS as it is (direct loads, the next step's in flight, page numbers
 // another step ahead), except that the 16-byte pieces of a row are permuted
 // by the row, so that neither of the two products meets bank conflicts:
-//   scores   S^T = K Q^T: each of eight waves has one page's 16 keys and, of
-//            the queries, half (MT 2) or half of their elements (MT 1), in
-//            registers throughout. Scores meet in LDS;
-//   values   O^T = V^T P^T: each wave has an eighth of the columns, for all
-//            64 keys. V^T is read by the transposing LDS loads from the same
-//            rows. Every wave forms all weights for itself, in the registers
-//            where the product wants them, as bf16 high and low parts, so
-//            they keep 16 bits.
+//   scores   S^T = K Q^T: each wave has one page's 16 keys and 16 queries, in
+//            registers throughout (with 16 queries in all, half the waves).
+//            It forms their weights, once the waves have exchanged maxima;
+//   values   O^T = V^T P^T: each of the eight waves has an eighth of the
+//            columns, for all 64 keys. V^T is read by the transposing LDS
+//            loads from the same rows, weights through LDS as bf16 high and
+//            low parts, so they keep 16 bits.
 // Long contexts are split over workgroups and merged by attn_ctx_merge.
 #include "attention_ctx.h"
 
@@ -36,6 +35,12 @@ DEV_INLINE void load_to_lds(const void* g, void* lds) {
       (__attribute__((address_space(3))) unsigned int*)lds, 16, 0, 0);
 }
 
+DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
+  unsigned r;
+  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(lo), "v"(hi));
+  return r;
+}
+
 // Waits for LDS only: the next step's loads stay in flight.
 DEV_INLINE void lds_barrier() {
   asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
@@ -49,16 +54,18 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
                         float* __restrict__ part_ml) {
   constexpr int QT = MT * 16;
   constexpr int RC = KS * 4;                     // 16-byte pieces per LDS row
-  constexpr int QS = MT == 2 ? KS : KS / 2;      // key steps of one wave
-  constexpr int SS = MT == 2 ? 1 : 2;            // parts of a score
+  constexpr int PP = CH + 8;                     // padded row of weights
   constexpr int LOADS = PAGE * RC / WAVE / 2;    // of one wave per step
   static_assert(PAGE * RC % (2 * WAVE) == 0 && KS % 2 == 0);
   // one array: beside a second one the compiler guards every LDS read
   // against the direct loads in flight, and waits for them
-  __shared__ alignas(16) uint4 s_all[2 * CH * RC + SS * QT * (CH + 4) / 4];
+  __shared__ alignas(16) uint4
+      s_all[2 * CH * RC + 2 * QT * PP / 8 + PAGES * QT / 4];
   auto& s_c = *reinterpret_cast<uint4(*)[2][CH * RC]>(s_all);
-  auto& s_s = *reinterpret_cast<float(*)[SS][QT][CH + 4]>(
+  auto& s_p = *reinterpret_cast<short(*)[2][QT][PP]>(   // high and low parts
       s_all + 2 * CH * RC);
+  auto& s_m = *reinterpret_cast<float(*)[PAGES][QT]>(
+      s_all + 2 * CH * RC + 2 * QT * PP / 8);
 
   const int e = blockIdx.x, split = blockIdx.z;
   const Entry en = entry_of(a.seq_start, e);
@@ -83,23 +90,23 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
   int pg = page_at(st0);                         // of the step to load next
 
   // queries: lane = query, 8 consecutive elements
-  short8 q[QS];
-  const int ks0 = MT == 2 ? 0 : part * QS;
+  const bool scoring = part < MT;
+  const int mine = (scoring ? part : 0) * 16;
+  short8 q[KS];
+  int qpos;
   {
-    const int qi = min(q0 + (MT == 2 ? part * 16 : 0) + lo, nq - 1);
+    const int qi = min(q0 + mine + lo, nq - 1);
+    qpos = pos0 + qi / a.heads;
     const bf16_t* qp = a.q + (long)(en.row0 + qi / a.heads) * a.q_ld +
                        (long)(qi % a.heads) * a.dim;
     #pragma unroll
-    for (int ks = 0; ks < QS; ++ks) {
-      const int d = (ks0 + ks) * 32 + grp * 8;
-      q[ks] = d < a.dim ? *reinterpret_cast<const short8*>(qp + d)
-                        : (short8){0, 0, 0, 0, 0, 0, 0, 0};
+    for (int ks = 0; ks < KS; ++ks) {
+      const int d = ks * 32 + grp * 8;
+      q[ks] = scoring && d < a.dim
+          ? *reinterpret_cast<const short8*>(qp + d)
+          : (short8){0, 0, 0, 0, 0, 0, 0, 0};
     }
   }
-  int qpos[MT];
-  #pragma unroll
-  for (int mt = 0; mt < MT; ++mt)
-    qpos[mt] = pos0 + min(q0 + mt * 16 + lo, nq - 1) / a.heads;
 
   // the lane's pieces of its wave's half page
   const int pieces = a.dim / 8;
@@ -120,11 +127,11 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
                   &s_c[buf][page * PAGE * RC + (part * LOADS + i) * WAVE]);
   };
 
-  float m[MT], l[MT];
+  float m[MT], l = 0.f;                          // l: of the wave's own keys
   float4v o[CT][MT];
   #pragma unroll
   for (int mt = 0; mt < MT; ++mt) {
-    m[mt] = NEG; l[mt] = 0.f;
+    m[mt] = NEG;
     #pragma unroll
     for (int c = 0; c < CT; ++c) o[c][mt] = (float4v){0.f, 0.f, 0.f, 0.f};
   }
@@ -134,7 +141,7 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
   pg = page_at(st0 + 1);
   // queries are there before the loop, so that it never waits for them
   #pragma unroll
-  for (int ks = 0; ks < QS; ++ks) asm volatile("" : "+v"(q[ks]));
+  for (int ks = 0; ks < KS; ++ks) asm volatile("" : "+v"(q[ks]));
   for (int st = st0; st < st1; ++st) {
     const int buf = (st - st0) & 1;
     // the barrier at the end of the last step has released the other buffer
@@ -147,72 +154,77 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     }
     asm volatile("s_barrier" ::: "memory");
-    float4v s[2];
-    s[0] = s[1] = (float4v){0.f, 0.f, 0.f, 0.f};
-    const uint4* krow = &s_c[buf][(page * PAGE + lo) * RC];
-    #pragma unroll
-    for (int ks = 0; ks < QS; ++ks) {
-      const short8 k = *reinterpret_cast<const short8*>(
-          &krow[((ks0 + ks) * 4 + grp) ^ (lo & 7)]);
-      s[ks & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, q[ks], s[ks & 1],
-                                                          0, 0, 0);
-    }
-    *reinterpret_cast<float4v*>(
-        &s_s[MT == 2 ? 0 : part][(MT == 2 ? part * 16 : 0) + lo]
-            [page * PAGE + grp * 4]) = s[0] + s[1];
-    lds_barrier();
-
-    short8 ph[MT][2], pl[MT][2];                 // weights of keys
-    #pragma unroll
-    for (int mt = 0; mt < MT; ++mt) {            //   half * 32 + grp * 8 + j
-      float v[2][8];
+    float s[4];
+    if (scoring) {
+      float4v acc[2];
+      acc[0] = acc[1] = (float4v){0.f, 0.f, 0.f, 0.f};
+      const uint4* krow = &s_c[buf][(page * PAGE + lo) * RC];
+      #pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const short8 k = *reinterpret_cast<const short8*>(
+            &krow[(ks * 4 + grp) ^ (lo & 7)]);
+        acc[ks & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            k, q[ks], acc[ks & 1], 0, 0, 0);
+      }
+      const int key = st * CH + page * PAGE + grp * 4;
       float mx = NEG;
       #pragma unroll
-      for (int half = 0; half < 2; ++half)
-        #pragma unroll
-        for (int j4 = 0; j4 < 2; ++j4) {
-          const int k = half * 32 + grp * 8 + j4 * 4;
-          float4v f =
-              *reinterpret_cast<const float4v*>(&s_s[0][mt * 16 + lo][k]);
-          if constexpr (SS == 2)
-            f += *reinterpret_cast<const float4v*>(&s_s[1][mt * 16 + lo][k]);
-          #pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            const float x = st * CH + k + j <= qpos[mt] ? f[j] * scale2
-                                                        : -INFINITY;
-            v[half][j4 * 4 + j] = x;
-            mx = fmaxf(mx, x);
-          }
-        }
+      for (int i = 0; i < 4; ++i) {
+        s[i] = key + i <= qpos ? (acc[0][i] + acc[1][i]) * scale2 : -INFINITY;
+        mx = fmaxf(mx, s[i]);
+      }
       mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
       mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
-      const float mn = fmaxf(m[mt], mx);
-      const float keep = __builtin_amdgcn_exp2f(m[mt] - mn);
-      m[mt] = mn;
-      float sum = 0.f;
-      #pragma unroll
-      for (int half = 0; half < 2; ++half)
-        #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const float p = __builtin_amdgcn_exp2f(v[half][j] - mn);
-          sum += p;                              // exp2(-inf) is 0
-          const bf16_t h = f2bf(p), w = f2bf(p - bf2f(h));
-          ph[mt][half][j] = *reinterpret_cast<const short*>(&h);
-          pl[mt][half][j] = *reinterpret_cast<const short*>(&w);
-        }
-      sum += __shfl_xor(sum, 16, WAVE);
-      sum += __shfl_xor(sum, 32, WAVE);
-      l[mt] = l[mt] * keep + sum;
-      if (!__all(keep == 1.f)) {
-        #pragma unroll
-        for (int c = 0; c < CT; ++c) o[c][mt] *= keep;
-      }
+      if (grp == 0) s_m[page][mine + lo] = mx;
     }
+    lds_barrier();
+    float keep[MT];
+    #pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+      float mn = m[mt];
+      #pragma unroll
+      for (int p = 0; p < PAGES; ++p) mn = fmaxf(mn, s_m[p][mt * 16 + lo]);
+      keep[mt] = __builtin_amdgcn_exp2f(m[mt] - mn);
+      m[mt] = mn;
+    }
+    if (scoring) {
+      const float mn = MT == 2 && part == 1 ? m[MT - 1] : m[0];
+      float p[4], sum = 0.f;
+      #pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        p[i] = __builtin_amdgcn_exp2f(s[i] - mn);    // exp2(-inf) is 0
+        sum += p[i];
+      }
+      l = l * (MT == 2 && part == 1 ? keep[MT - 1] : keep[0]) + sum;
+      uint2 hi, low;
+      hi.x = cvt_pk_bf16(p[0], p[1]);
+      hi.y = cvt_pk_bf16(p[2], p[3]);
+      const float2 b0 = unpack_bf16x2(hi.x), b1 = unpack_bf16x2(hi.y);
+      low.x = cvt_pk_bf16(p[0] - b0.x, p[1] - b0.y);
+      low.y = cvt_pk_bf16(p[2] - b1.x, p[3] - b1.y);
+      const int at = page * PAGE + grp * 4;
+      *reinterpret_cast<uint2*>(&s_p[0][mine + lo][at]) = hi;
+      *reinterpret_cast<uint2*>(&s_p[1][mine + lo][at]) = low;
+    }
+    #pragma unroll
+    for (int mt = 0; mt < MT; ++mt)
+      if (!__all(keep[mt] == 1.f)) {
+        #pragma unroll
+        for (int c = 0; c < CT; ++c) o[c][mt] *= keep[mt];
+      }
+    lds_barrier();
     #pragma unroll
     for (int half = 0; half < 2; ++half) {
       // the lane's place in a transposing load: a key's four columns
       const int key = half * 32 + grp * 8 + (lo >> 2);
-      short8 vt[CT];
+      short8 vt[CT], ph[MT], pl[MT];
+      #pragma unroll
+      for (int mt = 0; mt < MT; ++mt) {
+        ph[mt] = *reinterpret_cast<const short8*>(
+            &s_p[0][mt * 16 + lo][half * 32 + grp * 8]);
+        pl[mt] = *reinterpret_cast<const short8*>(
+            &s_p[1][mt * 16 + lo][half * 32 + grp * 8]);
+      }
       #pragma unroll
       for (int c = 0; c < CT; ++c) {
         const int col = (wave * CT + c) * 16 + (lo & 3) * 4;
@@ -236,21 +248,29 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
         #pragma unroll
         for (int mt = 0; mt < MT; ++mt) {
           o[c][mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              vt[c], ph[mt][half], o[c][mt], 0, 0, 0);
+              vt[c], ph[mt], o[c][mt], 0, 0, 0);
           o[c][mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              vt[c], pl[mt][half], o[c][mt], 0, 0, 0);
+              vt[c], pl[mt], o[c][mt], 0, 0, 0);
         }
     }
     lds_barrier();
   }
 
+  // sums of all waves' keys
+  l += __shfl_xor(l, 16, WAVE);
+  l += __shfl_xor(l, 32, WAVE);
+  if (scoring && grp == 0) s_m[page][mine + lo] = l;
+  lds_barrier();
   #pragma unroll
   for (int mt = 0; mt < MT; ++mt) {
+    float sum = 0.f;
+    #pragma unroll
+    for (int p = 0; p < PAGES; ++p) sum += s_m[p][mt * 16 + lo];
     const int qi = q0 + mt * 16 + lo;
     if (qi >= nq) continue;
     const long row = (long)en.row0 * a.heads + qi;   // row and head
     const long at = row * splits + split;
-    const float f = splits == 1 ? 1.f / l[mt] : 1.f;
+    const float f = splits == 1 ? 1.f / sum : 1.f;
     #pragma unroll
     for (int c = 0; c < CT; ++c) {
       const int col = (wave * CT + c) * 16 + grp * 4;
@@ -263,15 +283,17 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
     }
     if (splits > 1 && wave == 0 && grp == 0) {
       part_ml[at * 2] = m[mt];
-      part_ml[at * 2 + 1] = l[mt];
+      part_ml[at * 2 + 1] = sum;
     }
   }
 }
 
-// Queries per workgroup: 32 where that leaves enough of them.
-int query_tile(int entries, int max_len, int heads) {
-  const long q = (long)max_len * heads;
-  return q > 16 && entries * ((q + 31) / 32) >= 192 ? 32 : 16;
+// Queries per workgroup: 32, which reads the latents once for as many heads,
+// where that leaves enough workgroups (or steps to split between them).
+int query_tile(int entries, int max_len, int heads, int span) {
+  const long q = (long)max_len * heads, groups = entries * ((q + 31) / 32);
+  if (q <= 16) return 16;
+  return groups >= 192 || (groups >= 64 && span >= 24 * CH) ? 32 : 16;
 }
 
 }  // namespace
@@ -284,18 +306,18 @@ bool attn_latent_supported(int dim, int vdim, int block_size) {
 // Workgroups that share one context: enough for every CU, but at least two
 // steps for each. `span`: most keys a row can see.
 int attn_latent_splits(int entries, int max_len, int heads, int span) {
-  const int qt = query_tile(entries, max_len, heads);
+  const int qt = query_tile(entries, max_len, heads, span);
   const long groups = (long)entries * (((long)max_len * heads + qt - 1) / qt);
   const int steps = (span + CH - 1) / CH;
   int s = 1;
-  while (s < 32 && groups * s * 3 < 512 && steps >= s * 4) s *= 2;
+  while (s < 32 && groups * s < 256 && steps >= s * 4) s *= 2;
   return s;
 }
 
 void launch_attn_latent(const AttnCtx<bf16_t>& a, int entries, int max_len,
-                        int splits, float* part_o, float* part_ml,
+                        int span, int splits, float* part_o, float* part_ml,
                         hipStream_t stream) {
-  const int qt = query_tile(entries, max_len, a.heads);
+  const int qt = query_tile(entries, max_len, a.heads, span);
   const dim3 grid(entries, ((long)max_len * a.heads + qt - 1) / qt, splits);
   auto go = [&](auto ks, auto ct) {
     constexpr int KS = decltype(ks)::value, CT = decltype(ct)::value;

@@ -252,7 +252,7 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
           po = torch::empty({rows, heads, splits, vdim}, opt);
           pml = torch::empty({rows, heads, splits, 2}, opt);
         }
-        launch_attn_latent(a, entries, longest, splits,
+        launch_attn_latent(a, entries, longest, span, splits,
                            splits > 1 ? ptr<float>(po) : nullptr,
                            splits > 1 ? ptr<float>(pml) : nullptr, stream());
         if (splits > 1)

@@ -36,6 +36,7 @@ struct GroupGemm {
   const T* table;          // row t at table + t * t_ld
   long t_ld;
   int vocab;
+  bool quads;              // set by launch_group_gemm: four columns at a time
 };
 
 struct Tile {
@@ -72,18 +73,46 @@ DEV_INLINE float gelu_tanh_f(float v) {
   return v * __builtin_amdgcn_rcpf(1.f + __expf(-2.f * in));
 }
 
-template <Act ACT, bool FAST, class T, class Y>
-DEV_INLINE float group_act(const GroupGemm<T, Y>& a, int r, int g, int n,
-                           float v) {
-  if constexpr (ACT == Act::GELU) return gelu_erf_f<FAST>(v);
+// N columns of a row from n on, all of them there.
+template <Act ACT, bool FAST, int N, class T, class Y>
+DEV_INLINE void group_act(const GroupGemm<T, Y>& a, int r, int g, int n,
+                          float* v) {
+  float f[N];
   if constexpr (ACT == Act::GATE)
-    return v * sigmoid_f(ld1(a.gate + (long)r * a.gate_ld +
-                             (long)g * a.gate_gs + n));
+    ldv<N>(a.gate + (long)r * a.gate_ld + (long)g * a.gate_gs + n, f);
   if constexpr (ACT == Act::SIDE) {
     const int t = min(max(a.tokens[r], 0), a.vocab - 1);
-    return gelu_tanh_f<FAST>(v) * ld1(a.table + (long)t * a.t_ld + n);
+    ldv<N>(a.table + (long)t * a.t_ld + n, f);
   }
-  return v;
+  #pragma unroll
+  for (int j = 0; j < N; ++j) {
+    if constexpr (ACT == Act::GELU) v[j] = gelu_erf_f<FAST>(v[j]);
+    if constexpr (ACT == Act::GATE) v[j] *= sigmoid_f(f[j]);
+    if constexpr (ACT == Act::SIDE) v[j] = gelu_tanh_f<FAST>(v[j]) * f[j];
+  }
+}
+
+typedef __attribute__((ext_vector_type(4))) float float4v;
+
+// Four consecutive columns of a row, as far as they are there.
+template <Act ACT, class Y>
+DEV_INLINE void store4(const GroupGemm<bf16_t, Y>& a, Tile t, int r, int n,
+                       float4v acc) {
+  if (r >= t.r1 || n >= a.n) return;
+  Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n;
+  if (a.quads) {
+    float v[4] = {acc[0], acc[1], acc[2], acc[3]};
+    group_act<ACT, true, 4>(a, r, t.g, n, v);
+    stv<4>(y, v);
+    return;
+  }
+  #pragma unroll
+  for (int c = 0; c < 4; ++c) {
+    float v = acc[c];
+    if (n + c >= a.n) return;
+    group_act<ACT, true, 1>(a, r, t.g, n + c, &v);
+    st1(y + c, v);
+  }
 }
 
 // Calls f(integral_constant<Act>) with the product's.

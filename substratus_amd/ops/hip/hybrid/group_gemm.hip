@@ -2,8 +2,9 @@
 //
 //   stream   bf16, few rows per group: bound by reading the weights once.
 //            Every wave takes a share of the inner dimension of a tile of
-//            BM rows and 64 columns (4 waves, or 16 where there are few
-//            tiles), with both operands going from memory
+//            rows and 64 columns (4 waves, or 16 where there are few tiles;
+//            where the inner dimension is short, a share of the rows), with
+//            both operands going from memory
 //            straight into the matrix cores' registers (a fragment is 16
 //            consecutive bytes of a row, so nothing is gained by LDS); there
 //            is no barrier until the partial tiles are added up.
@@ -16,7 +17,6 @@
 namespace {
 
 typedef __attribute__((ext_vector_type(8))) short short8;
-typedef __attribute__((ext_vector_type(4))) float float4v;
 
 constexpr int BN = 64;
 constexpr int KC = 32;         // inner step of one matrix instruction
@@ -29,17 +29,18 @@ DEV_INLINE short8 frag(const bf16_t* p, bool there) {
   else return *reinterpret_cast<const short8*>(p);
 }
 
-// NW waves: shares of the inner dimension
-template <class Y, Act ACT, int FM, int NW>
-__global__ __launch_bounds__(NW * WAVE)
+// KW waves share the inner dimension, RW the rows
+template <class Y, Act ACT, int FM, int KW, int RW>
+__global__ __launch_bounds__(KW * RW * WAVE)
 void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
-  constexpr int BM = FM * 16, FN = BN / 16, PAD = 4;
-  __shared__ alignas(16) float s_p[NW][BM][BN + PAD];
+  constexpr int BM = FM * 16 * RW, FN = BN / 16, PAD = 4;
+  static_assert(KW == 1 || RW == 1);
   const Tile t = tile_of(a, blockIdx.y, blockIdx.z, BM);
   if (t.r1 <= t.r0) return;
   const int n0 = blockIdx.x * BN;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int lo = lane & 15, kq = (lane >> 4) * 8;
+  const int r0 = t.r0 + (RW > 1 ? wave * FM * 16 : 0);
 
   const bf16_t* wp[FN];
   const bf16_t* xp[FM];
@@ -49,7 +50,7 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
             kq;
   #pragma unroll
   for (int f = 0; f < FM; ++f) {
-    const int r = min(t.r0 + f * 16 + lo, t.r1 - 1);
+    const int r = min(r0 + f * 16 + lo, t.r1 - 1);
     xp[f] = a.x + (long)(a.src != nullptr ? a.src[r] : r) * a.x_ld +
             t.g * a.x_gs + kq;
   }
@@ -60,7 +61,8 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
     for (int j = 0; j < FM; ++j) acc[i][j] = (float4v){0.f, 0.f, 0.f, 0.f};
 
   const int chunks = (a.k + KC - 1) / KC;
-  const int c0 = chunks * wave / NW, c1 = chunks * (wave + 1) / NW;
+  const int c0 = KW > 1 ? chunks * wave / KW : 0,
+            c1 = KW > 1 ? chunks * (wave + 1) / KW : chunks;
   // U chunks at a time: their loads are in flight together
   auto steps = [&](int c, auto u, bool whole) {
     constexpr int U = decltype(u)::value;
@@ -70,7 +72,7 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
       const int k = (c + i) * KC;
       const bool there = whole || k + kq < a.k;
       #pragma unroll
-      for (int f = 0; f < FN; ++f) wf[i][f] = frag<true>(wp[f] + k, there);
+      for (int f = 0; f < FN; ++f) wf[i][f] = frag<false>(wp[f] + k, there);
       #pragma unroll
       for (int f = 0; f < FM; ++f) xf[i][f] = frag<false>(xp[f] + k, there);
     }
@@ -92,39 +94,33 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
   for (; c < full; ++c) steps(c, std::integral_constant<int, 1>{}, true);
   if (c < c1) steps(c, std::integral_constant<int, 1>{}, false);
 
-  #pragma unroll
-  for (int i = 0; i < FN; ++i)
+  const int c4 = (lane >> 4) * 4;
+  if constexpr (KW == 1) {
     #pragma unroll
-    for (int j = 0; j < FM; ++j)
-      *reinterpret_cast<float4v*>(
-          &s_p[wave][j * 16 + lo][i * 16 + (lane >> 4) * 4]) = acc[i][j];
-  __syncthreads();
-  const bool quads = a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0;
-  for (int i = threadIdx.x; i < BM * BN / 4; i += NW * WAVE) {
-    const int r = t.r0 + i / (BN / 4), c4 = i % (BN / 4) * 4, n = n0 + c4;
-    if (r >= t.r1 || n >= a.n) continue;
-    float v[4] = {0.f, 0.f, 0.f, 0.f};
-    #pragma unroll
-    for (int w = 0; w < NW; ++w) {
-      const float4v p =
-          *reinterpret_cast<const float4v*>(&s_p[w][r - t.r0][c4]);
+    for (int i = 0; i < FN; ++i)
       #pragma unroll
-      for (int j = 0; j < 4; ++j) v[j] += p[j];
-    }
+      for (int j = 0; j < FM; ++j)
+        store4<ACT>(a, t, r0 + j * 16 + lo, n0 + i * 16 + c4, acc[i][j]);
+  } else {
+    __shared__ alignas(16) float s_p[KW][BM][BN + PAD];
     #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (n + j < a.n)
-        v[j] = group_act<ACT, true>(a, r, t.g, n + j, v[j]);
-    Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n;
-    if (quads) {
-      stv<4>(y, v);
-    } else {
+    for (int i = 0; i < FN; ++i)
       #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (n + j < a.n) st1(y + j, v[j]);
+      for (int j = 0; j < FM; ++j)
+        *reinterpret_cast<float4v*>(&s_p[wave][j * 16 + lo][i * 16 + c4]) =
+            acc[i][j];
+    __syncthreads();
+    for (int i = threadIdx.x; i < BM * BN / 4; i += KW * WAVE) {
+      const int r = i / (BN / 4), c = i % (BN / 4) * 4;
+      float4v v = {0.f, 0.f, 0.f, 0.f};
+      #pragma unroll
+      for (int w = 0; w < KW; ++w)
+        v += *reinterpret_cast<const float4v*>(&s_p[w][r][c]);
+      store4<ACT>(a, t, t.r0 + r, n0 + c, v);
     }
   }
-  if (a.tail && blockIdx.x == 0) copy_tail(a, t, threadIdx.x, NW * WAVE);
+  if (a.tail && blockIdx.x == 0)
+    copy_tail(a, t, threadIdx.x, KW * RW * WAVE);
 }
 
 // 32 x 32 outputs per workgroup, 2 x 2 per thread, operands through LDS.
@@ -164,9 +160,10 @@ void group_gemm_any_kernel(GroupGemm<T, Y> a) {
     #pragma unroll
     for (int j = 0; j < 2; ++j) {
       const int r = t.r0 + ty + 16 * i, n = n0 + tx + 16 * j;
-      if (r < t.r1 && n < a.n)
-        st1(a.y + (long)r * a.y_ld + t.g * a.y_gs + n,
-            group_act<ACT, false>(a, r, t.g, n, acc[i][j]));
+      if (r < t.r1 && n < a.n) {
+        group_act<ACT, false, 1>(a, r, t.g, n, &acc[i][j]);
+        st1(a.y + (long)r * a.y_ld + t.g * a.y_gs + n, acc[i][j]);
+      }
     }
   if (a.tail && blockIdx.x == 0) copy_tail(a, t, threadIdx.x, 256);
 }
@@ -200,40 +197,60 @@ bool group_gemm_takes(const GroupGemm<T, Y>& a, int tile) {
   return tile == AT;
 }
 
+// everything a store touches comes in aligned groups of four columns
 template <class T, class Y>
-void launch_group_gemm(const GroupGemm<T, Y>& a, int tile,
+bool by_quads(const GroupGemm<T, Y>& a) {
+  auto ok = [](const void* p, size_t item) {
+    return reinterpret_cast<uintptr_t>(p) % (4 * item) == 0;
+  };
+  return a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0 &&
+         ok(a.y, sizeof(Y)) && a.gate_ld % 4 == 0 && a.gate_gs % 4 == 0 &&
+         ok(a.gate, sizeof(T)) && a.t_ld % 4 == 0 && ok(a.table, sizeof(T));
+}
+
+template <class T, class Y>
+void launch_group_gemm(const GroupGemm<T, Y>& given, int tile,
                        hipStream_t stream) {
+  GroupGemm<T, Y> a = given;
+  a.quads = by_quads(a);
   const bool packed = a.tiles != nullptr;
   const int gz = packed ? 1 : a.groups;
   if constexpr (std::is_same_v<T, bf16_t>) {
-    if (!packed && tile > 64 && !group_gemm_takes(a, tile)) tile = 64;
+    if (!packed && tile > 64 &&
+        (!group_gemm_takes(a, tile) ||
+         (long)((a.n + tile - 1) / tile) * ((a.m + tile - 1) / tile) * gz <
+             128))
+      tile = 64;
     if (group_gemm_takes(a, tile) && pieces(a)) {
       if (tile > 64) {
         launch_group_gemm_tile(a, tile, stream);
         return;
       }
       const int nt = (a.n + BN - 1) / BN;
+      const bool flat = !packed && a.k <= 512 && tile == 64;
       // smaller tiles of unpacked rows while the chip is not full
-      while (!packed && tile > 16 &&
+      while (!packed && !flat && tile > 16 &&
              (long)nt * ((a.m + tile - 1) / tile) * gz < 512) tile /= 2;
       const int mt = packed ? a.max_tiles : (a.m + tile - 1) / tile;
       const dim3 grid(nt, mt, gz);
-      auto go = [&](auto fm, auto nw) {
-        constexpr int FM = decltype(fm)::value, NW = decltype(nw)::value;
+      auto go = [&](auto fm, auto kw, auto rw) {
+        constexpr int FM = decltype(fm)::value, KW = decltype(kw)::value,
+                      RW = decltype(rw)::value;
         by_act(a.act, [&](auto act) {
-          group_gemm_stream_kernel<Y, decltype(act)::value, FM, NW>
-              <<<grid, dim3(NW * WAVE), 0, stream>>>(a);
+          group_gemm_stream_kernel<Y, decltype(act)::value, FM, KW, RW>
+              <<<grid, dim3(KW * RW * WAVE), 0, stream>>>(a);
         });
       };
-      using std::integral_constant;
-      if (tile == 16 && (long)nt * mt * gz < 256 && a.k >= 1024)
-        go(integral_constant<int, 1>{}, integral_constant<int, 16>{});
-      else if (tile == 16)
-        go(integral_constant<int, 1>{}, integral_constant<int, 4>{});
-      else if (tile == 32)
-        go(integral_constant<int, 2>{}, integral_constant<int, 4>{});
-      else
-        go(integral_constant<int, 4>{}, integral_constant<int, 4>{});
+      constexpr std::integral_constant<int, 1> c1{};
+      constexpr std::integral_constant<int, 2> c2{};
+      constexpr std::integral_constant<int, 4> c4{};
+      constexpr std::integral_constant<int, 16> c16{};
+      if (flat) go(c1, c1, c4);
+      else if (tile == 16 && (long)nt * mt * gz < 256 && a.k >= 1024)
+        go(c1, c16, c1);
+      else if (tile == 16) go(c1, c4, c1);
+      else if (tile == 32) go(c2, c4, c1);
+      else go(c4, c4, c1);
       return;
     }
   }

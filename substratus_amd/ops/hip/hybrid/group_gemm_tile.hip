@@ -14,7 +14,6 @@
 namespace {
 
 typedef __attribute__((ext_vector_type(8))) short short8;
-typedef __attribute__((ext_vector_type(4))) float float4v;
 
 constexpr int BK = 64;
 constexpr int XCDS = 8;
@@ -40,25 +39,6 @@ DEV_INLINE Tile my_tile(const GroupGemm<bf16_t, Y>& a, int bm, int bn,
       (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + b / XCDS;
   *n0 = id % nt * bn;
   return tile_of(a, id / nt, blockIdx.y, bm);
-}
-
-// Four consecutive columns of a row.
-template <Act ACT, class Y>
-DEV_INLINE void store4(const GroupGemm<bf16_t, Y>& a, Tile t, int r, int n,
-                       float4v acc) {
-  if (r >= t.r1 || n >= a.n) return;
-  Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n;
-  float v[4];
-  #pragma unroll
-  for (int c = 0; c < 4; ++c)
-    v[c] = n + c < a.n ? group_act<ACT, true>(a, r, t.g, n + c, acc[c]) : 0.f;
-  if (a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0) {
-    stv<4>(y, v);
-  } else {
-    #pragma unroll
-    for (int c = 0; c < 4; ++c)
-      if (n + c < a.n) st1(y + c, v[c]);
-  }
 }
 
 // One step ahead, two barriers per step.

@@ -10,17 +10,21 @@
 
 namespace {
 
-// index of the largest value (the lowest such index) over the wave
-DEV_INLINE void wave_argmax(float& v, int& i) {
-  #pragma unroll
-  for (int off = 32; off > 0; off >>= 1) {
-    const float ov = __shfl_xor(v, off, WAVE);
-    const int oi = __shfl_xor(i, off, WAVE);
-    if (ov > v || (ov == v && oi < i)) { v = ov; i = oi; }
-  }
-}
-
 constexpr int SW = 4;           // tokens per workgroup
+
+// How many of n values (padded with -inf to fours) come before value v of
+// index i, that is, are larger, or equal with a lower index. NaNs come last.
+DEV_INLINE int rank_of(const float* s, int n, float v, int i) {
+  int r = 0;
+  for (int j = 0; j < n; j += 4) {
+    const float4 f = *reinterpret_cast<const float4*>(s + j);
+    r += f.x > v || (f.x == v && j < i);
+    r += f.y > v || (f.y == v && j + 1 < i);
+    r += f.z > v || (f.z == v && j + 2 < i);
+    r += f.w > v || (f.w == v && j + 3 < i);
+  }
+  return r;
+}
 
 // PL: experts per lane
 template <int PL>
@@ -28,87 +32,72 @@ __global__ __launch_bounds__(SW * WAVE)
 void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
                        const float* __restrict__ z, int rows, int experts,
                        int top, int groups, int keep) {
-  extern __shared__ float s_all[];
+  extern __shared__ float4 s_all[];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-  const long row = (long)blockIdx.x * SW + wave;
-  float* s_z = s_all + wave * experts;          // the token's scores
-  const bool live = row < rows;
+  const int pad = (experts + 3) / 4 * 4;
+  const long row = min((long)blockIdx.x * SW + wave, (long)rows - 1);
+  float* s_z = reinterpret_cast<float*>(s_all) + wave * 2 * pad;
+  float* s_g = s_z + pad;                       // best score of each group
+  const int size = experts / groups;
   float v[PL];
   float mx = -INFINITY;
+  // scores that are no numbers: weights are none either, but experts are
+  for (int r = lane; r < top; r += WAVE) ids[row * top + r] = 0;
   #pragma unroll
   for (int i = 0; i < PL; ++i) {
     const int e = lane + i * WAVE;
-    v[i] = live && e < experts ? z[row * experts + e] : -INFINITY;
-    if (e < experts) s_z[e] = v[i];
+    v[i] = e < experts ? z[row * experts + e] : -INFINITY;
+    if (e < pad) s_z[e] = v[i];
     mx = fmaxf(mx, v[i]);
   }
-  __syncthreads();
-  if (!live) return;
   mx = wave_max(mx);
   float sum = 0.f;
   #pragma unroll
   for (int i = 0; i < PL; ++i)
     if (lane + i * WAVE < experts) sum += expf(v[i] - mx);
   sum = wave_sum(sum);
+  __syncthreads();
 
   if (keep < groups) {
-    // best score of each group: lanes take groups in turn
-    const int size = experts / groups;
-    float gv[PL];
-    bool kept[PL];
+    float g[PL];
     #pragma unroll
     for (int i = 0; i < PL; ++i) {
-      gv[i] = -INFINITY;
-      kept[i] = false;
-      const int g = lane + i * WAVE;
-      if (g < groups)
-        for (int e = 0; e < size; ++e) gv[i] = fmaxf(gv[i], s_z[g * size + e]);
+      g[i] = -INFINITY;
+      const int n = lane + i * WAVE;
+      if (n < groups)
+        for (int e = 0; e < size; ++e) g[i] = fmaxf(g[i], s_z[n * size + e]);
+      if (n < pad) s_g[n] = g[i];
     }
-    for (int r = 0; r < keep; ++r) {
-      float bv = -INFINITY;
-      int bi = 0x7fffffff;
-      #pragma unroll
-      for (int i = 0; i < PL; ++i) {
-        const int g = lane + i * WAVE;
-        if (g < groups && !kept[i] && (bi == 0x7fffffff || gv[i] > bv)) {
-          bv = gv[i]; bi = g;
-        }
-      }
-      wave_argmax(bv, bi);
-      #pragma unroll
-      for (int i = 0; i < PL; ++i)
-        if (lane + i * WAVE == bi) kept[i] = true;
-    }
-    // experts of the other groups cannot be chosen
+    __syncthreads();
+    #pragma unroll
+    for (int i = 0; i < PL; ++i)
+      if (lane + i * WAVE < groups &&
+          rank_of(s_g, groups, g[i], lane + i * WAVE) >= keep)
+        g[i] = INFINITY;                        // marks a group left out
+    __syncthreads();
+    #pragma unroll
+    for (int i = 0; i < PL; ++i)
+      if (lane + i * WAVE < groups) s_g[lane + i * WAVE] = g[i];
+    __syncthreads();
     #pragma unroll
     for (int i = 0; i < PL; ++i) {
       const int e = lane + i * WAVE;
-      const int g = e < experts ? e / size : 0;
-      unsigned long long any[PL];
-      #pragma unroll
-      for (int j = 0; j < PL; ++j) any[j] = __ballot(kept[j]);
-      bool in = false;
-      #pragma unroll
-      for (int j = 0; j < PL; ++j)
-        if (g / WAVE == j) in = any[j] >> (g % WAVE) & 1;
-      if (!in) v[i] = -INFINITY;
+      if (e < experts && s_g[e / size] == INFINITY) {
+        v[i] = -INFINITY;
+        s_z[e] = -INFINITY;
+      }
     }
+    __syncthreads();
   }
-  for (int r = 0; r < top; ++r) {
-    float bv = -INFINITY;
-    int bi = 0x7fffffff;
-    #pragma unroll
-    for (int i = 0; i < PL; ++i)
-      if (v[i] > bv) { bv = v[i]; bi = lane + i * WAVE; }
-    wave_argmax(bv, bi);
-    if (lane == 0) {
-      // scores that are no numbers choose the first expert, with their weight
-      ids[row * top + r] = bi < experts ? bi : 0;
-      weights[row * top + r] = expf(bv - mx) / sum;
+  #pragma unroll
+  for (int i = 0; i < PL; ++i) {
+    const int e = lane + i * WAVE;
+    if (e >= experts) continue;
+    const int r = rank_of(s_z, experts, v[i], e);
+    if (r < top) {
+      ids[row * top + r] = e;
+      weights[row * top + r] = expf(v[i] - mx) / sum;
     }
-    #pragma unroll
-    for (int i = 0; i < PL; ++i)
-      if (lane + i * WAVE == bi) v[i] = -INFINITY;
   }
 }
 
@@ -170,8 +159,8 @@ void launch_moe_select(int* ids, float* weights, const float* z, int rows,
   auto go = [&](auto pl) {
     moe_select_kernel<decltype(pl)::value>
         <<<dim3((rows + SW - 1) / SW), dim3(SW * WAVE),
-           SW * experts * sizeof(float), stream>>>(ids, weights, z, rows,
-                                                   experts, top, groups, keep);
+           SW * 2 * ((experts + 3) / 4 * 4) * sizeof(float), stream>>>(
+            ids, weights, z, rows, experts, top, groups, keep);
   };
   if (experts <= WAVE) go(std::integral_constant<int, 1>{});
   else if (experts <= 4 * WAVE) go(std::integral_constant<int, 4>{});
