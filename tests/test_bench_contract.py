@@ -51,10 +51,11 @@ def test_bench_train_schema():
 
 
 @pytest.mark.timeout(300)
-def test_bench_hybrid_schema():
+@pytest.mark.parametrize("model", ["kakovik-tiny", "guronex-tiny"])
+def test_bench_hybrid_schema(model):
     out = subprocess.run(
         [sys.executable, "bench.py", "--mode", "hybrid", "--steps", "2",
-         "--warmup", "1", "--model", "kakovik-tiny"],
+         "--warmup", "1", "--model", model],
         cwd=ROOT, capture_output=True, text=True, timeout=280,
         env=dict(os.environ, HIP_VISIBLE_DEVICES=""))
     assert out.returncode == 0, out.stderr[-2000:]
@@ -62,7 +63,7 @@ def test_bench_hybrid_schema():
     assert REQUIRED <= set(r)
     assert r["metric"] == "hybrid_decode_tokens_per_s"
     models = {p["model"] for p in r["config"]["points"]}
-    assert models == {"kakovik-tiny", "llama-tiny"}
+    assert models == {model, "llama-tiny"}
     for p in r["config"]["points"]:
         assert p["prefill_tokens_per_s"] > 0 and p["decode_tokens_per_s"] > 0
 
