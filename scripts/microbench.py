@@ -256,9 +256,9 @@ def bench_latent():
                    pos), it), rows * (h * r * 2 + spec.row * 2) * 2)
         router = torch.randn(moe.experts, w, **bf) * 0.02
         ext = hy._ext()
-        z = torch.empty(rows, moe.experts, device="cuda")
+        z = ext.router_scores(x, router)
         report(f"  router_scores rows={rows} {w}->{moe.experts}",
-               timeit(lambda: ext.router_scores(z, x, router), it),
+               timeit(lambda: ext.router_scores(x, router), it),
                rows * w * 2 + router.numel() * 2, 2.0 * rows * w * moe.experts)
         ids = torch.empty(rows, moe.top, device="cuda", dtype=torch.int32)
         wts = torch.empty(rows, moe.top, device="cuda")

@@ -7,6 +7,7 @@ The libraries land at substratus_amd/_C*.so and substratus_amd/_hybrid*.so
 default all.
 """
 
+import glob
 import os
 
 from setuptools import find_packages, setup
@@ -25,6 +26,16 @@ HYBRID_DIR = os.path.join(HIP_DIR, "hybrid")
 def hip_sources(folder):
     return [os.path.join(folder, f) for f in sorted(os.listdir(folder))
             if f.endswith(".hip") and not f.endswith("_hip.hip")]
+
+
+def drop_stale_objects():
+    """Objects older than a header: the build itself only looks at sources."""
+    headers = glob.glob(os.path.join(HIP_DIR, "**", "*.h"), recursive=True)
+    newest = max(os.path.getmtime(h) for h in headers)
+    for obj in glob.glob(os.path.join(ROOT, "build", "temp*", "**", "*.o"),
+                         recursive=True):
+        if os.path.getmtime(obj) < newest:
+            os.remove(obj)
 
 
 def extension(name, sources):
@@ -46,6 +57,7 @@ extensions = {
     "_hybrid": hip_sources(HYBRID_DIR) + [
         os.path.join(HIP_DIR, "activation.hip")],
 }
+drop_stale_objects()
 wanted = os.environ.get("SUB_EXT", ",".join(extensions)).split(",")
 
 setup(

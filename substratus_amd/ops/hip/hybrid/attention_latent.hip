@@ -49,7 +49,7 @@ DEV_INLINE void lds_barrier() {
 // KS: 32-wide steps of the key size (even); CT: 16-wide column tiles per wave
 template <int KS, int CT, int MT>
 __global__ __launch_bounds__(NW * WAVE)
-void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
+void attn_latent_kernel(AttnCtx<bf16_t> a, int entries, int splits,
                         float* __restrict__ part_o,
                         float* __restrict__ part_ml) {
   constexpr int QT = MT * 16;
@@ -67,9 +67,9 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
   auto& s_m = *reinterpret_cast<float(*)[PAGES][QT]>(
       s_all + 2 * CH * RC + 2 * QT * PP / 8);
 
-  const int e = blockIdx.x, split = blockIdx.z;
+  const int e = blockIdx.x % entries, split = blockIdx.y;
   const Entry en = entry_of(a.seq_start, e);
-  const int q0 = blockIdx.y * QT, nq = en.n * a.heads;
+  const int q0 = blockIdx.x / entries * QT, nq = en.n * a.heads;
   if (q0 >= nq) return;
   // page numbers come by scalar loads, which the counted waits do not see
   const auto* bt = (const __attribute__((address_space(4))) int*)(
@@ -88,25 +88,6 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
     return bt[min(st * PAGES + page, pages - 1)];
   };
   int pg = page_at(st0);                         // of the step to load next
-
-  // queries: lane = query, 8 consecutive elements
-  const bool scoring = part < MT;
-  const int mine = (scoring ? part : 0) * 16;
-  short8 q[KS];
-  int qpos;
-  {
-    const int qi = min(q0 + mine + lo, nq - 1);
-    qpos = pos0 + qi / a.heads;
-    const bf16_t* qp = a.q + (long)(en.row0 + qi / a.heads) * a.q_ld +
-                       (long)(qi % a.heads) * a.dim;
-    #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      const int d = ks * 32 + grp * 8;
-      q[ks] = scoring && d < a.dim
-          ? *reinterpret_cast<const short8*>(qp + d)
-          : (short8){0, 0, 0, 0, 0, 0, 0, 0};
-    }
-  }
 
   // the lane's pieces of its wave's half page
   const int pieces = a.dim / 8;
@@ -127,6 +108,28 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
                   &s_c[buf][page * PAGE * RC + (part * LOADS + i) * WAVE]);
   };
 
+  if (st0 < st1) load(0);
+  pg = page_at(st0 + 1);
+
+  // queries: lane = query, 8 consecutive elements
+  const bool scoring = part < MT;
+  const int mine = (scoring ? part : 0) * 16;
+  short8 q[KS];
+  int qpos;
+  {
+    const int qi = min(q0 + mine + lo, nq - 1);
+    qpos = pos0 + qi / a.heads;
+    const bf16_t* qp = a.q + (long)(en.row0 + qi / a.heads) * a.q_ld +
+                       (long)(qi % a.heads) * a.dim;
+    #pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int d = ks * 32 + grp * 8;
+      q[ks] = scoring && d < a.dim
+          ? *reinterpret_cast<const short8*>(qp + d)
+          : (short8){0, 0, 0, 0, 0, 0, 0, 0};
+    }
+  }
+
   float m[MT], l = 0.f;                          // l: of the wave's own keys
   float4v o[CT][MT];
   #pragma unroll
@@ -136,9 +139,6 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int splits,
     for (int c = 0; c < CT; ++c) o[c][mt] = (float4v){0.f, 0.f, 0.f, 0.f};
   }
   const float scale2 = a.scale * LOG2E;
-
-  if (st0 < st1) load(0);
-  pg = page_at(st0 + 1);
   // queries are there before the loop, so that it never waits for them
   #pragma unroll
   for (int ks = 0; ks < KS; ++ks) asm volatile("" : "+v"(q[ks]));
@@ -318,15 +318,15 @@ void launch_attn_latent(const AttnCtx<bf16_t>& a, int entries, int max_len,
                         int span, int splits, float* part_o, float* part_ml,
                         hipStream_t stream) {
   const int qt = query_tile(entries, max_len, a.heads, span);
-  const dim3 grid(entries, ((long)max_len * a.heads + qt - 1) / qt, splits);
+  const dim3 grid(entries * (((long)max_len * a.heads + qt - 1) / qt), splits);
   auto go = [&](auto ks, auto ct) {
     constexpr int KS = decltype(ks)::value, CT = decltype(ct)::value;
     if (qt == 16)
       attn_latent_kernel<KS, CT, 1><<<grid, dim3(NW * WAVE), 0, stream>>>(
-          a, splits, part_o, part_ml);
+          a, entries, splits, part_o, part_ml);
     else
       attn_latent_kernel<KS, CT, 2><<<grid, dim3(NW * WAVE), 0, stream>>>(
-          a, splits, part_o, part_ml);
+          a, entries, splits, part_o, part_ml);
   };
   using std::integral_constant;
   if (a.dim <= 192 && a.vdim <= 128)

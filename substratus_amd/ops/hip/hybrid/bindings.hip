@@ -17,7 +17,7 @@ template <class T>
 void launch_latent_prepare(T*, long, int, int, int, int, int, const float*, float, const double*, int, const int*, T*, const int*, long, hipStream_t);
 void launch_latent_gather(void*, void*, const void*, int, int, int, const int*, int, const int*, int, int, hipStream_t);
 int moe_max_experts();
-void launch_moe_select(int*, float*, const float*, int, int, int, int, int, hipStream_t);
+void launch_moe_select(int*, float*, const float*, int, int, int, int, int, int, hipStream_t);
 void launch_moe_sort(int*, int*, int*, int*, const int*, int, int, int, int, hipStream_t);
 template <class T>
 void launch_embed_norm(T*, float*, const T*, const int*, const float*, long, int, int, float, float, hipStream_t);
@@ -409,6 +409,7 @@ GroupGemm<T, Y> product(const Tensor& y, const Tensor& x, const Tensor& w) {
   a.n = w.size(-2); a.k = w.size(-1);
   a.groups = w.dim() == 3 ? w.size(0) : 1;
   a.m = x.size(0);
+  a.splits = 1;
   a.act = Act::NONE;
   return a;
 }
@@ -436,7 +437,8 @@ void head_linear(Tensor out, Tensor x, Tensor w, OptTensor gate,
     a.y = ptr<T>(out); a.x = ptr<T>(x); a.w = ptr<T>(w);
     a.y_ld = heads * (n + tail); a.y_gs = n + tail;
     a.x_ld = x.stride(0); a.x_gs = x.stride(1);
-    a.m = rows; a.n = n; a.k = k; a.groups = heads; a.tail = tail;
+    a.m = rows; a.n = n; a.k = k; a.groups = heads; a.splits = 1;
+    a.tail = tail;
     a.act = Act::NONE;
     if (gate) {
       check_rows(*gate, Scalar<T>::type, "gate");
@@ -448,18 +450,27 @@ void head_linear(Tensor out, Tensor x, Tensor w, OptTensor gate,
   });
 }
 
-// z [rows, experts] in float32
-void router_scores(Tensor z, Tensor x, Tensor w) {
-  TORCH_CHECK(x.size(1) == w.size(1) && z.size(0) == x.size(0) &&
-              z.size(1) == w.size(0), "router_scores: shapes differ");
-  if (x.size(0) == 0) return;
+// Scores in float32, [splits, rows, experts]; sums over the first axis are
+// left to moe_select.
+Tensor router_scores(Tensor x, Tensor w) {
+  TORCH_CHECK(x.dim() == 2 && x.size(1) == w.size(1),
+              "router_scores: shapes differ");
+  const auto opt = x.options().dtype(torch::kFloat32);
+  const long rows = x.size(0), experts = w.size(0);
+  if (rows == 0) return torch::empty({1, rows, experts}, opt);
+  Tensor z;
   by_type(x, [&](auto tag) {
     using T = decltype(tag);
-    group_gemm(product<T, float>(z, x, w),
-               std::min(64, group_gemm_tile(
-                   x.size(0), 1, std::is_same_v<T, bf16_t>, w.size(1))),
+    // its place in memory is not part of the choice of splits
+    auto a = product<T, float>(torch::empty({0, experts}, opt), x, w);
+    a.splits = group_gemm_splits(a);
+    z = torch::empty({a.splits, rows, experts}, opt);
+    a.y = ptr<float>(z);
+    group_gemm(a, std::min(64, group_gemm_tile(
+                   rows, 1, std::is_same_v<T, bf16_t>, w.size(1))),
                "router_scores");
   });
+  return z;
 }
 
 // gelu_tanh(x w^T) * table[tokens, t_at : t_at + n]
@@ -487,7 +498,8 @@ void side_gate(Tensor out, Tensor x, Tensor w, Tensor tokens, Tensor table,
 
 void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
                 int64_t keep) {
-  const long rows = z.size(0), experts = z.size(1), top = ids.size(1);
+  TORCH_CHECK(z.dim() == 3, "z must be [splits, rows, experts]");
+  const long rows = z.size(1), experts = z.size(2), top = ids.size(1);
   check(ids, torch::kInt32, "ids");
   check(weights, torch::kFloat32, "weights");
   check(z, torch::kFloat32, "z");
@@ -498,8 +510,8 @@ void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
               keep <= groups && top > 0 && top <= experts / groups * keep,
               "moe_select: cannot choose so many");
   if (rows == 0) return;
-  launch_moe_select(ptr<int>(ids), ptr<float>(weights), ptr<float>(z), rows,
-                    experts, top, groups, keep, stream());
+  launch_moe_select(ptr<int>(ids), ptr<float>(weights), ptr<float>(z),
+                    z.size(0), rows, experts, top, groups, keep, stream());
   post("moe_select");
 }
 

@@ -24,6 +24,8 @@ struct GroupGemm {
   const T* w;              // [groups, n, k]
   long y_ld, y_gs, x_ld, x_gs;
   int m, n, k, groups;
+  int splits;              // > 1: shares of the inner dimension, share s to
+                           //   y + s * m * n (unpacked rows, one group)
   int tail;                // elements of x after k, appended to y as they are
   Act act;
   const int* src;          // packed row -> row of x, or null
@@ -145,6 +147,10 @@ int group_gemm_tile(long rows, int groups, bool bf16, int ks);
 // Whether packed rows may come in tiles of this size.
 template <class T, class Y>
 bool group_gemm_takes(const GroupGemm<T, Y>&, int tile);
+
+// Shares of the inner dimension that let one small product fill the chip.
+template <class T, class Y>
+int group_gemm_splits(const GroupGemm<T, Y>&);
 
 template <class T, class Y>
 void launch_group_gemm(const GroupGemm<T, Y>&, int tile, hipStream_t);

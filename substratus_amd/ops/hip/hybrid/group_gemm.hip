@@ -2,9 +2,9 @@
 //
 //   stream   bf16, few rows per group: bound by reading the weights once.
 //            Every wave takes a share of the inner dimension of a tile of
-//            rows and 64 columns (4 waves, or 16 where there are few tiles;
-//            where the inner dimension is short, a share of the rows), with
-//            both operands going from memory
+//            rows and 64 columns (4 waves; 16 and 32 columns where there are
+//            few tiles; where the inner dimension is short, a share of the
+//            rows), with both operands going from memory
 //            straight into the matrix cores' registers (a fragment is 16
 //            consecutive bytes of a row, so nothing is gained by LDS); there
 //            is no barrier until the partial tiles are added up.
@@ -18,7 +18,6 @@ namespace {
 
 typedef __attribute__((ext_vector_type(8))) short short8;
 
-constexpr int BN = 64;
 constexpr int KC = 32;         // inner step of one matrix instruction
 
 // ONCE: nobody reads it again
@@ -29,14 +28,17 @@ DEV_INLINE short8 frag(const bf16_t* p, bool there) {
   else return *reinterpret_cast<const short8*>(p);
 }
 
-// KW waves share the inner dimension, RW the rows
-template <class Y, Act ACT, int FM, int KW, int RW>
+// FM, FN: 16-wide pieces of a wave's rows and columns; KW waves share the
+// inner dimension, RW the rows
+template <class Y, Act ACT, int FM, int FN, int KW, int RW>
 __global__ __launch_bounds__(KW * RW * WAVE)
 void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
-  constexpr int BM = FM * 16 * RW, FN = BN / 16, PAD = 4;
+  constexpr int BM = FM * 16 * RW, BN = FN * 16, PAD = 4;
   static_assert(KW == 1 || RW == 1);
-  const Tile t = tile_of(a, blockIdx.y, blockIdx.z, BM);
+  const Tile t = tile_of(a, blockIdx.y, a.splits > 1 ? 0 : blockIdx.z, BM);
   if (t.r1 <= t.r0) return;
+  const int share = a.splits > 1 ? blockIdx.z : 0;
+  a.y += (long)share * a.m * a.n;
   const int n0 = blockIdx.x * BN;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int lo = lane & 15, kq = (lane >> 4) * 8;
@@ -60,9 +62,9 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
     #pragma unroll
     for (int j = 0; j < FM; ++j) acc[i][j] = (float4v){0.f, 0.f, 0.f, 0.f};
 
-  const int chunks = (a.k + KC - 1) / KC;
-  const int c0 = KW > 1 ? chunks * wave / KW : 0,
-            c1 = KW > 1 ? chunks * (wave + 1) / KW : chunks;
+  const int chunks = (a.k + KC - 1) / KC, shares = KW * a.splits,
+            part = share * KW + (KW > 1 ? wave : 0);
+  const int c0 = chunks * part / shares, c1 = chunks * (part + 1) / shares;
   // U chunks at a time: their loads are in flight together
   auto steps = [&](int c, auto u, bool whole) {
     constexpr int U = decltype(u)::value;
@@ -89,6 +91,9 @@ void group_gemm_stream_kernel(GroupGemm<bf16_t, Y> a) {
   constexpr int U = FM == 4 ? 2 : 4;
   const int full = min(c1, a.k / KC);
   int c = c0;
+  if constexpr (FM == 1 && FN == 2)
+    for (; c + 2 * U <= full; c += 2 * U)
+      steps(c, std::integral_constant<int, 2 * U>{}, true);
   for (; c + U <= full; c += U)
     steps(c, std::integral_constant<int, U>{}, true);
   for (; c < full; ++c) steps(c, std::integral_constant<int, 1>{}, true);
@@ -209,12 +214,25 @@ bool by_quads(const GroupGemm<T, Y>& a) {
 }
 
 template <class T, class Y>
+int group_gemm_splits(const GroupGemm<T, Y>& a) {
+  if constexpr (std::is_same_v<T, bf16_t>) {
+    if (!pieces(a) || a.tiles != nullptr || a.groups != 1) return 1;
+    const long groups = (long)((a.n + 31) / 32) * ((a.m + 15) / 16);
+    int s = 1;     // every wave keeps at least two chunks
+    while (s < 16 && groups * s < 128 && a.k / KC >= s * 16) s *= 2;
+    return s;
+  }
+  return 1;
+}
+
+template <class T, class Y>
 void launch_group_gemm(const GroupGemm<T, Y>& given, int tile,
                        hipStream_t stream) {
   GroupGemm<T, Y> a = given;
   a.quads = by_quads(a);
-  const bool packed = a.tiles != nullptr;
-  const int gz = packed ? 1 : a.groups;
+  const bool packed = a.tiles != nullptr, split = a.splits > 1;
+  const int gz = packed ? 1 : split ? a.splits : a.groups;
+  if (split) tile = 16;
   if constexpr (std::is_same_v<T, bf16_t>) {
     if (!packed && tile > 64 &&
         (!group_gemm_takes(a, tile) ||
@@ -226,18 +244,20 @@ void launch_group_gemm(const GroupGemm<T, Y>& given, int tile,
         launch_group_gemm_tile(a, tile, stream);
         return;
       }
-      const int nt = (a.n + BN - 1) / BN;
       const bool flat = !packed && a.k <= 512 && tile == 64;
+      auto groups = [&](int bn) {
+        return (long)((a.n + bn - 1) / bn) *
+               (packed ? a.max_tiles : (a.m + tile - 1) / tile) * gz;
+      };
       // smaller tiles of unpacked rows while the chip is not full
-      while (!packed && !flat && tile > 16 &&
-             (long)nt * ((a.m + tile - 1) / tile) * gz < 512) tile /= 2;
-      const int mt = packed ? a.max_tiles : (a.m + tile - 1) / tile;
-      const dim3 grid(nt, mt, gz);
-      auto go = [&](auto fm, auto kw, auto rw) {
-        constexpr int FM = decltype(fm)::value, KW = decltype(kw)::value,
-                      RW = decltype(rw)::value;
+      while (!packed && !flat && !split && tile > 16 && groups(64) < 512) tile /= 2;
+      auto go = [&](auto fm, auto fn, auto kw, auto rw) {
+        constexpr int FM = decltype(fm)::value, FN = decltype(fn)::value,
+                      KW = decltype(kw)::value, RW = decltype(rw)::value;
+        const dim3 grid((a.n + FN * 16 - 1) / (FN * 16),
+                        packed ? a.max_tiles : (a.m + tile - 1) / tile, gz);
         by_act(a.act, [&](auto act) {
-          group_gemm_stream_kernel<Y, decltype(act)::value, FM, KW, RW>
+          group_gemm_stream_kernel<Y, decltype(act)::value, FM, FN, KW, RW>
               <<<grid, dim3(KW * RW * WAVE), 0, stream>>>(a);
         });
       };
@@ -245,12 +265,13 @@ void launch_group_gemm(const GroupGemm<T, Y>& given, int tile,
       constexpr std::integral_constant<int, 2> c2{};
       constexpr std::integral_constant<int, 4> c4{};
       constexpr std::integral_constant<int, 16> c16{};
-      if (flat) go(c1, c1, c4);
-      else if (tile == 16 && (long)nt * mt * gz < 256 && a.k >= 1024)
-        go(c1, c16, c1);
-      else if (tile == 16) go(c1, c4, c1);
-      else if (tile == 32) go(c2, c4, c1);
-      else go(c4, c4, c1);
+      if (split) go(c1, c2, c4, c1);
+      else if (flat) go(c1, c4, c1, c4);
+      else if (tile == 16 && groups(64) < 256 && a.k >= 1024)
+        go(c1, c2, c16, c1);
+      else if (tile == 16) go(c1, c4, c4, c1);
+      else if (tile == 32) go(c2, c4, c4, c1);
+      else go(c4, c4, c4, c1);
       return;
     }
   }
@@ -262,6 +283,7 @@ void launch_group_gemm(const GroupGemm<T, Y>& given, int tile,
 }
 
 #define INSTANTIATE(T, Y)                                                    \
+  template int group_gemm_splits<T, Y>(const GroupGemm<T, Y>&);              \
   template bool group_gemm_takes<T, Y>(const GroupGemm<T, Y>&, int);         \
   template void launch_group_gemm<T, Y>(const GroupGemm<T, Y>&, int,         \
                                         hipStream_t);

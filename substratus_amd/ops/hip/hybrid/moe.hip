@@ -1,6 +1,7 @@
 // Choosing experts and packing tokens by expert.
 //
-//   select   one wave per token: softmax over all experts, the best groups
+//   select   one wave per token: scores (sums of a product's shares of the
+//            inner dimension), softmax over all experts, the best groups
 //            of neighbours, the best experts of those; all in 32 bits.
 //   sort     one workgroup: token rows packed by expert, and every expert's
 //            rows cut into tiles for the grouped products. The order of an
@@ -30,8 +31,8 @@ DEV_INLINE int rank_of(const float* s, int n, float v, int i) {
 template <int PL>
 __global__ __launch_bounds__(SW * WAVE)
 void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
-                       const float* __restrict__ z, int rows, int experts,
-                       int top, int groups, int keep) {
+                       const float* __restrict__ z, int splits, int rows,
+                       int experts, int top, int groups, int keep) {
   extern __shared__ float4 s_all[];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int pad = (experts + 3) / 4 * 4;
@@ -47,6 +48,9 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
   for (int i = 0; i < PL; ++i) {
     const int e = lane + i * WAVE;
     v[i] = e < experts ? z[row * experts + e] : -INFINITY;
+    if (e < experts)
+      for (int s = 1; s < splits; ++s)
+        v[i] += z[((long)s * rows + row) * experts + e];
     if (e < pad) s_z[e] = v[i];
     mx = fmaxf(mx, v[i]);
   }
@@ -153,14 +157,14 @@ void moe_sort_kernel(int* __restrict__ at, int* __restrict__ src,
 
 int moe_max_experts() { return SORT; }
 
-void launch_moe_select(int* ids, float* weights, const float* z, int rows,
-                       int experts, int top, int groups, int keep,
+void launch_moe_select(int* ids, float* weights, const float* z, int splits,
+                       int rows, int experts, int top, int groups, int keep,
                        hipStream_t stream) {
   auto go = [&](auto pl) {
     moe_select_kernel<decltype(pl)::value>
         <<<dim3((rows + SW - 1) / SW), dim3(SW * WAVE),
            SW * 2 * ((experts + 3) / 4 * 4) * sizeof(float), stream>>>(
-            ids, weights, z, rows, experts, top, groups, keep);
+            ids, weights, z, splits, rows, experts, top, groups, keep);
   };
   if (experts <= WAVE) go(std::integral_constant<int, 1>{});
   else if (experts <= 4 * WAVE) go(std::integral_constant<int, 4>{});

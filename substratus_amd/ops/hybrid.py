@@ -229,8 +229,7 @@ def experts(y: torch.Tensor, router: torch.Tensor, up: torch.Tensor,
                                    spec.keep))
     ext = _ext()
     i32 = dict(dtype=torch.int32, device=y.device)
-    z = torch.empty(rows, spec.experts, dtype=torch.float32, device=y.device)
-    ext.router_scores(z, y, router)
+    z = ext.router_scores(y, router)
     ids = torch.empty(rows, spec.top, **i32)
     weights = torch.empty(rows, spec.top, dtype=torch.float32,
                           device=y.device)

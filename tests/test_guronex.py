@@ -297,7 +297,7 @@ def test_routing(place, experts, top, groups):
     else:
         ids = torch.empty(40, top, dtype=torch.int32, device="cuda")
         wt = torch.empty(40, top, device="cuda")
-        ops._ext().moe_select(ids, wt, z.cuda(), count, keep)
+        ops._ext().moe_select(ids, wt, z.cuda()[None], count, keep)
     router = {"top": top}
     if groups:
         router["groups"] = {"count": count, "keep": keep}

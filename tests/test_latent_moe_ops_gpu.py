@@ -166,7 +166,8 @@ def test_moe_select(rows, z):
                 s = rand(rows, z, seed=z + groups + keep, scale=2.0)
                 ids = torch.empty(rows, top, dtype=torch.int32).cuda()
                 wt = torch.empty(rows, top).cuda()
-                ext.moe_select(ids, wt, s.cuda(), groups, keep)
+                ext.moe_select(ids, wt, torch.stack(
+                    [s.cuda() * 0.25] * 4), groups, keep)
                 ri, rw = ref.moe_select(s, top, groups, keep)
                 assert torch.equal(ids.cpu(), ri), (groups, keep, top)
                 assert torch.allclose(wt.cpu(), rw, rtol=1e-5), (groups, keep)
@@ -206,6 +207,17 @@ def test_moe_sort(n, top, experts, tile):
 
 def combined(p):
     return (p.rows[p.at.long()].float() * p.weights[:, :, None]).sum(1)
+
+
+@BOTH
+@pytest.mark.parametrize("rows,width,experts", [
+    (1, 4096, 32), (64, 4096, 33), (5, 77, 9), (300, 1024, 64), (20, 2048, 7)])
+def test_router_scores(rows, width, experts, dtype):
+    """32-bit sums, in shares of the width when there are few rows."""
+    x = rand(rows, width, seed=1, dtype=dtype)
+    w = rand(experts, width, seed=2, dtype=dtype, scale=width ** -0.5)
+    got = ops._ext().router_scores(x.cuda(), w.cuda()).sum(0)
+    close(got, x.double() @ w.double().T, F32)
 
 
 @BOTH
