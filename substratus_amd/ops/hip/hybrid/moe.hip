@@ -48,9 +48,11 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
   for (int i = 0; i < PL; ++i) {
     const int e = lane + i * WAVE;
     v[i] = e < experts ? z[row * experts + e] : -INFINITY;
-    if (e < experts)
+    if (e < experts) {
+      #pragma unroll 4
       for (int s = 1; s < splits; ++s)
         v[i] += z[((long)s * rows + row) * experts + e];
+    }
     if (e < pad) s_z[e] = v[i];
     mx = fmaxf(mx, v[i]);
   }

@@ -48,25 +48,42 @@ void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
     }
   } else {
     float dk[RCAP][VEC];
+    if constexpr (SRC == PICKED) {
+      constexpr int P = 4;                       // rows on their way at once
+      #pragma unroll
+      for (int kk = 0; kk < RCAP; ++kk)
+        #pragma unroll
+        for (int j = 0; j < VEC; ++j) dk[kk][j] = 0.f;
+      for (int p = 0; p < picks; p += P) {
+        const T* src[P];
+        float w[P];
+        #pragma unroll
+        for (int q = 0; q < P; ++q) {
+          const long i = row * picks + min(p + q, picks - 1);
+          src[q] = delta + (long)at[i] * width;
+          w[q] = p + q < picks ? wt[i] : 0.f;
+        }
+        #pragma unroll
+        for (int kk = 0; kk < RCAP; ++kk) {
+          const int i = threadIdx.x + kk * BLOCK;
+          if (i >= nvec) break;
+          float f[P][VEC];
+          #pragma unroll
+          for (int q = 0; q < P; ++q) ldv<VEC>(src[q] + i * VEC, f[q]);
+          #pragma unroll
+          for (int q = 0; q < P; ++q)
+            #pragma unroll
+            for (int j = 0; j < VEC; ++j) dk[kk][j] += w[q] * f[q][j];
+        }
+      }
+    }
     float ss = 0.f;
-    const T* dr = delta + row * width;
     #pragma unroll
     for (int kk = 0; kk < RCAP; ++kk) {
       const int i = threadIdx.x + kk * BLOCK;
       if (i >= nvec) break;
-      if constexpr (SRC == ROW) {
-        ldv<VEC>(dr + i * VEC, dk[kk]);
-      } else {
-        #pragma unroll
-        for (int j = 0; j < VEC; ++j) dk[kk][j] = 0.f;
-        for (int p = 0; p < picks; ++p) {
-          float f[VEC];
-          ldv<VEC>(delta + (long)at[row * picks + p] * width + i * VEC, f);
-          const float w = wt[row * picks + p];
-          #pragma unroll
-          for (int j = 0; j < VEC; ++j) dk[kk][j] += w * f[j];
-        }
-      }
+      if constexpr (SRC == ROW)
+        ldv<VEC>(delta + row * width + i * VEC, dk[kk]);
       ldv<VEC>(xr + i * VEC, xk[kk]);
       #pragma unroll
       for (int j = 0; j < VEC; ++j) ss += dk[kk][j] * dk[kk][j];

@@ -91,52 +91,6 @@ def tol(place):
     return 2e-4 if place[1] == "float32" else 2e-2
 
 
-@pytest.mark.parametrize("place", PLACES)
-def test_norms_around_the_residual(place):
-    g = torch.Generator().manual_seed(0)
-    d, x, wp, wn = (torch.randn(s, generator=g)
-                    for s in ((5, 96), (5, 96), (96,), (96,)))
-    d = put(d, place)
-    xs = x.to(place[0], copy=True)
-    y = ops.stream_norm(d, xs, wp.to(place[0]), wn.to(place[0]), 1.0, 1e-2,
-                        0.5)
-    want_x = x.double() + oracle.stream_norm(d.cpu().double(), wp, 1e-2)
-    want = oracle.stream_norm(want_x, wn, 1e-2) * 0.5
-    assert float((xs.cpu() - want_x).abs().max()) < 1e-5
-    assert xs.dtype == torch.float32
-    assert float((y.cpu().double() - want).abs().max()) < tol(place)
-
-
-@pytest.mark.parametrize("place", PLACES)
-def test_projection_norms_and_value_blend(place):
-    g = torch.Generator().manual_seed(1)
-    heads, kv, d, dv, n = 4, 2, 24, 16, 5
-    buf, first = torch.randn(n, heads * d + kv * (d + dv) + 8, generator=g), \
-        torch.randn(n, kv * dv, generator=g)
-    qw, kw = (1 + torch.randn(m * d, generator=g) for m in (heads, kv))
-    buf, first = put(buf, place), put(first, place)
-    batch, pages = request_batch(place, [(30, n)])
-    kc = torch.zeros(pages, kv, 16, d, dtype=buf.dtype, device=place[0])
-    vc = torch.zeros(pages, kv, 16, dv, dtype=buf.dtype, device=place[0])
-    ref = buf.cpu().double()
-    ops.qkv_prepare(buf, heads * d, qw.to(place[0]), kw.to(place[0]), 1e-3,
-                    first, torch.tensor(0.3, device=place[0]), kc, vc,
-                    batch.slots)
-    q, k, v = ref[:, :heads * d], ref[:, heads * d:(heads + kv) * d], \
-        ref[:, (heads + kv) * d:(heads + kv) * d + kv * dv]
-    blocks = batch.block_table[0].long()
-    rows = slice(30, 30 + n)
-
-    def cached(c):
-        return c[blocks].transpose(1, 2).reshape(-1, kv * c.shape[3])[rows] \
-            .cpu().double()
-    for got, want in (
-            (buf[:, :heads * d].cpu().double(), oracle.rms(q, 1e-3) * qw),
-            (cached(kc), oracle.rms(k, 1e-3) * kw),
-            (cached(vc), oracle.mix_values(v, first.cpu().double(), 0.3))):
-        assert float((got - want).abs().max()) < tol(place) * 2
-
-
 def engine_for(folder, place, **kw):
     args = dict(max_batch=3, max_seq_len=192, kv_blocks=64, prefill_chunk=48)
     args.update(kw)
