@@ -1,6 +1,7 @@
 from .config import ModelConfig, get_config, register
 from . import guronex as _guronex  # registers the architecture and its models
 from . import kakovik as _kakovik  # the same
+from . import vurazen as _vurazen  # the same
 from .hybrid import HybridLM
 from .model import CausalLM
 

@@ -13,13 +13,13 @@ import os
 from dataclasses import dataclass, field
 from typing import Callable, Optional
 
-from .layers import LayerSpec
+from .layers import LayerSpec, LoopSpec
 
 
 @dataclass
 class ModelConfig:
     name: str
-    family: str  # "llama" | "falcon" | "opt" | "kakovik" | "guronex"
+    family: str  # "llama" | "falcon" | "opt" | "kakovik" | "guronex" | "vurazen"
     hidden_size: int
     intermediate_size: int
     num_layers: int
@@ -48,6 +48,12 @@ class ModelConfig:
     residual_mult: float = 1.0  # factor of what sublayers add to the residual
     side_dim: int = 0         # per layer: size of an input for the token itself
     logit_scale: float = 1.0
+    # mixer and feed-forward read one norm of the residual and are added to it
+    # together, or one after the other
+    parallel_block: bool = False
+    embed_scale: float = 1.0
+    logit_softcap: float = 0.0  # > 0: logits are cap * tanh(logits / cap)
+    loop: Optional[LoopSpec] = None
 
     def __post_init__(self) -> None:
         if self.head_dim == 0 and self.num_heads:
@@ -56,6 +62,17 @@ class ModelConfig:
     @property
     def kv_dim(self) -> int:
         return self.num_kv_heads * self.head_dim
+
+    def runs(self) -> list[tuple[int, Optional[int]]]:
+        """The layers in the order they run, each with the number of the
+        loop's pass that begins with it, or None."""
+        n = len(self.layers)
+        loop = self.loop or LoopSpec(n, n, 0)
+        body = [(i, t if i == loop.start else None)
+                for t in range(loop.times)
+                for i in range(loop.start, loop.stop)]
+        return [(i, None) for i in range(loop.start)] + body + \
+            [(i, None) for i in range(loop.stop, n)]
 
     def param_count(self) -> int:
         h, f, L, v = self.hidden_size, self.intermediate_size, self.num_layers, self.vocab_size

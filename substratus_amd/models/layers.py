@@ -1,8 +1,9 @@
 """Descriptions of layers for models whose layers are not all alike.
 
 A model is a tuple of LayerSpec; the mixer's spec type selects the mixer
-(models/hybrid.py) and what the cache manager keeps for the layer
-(serve/kv_cache.py): pages of keys and values, or one state per request.
+(models/hybrid.py). A mixer's spec also names what the cache manager
+(serve/kv_cache.py) keeps for the layer: pages with a row per token, slots
+with a state per request.
 """
 
 from __future__ import annotations
@@ -16,7 +17,39 @@ import torch
 
 
 @dataclass(frozen=True)
-class AttentionSpec:
+class Pages:
+    """Part of a layer's cache with a row of `dim` per token and head."""
+    heads: int
+    dim: int
+
+
+@dataclass(frozen=True)
+class Slots:
+    """Part of a layer's cache with one state per request."""
+    shape: tuple[int, ...]
+    f32: bool = True         # 32-bit in every serving dtype; else as activations
+
+
+class MixerSpec:
+    """What all mixers' specs have."""
+
+    def cache(self) -> tuple[Union[Pages, Slots], ...]:
+        """What the layer keeps, in the order in which its mixer takes it."""
+        raise NotImplementedError
+
+    def kv_bytes(self, itemsize: int) -> int:
+        """Cache bytes per token."""
+        return sum(p.heads * p.dim * itemsize for p in self.cache()
+                   if isinstance(p, Pages))
+
+    def state_bytes(self, itemsize: int = 4) -> int:
+        """State bytes per request."""
+        return sum(math.prod(p.shape) * (4 if p.f32 else itemsize)
+                   for p in self.cache() if isinstance(p, Slots))
+
+
+@dataclass(frozen=True)
+class AttentionSpec(MixerSpec):
     heads: int
     kv_heads: int
     dim: int                 # query/key size of a head
@@ -29,12 +62,8 @@ class AttentionSpec:
     v_mix: bool = False      # blend in the first such layer's values
     out_gate: bool = False   # sigmoid gate per head on the output
 
-    def kv_bytes(self, itemsize: int) -> int:
-        """Cache bytes per token."""
-        return self.kv_heads * (self.dim + self.vdim) * itemsize
-
-    def state_bytes(self) -> int:
-        return 0
+    def cache(self) -> tuple:
+        return Pages(self.kv_heads, self.dim), Pages(self.kv_heads, self.vdim)
 
     def params(self, width: int) -> int:
         rows = (self.heads + self.kv_heads) * self.dim \
@@ -43,19 +72,15 @@ class AttentionSpec:
 
 
 @dataclass(frozen=True)
-class GLASpec:
+class GLASpec(MixerSpec):
     heads: int
     dim: int
     vdim: int
     tau: float               # decays are sigmoid(z) ** (1 / tau)
     rank: int                # inner size of the decay projection
 
-    def kv_bytes(self, itemsize: int) -> int:
-        return 0
-
-    def state_bytes(self) -> int:
-        """State bytes per request; 32-bit in every serving dtype."""
-        return self.heads * self.dim * self.vdim * 4
+    def cache(self) -> tuple:
+        return (Slots((self.heads, self.dim, self.vdim)),)
 
     def params(self, width: int) -> int:
         rows = 2 * self.heads * (self.dim + self.vdim) + self.rank
@@ -66,9 +91,11 @@ class GLASpec:
 @dataclass(frozen=True)
 class RotarySpec:
     """Rotation of the first `dims` elements of a vector: element i turns with
-    element i + dims / 2, at position p by p * base ** (-2 i / dims)."""
+    element i + dims / 2, or if interleaved 2 i with 2 i + 1, at position p by
+    p * base ** (-2 i / dims)."""
     base: float
     dims: int
+    interleaved: bool = False
 
     def turns(self, device=None) -> torch.Tensor:
         """float64 [dims / 2]: full turns per position. Whole turns drop out
@@ -78,7 +105,7 @@ class RotarySpec:
 
 
 @dataclass(frozen=True)
-class LatentAttentionSpec:
+class LatentAttentionSpec(MixerSpec):
     """Attention whose keys and values are projections of one latent vector
     per token, beside a rotated key part that all heads share."""
     heads: int
@@ -96,11 +123,8 @@ class LatentAttentionSpec:
         """Elements the cache holds per token: latent, rotated key part."""
         return self.rank + self.rot_dim
 
-    def kv_bytes(self, itemsize: int) -> int:
-        return self.row * itemsize if self.kv_from is None else 0
-
-    def state_bytes(self) -> int:
-        return 0
+    def cache(self) -> tuple:
+        return (Pages(1, self.row),) if self.kv_from is None else ()
 
     def params(self, width: int) -> int:
         rows = self.heads * (self.dim + self.rot_dim +
@@ -110,14 +134,136 @@ class LatentAttentionSpec:
 
 
 @dataclass(frozen=True)
+class ConvAttentionSpec(MixerSpec):
+    """Attention whose queries and keys pass a short causal convolution over
+    time and are rotated; the values are the keys ahead of their rotation."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    taps: int                # of the convolution
+    rot: RotarySpec
+    window: int = 0          # > 0: a position sees so many, itself included,
+    keep: int = 0            #   and the first `keep` of its sequence
+    softcap: float = 0.0     # > 0: scores are cap * tanh(score / cap)
+    sink: bool = False       # a learned share of the softmax without a value
+
+    def cache(self) -> tuple:
+        rows = (self.heads + self.kv_heads) * self.dim
+        return Pages(self.kv_heads, self.dim), \
+            Pages(self.kv_heads, self.dim), \
+            Slots((self.taps - 1, rows), False)
+
+    def params(self, width: int) -> int:
+        rows = (self.heads + self.kv_heads) * self.dim
+        return width * (rows + self.heads * self.dim) + rows * self.taps
+
+
+@dataclass(frozen=True)
+class DeltaSpec(MixerSpec):
+    """Gated delta rule with a decay per key channel."""
+    heads: int
+    kv_heads: int            # heads of queries and keys
+    dim: int
+    vdim: int
+    taps: int                # of the convolution of q, k and v
+    decay_rank: int          # inner sizes of the decays' and the output
+    gate_rank: int           #   gate's projection
+
+    @property
+    def conv_rows(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    def cache(self) -> tuple:
+        return Slots((self.heads, self.dim, self.vdim)), \
+            Slots((self.taps - 1, self.conv_rows), False)
+
+    def params(self, width: int) -> int:
+        hv = self.heads * self.vdim
+        return width * (self.conv_rows + self.heads + self.decay_rank +
+                        self.gate_rank + hv) + self.conv_rows * self.taps \
+            + self.heads * self.dim * self.decay_rank + hv * self.gate_rank
+
+
+@dataclass(frozen=True)
+class MambaSpec(MixerSpec):
+    """Selective scan: a state of `state` numbers per channel."""
+    inner: int               # channels
+    state: int
+    rank: int                # inner size of the step sizes' projection
+    taps: int
+
+    def cache(self) -> tuple:
+        return Slots((self.inner, self.state)), \
+            Slots((self.taps - 1, self.inner), False)
+
+    def params(self, width: int) -> int:
+        return self.inner * (3 * width + 2 * self.rank + 3 * self.state +
+                             self.taps)
+
+
+@dataclass(frozen=True)
+class LightningSpec(MixerSpec):
+    """Linear attention with a constant decay per head, normed over all heads
+    at once."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple[float, ...]
+
+    def __post_init__(self) -> None:
+        if len(self.decay) != self.heads:
+            raise ValueError(f"{len(self.decay)} decays for {self.heads} "
+                             "heads")
+
+    def cache(self) -> tuple:
+        return (Slots((self.heads, self.dim, self.vdim)),)
+
+    def params(self, width: int) -> int:
+        return width * self.heads * (2 * self.dim + 3 * self.vdim)
+
+
+@dataclass(frozen=True)
+class SideBySideSpec(MixerSpec):
+    """Two mixers that read the same input, and the scaled sum of both."""
+    left: MixerSpec
+    right: MixerSpec
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+    def cache(self) -> tuple:
+        return self.left.cache() + self.right.cache()
+
+    def params(self, width: int) -> int:
+        return self.left.params(width) + self.right.params(width)
+
+
+@dataclass(frozen=True)
+class GluSpec:
+    """How a gated feed-forward forms its hidden values from gate g and u:
+    silu      silu(g) * u
+    relu      max(g, 0) * u
+    clamped   g * sigmoid(1.702 g) * (u + 1), of g up to `limit` and u within
+              `limit` of zero"""
+    act: str = "silu"
+    limit: float = 0.0
+
+
+@dataclass(frozen=True)
 class MoESpec:
     """Experts, of which a token uses the `top` best of the `keep` best
-    groups of neighbours; weights are softmax scores over all experts."""
+    groups of neighbours. Weights are softmax scores over all experts, or
+    over the chosen ones."""
     experts: int
     top: int
     ff: int                  # inner size of one expert
     groups: int = 1
     keep: int = 1
+    glu: Optional[GluSpec] = None   # experts are gated; None: gelu
+    over_chosen: bool = False
+    bias: bool = False       # of the router's scores
+    shared_ff: int = 0       # an expert for every token, 0: none
+    shared_glu: Optional[GluSpec] = None
 
     def __post_init__(self) -> None:
         if self.experts % self.groups or not 0 < self.keep <= self.groups:
@@ -128,18 +274,30 @@ class MoESpec:
                              f"{self.experts // self.groups} experts")
 
     def params(self, width: int) -> int:
-        return width * self.experts * (1 + 2 * self.ff)
+        return width * (self.experts * (1 + (3 if self.glu else 2) * self.ff)
+                        + 3 * self.shared_ff)
 
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[AttentionSpec, GLASpec, LatentAttentionSpec]
+    mixer: MixerSpec
     ff: int = 0              # inner size of the gated feed-forward, 0: none
     moe: Optional[MoESpec] = None   # experts instead of it
+    glu: GluSpec = GluSpec()
 
     def params(self, width: int) -> int:
         return self.mixer.params(width) + 3 * width * self.ff \
             + (self.moe.params(width) if self.moe else 0)
+
+
+@dataclass(frozen=True)
+class LoopSpec:
+    """Layers start .. stop - 1 run `times` times in a row, with the same
+    weights and caches of their own. Every pass begins with a learned vector
+    added to the residual; every one but the first, also with the embedding."""
+    start: int
+    stop: int
+    times: int
 
 
 def distance_bucket(n: int, rows: int, furthest: int) -> int:

@@ -29,12 +29,14 @@ def to_native(sd: dict, mcfg: ModelConfig) -> dict:
     from . import hf_compat as hf
     from .guronex import guronex_to_native, is_guronex_state_dict
     from .kakovik import is_kakovik_state_dict, kakovik_to_native
+    from .vurazen import is_vurazen_state_dict, vurazen_to_native
     for known, convert in (
             (hf.is_hf_llama_state_dict, hf.hf_llama_to_native),
             (hf.is_hf_falcon_state_dict, hf.hf_falcon_to_native),
             (hf.is_hf_opt_state_dict, hf.hf_opt_to_native),
             (is_kakovik_state_dict, kakovik_to_native),
-            (is_guronex_state_dict, guronex_to_native)):
+            (is_guronex_state_dict, guronex_to_native),
+            (is_vurazen_state_dict, vurazen_to_native)):
         if known(sd):
             return convert(sd, mcfg)
     return sd

@@ -1,7 +1,8 @@
 """Ops of models whose layers differ from one another (models/hybrid.py):
 norms around a 32-bit residual, attention that reads the paged cache for
 single tokens and prompt portions alike, attention over a cache of latents,
-gated linear attention with a recurrent state per request, mixtures of experts.
+linear attention, delta-rule and selective-scan recurrences with a state per
+request, short convolutions over time, mixtures of experts.
 
 Same policy as the rest of ops: GPU tensors need the HIP extension
 (substratus_amd._hybrid), CPU tensors run the plain implementations in ref.py.
@@ -90,23 +91,36 @@ def qkv_prepare(buf: torch.Tensor, nq: int, q_norm: Optional[torch.Tensor],
 
 def attn_ctx(q: torch.Tensor, gate: Optional[torch.Tensor],
              k_cache: torch.Tensor, v_cache: torch.Tensor,
-             bias: Optional[torch.Tensor], batch, scale: float, chunk: int,
-             any_size: bool = False) -> torch.Tensor:
+             bias: Optional[torch.Tensor], batch, scale: float, chunk: int = 0,
+             any_size: bool = False, window: int = 0, keep: int = 0,
+             softcap: float = 0.0, sink: Optional[torch.Tensor] = None,
+             mult: float = 1.0,
+             out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of a batch's rows over the paged cache, which already holds
     their own keys and values.
 
-    q [rows, heads * dim] and gate [rows, heads] may be views of one buffer.
-    bias [heads, n]: added to the score by distance, the last column also for
-    every larger distance. chunk > 0: rows see keys of their own chunk of
-    positions only. any_size takes the untiled kernel on the GPU."""
+    q [rows, heads * dim] and gate [rows, heads] may be views of one buffer,
+    out [rows, heads * vdim] a view of wider rows. bias [heads, n]: added to
+    the score by distance, the last column also for every larger distance.
+    chunk > 0: rows see keys of their own chunk of positions only. window > 0:
+    rows see that many keys up to their own, and the first `keep`. softcap > 0:
+    scores are cap * tanh(score / cap) ahead of the bias. sink [heads]: a score
+    in the softmax that has no value. mult multiplies the result. any_size
+    takes the untiled kernel on the GPU."""
     heads = q.shape[1] // k_cache.shape[3]
-    out = q.new_empty(q.shape[0], heads * v_cache.shape[3])
-    span = batch.max_context if chunk == 0 else min(chunk, batch.max_context)
+    if out is None:
+        out = q.new_empty(q.shape[0], heads * v_cache.shape[3])
+    span = batch.max_context
+    if chunk:
+        span = min(chunk, span)
+    if window:
+        span = min(window + keep, span)
     fn = _ext().attn_ctx if q.is_cuda else ref.attn_ctx
     for rows, ents, seq_start, max_len in batch.parts():
         fn(out[rows], q[rows], None if gate is None else gate[rows], k_cache,
-           v_cache, bias, batch.positions[rows], seq_start,
-           batch.block_table[ents], scale, chunk, max_len, span, any_size)
+           v_cache, bias, sink, batch.positions[rows], seq_start,
+           batch.block_table[ents], scale, chunk, window, keep, softcap, mult,
+           max_len, span, any_size)
     return out
 
 
@@ -148,9 +162,9 @@ def _latent_absorbed(out, q, gate, cache, w_uv, uk_t, batch, rows, ents,
                      tail=spec.rot_dim)
     o = q.new_empty(n, spec.heads * spec.rank)
     fn = _ext().attn_ctx if q.is_cuda else ref.attn_ctx
-    fn(o, qa.view(n, -1), None, cache, cache[..., :spec.rank], None,
+    fn(o, qa.view(n, -1), None, cache, cache[..., :spec.rank], None, None,
        batch.positions[rows], seq_start, batch.block_table[ents], spec.scale,
-       0, max_len, batch.max_context, False)
+       0, 0, 0, 0.0, 1.0, max_len, batch.max_context, False)
     head_linear(o.view(n, spec.heads, spec.rank), w_uv, gate, out=out)
 
 
@@ -220,20 +234,22 @@ def latent_attn(q: torch.Tensor, gate: Optional[torch.Tensor],
 
 
 def experts(y: torch.Tensor, router: torch.Tensor, up: torch.Tensor,
-            down: torch.Tensor, spec) -> Picked:
-    """A mixture of experts: y [rows, width], router [experts, width], up
-    [experts, ff, width], down [experts, width, ff]. Scores are 32-bit."""
+            down: torch.Tensor, spec,
+            bias: Optional[torch.Tensor] = None) -> Picked:
+    """A mixture of experts: y [rows, width], router [experts, width], bias
+    [experts], up [experts, ff, width] (gated experts: twice as many rows, of
+    gate and up in turn), down [experts, width, ff]. Scores are 32-bit."""
     rows = y.shape[0]
     if not y.is_cuda:
-        return Picked(*ref.experts(y, router, up, down, spec.top, spec.groups,
-                                   spec.keep))
+        return Picked(*ref.experts(y, router, bias, up, down, spec))
     ext = _ext()
     i32 = dict(dtype=torch.int32, device=y.device)
     z = ext.router_scores(y, router)
     ids = torch.empty(rows, spec.top, **i32)
     weights = torch.empty(rows, spec.top, dtype=torch.float32,
                           device=y.device)
-    ext.moe_select(ids, weights, z, spec.groups, spec.keep)
+    ext.moe_select(ids, weights, z, spec.groups, spec.keep, bias,
+                   spec.over_chosen)
     packed = rows * spec.top
     tile = ext.moe_tile(packed, spec.experts, y.dtype == torch.bfloat16,
                         y.shape[1], spec.ff)
@@ -244,9 +260,11 @@ def experts(y: torch.Tensor, router: torch.Tensor, up: torch.Tensor,
                                  min(spec.experts, packed)), **i32)
     ext.moe_sort(at, src, start, tiles, ids, tile)
     h = y.new_empty(packed, spec.ff)
-    ext.expert_linear(h, y, up, src, start, tiles, tile, True)
+    act, limit = ("gelu", 0.0) if spec.glu is None else \
+        (spec.glu.act, spec.glu.limit)
+    ext.expert_linear(h, y, up, src, start, tiles, tile, act, limit)
     out = y.new_empty(packed, y.shape[1])
-    ext.expert_linear(out, h, down, None, start, tiles, tile, False)
+    ext.expert_linear(out, h, down, None, start, tiles, tile, "none", 0.0)
     return Picked(out, at, weights)
 
 
@@ -281,3 +299,155 @@ def silu_mul(x: torch.Tensor) -> torch.Tensor:
     out = x.new_empty(*x.shape[:-1], x.shape[-1] // 2)
     _ext().silu_mul(out, x.contiguous())
     return out
+
+
+def glu(x: torch.Tensor, spec, out: torch.Tensor) -> None:
+    """out = the gated feed-forward's hidden values of x [rows, 2 f], gate
+    then up; both may be views of wider rows."""
+    (_ext() if x.is_cuda else ref).glu(out, x, spec.act, spec.limit)
+
+
+def add_norm(x: Optional[torch.Tensor], w: torch.Tensor,
+             b: Optional[torch.Tensor], eps: float, dtype: torch.dtype,
+             rows: Optional[torch.Tensor] = None,
+             picked: Optional[Picked] = None,
+             embedded: Optional[tuple] = None,
+             vec: Optional[torch.Tensor] = None
+             ) -> tuple[torch.Tensor, torch.Tensor]:
+    """Adds to the residual x, in place, whatever is given: rows [rows,
+    width]; the weighed sum of picked rows; embedded = (tokens, table, scale),
+    scale * table[tokens]; vec [width]. x None: the residual begins here.
+    Returns x and its layer norm with weight w and bias b, or without b its RMS
+    norm, as dtype."""
+    if x is None:
+        n = embedded[0].shape[0]
+        fresh = torch.empty if w.is_cuda else torch.zeros
+        x, new = fresh(n, w.shape[0], dtype=torch.float32,
+                       device=w.device), True
+    else:
+        new = False
+    pool, at, weights = picked if picked is not None else (None,) * 3
+    tokens, table, scale = embedded if embedded is not None else \
+        (None, None, 1.0)
+    if not x.is_cuda:
+        return x, ref.add_norm(x, rows, at, weights, pool, tokens, table,
+                               scale, vec, w, b, eps, dtype)
+    y = torch.empty(x.shape, dtype=dtype, device=x.device)
+    _ext().add_norm(y, x, new, rows, pool, at, weights, tokens, table, scale,
+                    vec, w, b, eps)
+    return x, y
+
+
+def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap * tanh(x / cap), in place."""
+    (_ext() if x.is_cuda else ref).softcap(x, cap)
+    return x
+
+
+def linear32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x @ w.T in float32, unrounded; x may be a view of wider rows."""
+    if x.dtype == torch.float32 or not x.is_cuda:
+        return torch.nn.functional.linear(x.float(), w.float())
+    return _ext().linear32(x, w)
+
+
+def rope_table(batch, rot, turns: torch.Tensor, shared: dict) -> torch.Tensor:
+    """Cosines and sines of a batch's rows, float32 [rows, dims / 2, 2]; made
+    once per batch for all layers that rotate alike."""
+    held = shared.get(rot)
+    if held is None:
+        if turns.is_cuda:
+            held = torch.empty(batch.positions.shape[0], turns.shape[0], 2,
+                               dtype=torch.float32, device=turns.device)
+            _ext().rope_table(held, batch.positions, turns)
+        else:
+            held = ref.rope_table(batch.positions, turns)
+        shared[rot] = held
+    return held
+
+
+def short_conv(x: torch.Tensor, weight: torch.Tensor,
+               bias: Optional[torch.Tensor], act: bool, state: torch.Tensor,
+               batch) -> torch.Tensor:
+    """A causal convolution over time per channel, then silu if act: x [rows,
+    channels] may be a view of wider rows; weight [channels, taps], the last
+    tap is the row's own. state [slots, taps - 1, channels] has each request's
+    last inputs and is updated."""
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    fn = (_ext() if x.is_cuda else ref).short_conv
+    for rows, ents, seq_start, max_len in batch.parts():
+        fn(out[rows], x[rows], None, weight, bias, act, state,
+           batch.state_slots[ents], batch.positions[rows], seq_start, max_len)
+    return out
+
+
+def conv_rope(buf: torch.Tensor, in_bias: Optional[torch.Tensor],
+              weight: torch.Tensor, state: torch.Tensor, rope: torch.Tensor,
+              k_cache: torch.Tensor, v_cache: torch.Tensor,
+              batch) -> torch.Tensor:
+    """buf rows are [q | k | ...]. in_bias is added to both, then they pass a
+    short convolution (as short_conv); what that makes of k is also the value
+    and goes to v_cache; q and k are rotated (rope: rope_table, neighbouring
+    elements are pairs) and k goes to k_cache. Returns q."""
+    kv, dim = k_cache.shape[1], k_cache.shape[3]
+    q = buf.new_empty(buf.shape[0], weight.shape[0] - kv * dim)
+    fn = (_ext() if buf.is_cuda else ref).conv_rope
+    for rows, ents, seq_start, max_len in batch.parts():
+        fn(q[rows], buf[rows], in_bias, weight, state,
+           batch.state_slots[ents], rope[rows], k_cache, v_cache,
+           batch.positions[rows], batch.slots[rows], seq_start, max_len)
+    return q
+
+
+def selective_scan(u: torch.Tensor, gate: torch.Tensor, z: torch.Tensor,
+                   z_bias: torch.Tensor, low: torch.Tensor, b_at: int,
+                   a: torch.Tensor, d: torch.Tensor, state: torch.Tensor,
+                   batch, out: torch.Tensor, recurrent: bool = False) -> None:
+    """Per channel c with state S[c, :], updated from token to token:
+        dt = softplus(z + z_bias)
+        S <- exp(dt a) S + dt u B,   out = (S . C + d u) silu(gate)
+    u, gate, out [rows, channels] (gate and out may be views), z float32; low
+    rows have B and C from column b_at on; a [channels, n] float32. recurrent
+    walks portions without cutting them into segments."""
+    fn = (_ext() if u.is_cuda else ref).selective_scan
+    for rows, ents, seq_start, max_len in batch.parts():
+        fn(out[rows], u[rows], gate[rows], z[rows], z_bias, low[rows], b_at,
+           a, d, state, batch.state_slots[ents], batch.positions[rows],
+           seq_start, max_len, recurrent)
+
+
+def lightning(x: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+              batch, recurrent: bool = False) -> torch.Tensor:
+    """x rows are [q | k | v | ...], each of which passes silu; per head
+    S <- decay S + k v^T and o = S^T q. Returns [rows, heads * vdim]."""
+    out = x.new_empty(x.shape[0], state.shape[1] * state.shape[3])
+    fn = (_ext() if x.is_cuda else ref).lightning
+    for rows, ents, seq_start, max_len in batch.parts():
+        fn(out[rows], x[rows], decay, state, batch.state_slots[ents],
+           batch.positions[rows], seq_start, max_len, recurrent)
+    return out
+
+
+def joint_gate(o: torch.Tensor, norm: torch.Tensor, gate: torch.Tensor,
+               eps: float, out: torch.Tensor) -> None:
+    """out = rms(o) over whole rows * norm * sigmoid(gate)."""
+    (_ext() if o.is_cuda else ref).joint_gate(out, o, norm, gate, eps)
+
+
+def delta(qkv: torch.Tensor, z: torch.Tensor, z_bias: torch.Tensor,
+          rate: torch.Tensor, beta: torch.Tensor, norm: torch.Tensor,
+          gate: torch.Tensor, state: torch.Tensor, batch, kv_heads: int,
+          eps: float, mult: float, out: torch.Tensor,
+          recurrent: bool = False) -> None:
+    """Gated delta rule. Per head, with k and q made unit vectors (q also
+    times dim^-1/2) and a decay per key channel:
+        S <- exp(-rate softplus(z + z_bias)) S,  u = sigmoid(beta) (v - S^T k)
+        S <- S + k u^T,   out = rms(S^T q) norm sigmoid(gate) mult
+    qkv rows are [q | k | v], q and k with kv_heads heads; z [rows, heads *
+    dim] float32; beta [rows, heads], gate and out [rows, heads * vdim], all
+    three maybe views of wider rows."""
+    fn = (_ext() if qkv.is_cuda else ref).delta
+    for rows, ents, seq_start, max_len in batch.parts():
+        fn(out[rows], qkv[rows], z[rows], z_bias, rate, beta[rows], norm,
+           gate[rows], state, batch.state_slots[ents], batch.positions[rows],
+           seq_start, kv_heads, eps, mult, max_len, recurrent)

@@ -255,6 +255,162 @@ def embed_norm(tokens, table, w_pre, offset, eps):
     return x, y.to(table.dtype, copy=True)
 
 
+def add_norm(x, rows, at, weights, pool, tokens, table, scale, vec, w, b, eps,
+             dtype):
+    if rows is not None:
+        x += rows.float()
+    if pool is not None:
+        x += (pool[at.long()].float() * weights[:, :, None]).sum(1)
+    if table is not None:
+        x += table[tokens.long()].float() * scale
+    if vec is not None:
+        x += vec
+    if b is None:
+        return (_rms(x, eps) * w).to(dtype)
+    d = x - x.mean(-1, keepdim=True)
+    return (_rms(d, eps) * w + b).to(dtype)
+
+
+def softcap(x, cap):
+    x.copy_(cap * torch.tanh(x.float() / cap))
+
+
+def rope_table(positions, turns):
+    t = positions.double()[:, None] * turns
+    a = ((t - t.round()) * (2 * math.pi)).float()
+    return torch.stack([a.cos(), a.sin()], -1)
+
+
+def short_conv(out, x, in_bias, weight, bias, act, state, state_slots,
+               positions, seq_start, max_len):
+    taps = weight.shape[1]
+    for e, (a, b) in enumerate(_entry_rows(seq_start, x.shape[0])):
+        slot = int(state_slots[e])
+        u = x[a:b].float() if in_bias is None else x[a:b].float() + in_bias
+        old = torch.zeros(taps - 1, x.shape[1], device=x.device)
+        if slot >= 0 and int(positions[a]) > 0:
+            old = state[slot].float()
+            # inputs before the sequence's start are zeros, not biases
+            n = min(taps - 1, int(positions[a]))
+            if in_bias is not None and n:
+                old = old.clone()
+                old[taps - 1 - n:] += in_bias
+        held = torch.cat([old, u])
+        y = sum(held[j:j + b - a] * weight[:, j] for j in range(taps))
+        if bias is not None:
+            y = y + bias
+        if slot >= 0 and taps > 1:
+            raw = torch.cat([state[slot] if int(positions[a]) > 0 else
+                             torch.zeros_like(state[slot]),
+                             x[a:b].to(state.dtype)])
+            state[slot] = raw[-(taps - 1):]
+        out[a:b] = (torch.nn.functional.silu(y) if act else y).to(out.dtype)
+
+
+def conv_rope(q, buf, in_bias, weight, state, state_slots, rope, k_cache,
+              v_cache, positions, slots, seq_start, max_len):
+    rows = weight.shape[0]
+    y = torch.empty(buf.shape[0], rows, device=buf.device)
+    short_conv(y, buf[:, :rows], in_bias, weight, None, False, state,
+               state_slots, positions, seq_start, max_len)
+    kv, dim = k_cache.shape[1], k_cache.shape[3]
+    y = y.view(buf.shape[0], -1, dim)
+    v = y[:, -kv:].clone()
+    half = rope.shape[1]
+    cos, sin = rope[:, None, :, 0], rope[:, None, :, 1]
+    a, b = y[..., 0:2 * half:2].clone(), y[..., 1:2 * half:2].clone()
+    y[..., 0:2 * half:2] = a * cos - b * sin
+    y[..., 1:2 * half:2] = b * cos + a * sin
+    q.copy_(y[:, :-kv].reshape(q.shape).to(q.dtype))
+    kv_append(y[:, -kv:], v, k_cache, v_cache, slots)
+
+
+def selective_scan(out, u, gate, z, z_bias, low, b_at, a, d, state,
+                   state_slots, positions, seq_start, max_len, recurrent):
+    n = a.shape[1]
+    dt = torch.nn.functional.softplus(z + z_bias)
+    x, lowf = u.float(), low[:, b_at:b_at + 2 * n].float()
+    for e, (r0, r1) in enumerate(_entry_rows(seq_start, u.shape[0])):
+        slot = int(state_slots[e])
+        s = torch.zeros_like(a) if slot < 0 or int(positions[r0]) == 0 \
+            else state[slot]
+        for t in range(r0, r1):
+            s = torch.exp(dt[t][:, None] * a) * s \
+                + (dt[t] * x[t])[:, None] * lowf[t, :n]
+            y = s @ lowf[t, n:] + d * x[t]
+            out[t] = (y * torch.nn.functional.silu(gate[t].float())).to(
+                out.dtype)
+        if slot >= 0:
+            state[slot] = s
+
+
+def lightning(out, x, decay, state, state_slots, positions, seq_start,
+              max_len, recurrent):
+    _, heads, dim, vdim = state.shape
+    f = torch.nn.functional.silu(x[:, :heads * (2 * dim + vdim)].float()).to(
+        x.dtype).float()
+    q, k, v = f.split([heads * dim] * 2 + [heads * vdim], dim=1)
+    q, k = (t.reshape(-1, heads, dim, 1) for t in (q, k))
+    v = v.reshape(-1, heads, 1, vdim)
+    for e, (a, b) in enumerate(_entry_rows(seq_start, x.shape[0])):
+        slot = int(state_slots[e])
+        s = torch.zeros(heads, dim, vdim, device=x.device) \
+            if slot < 0 or int(positions[a]) == 0 else state[slot]
+        for t in range(a, b):
+            s = decay[:, None, None] * s + k[t] * v[t]
+            out[t] = (s * q[t]).sum(1).reshape(-1).to(out.dtype)
+        if slot >= 0:
+            state[slot] = s
+
+
+def joint_gate(out, o, norm, gate, eps):
+    y = _rms(o.float(), eps) * norm * torch.sigmoid(gate.float())
+    out.copy_(y.to(out.dtype))
+
+
+def delta(out, qkv, z, z_bias, rate, beta, norm, gate, state, state_slots,
+          positions, seq_start, kv_heads, eps, mult, max_len, recurrent):
+    _, heads, dim, vdim = state.shape
+    f = qkv.float()
+    q, k, v = f.split([kv_heads * dim] * 2 + [heads * vdim], dim=1)
+
+    def unit(t):
+        t = t.reshape(-1, kv_heads, dim)
+        t = t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)
+        return t.repeat_interleave(heads // kv_heads, 1)[..., None]
+    q, k = unit(q) * dim ** -0.5, unit(k)
+    v = v.reshape(-1, heads, vdim)
+    g = torch.exp(-rate[:, None] * torch.nn.functional.softplus(
+        z + z_bias).view(-1, heads, dim))[..., None]
+    b = torch.sigmoid(beta.float())[..., None]
+    for e, (r0, r1) in enumerate(_entry_rows(seq_start, qkv.shape[0])):
+        slot = int(state_slots[e])
+        s = torch.zeros(heads, dim, vdim, device=f.device) \
+            if slot < 0 or int(positions[r0]) == 0 else state[slot]
+        for t in range(r0, r1):
+            s = g[t] * s
+            new = b[t] * (v[t] - (s * k[t]).sum(1))
+            s = s + k[t] * new[:, None]
+            o = _rms((s * q[t]).sum(1), eps) * norm
+            o = o.reshape(-1) * torch.sigmoid(gate[t].float()) * mult
+            out[t] = o.to(out.dtype)
+        if slot >= 0:
+            state[slot] = s
+
+
+def glu_values(g, u, act, limit):
+    if act == "clamped":
+        g, u = g.clamp(max=limit), u.clamp(-limit, limit) + 1
+        return g * torch.sigmoid(1.702 * g) * u
+    return (g.clamp(min=0) if act == "relu"
+            else torch.nn.functional.silu(g)) * u
+
+
+def glu(out, x, act, limit):
+    out.copy_(glu_values(*x.float().chunk(2, dim=-1), act, limit).to(
+        out.dtype))
+
+
 def _rotate(x, turns, positions):
     """x [rows, ..., n] float, its first 2 * len(turns) elements turned."""
     half = turns.shape[0]
@@ -294,26 +450,34 @@ def head_linear(out, x, w, gate, tail):
         out[..., w.shape[1]:] = x[..., k:k + tail]
 
 
-def moe_select(z, top, groups, keep):
+def moe_select(z, top, groups, keep, over_chosen=False):
     """(ids [rows, top] int32, weights float32), best first, of scores z."""
     s = torch.softmax(z, -1)
-    best = s.view(-1, groups, s.shape[1] // groups).amax(-1)
+    best = z.view(-1, groups, s.shape[1] // groups).amax(-1)
     kept = torch.zeros_like(best, dtype=torch.bool).scatter_(
         1, best.topk(keep, 1).indices, True)
     kept = kept.repeat_interleave(s.shape[1] // groups, 1)
-    weights, ids = s.masked_fill(~kept, -1.0).topk(top, 1)
-    return ids.int(), weights
+    chosen, ids = z.masked_fill(~kept, float("-inf")).topk(top, 1)
+    return ids.int(), torch.softmax(chosen, -1) if over_chosen \
+        else s.gather(1, ids)
 
 
-def experts(y, router, up, down, top, groups, keep):
-    """(rows, at, weights) of the chosen experts' outputs, token by token."""
-    f = y.float()
-    ids, weights = moe_select(f @ router.float().T, top, groups, keep)
+def experts(y, router, bias, up, down, spec):
+    """(rows, at, weights) of the chosen experts' outputs, token by token.
+    Gated experts' matrices have the rows of gate and up in turn."""
+    f, top = y.float(), spec.top
+    z = f @ router.float().T
+    if bias is not None:
+        z = z + bias
+    ids, weights = moe_select(z, top, spec.groups, spec.keep,
+                              spec.over_chosen)
     out = y.new_zeros(y.shape[0] * top, y.shape[1])
     flat = ids.reshape(-1)
     for e in flat.unique().tolist():
         r = (flat == e).nonzero()[:, 0]
-        h = torch.nn.functional.gelu(f[r // top] @ up[e].float().T)
+        h = f[r // top] @ up[e].float().T
+        h = torch.nn.functional.gelu(h) if spec.glu is None else glu_values(
+            h[:, ::2], h[:, 1::2], spec.glu.act, spec.glu.limit)
         out[r] = (h.to(y.dtype).float() @ down[e].float().T).to(y.dtype)
     at = torch.arange(flat.shape[0], dtype=torch.int32).view(-1, top)
     return out, at.to(y.device), weights
@@ -347,8 +511,9 @@ def _entry_rows(seq_start, rows):
     return list(zip(s[:-1], s[1:]))
 
 
-def attn_ctx(out, q, gate, k_cache, v_cache, bias, positions, seq_start,
-             block_table, scale, chunk, max_len, span, any_size):
+def attn_ctx(out, q, gate, k_cache, v_cache, bias, sink, positions, seq_start,
+             block_table, scale, chunk, window, keep, cap, mult, max_len, span,
+             any_size):
     kv, bs, dim = k_cache.shape[1:]
     vdim = v_cache.shape[3]
     for e, (a, b) in enumerate(_entry_rows(seq_start, q.shape[0])):
@@ -359,6 +524,8 @@ def attn_ctx(out, q, gate, k_cache, v_cache, bias, positions, seq_start,
                 .float() for c in (k_cache, v_cache))
         qe = q[a:b].float().view(b - a, kv, -1, dim)
         s = torch.einsum("ikgd,jkd->kgij", qe, k) * scale
+        if cap:
+            s = cap * torch.tanh(s / cap)
         dist = pos[:, None] - torch.arange(n, device=pos.device)
         if bias is not None:
             s = s + bias[:, dist.clamp(0, bias.shape[1] - 1)].view(
@@ -367,11 +534,18 @@ def attn_ctx(out, q, gate, k_cache, v_cache, bias, positions, seq_start,
         if chunk:
             seen &= (pos // chunk)[:, None] == torch.arange(
                 n, device=pos.device) // chunk
-        p = torch.softmax(s.masked_fill(~seen, float("-inf")), -1)
+        if window:
+            seen &= (dist < window) | (torch.arange(
+                n, device=pos.device) < keep)
+        s = s.masked_fill(~seen, float("-inf"))
+        if sink is not None:    # a key without a value
+            s = torch.cat([s, sink.view(kv, -1, 1, 1).expand(
+                kv, s.shape[1], b - a, 1)], -1)
+        p = torch.softmax(s, -1)[..., :n]
         o = torch.einsum("kgij,jkd->ikgd", p, v).reshape(b - a, -1, vdim)
         if gate is not None:
             o = o * torch.sigmoid(gate[a:b].float())[:, :, None]
-        out[a:b] = o.reshape(b - a, -1).to(out.dtype)
+        out[a:b] = (o.reshape(b - a, -1) * mult).to(out.dtype)
 
 
 def gla(out, x, a2, a2_bias, norm, state, state_slots, positions, seq_start,

@@ -6,10 +6,12 @@ block_size × head_dim panel (16×128 bf16 = 4 KiB), the unit the decode
 attention kernel streams through LDS/registers with wide coalesced loads.
 
 Models of unlike layers (ModelConfig.layers) keep per layer what its mixer
-asks for: pages with its own head sizes, pages of latents, or a 32-bit recurrent
-state for each of `state_slots` requests. A layer's entry in `layers` is (k, v),
-(latents,) or (state,). A layer that attends to another one's latents has that
-layer's very entry, and takes no memory of its own.
+asks for (MixerSpec.cache): pages with its own head sizes, pages of latents,
+a 32-bit recurrent state or a convolution's last inputs for each of
+`state_slots` requests. A layer's entry in `layers` has these in the mixer's
+order. A layer that attends to another one's latents has that layer's very
+entry, and takes no memory of its own. Layers that run more than once have an
+entry for every time they run, in the order they run.
 """
 
 from __future__ import annotations
@@ -19,7 +21,7 @@ from dataclasses import dataclass, field
 import torch
 
 from ..models.config import ModelConfig
-from ..models.layers import LatentAttentionSpec
+from ..models.layers import Pages
 
 DEFAULT_BLOCK_SIZE = 16
 
@@ -84,24 +86,20 @@ class PagedKVCache:
         self.slots = SlotAllocator(
             state_slots if any(s.mixer.state_bytes() for s in cfg.layers)
             else 0)
-        for spec in cfg.layers:
-            m = spec.mixer
-            if isinstance(m, LatentAttentionSpec):
-                # one row per token, as one key head of which the first
-                # columns are also the values
-                self.layers.append(
-                    self.layers[m.kv_from] if m.kv_from is not None else
-                    (torch.zeros(num_blocks, 1, block_size, m.row,
-                                 device=device, dtype=dtype),))
-            elif m.state_bytes():
-                self.layers.append((torch.zeros(
-                    state_slots, m.heads, m.dim, m.vdim, device=device,
-                    dtype=torch.float32),))
-            else:
-                self.layers.append(tuple(
-                    torch.zeros(num_blocks, m.kv_heads, block_size, d,
-                                device=device, dtype=dtype)
-                    for d in (m.dim, m.vdim)))
+
+        def part(p):
+            if isinstance(p, Pages):
+                return torch.zeros(num_blocks, p.heads, block_size, p.dim,
+                                   device=device, dtype=dtype)
+            return torch.zeros(state_slots, *p.shape, device=device,
+                               dtype=torch.float32 if p.f32 else dtype)
+        latest: dict[int, tuple] = {}    # layer -> its last run's entry
+        for i, _ in cfg.runs():
+            m = cfg.layers[i].mixer
+            src = getattr(m, "kv_from", None)
+            latest[i] = latest[src] if src is not None else \
+                tuple(part(p) for p in m.cache())
+            self.layers.append(latest[i])
         for _ in range(0 if cfg.layers else cfg.num_layers):
             k = torch.zeros(num_blocks, n_kv_heads_local, block_size,
                             cfg.head_dim, device=device, dtype=dtype)
@@ -136,7 +134,8 @@ class PagedKVCache:
 
     @staticmethod
     def state_bytes(cfg: ModelConfig, state_slots: int) -> int:
-        return state_slots * sum(s.mixer.state_bytes() for s in cfg.layers)
+        return state_slots * sum(cfg.layers[i].mixer.state_bytes()
+                                 for i, _ in cfg.runs())
 
     @staticmethod
     def blocks_for_memory(cfg: ModelConfig, n_kv_heads_local: int,
@@ -144,8 +143,9 @@ class PagedKVCache:
                           block_size: int = DEFAULT_BLOCK_SIZE,
                           dtype_bytes: int = 2) -> int:
         if cfg.layers:
-            per_block = block_size * sum(s.mixer.kv_bytes(dtype_bytes)
-                                         for s in cfg.layers)
+            per_block = block_size * sum(
+                cfg.layers[i].mixer.kv_bytes(dtype_bytes)
+                for i, _ in cfg.runs())
         else:
             per_block = (2 * cfg.num_layers * n_kv_heads_local * block_size *
                          cfg.head_dim * dtype_bytes)
