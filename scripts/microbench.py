@@ -295,12 +295,13 @@ def bench_latent():
         wb = live * moe.ff * w * 2
         report(f"  expert_linear up packed={packed} {w}->{moe.ff} "
                f"x{live}", timeit(lambda: ext.expert_linear(
-                   hid, x, up, src, start, tiles, tile, True), it),
+                   hid, x, up, src, start, tiles, tile, "gelu", 0.0), it),
                wb + rows * w * 2 + packed * moe.ff * 2,
                2.0 * packed * w * moe.ff)
         report(f"  expert_linear down packed={packed} {moe.ff}->{w}",
                timeit(lambda: ext.expert_linear(
-                   out, hid, down, None, start, tiles, tile, False), it),
+                   out, hid, down, None, start, tiles, tile, "none", 0.0),
+                   it),
                wb + packed * (moe.ff + w) * 2, 2.0 * packed * w * moe.ff)
         del up, down, hid, out, dense, dn, y
         side = 256
@@ -346,8 +347,9 @@ def bench_latent():
         o = torch.empty(b, h * rank, **bf)
         report(f"  attn_latent single b={b} ctx={ctx} {h}x{spec.row}",
                timeit(lambda: hy._ext().attn_ctx(
-                   o, qa, None, cache, cache[..., :rank], None, sb.positions,
-                   None, sb.block_table, spec.scale, 0, 1, ctx, False), 50),
+                   o, qa, None, cache, cache[..., :rank], None, None,
+                   sb.positions, None, sb.block_table, spec.scale, 0, 0, 0,
+                   0.0, 1.0, 1, ctx, False), 50),
                b * ctx * spec.row * 2 + b * h * (spec.row + rank) * 2,
                2.0 * b * ctx * h * (spec.row + rank))
 
@@ -384,9 +386,9 @@ def bench_latent():
         o = torch.empty(b * n, h * rank, **bf)
         report(f"  attn_latent portions b={b} {n} after {first}",
                timeit(lambda: hy._ext().attn_ctx(
-                   o, qa, None, cache, cache[..., :rank], None, sb.positions,
-                   sb.seq_start, sb.block_table, spec.scale, 0, n, first + n,
-                   False), 20),
+                   o, qa, None, cache, cache[..., :rank], None, None,
+                   sb.positions, sb.seq_start, sb.block_table, spec.scale, 0,
+                   0, 0, 0.0, 1.0, n, first + n, False), 20),
                b * (first + n) * spec.row * 2 + b * n * h * 2 * (
                    spec.row + rank),
                2.0 * b * n * (first + n / 2) * h * (spec.row + rank))

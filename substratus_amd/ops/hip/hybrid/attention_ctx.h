@@ -7,7 +7,7 @@
 
 template <class T>
 struct AttnCtx {
-  T* out;                  // [rows, heads * vdim]
+  T* out;                  // row r, head h at out + r * out_ld + h * vdim
   const T* q;              // row r, head h at q + r * q_ld + h * dim
   const T* gate;           // row r, head h at gate + r * g_ld + h, or null;
                            // flat: column c at gate + r * g_ld + h * vdim + c
@@ -15,12 +15,18 @@ struct AttnCtx {
   const T* vc;             // [blocks, kv_heads, block_size, vdim], rows of
                            // v_ld elements (values may be part of the keys)
   const float* bias;       // [heads, nbias] by distance, or null
+  const float* sink;       // [heads], or null
   const int* positions;    // [rows]
   const int* seq_start;    // [entries + 1] row offsets, or null: one row each
   const int* block_table;  // [entries, max_blocks]
-  long q_ld, g_ld, v_ld;
+  long q_ld, g_ld, v_ld, out_ld;
   int heads, kv_heads, dim, vdim, nbias, chunk, max_blocks, block_size;
+  int window;              // > 0: keys that a row sees, its own included
+  int keep;                // with a window: a sequence's first keys, too
   float scale;
+  float cap;               // > 0: scores are cap * tanh(score / cap)
+  float mult;              // of the result
+  bool quads;              // out: four columns at a time may be stored
   // flat: keys and values are not paged; key j of entry e is row
   // ctx_start[e] + j of kc and vc, whose rows are v_ld apart and hold one
   // piece per head; the last `shared` elements of every head's key are kr's
@@ -30,6 +36,30 @@ struct AttnCtx {
 };
 
 constexpr float LOG2E = 1.44269504088896340736f;
+
+// First key that a row at `pos` sees, apart from the kept ones.
+template <class T>
+DEV_INLINE int first_seen(const AttnCtx<T>& a, int pos) {
+  if (a.chunk > 0) return pos / a.chunk * a.chunk;
+  return a.window > 0 ? max(pos - a.window + 1, 0) : 0;
+}
+
+// Pieces of a context (pages, steps) that hold visible keys, in order: those
+// of the kept keys, then those from key `lo` to the last piece.
+struct Pieces {
+  int kept, skip, n;
+  DEV_INLINE Pieces(int keep, int lo, int pieces, int size) {
+    kept = min((keep + size - 1) / size, pieces);
+    skip = max(lo / size - kept, 0);
+    n = pieces - skip;
+  }
+  DEV_INLINE int at(int i) const { return i < kept ? i : i + skip; }
+};
+
+// tanh(z) = 1 - 2 / (e^(2z) + 1), to 1e-7 absolute; `z2` is 2 z log2(e)
+DEV_INLINE float tanh_exp2(float z2) {
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(z2) + 1.f);
+}
 
 constexpr int ATTN_ANY_VDIM = 1024;   // largest value size
 

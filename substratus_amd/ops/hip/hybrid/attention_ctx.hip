@@ -1,9 +1,13 @@
 // Attention over a paged cache for any head sizes, in float or bf16, for
 // single tokens and portions of prompts: one wave per (row, query head).
 //
-//   score(i, j) = scale * q_i . k_j + bias[h][min(i - j, nbias - 1)]
-//   visible: j <= i, and i / chunk == j / chunk when chunk > 0
-//   out_h = softmax(score) v * sigmoid(gate_h)          (gate optional)
+//   score(i, j) = f(scale * q_i . k_j) + bias[h][min(i - j, nbias - 1)]
+//                 with f(s) = s, or cap * tanh(s / cap) when cap > 0
+//   visible: j <= i, and i / chunk == j / chunk when chunk > 0,
+//            and i - j < window or j < keep when window > 0
+//   out_h = softmax(score) v * sigmoid(gate_h) * mult   (gate optional)
+//
+// With a sink, the softmax's denominator has e^(sink_h) besides the keys.
 //
 // Query head h reads key/value head h / (heads / kv_heads). 64 keys at a
 // time: lane = key for the scores, lane = column for the values. This is the
@@ -23,7 +27,8 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
   const int h = blockIdx.y, lane = threadIdx.x;
   const int kvh = h / (a.heads / a.kv_heads);
   const int pos = a.positions[row];
-  const int lo = a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
+  const int lo = first_seen(a, pos);
+  const Pieces part(a.keep, lo, pos / WAVE + 1, WAVE);
   const int* bt = a.block_table + (long)blockIdx.z * a.max_blocks;
 
   const T* q = a.q + row * a.q_ld + (long)h * a.dim;
@@ -34,19 +39,21 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
   #pragma unroll
   for (int c = 0; c < CMAX; ++c) acc[c] = 0.f;
   float m = -INFINITY, l = 0.f;
-  for (int k0 = lo; k0 <= pos; k0 += WAVE) {
-    const int key = k0 + lane;
+  if (a.sink != nullptr) { m = a.sink[h]; l = 1.f; }
+  for (int i = 0; i < part.n; ++i) {
+    const int k0 = part.at(i) * WAVE, key = k0 + lane;
     float s = -INFINITY;
-    if (key <= pos) {
+    if (key <= pos && (key >= lo || key < a.keep)) {
       const long page = bt[key / a.block_size];
       const T* k = a.kc + ((page * a.kv_heads + kvh) * a.block_size +
                            key % a.block_size) * a.dim;
       s = 0.f;
       for (int i = 0; i < a.dim; ++i) s += s_q[i] * ld1(k + i);
+      if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
       if (a.bias != nullptr)
         s += a.bias[(long)h * a.nbias + min(pos - key, a.nbias - 1)];
     }
-    const float mn = fmaxf(m, wave_max(s));      // finite: key k0 is visible
+    const float mn = fmaxf(m, wave_max(s));      // finite: some key is visible
     const float p = expf(s - mn);
     const float keep = expf(m - mn);
     l = l * keep + wave_sum(p);
@@ -70,9 +77,9 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
     }
     __syncthreads();
   }
-  float g = 1.f / l;
+  float g = a.mult / l;
   if (a.gate != nullptr) g *= sigmoid_f(ld1(a.gate + row * a.g_ld + h));
-  T* out = a.out + (row * a.heads + h) * a.vdim;
+  T* out = a.out + row * a.out_ld + (long)h * a.vdim;
   #pragma unroll
   for (int c = 0; c < CMAX; ++c) {
     const int col = lane + c * WAVE;

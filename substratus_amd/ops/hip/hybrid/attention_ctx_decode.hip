@@ -44,7 +44,8 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   const int nh = min(GQ, per - g0);
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int pos = a.positions[b];
-  const int lo = a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
+  const int lo = first_seen(a, pos);
+  const Pieces part(a.keep, lo, pos / PAGE + 1, PAGE);
   const int* bt = a.block_table + (long)b * a.max_blocks;
 
   for (int i = threadIdx.x; i < GQ * DCH * 16; i += NW * WAVE) {
@@ -58,9 +59,11 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   const int key = lane >> 2, sub = lane & 3;
   const int col = lane % CL, rg = lane / CL;
   const int kch = a.dim / 8, vch = a.vdim / 8;
-  const int first = lo / PAGE + split * NW + wave, last = pos / PAGE;
-  const int stride = splits * NW;
+  const int first = split * NW + wave, stride = splits * NW;
+  // a capped score: cap tanh(s scale / cap), by tanh_exp2
   const float scale2 = a.scale * LOG2E;
+  const float cap2 = a.cap * LOG2E;
+  const float cscale = a.cap > 0.f ? 2.f * scale2 / a.cap : 0.f;
 
   uint4v kr[DCH], vr[NV];
   float br[GQ];
@@ -92,8 +95,9 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     #pragma unroll
     for (int j = 0; j < 8; ++j) acc[g][j] = 0.f;
   }
-  if (first <= last) load(first);
-  for (int pg = first; pg <= last; pg += stride) {
+  if (first < part.n) load(part.at(first));
+  for (int it = first; it < part.n; it += stride) {
+    const int pg = part.at(it);
     uint4v kn[DCH], vn[NV];
     float bn[GQ];
     #pragma unroll
@@ -102,7 +106,7 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     for (int i = 0; i < NV; ++i) vn[i] = vr[i];
     #pragma unroll
     for (int g = 0; g < GQ; ++g) bn[g] = br[g];
-    if (pg + stride <= last) load(pg + stride);
+    if (it + stride < part.n) load(part.at(it + stride));
 
     float s[GQ];
     #pragma unroll
@@ -120,12 +124,13 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
       }
     }
     const int kpos = pg * PAGE + key;
-    const bool live = kpos >= lo && kpos <= pos;
+    const bool live = kpos <= pos && (kpos >= lo || kpos < a.keep);
     #pragma unroll
     for (int g = 0; g < GQ; ++g) {
       s[g] += __shfl_xor(s[g], 1, WAVE);
       s[g] += __shfl_xor(s[g], 2, WAVE);
-      s[g] = live ? s[g] * scale2 + bn[g] : NEG;
+      s[g] = a.cap > 0.f ? cap2 * tanh_exp2(s[g] * cscale) : s[g] * scale2;
+      s[g] = live ? s[g] + bn[g] : NEG;
       float mx = s[g];
       #pragma unroll
       for (int off = 4; off < WAVE; off <<= 1)
@@ -177,6 +182,11 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     #pragma unroll
     for (int w = 1; w < NW; ++w) M = fmaxf(M, s_ml[w][g][0]);
     float L = 0.f, o = 0.f;
+    if (a.sink != nullptr && splits == 1) {
+      const float s = a.sink[h] * LOG2E;
+      M = fmaxf(M, s);
+      L = __builtin_amdgcn_exp2f(s - M);
+    }
     #pragma unroll
     for (int w = 0; w < NW; ++w) {
       const float f = __builtin_amdgcn_exp2f(s_ml[w][g][0] - M);
@@ -184,10 +194,10 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
       o += s_o[w][g][c] * f;
     }
     if (splits == 1) {
-      float f = 1.f / L;
+      float f = a.mult / L;
       if (a.gate != nullptr)
         f *= sigmoid_f(bf2f(a.gate[(long)b * a.g_ld + h]));
-      a.out[((long)b * a.heads + h) * a.vdim + c] = f2bf(o * f);
+      a.out[(long)b * a.out_ld + (long)h * a.vdim + c] = f2bf(o * f);
     } else {
       const long at = ((long)b * a.heads + h) * splits + split;
       part_o[at * a.vdim + c] = o;
@@ -209,6 +219,11 @@ void attn_ctx_merge_kernel(AttnCtx<bf16_t> a, int splits,
   float M = NEG;
   for (int s = 0; s < splits; ++s) M = fmaxf(M, part_ml[(at + s) * 2]);
   float L = 0.f, o[VEC];
+  if (a.sink != nullptr) {
+    const float s = a.sink[h] * LOG2E;
+    M = fmaxf(M, s);
+    L = __builtin_amdgcn_exp2f(s - M);
+  }
   #pragma unroll
   for (int j = 0; j < VEC; ++j) o[j] = 0.f;
   #pragma unroll 4
@@ -220,11 +235,17 @@ void attn_ctx_merge_kernel(AttnCtx<bf16_t> a, int splits,
     #pragma unroll
     for (int j = 0; j < VEC; ++j) o[j] += p[j] * f;
   }
-  float f = 1.f / L;
+  float f = a.mult / L;
   if (a.gate != nullptr) f *= sigmoid_f(bf2f(a.gate[b * a.g_ld + h]));
   #pragma unroll
   for (int j = 0; j < VEC; ++j) o[j] *= f;
-  stv<VEC>(a.out + (b * a.heads + h) * a.vdim + c, o);
+  bf16_t* out = a.out + b * a.out_ld + (long)h * a.vdim + c;
+  if (a.quads) {
+    stv<VEC>(out, o);
+  } else {
+    #pragma unroll
+    for (int j = 0; j < VEC; ++j) st1(out + j, o[j]);
+  }
 }
 
 constexpr int pick_gq(int per) { return per >= 4 ? 4 : per >= 2 ? 2 : 1; }

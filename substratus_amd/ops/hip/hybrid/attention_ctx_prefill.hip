@@ -42,7 +42,8 @@ DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
 }
 
 // KK: 16-wide steps of the key size; DC: 32-wide tiles of the value size
-template <int KK, int DC, int WAVES, bool FLAT>
+// CAP: scores are capped
+template <int KK, int DC, int WAVES, bool FLAT, bool CAP>
 __global__ __launch_bounds__(WAVES * WAVE)
 void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   constexpr int THREADS = WAVES * WAVE;
@@ -76,13 +77,12 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   const bool wave_live = qw0 < total;
   const int qpos = qw0 + lo5;
   const int row = min(q0_tile + wave * 32 + lo5, en.n - 1);
-  const int lo = a.chunk > 0 ? qpos / a.chunk * a.chunk : 0;
-  const int lo_wave = a.chunk > 0 ? qw0 / a.chunk * a.chunk : 0;
+  const int lo = first_seen(a, qpos), lo_wave = first_seen(a, qw0);
   const int hi_wave = min(qw0 + 31, total - 1);
-  // lo of the wave's last row: keys at or above it are inside every chunk
-  const int lo_last = a.chunk > 0 ? (qw0 + 31) / a.chunk * a.chunk : 0;
-  const int first = (a.chunk > 0 ? qa0 / a.chunk * a.chunk : 0) / CH;
-  const int steps = (min(qa0 + QT, total) + CH - 1) / CH;
+  // lo of the wave's last row: keys at or above it are inside every range
+  const int lo_last = first_seen(a, qw0 + 31);
+  const Pieces part(a.keep, first_seen(a, qa0),
+                    (min(qa0 + QT, total) + CH - 1) / CH, CH);
 
   short8 qreg[KK];
   {
@@ -96,30 +96,35 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
     }
   }
   float m = -INFINITY, l = 0.f;
+  if (a.sink != nullptr) { m = a.sink[head] * LOG2E; l = 1.f; }
   float16v o_t[DC];
   #pragma unroll
   for (int c = 0; c < DC; ++c) o_t[c] = (float16v){};
 
   const float scale2 = a.scale * LOG2E;
+  const float cap2 = a.cap * LOG2E;
+  const float cscale = a.cap > 0.f ? 2.f * scale2 / a.cap : 0.f;
   int pgk[LK], pgv[LV];                          // page bases, -1: no key
   uint4 st_k[LK], st_v[LV];
   float st_b = 0.f;
 
-  auto pages = [&](int st) {
+  auto pages = [&](int it) {
+    const int st = part.at(it);
     #pragma unroll
     for (int i = 0; i < LK; ++i) {
       const int key = st * CH + (i * THREADS + tid) / (KK * 2);
-      pgk[i] = st < steps && key < total && key < st * CH + CH
+      pgk[i] = it < part.n && key < total && key < st * CH + CH
           ? (FLAT ? key : bt[key / PAGE]) : -1;
     }
     #pragma unroll
     for (int i = 0; i < LV; ++i) {
       const int key = st * CH + (i * THREADS + tid) / (DC * 4);
-      pgv[i] = st < steps && key < total && key < st * CH + CH
+      pgv[i] = it < part.n && key < total && key < st * CH + CH
           ? (FLAT ? key : bt[key / PAGE]) : -1;
     }
   };
-  auto stage_load = [&](int st) {
+  auto stage_load = [&](int it) {
+    const int st = part.at(it);
     #pragma unroll
     for (int i = 0; i < LK; ++i) {
       const int f = i * THREADS + tid;
@@ -179,20 +184,21 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
     s_b[buf][tid] = st_b;
   };
 
-  pages(first);
-  stage_load(first);
-  pages(first + 1);
+  pages(0);
+  stage_load(0);
+  pages(1);
   stage_write(0);
   __syncthreads();
 
-  for (int st = first; st < steps; ++st) {
-    const int cur = (st - first) & 1;
-    if (st + 1 < steps) {
-      stage_load(st + 1);
-      pages(st + 2);
+  for (int it = 0; it < part.n; ++it) {
+    const int cur = it & 1;
+    if (it + 1 < part.n) {
+      stage_load(it + 1);
+      pages(it + 2);
     }
-    const int kbase = st * CH;
-    if (wave_live && kbase <= hi_wave && kbase + CH > lo_wave) {
+    const int kbase = part.at(it) * CH;
+    if (wave_live && kbase <= hi_wave &&
+        (kbase + CH > lo_wave || kbase < a.keep)) {
       float16v sacc[CH / 32];
       #pragma unroll
       for (int sc = 0; sc < CH / 32; ++sc) {
@@ -211,7 +217,8 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
       for (int sc = 0; sc < CH / 32; ++sc)
         #pragma unroll
         for (int r = 0; r < 16; ++r)
-          sv[sc][r] = sacc[sc][r] * scale2 +
+          sv[sc][r] = (CAP ? cap2 * tanh_exp2(sacc[sc][r] * cscale)
+                           : sacc[sc][r] * scale2) +
                       bw[-(sc * 32 + (r & 3) + 8 * (r >> 2))];
       // steps inside every row's range need no mask
       if (kbase < lo_last || kbase + CH - 1 > qw0 || qw0 + 31 >= total) {
@@ -221,7 +228,8 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
           for (int r = 0; r < 16; ++r) {
             const int kpos =
                 kbase + sc * 32 + (r & 3) + 8 * (r >> 2) + 4 * hi;
-            if (!(kpos <= qpos && kpos >= lo && qpos < total))
+            if (!(kpos <= qpos && (kpos >= lo || kpos < a.keep) &&
+                  qpos < total))
               sv[sc][r] = -INFINITY;
           }
       }
@@ -282,16 +290,16 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
       }
       l += sum + __shfl_xor(sum, 32, WAVE);
     }
-    if (st + 1 < steps) stage_write(cur ^ 1);
+    if (it + 1 < part.n) stage_write(cur ^ 1);
     __syncthreads();
   }
 
   if (wave_live && qpos < total) {
     const long r = en.row0 + row;
-    float f = 1.f / l;
+    float f = a.mult / l;
     if (!FLAT && a.gate != nullptr)
       f *= sigmoid_f(bf2f(a.gate[r * a.g_ld + head]));
-    bf16_t* op = a.out + (r * a.heads + head) * a.vdim;
+    bf16_t* op = a.out + r * a.out_ld + (long)head * a.vdim;
     #pragma unroll
     for (int c = 0; c < DC; ++c) {
       #pragma unroll
@@ -307,7 +315,12 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
             #pragma unroll
             for (int j = 0; j < 4; ++j) o[j] *= sigmoid_f(g[j]);
           }
-          stv<4>(op + d0, o);
+          if (a.quads) {
+            stv<4>(op + d0, o);
+          } else {
+            #pragma unroll
+            for (int j = 0; j < 4; ++j) st1(op + d0 + j, o[j]);
+          }
         }
       }
     }
@@ -326,12 +339,17 @@ void launch_attn_ctx_prefill(const AttnCtx<bf16_t>& a, int entries,
   auto go = [&](auto kk, auto dc, auto waves) {
     constexpr int W = decltype(waves)::value;
     const dim3 grid(entries, a.heads, (max_len + W * 32 - 1) / (W * 32));
+    constexpr int K = decltype(kk)::value, D = decltype(dc)::value;
+    const dim3 block(W * WAVE);
     if (a.ctx_start != nullptr)
-      attn_ctx_prefill_kernel<decltype(kk)::value, decltype(dc)::value, W,
-                              true><<<grid, dim3(W * WAVE), 0, stream>>>(a);
+      attn_ctx_prefill_kernel<K, D, W, true, false>
+          <<<grid, block, 0, stream>>>(a);
+    else if (a.cap > 0.f)
+      attn_ctx_prefill_kernel<K, D, W, false, true>
+          <<<grid, block, 0, stream>>>(a);
     else
-      attn_ctx_prefill_kernel<decltype(kk)::value, decltype(dc)::value, W,
-                              false><<<grid, dim3(W * WAVE), 0, stream>>>(a);
+      attn_ctx_prefill_kernel<K, D, W, false, false>
+          <<<grid, block, 0, stream>>>(a);
   };
   using std::integral_constant;
   auto by_dc = [&](auto kk) {

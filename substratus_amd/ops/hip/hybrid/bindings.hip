@@ -1,14 +1,13 @@
 // Python bindings of the hybrid-model kernels (substratus_amd._hybrid): norms
-// of a 32-bit residual, cache-reading attention, gated linear attention.
+// of a 32-bit residual, cache-reading attention, mixtures of experts; mixers
+// with a state per request are in bindings_mixers.hip.
 // Every op takes float or bf16 activations. Shapes are checked here; kernels
 // are thin and trusting.
-#include <torch/extension.h>
-#include <ATen/cuda/CUDAContext.h>
+#include "bindings.h"
 
 #include <numeric>
 
 #include "attention_ctx.h"
-#include "gla.h"
 #include "group_gemm.h"
 
 template <class T>
@@ -17,7 +16,7 @@ template <class T>
 void launch_latent_prepare(T*, long, int, int, int, int, int, const float*, float, const double*, int, const int*, T*, const int*, long, hipStream_t);
 void launch_latent_gather(void*, void*, const void*, int, int, int, const int*, int, const int*, int, int, hipStream_t);
 int moe_max_experts();
-void launch_moe_select(int*, float*, const float*, int, int, int, int, int, int, hipStream_t);
+void launch_moe_select(int*, float*, const float*, int, int, int, int, int, int, const float*, bool, hipStream_t);
 void launch_moe_sort(int*, int*, int*, int*, const int*, int, int, int, int, hipStream_t);
 template <class T>
 void launch_embed_norm(T*, float*, const T*, const int*, const float*, long, int, int, float, float, hipStream_t);
@@ -29,47 +28,6 @@ void launch_silu_mul_any(float*, const float*, long, int, hipStream_t);
 void launch_silu_mul_any(bf16_t*, const bf16_t*, long, int, hipStream_t);
 
 namespace {
-
-using torch::Tensor;
-using OptTensor = std::optional<Tensor>;
-
-hipStream_t stream() { return at::cuda::getCurrentCUDAStream().stream(); }
-
-template <class T> struct Scalar;
-template <> struct Scalar<float> { static constexpr auto type = torch::kFloat32; };
-template <> struct Scalar<bf16_t> { static constexpr auto type = torch::kBFloat16; };
-
-void check(const Tensor& t, torch::ScalarType type, const char* name,
-           bool contiguous = true) {
-  TORCH_CHECK(t.is_cuda(), name, " must be on the GPU");
-  TORCH_CHECK(t.scalar_type() == type, name, " must be ", type, ", is ",
-              t.scalar_type());
-  TORCH_CHECK(!contiguous || t.is_contiguous(), name, " must be contiguous");
-}
-
-template <class T>
-T* ptr(const Tensor& t) { return reinterpret_cast<T*>(t.data_ptr()); }
-template <class T>
-T* ptr(const OptTensor& t) { return t ? ptr<T>(*t) : nullptr; }
-
-// [rows, n] view whose rows are `stride(0)` apart
-void check_rows(const Tensor& t, torch::ScalarType type, const char* name) {
-  check(t, type, name, false);
-  TORCH_CHECK(t.dim() == 2 && (t.stride(1) == 1 || t.size(1) == 1), name,
-              " must be [rows, n] with contiguous rows");
-}
-
-void post(const char* op) {
-  const hipError_t e = hipGetLastError();
-  TORCH_CHECK(e == hipSuccess, op, ": launch failed: ", hipGetErrorString(e));
-}
-
-template <class F>
-void by_type(const Tensor& t, F f) {
-  if (t.scalar_type() == torch::kBFloat16) f(bf16_t{});
-  else if (t.scalar_type() == torch::kFloat32) f(float{});
-  else TORCH_CHECK(false, "activations must be float32 or bfloat16");
-}
 
 // rows [pool, width], picked by at and weights [rows of x, picks], or
 // [rows of x, width] without those
@@ -179,9 +137,10 @@ void qkv_prepare(Tensor buf, int64_t nq, OptTensor qw, OptTensor kw,
 // `rows` are those of q; span: most keys a row can see; any: take the
 // untiled kernel.
 void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
-              OptTensor bias, Tensor positions, OptTensor seq_start,
-              Tensor block_table, double scale, int64_t chunk,
-              int64_t max_len, int64_t span, bool any) {
+              OptTensor bias, OptTensor sink, Tensor positions,
+              OptTensor seq_start, Tensor block_table, double scale,
+              int64_t chunk, int64_t window, int64_t keep, double cap,
+              double mult, int64_t max_len, int64_t span, bool any) {
   const int kv = kc.size(1), dim = kc.size(3), vdim = vc.size(3);
   const long rows = q.size(0);
   TORCH_CHECK(q.size(1) % dim == 0, "q is not heads * dim wide");
@@ -207,11 +166,16 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     check(*bias, torch::kFloat32, "bias");
     TORCH_CHECK(bias->dim() == 2 && bias->size(0) == heads, "bias heads");
   }
+  if (sink) {
+    check(*sink, torch::kFloat32, "sink");
+    TORCH_CHECK(sink->numel() == heads, "sink heads");
+  }
+  TORCH_CHECK(chunk == 0 || window == 0, "a chunk or a window, not both");
   if (rows == 0) return;
   by_type(q, [&](auto tag) {
     using T = decltype(tag);
     check_rows(q, Scalar<T>::type, "q");
-    check(out, Scalar<T>::type, "out");
+    check_rows(out, Scalar<T>::type, "out");
     check(kc, Scalar<T>::type, "kc");
     // values may be the first columns of wider rows
     check(vc, Scalar<T>::type, "vc", false);
@@ -236,13 +200,20 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     a.nbias = bias ? bias->size(1) : 1; a.chunk = chunk;
     a.max_blocks = block_table.size(1); a.block_size = kc.size(2);
     a.scale = scale;
+    a.sink = ptr<float>(sink);
+    a.window = window; a.keep = window > 0 ? keep : 0;
+    a.cap = cap; a.mult = mult;
+    a.out_ld = out.stride(0);
+    a.quads = vdim % 4 == 0 && a.out_ld % 4 == 0 &&
+              reinterpret_cast<uintptr_t>(a.out) % (4 * sizeof(T)) == 0;
     if constexpr (std::is_same_v<T, bf16_t>) {
       // the tiled kernels read q rows in 16-byte pieces
       const bool aligned = a.q_ld % 8 == 0 &&
           reinterpret_cast<uintptr_t>(a.q) % 16 == 0;
       any = any || v_ld % 8 != 0;
       if (!any && aligned && kv == 1 && a.kc == a.vc && v_ld == dim && !bias &&
-          !gate && chunk == 0 &&
+          !gate && chunk == 0 && window == 0 && !sink && cap == 0 &&
+          mult == 1 && out.is_contiguous() &&
           attn_latent_supported(dim, vdim, a.block_size)) {
         const int longest = seq_start ? max_len : 1;
         const int splits = attn_latent_splits(entries, longest, heads, span);
@@ -330,7 +301,8 @@ void attn_flat(Tensor out, Tensor q, OptTensor gate, Tensor kv, Tensor kr,
   a.q_ld = q.stride(0); a.g_ld = gate ? gate->stride(0) : 0;
   a.v_ld = kv.size(1);
   a.heads = a.kv_heads = heads; a.nbias = 1; a.block_size = 16;
-  a.scale = scale;
+  a.scale = scale; a.mult = 1.f;
+  a.out_ld = out.stride(0); a.quads = vdim % 4 == 0;
   launch_attn_ctx_prefill(a, entries, max_len, stream());
   post("attn_flat");
 }
@@ -496,8 +468,25 @@ void side_gate(Tensor out, Tensor x, Tensor w, Tensor tokens, Tensor table,
   });
 }
 
+// x w^T in float32, unrounded
+Tensor linear32(Tensor x, Tensor w) {
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && x.size(1) == w.size(1),
+              "linear32: shapes differ");
+  Tensor y = torch::empty({x.size(0), w.size(0)},
+                          x.options().dtype(torch::kFloat32));
+  if (x.size(0) == 0) return y;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    auto a = product<T, float>(y, x, w);
+    group_gemm(a, std::min(128, group_gemm_tile(
+                   x.size(0), 1, std::is_same_v<T, bf16_t>, w.size(1))),
+               "linear32");
+  });
+  return y;
+}
+
 void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
-                int64_t keep) {
+                int64_t keep, OptTensor bias, bool over_chosen) {
   TORCH_CHECK(z.dim() == 3, "z must be [splits, rows, experts]");
   const long rows = z.size(1), experts = z.size(2), top = ids.size(1);
   check(ids, torch::kInt32, "ids");
@@ -506,12 +495,17 @@ void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
   TORCH_CHECK(ids.size(0) == rows && ids.sizes() == weights.sizes(),
               "moe_select: shapes differ");
   TORCH_CHECK(experts <= moe_max_experts(), "too many experts");
+  if (bias) {
+    check(*bias, torch::kFloat32, "bias");
+    TORCH_CHECK(bias->numel() == experts, "one bias per expert");
+  }
   TORCH_CHECK(groups > 0 && experts % groups == 0 && keep > 0 &&
               keep <= groups && top > 0 && top <= experts / groups * keep,
               "moe_select: cannot choose so many");
   if (rows == 0) return;
   launch_moe_select(ptr<int>(ids), ptr<float>(weights), ptr<float>(z),
-                    z.size(0), rows, experts, top, groups, keep, stream());
+                    z.size(0), rows, experts, top, groups, keep,
+                    ptr<float>(bias), over_chosen, stream());
   post("moe_select");
 }
 
@@ -540,13 +534,18 @@ void moe_sort(Tensor at, Tensor src, Tensor start, Tensor tiles, Tensor ids,
 }
 
 // Every packed row by its expert's matrix: out [packed, n], w [experts, n, k];
-// packed row r is row src[r] of x, or row r.
+// packed row r is row src[r] of x, or row r. act: none, gelu, or a gated
+// feed-forward's (w has the rows of gate and up in turn, out half as many
+// columns).
 void expert_linear(Tensor out, Tensor x, Tensor w, OptTensor src,
-                   Tensor start, Tensor tiles, int64_t tile, bool gelu) {
+                   Tensor start, Tensor tiles, int64_t tile,
+                   const std::string& act, double limit) {
+  const bool glu = act != "none" && act != "gelu";
   check(start, torch::kInt32, "start");
   check(tiles, torch::kInt32, "tiles");
   TORCH_CHECK(w.dim() == 3 && start.numel() == w.size(0) + 1 &&
-              x.size(1) == w.size(2) && out.size(1) == w.size(1),
+              x.size(1) == w.size(2) &&
+              (glu ? 2 : 1) * out.size(1) == w.size(1),
               "expert_linear: shapes differ");
   if (src) {
     check(*src, torch::kInt32, "src");
@@ -561,74 +560,10 @@ void expert_linear(Tensor out, Tensor x, Tensor w, OptTensor src,
     a.m = out.size(0);
     a.src = ptr<int>(src); a.start = ptr<int>(start);
     a.tiles = ptr<int>(tiles); a.max_tiles = (tiles.numel() - 1) / 2;
-    if (gelu) a.act = Act::GELU;
+    if (act == "gelu") a.act = Act::GELU;
+    if (glu) { a.act = Act::GLU; a.glu = glu_of(act); a.limit = limit; }
     group_gemm(a, tile, "expert_linear");
   });
-}
-
-// x [rows, >= q | k | v | g | A1 h]; state [slots, heads, dim, vdim]
-void gla(Tensor out, Tensor x, Tensor a2, Tensor a2b, Tensor norm,
-         Tensor state, Tensor state_slots, Tensor positions,
-         OptTensor seq_start, double inv_tau, double eps, int64_t max_len,
-         bool recurrent) {
-  const int heads = state.size(1), dim = state.size(2), vdim = state.size(3);
-  const int rank = a2.size(1);
-  const long rows = x.size(0);
-  check(a2, torch::kFloat32, "a2");
-  check(a2b, torch::kFloat32, "a2b");
-  check(norm, torch::kFloat32, "norm");
-  check(state, torch::kFloat32, "state");
-  check(state_slots, torch::kInt32, "state_slots");
-  check(positions, torch::kInt32, "positions");
-  const int entries = state_slots.numel();
-  if (seq_start) {
-    check(*seq_start, torch::kInt32, "seq_start");
-    TORCH_CHECK(seq_start->numel() == entries + 1, "entries differ");
-  } else {
-    TORCH_CHECK(rows == entries, "one row per entry");
-  }
-  TORCH_CHECK(a2.size(0) == heads * dim && a2b.numel() == heads * dim &&
-              norm.numel() == vdim && positions.numel() == rows,
-              "gla: shapes differ");
-  TORCH_CHECK(x.size(1) >= 2 * heads * (dim + vdim) + rank, "x too narrow");
-  TORCH_CHECK(dim <= 2048 && vdim <= 2048, "head size over 2048");
-  TORCH_CHECK(out.size(0) == rows && out.size(1) == heads * vdim,
-              "out must be [rows, heads * vdim]");
-  if (rows == 0) return;
-  by_type(x, [&](auto tag) {
-    using T = decltype(tag);
-    check_rows(x, Scalar<T>::type, "x");
-    check(out, Scalar<T>::type, "out");
-    Gla<T> a{};
-    a.out = ptr<T>(out); a.x = ptr<T>(x); a.ld = x.stride(0);
-    a.k_off = heads * dim; a.v_off = 2 * heads * dim;
-    a.g_off = a.v_off + heads * vdim; a.a_off = a.g_off + heads * vdim;
-    a.a2 = ptr<float>(a2); a.a2b = ptr<float>(a2b);
-    a.norm = ptr<float>(norm); a.state = ptr<float>(state);
-    a.state_slots = ptr<int>(state_slots);
-    a.positions = ptr<int>(positions); a.seq_start = ptr<int>(seq_start);
-    a.heads = heads; a.dim = dim; a.vdim = vdim; a.rank = rank;
-    a.qscale = 1.f / std::sqrt((float)dim); a.inv_tau = inv_tau; a.eps = eps;
-    if constexpr (std::is_same_v<T, bf16_t>) {
-      // the chunk kernel addresses a segment's rows with 32-bit offsets
-      if (seq_start && !recurrent && gla_chunk_supported(dim, vdim, rank) &&
-          max_len * a.ld * 2 < 0x7ffffff0 - (1 << 20)) {
-        const int nseg = gla_chunk_segments(entries, heads, max_len);
-        Tensor ws, wd;
-        if (nseg > 1) {
-          const auto opt = state.options();
-          ws = torch::empty({entries, nseg, heads, dim, vdim}, opt);
-          wd = torch::empty({entries, nseg, heads, dim}, opt);
-        }
-        launch_gla_chunk(a, entries, max_len, nseg,
-                         nseg > 1 ? ptr<float>(ws) : nullptr,
-                         nseg > 1 ? ptr<float>(wd) : nullptr, stream());
-        return;
-      }
-    }
-    launch_gla_recurrent<T>(a, entries, stream());
-  });
-  post("gla");
 }
 
 void silu_mul(Tensor out, Tensor x) {
@@ -659,7 +594,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("embed_norm", &embed_norm);
   m.def("qkv_prepare", &qkv_prepare);
   m.def("attn_ctx", &attn_ctx);
-  m.def("gla", &gla);
   m.def("silu_mul", &silu_mul);
   m.def("attn_flat", &attn_flat);
   m.def("latent_gather", &latent_gather);
@@ -667,8 +601,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("head_linear", &head_linear);
   m.def("router_scores", &router_scores);
   m.def("side_gate", &side_gate);
-  m.def("moe_select", &moe_select);
+  m.def("moe_select", &moe_select, py::arg("ids"), py::arg("weights"),
+        py::arg("z"), py::arg("groups"), py::arg("keep"),
+        py::arg("bias") = py::none(), py::arg("over_chosen") = false);
   m.def("moe_tile", &moe_tile);
   m.def("moe_sort", &moe_sort);
   m.def("expert_linear", &expert_linear);
+  m.def("linear32", &linear32);
+  bind_mixers(m);
 }

@@ -8,6 +8,8 @@
 // take key channels in turn.
 #include "gla.h"
 
+#include <type_traits>
+
 namespace {
 
 constexpr int BLOCK = 256;
@@ -37,7 +39,8 @@ DEV_INLINE void st_state(float* p, const float* f) {
   }
 }
 
-template <class T, int VEC>
+// CONST: constant decays
+template <class T, int VEC, bool CONST>
 __global__ __launch_bounds__(BLOCK)
 void gla_recurrent_kernel(Gla<T> a, int lpr) {
   extern __shared__ float smem[];
@@ -59,6 +62,12 @@ void gla_recurrent_kernel(Gla<T> a, int lpr) {
     const bool fresh = state == nullptr || a.positions[row] == 0;
     for (int d = tid; d < a.dim; d += BLOCK) {
       const int c = h * a.dim + d;
+      if constexpr (CONST) {
+        s_a[d] = a.decay[h];
+        s_q[d] = silu_as<T>(ld1(x + c));
+        s_k[d] = silu_as<T>(ld1(x + a.k_off + c));
+        continue;
+      }
       float z = a.a2b[c];
       for (int r = 0; r < a.rank; ++r)
         z += a.a2[(long)c * a.rank + r] * ld1(x + a.a_off + r);
@@ -71,7 +80,10 @@ void gla_recurrent_kernel(Gla<T> a, int lpr) {
       float v[VEC], o[VEC];
       ldv<VEC>(x + a.v_off + h * a.vdim + c0, v);
       #pragma unroll
-      for (int j = 0; j < VEC; ++j) o[j] = 0.f;
+      for (int j = 0; j < VEC; ++j) {
+        if constexpr (CONST) v[j] = silu_as<T>(v[j]);
+        o[j] = 0.f;
+      }
       for (int d0 = grp; d0 < a.dim; d0 += groups * UNROLL) {
         float s[UNROLL][VEC];
         #pragma unroll
@@ -107,8 +119,16 @@ void gla_recurrent_kernel(Gla<T> a, int lpr) {
     for (int c = tid; c < a.vdim; c += BLOCK) {
       float o = 0.f;
       for (int g = 0; g < groups; ++g) o += s_o[g * a.vdim + c];
+      if constexpr (CONST) {
+        st1(a.out + (row * a.heads + h) * a.vdim + c, o);
+        continue;
+      }
       s_o[c] = o;                     // column c of group 0: this thread's
       ss += o * o;
+    }
+    if constexpr (CONST) {
+      __syncthreads();
+      continue;
     }
     ss = block_sum<BLOCK / WAVE>(ss, scratch);
     const float inv = 1.f / sqrtf(ss / (float)a.vdim + a.eps);
@@ -133,10 +153,16 @@ void launch_gla_recurrent(const Gla<T>& a, int entries, hipStream_t stream) {
   while (lpr < BLOCK && (BLOCK / lpr) * a.vdim > 8192) lpr *= 2;
   const size_t lds = sizeof(float) * (3 * a.dim + (BLOCK / lpr) * a.vdim);
   const dim3 grid(entries, a.heads);
-  if (vec)
-    gla_recurrent_kernel<T, 4><<<grid, dim3(BLOCK), lds, stream>>>(a, lpr);
-  else
-    gla_recurrent_kernel<T, 1><<<grid, dim3(BLOCK), lds, stream>>>(a, lpr);
+  auto go = [&](auto v, auto constant) {
+    gla_recurrent_kernel<T, decltype(v)::value, decltype(constant)::value>
+        <<<grid, dim3(BLOCK), lds, stream>>>(a, lpr);
+  };
+  auto by_vec = [&](auto constant) {
+    if (vec) go(std::integral_constant<int, 4>{}, constant);
+    else go(std::integral_constant<int, 1>{}, constant);
+  };
+  if (a.decay != nullptr) by_vec(std::true_type{});
+  else by_vec(std::false_type{});
 }
 
 template void launch_gla_recurrent<float>(const Gla<float>&, int, hipStream_t);

@@ -31,6 +31,8 @@
 // the segments' initial states, and the second pass writes outputs.
 #include "gla.h"
 
+#include <type_traits>
+
 typedef __attribute__((ext_vector_type(8))) short short8;
 typedef __attribute__((ext_vector_type(4))) short short4v;
 typedef __attribute__((ext_vector_type(16))) float float16v;
@@ -48,6 +50,10 @@ constexpr int OUT_OF_RANGE = 0x7ffffff0;   // beyond any buffer's end
 // place of element i (of 16) so that a lane half reads 8 in a row
 DEV_INLINE int perm16(int i) {
   return (i & ~12) | (i & 4) << 1 | (i & 8) >> 1;
+}
+
+DEV_INLINE unsigned raw16(bf16_t x) {
+  return *reinterpret_cast<unsigned short*>(&x);
 }
 
 DEV_INLINE float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
@@ -94,14 +100,14 @@ struct Lds {
 };
 
 // OUT: write outputs and the final state; else leave the segment's own state
-// and decay in the workspace.
+// and decay in the workspace. CONST: constant decays (gla.h).
 //
 // Making q~, k~ and k^ is divided into tasks of 32 channels: one kind makes
 // q~, the other k~ and k^. Both begin with the channel block's decays, a
 // product of the rows' A1 h with A2 on the matrix cores whose accumulators
 // hold a channel per lane and the tokens in registers. A wave takes its tasks
 // with their rows loaded a chunk ahead.
-template <int DT, bool OUT>
+template <int DT, bool OUT, bool CONST>
 __global__ __launch_bounds__(MAXW * WAVE)
 void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
                       float* __restrict__ ws, float* __restrict__ ws_decay) {
@@ -145,7 +151,15 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
           ? init[d * a.vdim + col] : 0.f;
     }
   const float inv_vdim = 1.f / (float)a.vdim;
-  const float nweight = OUT && col_ok ? a.norm[col] : 0.f;
+  const float nweight = OUT && !CONST && col_ok ? a.norm[col] : 0.f;
+  // per token, base 2
+  const float ldecay = CONST ? fmaxf(log2f(a.decay[h]), -1e4f) : 0.f;
+  // a projected value as it enters the recurrence
+  auto value = [&](unsigned raw) {
+    const float f = __uint_as_float(raw << 16);
+    if constexpr (CONST) return silu_as<bf16_t>(f);
+    else return f;
+  };
   if (tid < 2) s.direct[tid] = 0;
   for (int d = tid; d < DP; d += blockDim.x) s.total[d] = 0.f;
   __syncthreads();
@@ -174,6 +188,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
                min(32 * tile + lo5, a.dim - 1), f);
   };
   auto load_a1 = [&](int c0, int r0, unsigned* f) {
+    if constexpr (CONST) return;
     const int off = ((c0 + lo5) * ld + a.a_off) * 2;
     #pragma unroll
     for (int j = 0; j < 8; ++j)
@@ -188,6 +203,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
   };
   // rows of A2 for channel block `tile`, zero outside rank and head
   auto load_a2 = [&](int tile, int r0, short8* wh, short8* wl) {
+    if constexpr (CONST) return;
     const int d = 32 * tile + lo5;
     const float* w2 = a.a2 + (long)(h * a.dim + min(d, a.dim - 1)) * a.rank;
     float w[8];
@@ -204,6 +220,12 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
   auto logs = [&](int c0, int tile, const unsigned* a1, short8 wh, short8 wl,
                   float* b) {
     const int d = 32 * tile + lo5;
+    if constexpr (CONST) {
+      const float by = d < a.dim ? ldecay : 0.f;
+      #pragma unroll
+      for (int r = 0; r < 16; ++r) b[r] = by * min(crow(r) + 1, len - c0);
+      return by * min(C, len - c0);
+    }
     float16v z = {};
     z = mma(pack8(a1), wh, z);
     z = mma(pack8(a1), wl, z);
@@ -264,7 +286,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
       const float scale = d < a.dim ? a.qscale : 0.f;
       #pragma unroll
       for (int r = 0; r < 16; ++r)
-        f[r] = __uint_as_float(rows[r] << 16) * scale * exp2_f(b[r]);
+        f[r] = value(rows[r]) * scale * exp2_f(b[r]);
       put_rows(s.q, tile, f);
       return;
     }
@@ -273,7 +295,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
     #pragma unroll
     for (int r = 0; r < 16; ++r)
       k[r] = (r & 3) + 8 * (r >> 2) < lim
-          ? __uint_as_float(rows[r] << 16) : 0.f;
+          ? value(rows[r]) : 0.f;
     #pragma unroll
     for (int r = 0; r < 16; ++r) f[r] = k[r] * exp2_f(end - b[r]);
     short8 kh, kl;
@@ -297,7 +319,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
 
   // the wave's first task comes loaded; its part of A2 stays for the segment
   const int vcol = h * a.vdim + min(col, a.vdim - 1);
-  unsigned task_rows[16], vraw[16], a1[8];
+  unsigned task_rows[16], vraw[16], a1[8] = {};
   short8 wh0 = {}, wl0 = {};
   if (wave < TASKS) {
     load_task(0, wave, task_rows);
@@ -319,6 +341,11 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
     }
     // V as the second operand of both products: token order as in the
     // accumulators
+    if constexpr (CONST) {
+      #pragma unroll
+      for (int r = 0; r < 16; ++r)
+        vraw[r] = __float_as_uint(value(vraw[r])) >> 16;
+    }
     const short8 vf[2] = {pack8(vraw), pack8(vraw + 8)};
     __syncthreads();
     const bool direct = OUT && s.direct[par] != 0;    // uniform
@@ -342,8 +369,8 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
         float acc = 0.f;
         if (ks <= qt && c0 + qt < len) {
           for (int d = 0; d < a.dim; ++d)
-            acc += bf2f(x[qt * ld + d]) * a.qscale *
-                   bf2f(x[ks * ld + a.k_off + d]) *
+            acc += value(raw16(x[qt * ld + d])) * a.qscale *
+                   value(raw16(x[ks * ld + a.k_off + d])) *
                    exp2_f(sb[qt][d] - sb[ks][d]);
         }
         s.score[ks][qt] = acc;
@@ -352,7 +379,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
     }
 
     unsigned graw[16];
-    if (OUT) load16(c0, a.g_off + vcol, graw);
+    if (OUT && !CONST) load16(c0, a.g_off + vcol, graw);
     if (c0 + C < len) {
       if (wave < TASKS) load_task(c0 + C, wave, task_rows);
       load_a1(c0 + C, 0, a1);
@@ -418,7 +445,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
       }
     }
 
-    if (OUT) {
+    if (OUT && !CONST) {
       // sum of squares of each token over the wave's 32 columns: halve the
       // set of tokens a lane holds at every exchange
       float q[16];
@@ -438,7 +465,7 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
       if ((lane & 16) == 0) s.ssq[wave][crow(lane & 15)] = q[0];
     }
     __syncthreads();
-    if (OUT) {
+    if constexpr (OUT && !CONST) {
       float ss[16];
       #pragma unroll
       for (int r = 0; r < 16; ++r) ss[r] = 0.f;
@@ -457,6 +484,8 @@ void gla_chunk_kernel(Gla<bf16_t> a, int nseg, int seg_len,
         o[r] *= __builtin_amdgcn_rsqf(ss[r] * inv_vdim + a.eps) * nweight *
                 g * __builtin_amdgcn_rcpf(1.f + exp2_f(-g * LOG2E));
       }
+    }
+    if constexpr (OUT) {
       const int off = col_ok
           ? ((c0 + 4 * hi) * out_ld + h * a.vdim + col) * 2 : OUT_OF_RANGE;
       #pragma unroll
@@ -509,7 +538,7 @@ void gla_scan_kernel(Gla<bf16_t> a, int nseg, int seg_len,
   }
 }
 
-template <int DT>
+template <int DT, bool CONST>
 void run(const Gla<bf16_t>& a, int entries, int max_len, int nseg, float* ws,
          float* ws_decay, hipStream_t stream) {
   const int waves = (a.vdim + 31) / 32;
@@ -517,12 +546,12 @@ void run(const Gla<bf16_t>& a, int entries, int max_len, int nseg, float* ws,
   seg_len = (seg_len + C - 1) / C * C;
   const dim3 grid(entries * nseg, a.heads), block(waves * WAVE);
   if (nseg > 1) {
-    gla_chunk_kernel<DT, false><<<grid, block, 0, stream>>>(
+    gla_chunk_kernel<DT, false, CONST><<<grid, block, 0, stream>>>(
         a, nseg, seg_len, ws, ws_decay);
     gla_scan_kernel<<<dim3((a.dim * a.vdim + 255) / 256, entries, a.heads),
                       dim3(256), 0, stream>>>(a, nseg, seg_len, ws, ws_decay);
   }
-  gla_chunk_kernel<DT, true><<<grid, block, 0, stream>>>(
+  gla_chunk_kernel<DT, true, CONST><<<grid, block, 0, stream>>>(
       a, nseg, seg_len, ws, ws_decay);
 }
 
@@ -542,8 +571,16 @@ int gla_chunk_segments(int entries, int heads, int max_len) {
 
 void launch_gla_chunk(const Gla<bf16_t>& a, int entries, int max_len, int nseg,
                       float* ws, float* ws_decay, hipStream_t stream) {
-  if (a.dim <= 32) run<1>(a, entries, max_len, nseg, ws, ws_decay, stream);
-  else if (a.dim <= 64) run<2>(a, entries, max_len, nseg, ws, ws_decay, stream);
-  else if (a.dim <= 128) run<4>(a, entries, max_len, nseg, ws, ws_decay, stream);
-  else run<8>(a, entries, max_len, nseg, ws, ws_decay, stream);
+  auto go = [&](auto dt) {
+    constexpr int DT = decltype(dt)::value;
+    if (a.decay != nullptr)
+      run<DT, true>(a, entries, max_len, nseg, ws, ws_decay, stream);
+    else
+      run<DT, false>(a, entries, max_len, nseg, ws, ws_decay, stream);
+  };
+  using std::integral_constant;
+  if (a.dim <= 32) go(integral_constant<int, 1>{});
+  else if (a.dim <= 64) go(integral_constant<int, 2>{});
+  else if (a.dim <= 128) go(integral_constant<int, 4>{});
+  else go(integral_constant<int, 8>{});
 }

@@ -15,6 +15,7 @@ enum class Act {
   GELU,      // exact gelu
   GATE,      // times sigmoid(gate[row][g][n])
   SIDE,      // gelu_tanh, times table[tokens[row]][n]
+  GLU,       // columns are gate and up in turn; y has half as many
 };
 
 template <class T, class Y>
@@ -38,6 +39,8 @@ struct GroupGemm {
   const T* table;          // row t at table + t * t_ld
   long t_ld;
   int vocab;
+  Glu glu;
+  float limit;             // of Glu::CLAMPED
   bool quads;              // set by launch_group_gemm: four columns at a time
 };
 
@@ -101,6 +104,19 @@ template <Act ACT, class Y>
 DEV_INLINE void store4(const GroupGemm<bf16_t, Y>& a, Tile t, int r, int n,
                        float4v acc) {
   if (r >= t.r1 || n >= a.n) return;
+  if constexpr (ACT == Act::GLU) {
+    Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n / 2;
+    const float v0 = glu_f(a.glu, acc[0], acc[1], a.limit);
+    const float v1 = glu_f(a.glu, acc[2], acc[3], a.limit);
+    if (a.quads) {
+      const float v[2] = {v0, v1};
+      stv<2>(y, v);
+    } else {
+      st1(y, v0);
+      if (n + 2 < a.n) st1(y + 1, v1);
+    }
+    return;
+  }
   Y* y = a.y + (long)r * a.y_ld + t.g * a.y_gs + n;
   if (a.quads) {
     float v[4] = {acc[0], acc[1], acc[2], acc[3]};
@@ -125,6 +141,7 @@ void by_act(Act act, F f) {
     case Act::GELU: f(std::integral_constant<Act, Act::GELU>{}); break;
     case Act::GATE: f(std::integral_constant<Act, Act::GATE>{}); break;
     case Act::SIDE: f(std::integral_constant<Act, Act::SIDE>{}); break;
+    case Act::GLU: f(std::integral_constant<Act, Act::GLU>{}); break;
   }
 }
 

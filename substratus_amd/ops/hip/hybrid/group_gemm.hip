@@ -165,7 +165,12 @@ void group_gemm_any_kernel(GroupGemm<T, Y> a) {
     #pragma unroll
     for (int j = 0; j < 2; ++j) {
       const int r = t.r0 + ty + 16 * i, n = n0 + tx + 16 * j;
-      if (r < t.r1 && n < a.n) {
+      if constexpr (ACT == Act::GLU) {
+        const float up = __shfl_xor(acc[i][j], 1, WAVE);
+        if (r < t.r1 && n < a.n && tx % 2 == 0)
+          st1(a.y + (long)r * a.y_ld + t.g * a.y_gs + n / 2,
+              glu_f(a.glu, acc[i][j], up, a.limit));
+      } else if (r < t.r1 && n < a.n) {
         group_act<ACT, false, 1>(a, r, t.g, n, &acc[i][j]);
         st1(a.y + (long)r * a.y_ld + t.g * a.y_gs + n, acc[i][j]);
       }
@@ -208,6 +213,9 @@ bool by_quads(const GroupGemm<T, Y>& a) {
   auto ok = [](const void* p, size_t item) {
     return reinterpret_cast<uintptr_t>(p) % (4 * item) == 0;
   };
+  if (a.act == Act::GLU)      // pairs
+    return a.n % 4 == 0 && a.y_ld % 2 == 0 && a.y_gs % 2 == 0 &&
+           reinterpret_cast<uintptr_t>(a.y) % (2 * sizeof(Y)) == 0;
   return a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0 &&
          ok(a.y, sizeof(Y)) && a.gate_ld % 4 == 0 && a.gate_gs % 4 == 0 &&
          ok(a.gate, sizeof(T)) && a.t_ld % 4 == 0 && ok(a.table, sizeof(T));

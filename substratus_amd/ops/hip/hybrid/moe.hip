@@ -3,6 +3,7 @@
 //   select   one wave per token: scores (sums of a product's shares of the
 //            inner dimension), softmax over all experts, the best groups
 //            of neighbours, the best experts of those; all in 32 bits.
+//            Or the softmax is over the chosen experts only.
 //   sort     one workgroup: token rows packed by expert, and every expert's
 //            rows cut into tiles for the grouped products. The order of an
 //            expert's rows is left to chance: no row's result depends on it,
@@ -32,7 +33,8 @@ template <int PL>
 __global__ __launch_bounds__(SW * WAVE)
 void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
                        const float* __restrict__ z, int splits, int rows,
-                       int experts, int top, int groups, int keep) {
+                       int experts, int top, int groups, int keep,
+                       const float* __restrict__ bias, bool over_chosen) {
   extern __shared__ float4 s_all[];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int pad = (experts + 3) / 4 * 4;
@@ -52,6 +54,7 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
       #pragma unroll 4
       for (int s = 1; s < splits; ++s)
         v[i] += z[((long)s * rows + row) * experts + e];
+      if (bias != nullptr) v[i] += bias[e];
     }
     if (e < pad) s_z[e] = v[i];
     mx = fmaxf(mx, v[i]);
@@ -95,14 +98,20 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
     }
     __syncthreads();
   }
+  int r[PL];
+  float chosen = 0.f;
   #pragma unroll
   for (int i = 0; i < PL; ++i) {
     const int e = lane + i * WAVE;
-    if (e >= experts) continue;
-    const int r = rank_of(s_z, experts, v[i], e);
-    if (r < top) {
-      ids[row * top + r] = e;
-      weights[row * top + r] = expf(v[i] - mx) / sum;
+    r[i] = e < experts ? rank_of(s_z, experts, v[i], e) : top;
+    if (r[i] < top) chosen += expf(v[i] - mx);
+  }
+  if (over_chosen) sum = wave_sum(chosen);
+  #pragma unroll
+  for (int i = 0; i < PL; ++i) {
+    if (r[i] < top) {
+      ids[row * top + r[i]] = lane + i * WAVE;
+      weights[row * top + r[i]] = expf(v[i] - mx) / sum;
     }
   }
 }
@@ -161,12 +170,14 @@ int moe_max_experts() { return SORT; }
 
 void launch_moe_select(int* ids, float* weights, const float* z, int splits,
                        int rows, int experts, int top, int groups, int keep,
+                       const float* bias, bool over_chosen,
                        hipStream_t stream) {
   auto go = [&](auto pl) {
     moe_select_kernel<decltype(pl)::value>
         <<<dim3((rows + SW - 1) / SW), dim3(SW * WAVE),
            SW * 2 * ((experts + 3) / 4 * 4) * sizeof(float), stream>>>(
-            ids, weights, z, splits, rows, experts, top, groups, keep);
+            ids, weights, z, splits, rows, experts, top, groups, keep, bias,
+            over_chosen);
   };
   if (experts <= WAVE) go(std::integral_constant<int, 1>{});
   else if (experts <= 4 * WAVE) go(std::integral_constant<int, 4>{});

@@ -36,6 +36,8 @@ template <int VEC>
 DEV_INLINE void stv(float* p, const float* f) {
   if constexpr (VEC == 4) {
     *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+  } else if constexpr (VEC == 2) {
+    *reinterpret_cast<float2*>(p) = make_float2(f[0], f[1]);
   } else {
     #pragma unroll
     for (int i = 0; i < VEC; ++i) p[i] = f[i];
@@ -47,6 +49,8 @@ DEV_INLINE void stv(bf16_t* p, const float* f) {
   if constexpr (VEC == 4) {
     *reinterpret_cast<uint2*>(p) =
         make_uint2(pack_bf16x2(f[0], f[1]), pack_bf16x2(f[2], f[3]));
+  } else if constexpr (VEC == 2) {
+    *reinterpret_cast<unsigned*>(p) = pack_bf16x2(f[0], f[1]);
   } else {
     #pragma unroll
     for (int i = 0; i < VEC; ++i) p[i] = f2bf(f[i]);
@@ -58,6 +62,28 @@ DEV_INLINE float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 // ln(sigmoid(z)) without overflow at either end
 DEV_INLINE float log_sigmoid_f(float z) {
   return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+}
+
+// Hidden values of a gated feed-forward.
+enum class Glu {
+  SILU,      // silu(g) u
+  RELU,      // max(g, 0) u
+  CLAMPED,   // g sigmoid(1.702 g) (u + 1), g up to limit, u within it
+};
+
+DEV_INLINE float glu_f(Glu kind, float g, float u, float limit) {
+  if (kind == Glu::RELU) return fmaxf(g, 0.f) * u;
+  float s = 1.f;
+  if (kind == Glu::CLAMPED) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit) + 1.f;
+    s = 1.702f;
+  }
+  return g * sigmoid_f(s * g) * u;
+}
+
+DEV_INLINE float softplus_f(float z) {
+  return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
 }
 
 // One request's place in the batch, for kernels over single tokens and over

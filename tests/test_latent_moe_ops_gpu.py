@@ -258,7 +258,8 @@ def test_expert_tiles(tile, k, n):
     ext = ops._ext()
     ext.moe_sort(at, src, start, tiles, ids.cuda(), tile)
     out = torch.full((total, n), 9.0, dtype=BF16, device="cuda")
-    ext.expert_linear(out, x.cuda(), w.cuda(), src, start, tiles, tile, True)
+    ext.expert_linear(out, x.cuda(), w.cuda(), src, start, tiles, tile, "gelu",
+                      0.0)
     want = torch.empty(total, n)
     for i in range(e):
         r = ids[:, 0] == i
