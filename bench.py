@@ -236,8 +236,8 @@ def bench_train(args) -> None:
     run_train_bench(args)
 
 
-# hybrid-layer model, the uniform model of equal width, depth and feed-forward,
-# and (batch, prompt length) points
+# hybrid-layer model, the model of equal width and depth closest to it, and
+# (batch, prompt length) points
 HYBRID_PAIRS = [
     ("kakovik-1b", "llama-1b", [(8, 512), (64, 512), (256, 512), (16, 3072)]),
     ("kakovik-7b", "llama2-7b", [(8, 512), (64, 512), (256, 512),
@@ -245,9 +245,14 @@ HYBRID_PAIRS = [
     ("guronex-1b", "llama-1b", [(8, 512), (64, 512), (256, 512), (16, 3072)]),
     ("guronex-7b", "llama2-7b", [(8, 512), (64, 512), (256, 512),
                                  (16, 3072)]),
+    ("vurazen-1b", "kakovik-1b", [(8, 512), (64, 512), (256, 512),
+                                  (16, 3072)]),
+    ("vurazen-7b", "kakovik-7b", [(8, 512), (64, 512), (256, 512),
+                                  (16, 3072)]),
 ]
 HYBRID_TINY = [("kakovik-tiny", "llama-tiny", [(2, 24)]),
-               ("guronex-tiny", "llama-tiny", [(2, 24)])]
+               ("guronex-tiny", "llama-tiny", [(2, 24)]),
+               ("vurazen-tiny", "kakovik-tiny", [(2, 24)])]
 
 
 def bench_hybrid(args) -> None:
@@ -258,7 +263,9 @@ def bench_hybrid(args) -> None:
     device = "cuda:0" if on_gpu else "cpu"
     pairs = HYBRID_PAIRS if on_gpu else HYBRID_TINY
     if args.model:
-        pairs = [p for p in HYBRID_PAIRS + HYBRID_TINY if args.model in p[:2]]
+        known = HYBRID_PAIRS + HYBRID_TINY
+        pairs = [p for p in known if args.model == p[0]] or \
+            [p for p in known if args.model == p[1]]
 
     def sync():
         if on_gpu:

@@ -27,9 +27,9 @@ def clear_router(codes, experts, top, gen):
     """Of many random routers, (rows, biases) with the clearest decisions."""
     best, best_gap = None, -1.0
     for _ in range(1500):
-        w = 2.0 * torch.randn(experts, CODE, generator=gen)
+        w = 0.8 * torch.randn(experts, CODE, generator=gen)
         # multiples of 1/64 that add up to zero also in bfloat16
-        w = (w * 16).round() / 16
+        w = (w * 64).round() / 64
         w[:, -1] -= w.sum(1)
         b = (0.4 * torch.randn(experts, generator=gen)).bfloat16().float()
         if top == experts:
@@ -40,7 +40,7 @@ def clear_router(codes, experts, top, gen):
         gap = float((z[:, top - 1] - z[:, top]).min())
         if gap > best_gap:
             best, best_gap = (w, b), gap
-    assert best_gap > 0.04, best_gap
+    assert best_gap > 0.03, best_gap
     return best
 
 
@@ -56,12 +56,12 @@ def lightning(heads, dim, vdim, decay):
             "mlp": None}
 
 
-def att(heads, kv_heads, dim, taps, size, keep, dims, base=100.0, cap=20.0,
+def att(heads, kv_heads, dim, taps, size, keep, dims, base=100.0, cap=8.0,
         scale=None):
     return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
             "conv": taps, "mask": {"size": size, "keep_first": keep},
             "rot": {"base": base, "dims": dims}, "softcap": cap,
-            "scale": scale or 1.5 * dim ** -0.5}
+            "scale": scale or 2.5 * dim ** -0.5}
 
 
 def delta(heads, kv_heads, dim, vdim, taps):
@@ -87,7 +87,7 @@ def moe(layer, experts, top, ff, limit, shared=None):
     return dict(layer, mlp=doc)
 
 
-def config(width, vocab, layers, loop=None, eps=1e-5, scale=1.0, cap=25.0):
+def config(width, vocab, layers, loop=None, eps=1e-5, scale=1.0, cap=9.0):
     doc = {"architecture": "Vurazen", "width": width, "vocab": vocab,
            "norm": {"eps": eps}, "embedding": {"scale": scale},
            "logit_softcap": cap, "layers": layers}

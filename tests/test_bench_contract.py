@@ -51,8 +51,10 @@ def test_bench_train_schema():
 
 
 @pytest.mark.timeout(300)
-@pytest.mark.parametrize("model", ["kakovik-tiny", "guronex-tiny"])
-def test_bench_hybrid_schema(model):
+@pytest.mark.parametrize("model,beside", [
+    ("kakovik-tiny", "llama-tiny"), ("guronex-tiny", "llama-tiny"),
+    ("vurazen-tiny", "kakovik-tiny")])
+def test_bench_hybrid_schema(model, beside):
     out = subprocess.run(
         [sys.executable, "bench.py", "--mode", "hybrid", "--steps", "2",
          "--warmup", "1", "--model", model],
@@ -63,7 +65,7 @@ def test_bench_hybrid_schema(model):
     assert REQUIRED <= set(r)
     assert r["metric"] == "hybrid_decode_tokens_per_s"
     models = {p["model"] for p in r["config"]["points"]}
-    assert models == {model, "llama-tiny"}
+    assert models == {model, beside}
     for p in r["config"]["points"]:
         assert p["prefill_tokens_per_s"] > 0 and p["decode_tokens_per_s"] > 0
 

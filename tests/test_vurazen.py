@@ -57,7 +57,7 @@ def test_config_is_read_from_the_folder(folder):
     cfg = get_config(folder("mixed")[0])
     assert cfg.family == "vurazen" and cfg.num_layers == 5
     assert (cfg.hidden_size, cfg.vocab_size) == (80, 101)
-    assert (cfg.embed_scale, cfg.logit_softcap) == (1.5, 25.0)
+    assert (cfg.embed_scale, cfg.logit_softcap) == (1.5, 9.0)
     assert cfg.loop == LoopSpec(1, 4, 2)
     assert [(i, t) for i, t in cfg.runs()] == \
         oracle.passes(models.CONFIGS["mixed"][0])
@@ -66,7 +66,7 @@ def test_config_is_read_from_the_folder(folder):
     assert (both.left_scale, both.right_scale) == (0.7, 1.2)
     assert (a.heads, a.kv_heads, a.dim, a.taps, a.window, a.keep) == \
         (4, 2, 24, 3, 24, 3)
-    assert (a.softcap, a.sink, a.rot) == (20.0, True,
+    assert (a.softcap, a.sink, a.rot) == (8.0, True,
                                           RotarySpec(100.0, 12, True))
     assert (d.heads, d.kv_heads, d.dim, d.vdim, d.taps, d.decay_rank,
             d.gate_rank) == (4, 2, 16, 24, 4, 8, 12)
