@@ -394,6 +394,191 @@ def bench_latent():
                2.0 * b * n * (first + n / 2) * h * (spec.row + rank))
 
 
+EXP = 256 * 16 * 2.4e9    # exponentials/s of the vector units
+FMA = 256 * 64 * 2.4e9    # 32-bit vector instructions/s, unpacked
+
+
+def bench_mixers():
+    """Kernels of models with recurrent mixers, windowed attention and gated
+    experts beside the like kernels of Kakovik and Guronex, at 7b sizes."""
+    from substratus_amd.models.layers import GluSpec, MoESpec, RotarySpec
+    from substratus_amd.ops import hybrid as hy
+    from substratus_amd.serve.batch import StepBatch
+    torch.manual_seed(0)
+    bf = dict(device="cuda", dtype=torch.bfloat16)
+    f32 = dict(device="cuda")
+
+    def batch_of(n, first, tokens):
+        need = (first + tokens + 15) // 16
+        return StepBatch.build(
+            [([1] * tokens, first, list(range(i * need, (i + 1) * need)), i,
+              []) for i in range(n)], 16, torch.device("cuda"))
+
+    w, h, d, inner, ns, rank = 4096, 32, 128, 8192, 16, 256
+    for rows in (64, 256, 16384):
+        it = 200 if rows < 1000 else 30
+        x, xf = torch.randn(rows, w, **bf), torch.randn(rows, w, **f32)
+        w32 = torch.randn(w, **f32)
+        report(f"stream_norm rows={rows} w={w}",
+               timeit(lambda: hy.stream_norm(x, xf, w32, w32, 1.0, 1e-5), it),
+               rows * w * 12)
+        at = torch.randperm(rows * 8, device="cuda").int().view(rows, 8)
+        pk = hy.Picked(torch.randn(rows * 8, w, **bf), at,
+                       torch.rand(rows, 8, device="cuda"))
+        report(f"stream_norm of 8 picks rows={rows} w={w}",
+               timeit(lambda: hy.stream_norm(pk, xf, w32, None, 0.0, 1e-5),
+                      it), rows * w * 26)
+        report(f"  add_norm rows={rows} w={w}",
+               timeit(lambda: hy.add_norm(xf, w32, w32, 1e-5, x.dtype, x), it),
+               rows * w * 12)
+        report(f"  add_norm and 8 picks rows={rows} w={w}",
+               timeit(lambda: hy.add_norm(xf, w32, w32, 1e-5, x.dtype, x, pk),
+                      it), rows * w * 28)
+        del pk
+        buf = torch.randn(rows, 3 * h * d + 32, **bf)
+        kc = torch.zeros((rows + 15) // 16, h, 16, d, **bf)
+        vc, vf = torch.zeros_like(kc), torch.randn(rows, h * d, **bf)
+        pos = torch.arange(rows, device="cuda", dtype=torch.int32)
+        wn, lam = torch.ones(h * d, **f32), torch.tensor(0.5, device="cuda")
+        report(f"qkv_prepare rows={rows} {h}x{d}",
+               timeit(lambda: hy.qkv_prepare(buf, h * d, wn, wn, 1e-5, vf, lam,
+                                             kc, vc, pos), it),
+               rows * h * d * 2 * 7)
+        sb = batch_of(rows, 20, 1) if rows < 1000 else batch_of(8, 0, 2048)
+        n = sb.state_slots.numel()
+        kc = torch.zeros(rows * 2 if rows < 1000 else rows // 16, h, 16, d,
+                         **bf)
+        vc = torch.zeros_like(kc)
+        cs = torch.zeros(n, 3, 2 * h * d, **bf)
+        cw, cb = torch.randn(2 * h * d, 4, **f32), torch.randn(2 * h * d,
+                                                               **f32)
+        rot = RotarySpec(1e4, d, True)
+        turns = rot.turns("cuda")
+        rope = hy.rope_table(sb, rot, turns, {})
+        taps = n * 3 * 2 * h * d * 4
+        report(f"  conv_rope rows={rows} {h}x{d} 4 taps",
+               timeit(lambda: hy.conv_rope(buf, cb, cw, cs, rope, kc, vc, sb),
+                      it), rows * h * d * 2 * 5 + taps + rows * d * 4)
+        for ch in (3 * h * d, inner):
+            cs = torch.zeros(n, 3, ch, **bf)
+            cw, x2 = torch.randn(ch, 4, **f32), torch.randn(rows, ch, **bf)
+            report(f"  short_conv rows={rows} {ch} 4 taps",
+                   timeit(lambda: hy.short_conv(x2, cw, None, True, cs, sb),
+                          it), rows * ch * 4 + n * 3 * ch * 4)
+        up = torch.randn(rows, 2 * 11008, **bf)
+        report(f"silu_mul rows={rows} 11008",
+               timeit(lambda: hy.silu_mul(up), it), rows * 11008 * 6)
+        out = torch.empty(rows, 11008, **bf)
+        report(f"  glu relu rows={rows} 11008",
+               timeit(lambda: hy.glu(up, GluSpec("relu"), out), it),
+               rows * 11008 * 6)
+        o, nw = torch.randn(rows, h * d, **bf), torch.ones(h * d, **f32)
+        report(f"  joint_gate rows={rows} {h * d}",
+               timeit(lambda: hy.joint_gate(o, nw, up[:, :h * d], 1e-5, x),
+                      it), rows * h * d * 6)
+        for k, n2 in ((rank, inner), (d, h * d)):
+            low, wl = torch.randn(rows, k, **bf), torch.randn(n2, k, **bf)
+            report(f"  linear32 rows={rows} {k}->{n2}",
+                   timeit(lambda: hy.linear32(low, wl), it),
+                   (rows * k + n2 * k) * 2 + rows * n2 * 4,
+                   2.0 * rows * k * n2)
+        for name, moe, f in (
+                ("gelu 8 of 32 x 2048", MoESpec(32, 8, 2048, 8, 4), 1),
+                ("gated 8 of 32 x 1024", MoESpec(
+                    32, 8, 1024, glu=GluSpec("clamped", 7.0),
+                    over_chosen=True), 2)):
+            wu = torch.randn(32, f * moe.ff, w, **bf) * 0.02
+            wd = torch.randn(32, w, moe.ff, **bf) * 0.02
+            router = torch.randn(32, w, **bf) * 0.02
+            report(f"{'  ' if f == 2 else ''}experts rows={rows} {name}",
+                   timeit(lambda: hy.experts(x, router, wu, wd, moe), it),
+                   (wu.numel() + wd.numel() + rows * 8 * (w + 2 * moe.ff)) * 2,
+                   2.0 * rows * 8 * moe.ff * w * (f + 1))
+            del wu, wd
+        del buf, kc, vc, up
+
+    sink = torch.zeros(h, **f32)
+    bias = torch.randn(h, 4096, **f32)
+    for b, ctx in ((8, 512), (64, 512), (256, 512), (64, 2048)):
+        nb = b * ctx // 16
+        kc = torch.randn(nb, h, 16, d, **bf)
+        vc, q = torch.randn_like(kc), torch.randn(b, h * d, **bf)
+        sb, gate = batch_of(b, ctx - 1, 1), torch.randn(b, h, **bf)
+        report(f"attn_ctx single b={b} ctx={ctx} chunk",
+               timeit(lambda: hy.attn_ctx(q, gate, kc, vc, bias, sb,
+                                          d ** -0.5, 4096), 100),
+               4 * b * ctx * h * d)
+        report(f"  attn_ctx single b={b} ctx={ctx} window 1024, cap, sink",
+               timeit(lambda: hy.attn_ctx(
+                   q, None, kc, vc, None, sb, d ** -0.5, window=1024, keep=4,
+                   softcap=30.0, sink=sink), 100),
+               4 * b * min(ctx, 1028) * h * d)
+        del kc, vc
+    for b, s_ in ((32, 512), (8, 2048), (4, 4096)):
+        t = b * s_
+        q, kc = torch.randn(t, h * d, **bf), torch.randn(t // 16, h, 16, d,
+                                                         **bf)
+        vc, sb = torch.randn_like(kc), batch_of(b, 0, s_)
+        gate, k = torch.randn(t, h, **bf), min(s_, 1024)
+        report(f"attn_ctx portions b={b} s={s_} chunk",
+               timeit(lambda: hy.attn_ctx(q, gate, kc, vc, bias, sb,
+                                          d ** -0.5, 4096), 20),
+               8 * t * h * d, 4.0 * b * h * (s_ * (s_ + 1) / 2) * d)
+        report(f"  attn_ctx portions b={b} s={s_} window 1024, cap, sink",
+               timeit(lambda: hy.attn_ctx(
+                   q, None, kc, vc, None, sb, d ** -0.5, window=1024, keep=4,
+                   softcap=30.0, sink=sink), 20), 8 * t * h * d,
+               4.0 * b * h * d * (k * (k + 1) / 2 + (s_ - k) * (k + 4)))
+        del q, kc, vc
+
+    gh, gv = 16, 256
+    a2, ab = torch.randn(gh * d, 16, **f32) * 0.25, torch.randn(gh * d, **f32)
+    nw, nv = torch.ones(gv, **f32), torch.ones(d, **f32)
+    decay = torch.full((h,), 0.99, **f32)
+    rate, zb = torch.full((h,), 0.5, **f32), torch.full((h * d,), -4.0, **f32)
+    la, ld_ = -torch.rand(inner, ns, **f32) * 8, torch.ones(inner, **f32)
+    zs = torch.full((inner,), -4.0, **f32)
+    for b, s_ in ((8, 1), (64, 1), (256, 1), (32, 512), (8, 2048), (1, 8192)):
+        t, it = b * s_, 100 if s_ == 1 else 20
+        sb = batch_of(b, 100 if s_ == 1 else 0, s_)
+        what = f"single b={b}" if s_ == 1 else f"portions b={b} s={s_}"
+        c = 32.0 if s_ > 1 else 0.0
+        # state products and, within chunks of 32, score products
+        state, x = torch.zeros(b, gh, d, gv, **f32), torch.randn(
+            t, 2 * gh * (d + gv) + 16, **bf)
+        held = state.numel() * 8
+        report(f"gla {what} {gh}x{d}x{gv}",
+               timeit(lambda: hy.gla(x, a2, ab, nw, state, sb, 16.0, 1e-5),
+                      it), held + x.numel() * 2 + t * gh * gv * 2,
+               t * gh * (4.0 * d * gv + c * (d + gv)) if s_ > 1 else 0)
+        state, x = torch.zeros(b, h, d, d, **f32), torch.randn(
+            t, 4 * h * d, **bf)
+        report(f"  lightning {what} {h}x{d}x{d}",
+               timeit(lambda: hy.lightning(x, decay, state, sb), it),
+               held + t * h * d * 8,
+               t * h * (4.0 * d * d + c * 2 * d) if s_ > 1 else 0)
+        x = torch.randn(t, 3 * h * d, **bf)
+        z, beta = torch.randn(t, h * d, **f32), torch.randn(t, h, **bf)
+        gate, out = torch.randn(t, h * d, **bf), torch.empty(t, h * d, **bf)
+        report(f"  delta {what} {h}x{d}x{d}",
+               timeit(lambda: hy.delta(x, z, zb, rate, beta, nv, gate, state,
+                                       sb, h, 1e-5, 1.0, out), it),
+               held + t * h * d * 14,
+               t * h * (6.0 * d * d + c * 4 * d) if s_ > 1 else 0)
+        state = torch.zeros(b, inner, ns, **f32)
+        u, g = torch.randn(t, inner, **bf), torch.randn(t, 2 * inner, **bf)
+        z, o = torch.randn(t, inner, **f32), torch.empty(t, inner, **bf)
+        low = torch.randn(t, rank + 2 * ns, **bf)
+        # one exponential and four other instructions per state and token
+        steps = t * inner * ns
+        report(f"  selective_scan {what} {inner}x{ns}",
+               timeit(lambda: hy.selective_scan(
+                   u, g[:, inner:], z, zs, low, rank, la, ld_, state, sb, o),
+                   it),
+               max(state.numel() * 8 + t * inner * 10,
+                   HBM * steps * (1 / EXP + 4 / FMA)))
+
+
 def bench_sample(B=64, V=32000):
     logits = torch.randn(B, V, device="cuda").bfloat16()
     temp = torch.zeros(B, device="cuda")
@@ -627,6 +812,8 @@ if __name__ == "__main__":
         bench_hybrid()
     if a.which == "latent":
         bench_latent()
+    if a.which == "mixers":
+        bench_mixers()
     if a.which in ("all", "norm"):
         bench_norm()
     if a.which in ("all", "sample"):

@@ -9,6 +9,8 @@
 #include "scan.h"
 #include "short_conv.h"
 
+#include <algorithm>
+
 namespace {
 
 // Number of entries, with state slots, positions and seq_start checked.
@@ -261,6 +263,9 @@ void selective_scan(Tensor out, Tensor u, Tensor gate, Tensor z, Tensor zb,
   post("selective_scan");
 }
 
+constexpr int DELTA_CHUNK_FROM = 8;             // tokens of a portion
+constexpr long DELTA_WORKSPACE = 2l << 30;      // bytes
+
 void delta(Tensor out, Tensor qkv, Tensor z, Tensor zb, Tensor rate,
            Tensor beta, Tensor norm, Tensor gate, Tensor state,
            Tensor state_slots, Tensor positions, OptTensor seq_start,
@@ -295,6 +300,21 @@ void delta(Tensor out, Tensor qkv, Tensor z, Tensor zb, Tensor rate,
     a.g_ld = gate.stride(0);
     a.heads = heads; a.kv_heads = kv_heads; a.dim = dim; a.vdim = vdim;
     a.eps = eps; a.mult = mult;
+    if constexpr (std::is_same_v<T, bf16_t>) {
+      if (seq_start && !recurrent && max_len >= DELTA_CHUNK_FROM &&
+          delta_chunk_supported(a)) {
+        TORCH_CHECK(entries <= 65535, "too many portions");
+        const long bytes = delta_chunk_bytes(dim, rows, entries);
+        const int some = std::clamp<long>(DELTA_WORKSPACE / bytes, 1, heads);
+        Tensor ws = torch::empty({some * bytes},
+                                 state.options().dtype(torch::kUInt8));
+        for (int h0 = 0; h0 < heads; h0 += some)
+          launch_delta_chunk(a, entries, max_len, h0,
+                             std::min(some, heads - h0), ws.data_ptr(),
+                             stream());
+        return;
+      }
+    }
     launch_delta_recurrent<T>(a, entries, stream());
   });
   post("delta");

@@ -35,3 +35,10 @@ constexpr float UNIT_EPS = 1e-6f;    // under the root of a unit vector's length
 
 template <class T>
 void launch_delta_recurrent(const Delta<T>&, int entries, hipStream_t);
+
+// Portions by chunks of tokens: heads h0 .. h0 + heads - 1, with a workspace
+// of delta_chunk_bytes per head.
+bool delta_chunk_supported(const Delta<bf16_t>&);
+long delta_chunk_bytes(int dim, long rows, int entries);
+void launch_delta_chunk(const Delta<bf16_t>&, int entries, int max_len, int h0,
+                        int heads, void* ws, hipStream_t);
