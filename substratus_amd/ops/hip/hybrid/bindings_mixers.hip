@@ -302,7 +302,7 @@ void delta(Tensor out, Tensor qkv, Tensor z, Tensor zb, Tensor rate,
     a.eps = eps; a.mult = mult;
     if constexpr (std::is_same_v<T, bf16_t>) {
       if (seq_start && !recurrent && max_len >= DELTA_CHUNK_FROM &&
-          delta_chunk_supported(a)) {
+          delta_chunk_supported(a, max_len)) {
         TORCH_CHECK(entries <= 65535, "too many portions");
         const long bytes = delta_chunk_bytes(dim, rows, entries);
         const int some = std::clamp<long>(DELTA_WORKSPACE / bytes, 1, heads);

@@ -14,6 +14,8 @@ namespace {
 constexpr int C = 32;               // tokens per chunk
 constexpr float DIRECT_BELOW = -86.f;      // in powers of two: e^-60
 constexpr float LOG2E = 1.44269504088896340736f;
+constexpr int BUFFER_FLAGS = 0x00020000;   // untyped, offset-checked
+constexpr int OUT_OF_RANGE = 0x7ffffff0;   // beyond any buffer's end
 
 DEV_INLINE float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 

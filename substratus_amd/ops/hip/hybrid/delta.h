@@ -38,7 +38,7 @@ void launch_delta_recurrent(const Delta<T>&, int entries, hipStream_t);
 
 // Portions by chunks of tokens: heads h0 .. h0 + heads - 1, with a workspace
 // of delta_chunk_bytes per head.
-bool delta_chunk_supported(const Delta<bf16_t>&);
+bool delta_chunk_supported(const Delta<bf16_t>&, int max_len);
 long delta_chunk_bytes(int dim, long rows, int entries);
 void launch_delta_chunk(const Delta<bf16_t>&, int entries, int max_len, int h0,
                         int heads, void* ws, hipStream_t);

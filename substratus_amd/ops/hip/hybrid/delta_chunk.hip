@@ -14,10 +14,10 @@
 //
 // Only products with S have to wait for the chunk before. So a first kernel
 // makes q~, k~, k^, P and T of all chunks side by side, and leaves them as
-// matrix-core operands: what a wave loads is what it multiplies, no LDS, no
-// barrier. The second kernel walks a portion's chunks with a workgroup per
-// (portion, head), a wave per 32 value columns, its columns of S in
-// accumulators.
+// matrix-core operands. The second kernel walks a portion's chunks with a
+// workgroup per (portion, head), a wave per 32 value columns, its columns of S
+// in accumulators; the next chunk's operands are in flight meanwhile, and go
+// through LDS as they are.
 //
 // Factors are split into bf16 high and low parts (2^-16 relative), V is bf16
 // already. Contraction indices run in the order in which accumulators hold
@@ -29,6 +29,8 @@
 // positive.
 #include "chunk.h"
 #include "delta.h"
+
+#include <algorithm>
 
 namespace {
 
@@ -258,22 +260,25 @@ DEV_INLINE void lds_barrier() {
   asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
 }
 
-template <int N>
-DEV_INLINE void load_operands(const short* p, int lane, short8* f) {
-  #pragma unroll
-  for (int i = 0; i < N; ++i)
-    f[i] = *reinterpret_cast<const short8*>(p + (i * WAVE + lane) * 8);
+DEV_INLINE short8 operand(const short* p, int lane) {
+  return *reinterpret_cast<const short8*>(p + 8 * lane);
 }
 
-template <int DT, int MAXW>
-__global__ __launch_bounds__(MAXW * WAVE)
+// NW waves; those past the value columns only help to load.
+template <int DT, int NW>
+__global__ __launch_bounds__(NW * WAVE, 2)
 void delta_chunk_kernel(Delta<bf16_t> a, int h0,
                         const Operands<DT>* __restrict__ ws) {
-  __shared__ float ssq[2][MAXW][C];
+  constexpr int THREADS = NW * WAVE, PIECES = sizeof(Operands<DT>) / 16;
+  constexpr int MINE = (PIECES + THREADS - 1) / THREADS;
+  __shared__ struct {
+    alignas(16) Operands<DT> in;
+    float ssq[NW][C];
+  } s;
   const int e = blockIdx.x, h = h0 + blockIdx.y;
   const Entry en = entry_of(a.seq_start, e);
   if (en.n <= 0) return;
-  const int nw = blockDim.x / WAVE, tid = threadIdx.x;
+  const int tid = threadIdx.x;
   const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int lane = tid % WAVE, lo5 = lane & 31, hi = lane >> 5;
   const int col = wave * 32 + lo5;
@@ -295,96 +300,121 @@ void delta_chunk_kernel(Delta<bf16_t> a, int h0,
     }
   const float nweight = col_ok ? a.norm[col] * a.mult : 0.f;
   const float inv_vdim = 1.f / (float)a.vdim;
-  const bf16_t* v = a.qkv + 2 * a.kv_heads * a.dim + vcol;
+  // The portion's rows as bounded buffers: rows past its end read as zero and
+  // are not written.
+  auto buffer = [&](const bf16_t* p, long ld) {
+    return __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<bf16_t*>(p) + en.row0 * ld, 0, (int)(en.n * ld * 2),
+        BUFFER_FLAGS);
+  };
+  const auto v_in = buffer(a.qkv, a.ld), g_in = buffer(a.gate, a.g_ld);
+  const auto out = buffer(a.out, a.out_ld);
+  const int v_at = 2 * a.kv_heads * a.dim + vcol;
+  auto load16 = [&](auto from, int ld, int at, int c0, unsigned* f) {
+    const int off = ((c0 + 4 * hi) * ld + at) * 2;
+    #pragma unroll
+    for (int r = 0; r < 16; ++r)
+      f[r] = __builtin_amdgcn_raw_buffer_load_b16(
+          from, off + ((r & 3) + 8 * (r >> 2)) * ld * 2, 0, 0);
+  };
 
   const Operands<DT>* w = ws + chunk_at(en.row0, e, 0) * gridDim.y +
                           blockIdx.y;
-  short8 kf[4 * DT], qf[4 * DT];
-  load_operands<4 * DT>(&w->k[0][0][0][0], lane, kf);
-  load_operands<4 * DT>(&w->q[0][0][0][0], lane, qf);
-  float vv[16];
-  auto load_v = [&](int c0) {
+  short8 next[MINE];
+  unsigned vn[16];
+  auto load = [&](int c0) {
+    const auto from = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<Operands<DT>*>(w), 0, sizeof(Operands<DT>), BUFFER_FLAGS);
     #pragma unroll
-    for (int r = 0; r < 16; ++r)
-      vv[r] = ld1(v + (en.row0 + min(c0 + crow(r), en.n - 1)) * a.ld);
+    for (int i = 0; i < MINE; ++i)
+      next[i] = __builtin_bit_cast(
+          short8, __builtin_amdgcn_raw_buffer_load_b128(
+              from, tid * 16, i * THREADS * 16, 0));
+    load16(v_in, a.ld, v_at, c0, vn);
+    w += gridDim.y;
   };
-  load_v(0);
+  auto to_lds = [&]() {
+    short8* to = reinterpret_cast<short8*>(&s.in);
+    #pragma unroll
+    for (int i = 0; i < MINE; ++i)
+      if (tid + i * THREADS < PIECES) to[tid + i * THREADS] = next[i];
+  };
+  load(0);
+  to_lds();
+  lds_barrier();
 
   for (int c0 = 0; c0 < en.n; c0 += C) {
-    short8 tf[4], pf[4], ktf[4 * DT];
-    load_operands<4>(&w->t[0][0][0][0], lane, tf);
-    load_operands<4>(&w->p[0][0][0][0], lane, pf);
-    load_operands<4 * DT>(&w->kt[0][0][0][0], lane, ktf);
-    float g[16], end[DT][16];
+    float16v ks, o = {};            // k~ S - V
     #pragma unroll
-    for (int r = 0; r < 16; ++r)
-      g[r] = ld1(a.gate + (en.row0 + min(c0 + crow(r), en.n - 1)) * a.g_ld +
-                 vcol);
-    #pragma unroll
-    for (int i = 0; i < DT; ++i)
-      #pragma unroll
-      for (int r = 0; r < 16; r += 4)
-        ldv<4>(&w->end[32 * i + crow(r)], &end[i][r]);
+    for (int r = 0; r < 16; ++r) ks[r] = -__uint_as_float(vn[r] << 16);
+    if (c0 + C < en.n) load(c0 + C);
 
-    float16v ks = {}, o = {};
     #pragma unroll
     for (int i = 0; i < DT; ++i) {
       #pragma unroll
       for (int y = 0; y < 2; ++y) {
-        const int at = 2 * (2 * i + y);
+        const int it = 2 * i + y;
         short8 sh, sl;
         if (y == 0) split_rows<0>(st[i], &sh, &sl);
         else split_rows<8>(st[i], &sh, &sl);
-        ks = mma(kf[at], sh, ks);
-        o = mma(qf[at], sh, o);
-        ks = mma(kf[at], sl, ks);
-        o = mma(qf[at], sl, o);
-        ks = mma(kf[at + 1], sh, ks);
-        o = mma(qf[at + 1], sh, o);
+        const short8 kh = operand(s.in.k[it][0][0], lane);
+        const short8 qh = operand(s.in.q[it][0][0], lane);
+        ks = mma(kh, sh, ks);
+        o = mma(qh, sh, o);
+        ks = mma(kh, sl, ks);
+        o = mma(qh, sl, o);
+        ks = mma(operand(s.in.k[it][1][0], lane), sh, ks);
+        o = mma(operand(s.in.q[it][1][0], lane), sh, o);
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
     #pragma unroll
-    for (int r = 0; r < 16; ++r) ks[r] = vv[r] - ks[r];
-    w += gridDim.y;
-    if (c0 + C < en.n) {
-      load_operands<4 * DT>(&w->k[0][0][0][0], lane, kf);
-      load_operands<4 * DT>(&w->q[0][0][0][0], lane, qf);
-      load_v(c0 + C);
-    }
+    for (int r = 0; r < 16; ++r) ks[r] = -ks[r];
+    __builtin_amdgcn_sched_barrier(0);
     float16v u = {};
     #pragma unroll
     for (int y = 0; y < 2; ++y) {
       short8 rh, rl;
       if (y == 0) split_rows<0>(ks, &rh, &rl);
       else split_rows<8>(ks, &rh, &rl);
-      u = mma(tf[2 * y], rh, u);
-      u = mma(tf[2 * y], rl, u);
-      u = mma(tf[2 * y + 1], rh, u);
+      const short8 th = operand(s.in.t[y][0][0], lane);
+      u = mma(th, rh, u);
+      u = mma(th, rl, u);
+      u = mma(operand(s.in.t[y][1][0], lane), rh, u);
     }
     short8 uh[2], ul[2];
     split_rows<0>(u, &uh[0], &ul[0]);
     split_rows<8>(u, &uh[1], &ul[1]);
     #pragma unroll
-    for (int i = 0; i < DT; ++i)
-      #pragma unroll
-      for (int r = 0; r < 16; ++r) st[i][r] *= end[i][r];
-    #pragma unroll
     for (int y = 0; y < 2; ++y) {
-      o = mma(pf[2 * y], uh[y], o);
-      o = mma(pf[2 * y], ul[y], o);
-      o = mma(pf[2 * y + 1], uh[y], o);
-      #pragma unroll
-      for (int i = 0; i < DT; ++i) {
-        const int at = 2 * (2 * i + y);
-        st[i] = mma(ktf[at], uh[y], st[i]);
-        st[i] = mma(ktf[at], ul[y], st[i]);
-        st[i] = mma(ktf[at + 1], uh[y], st[i]);
-      }
+      const short8 ph = operand(s.in.p[y][0][0], lane);
+      o = mma(ph, uh[y], o);
+      o = mma(ph, ul[y], o);
+      o = mma(operand(s.in.p[y][1][0], lane), uh[y], o);
     }
+    #pragma unroll
+    for (int i = 0; i < DT; ++i) {
+      #pragma unroll
+      for (int r = 0; r < 16; r += 4) {
+        float end[4];
+        ldv<4>(&s.in.end[32 * i + crow(r)], end);
+        #pragma unroll
+        for (int j = 0; j < 4; ++j) st[i][r + j] *= end[j];
+      }
+      #pragma unroll
+      for (int y = 0; y < 2; ++y) {
+        const short8 kh = operand(s.in.kt[2 * i + y][0][0], lane);
+        st[i] = mma(kh, uh[y], st[i]);
+        st[i] = mma(kh, ul[y], st[i]);
+        st[i] = mma(operand(s.in.kt[2 * i + y][1][0], lane), uh[y], st[i]);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    unsigned g[16];
+    load16(g_in, a.g_ld, vcol, c0, g);
 
     // sum of squares of each token over the wave's 32 columns: halve the set
     // of tokens a lane holds at every exchange
-    const int par = (c0 / C) & 1;
     float q[16];
     #pragma unroll
     for (int r = 0; r < 16; ++r) q[r] = col_ok ? o[r] * o[r] : 0.f;
@@ -398,31 +428,45 @@ void delta_chunk_kernel(Delta<bf16_t> a, int h0,
       }
     }
     q[0] += __shfl_xor(q[0], 16, WAVE);
-    if ((lane & 16) == 0) ssq[par][wave][crow(lane & 15)] = q[0];
-    lds_barrier();
-    // (written again two chunks on, past the next barrier)
+    if ((lane & 16) == 0) s.ssq[wave][crow(lane & 15)] = q[0];
+    lds_barrier();                  // the chunk's operands have been read
+    if (c0 + C < en.n) to_lds();
     float ss[16];
     #pragma unroll
     for (int r = 0; r < 16; ++r) ss[r] = 0.f;
-    for (int n = 0; n < nw; ++n)
+    #pragma unroll 1
+    for (int n = 0; n < NW; ++n)
       #pragma unroll
-      for (int r = 0; r < 16; ++r) ss[r] += ssq[par][n][crow(r)];
+      for (int r = 0; r < 16; r += 4) {
+        float f[4];
+        ldv<4>(&s.ssq[n][crow(r)], f);
+        #pragma unroll
+        for (int j = 0; j < 4; ++j) ss[r + j] += f[j];
+      }
+    lds_barrier();
+    const int off = ((c0 + 4 * hi) * (int)a.out_ld + vcol) * 2;
     #pragma unroll
     for (int r = 0; r < 16; ++r) {
-      const int t = c0 + crow(r);
-      if (t < en.n && col_ok)
-        st1(a.out + (en.row0 + t) * a.out_ld + vcol,
-            o[r] / sqrtf(ss[r] * inv_vdim + a.eps) * nweight *
-                sigmoid_f(g[r]));
+      const float f = o[r] * __builtin_amdgcn_rsqf(ss[r] * inv_vdim + a.eps) *
+          nweight * __builtin_amdgcn_rcpf(
+              1.f + exp2_f(-__uint_as_float(g[r] << 16) * LOG2E));
+      __builtin_amdgcn_raw_buffer_store_b16(
+          cvt_pk_bf16(f, f), out, col_ok
+              ? off + ((r & 3) + 8 * (r >> 2)) * (int)a.out_ld * 2
+              : OUT_OF_RANGE, 0, 0);
     }
   }
   if (state != nullptr && col_ok) {
+    // addresses are formed anew: those of the beginning would have to stay in
+    // registers all the while
+    int to = col, dim = a.dim;
+    asm volatile("" : "+v"(to), "+s"(dim));
     #pragma unroll
     for (int i = 0; i < DT; ++i)
       #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int d = 32 * i + crow(r);
-        if (d < a.dim) state[d * a.vdim + col] = st[i][r];
+        if (d < dim) state[d * a.vdim + to] = st[i][r];
       }
   }
 }
@@ -434,21 +478,22 @@ void run(const Delta<bf16_t>& a, int entries, int max_len, int h0, int heads,
   delta_prep_kernel<DT>
       <<<dim3((max_len + C - 1) / C, entries, heads), PREP, 0, stream>>>(
           a, h0, ops);
-  const int waves = (a.vdim + 31) / 32;
-  const dim3 grid(entries, heads), block(waves * WAVE);
-  if (waves <= 4)
-    delta_chunk_kernel<DT, 4><<<grid, block, 0, stream>>>(a, h0, ops);
+  const dim3 grid(entries, heads);
+  if (a.vdim <= 128)
+    delta_chunk_kernel<DT, 4><<<grid, 4 * WAVE, 0, stream>>>(a, h0, ops);
   else
-    delta_chunk_kernel<DT, 8><<<grid, block, 0, stream>>>(a, h0, ops);
+    delta_chunk_kernel<DT, 8><<<grid, 8 * WAVE, 0, stream>>>(a, h0, ops);
 }
 
 int tiles(int dim) { return dim <= 32 ? 1 : dim <= 64 ? 2 : 4; }
 
 }  // namespace
 
-bool delta_chunk_supported(const Delta<bf16_t>& a) {
+bool delta_chunk_supported(const Delta<bf16_t>& a, int max_len) {
+  // a portion's rows are addressed with 32-bit offsets
+  const long far = (max_len + C) * std::max({a.ld, a.out_ld, a.g_ld}) * 2;
   return a.dim <= 128 && a.dim % 4 == 0 && a.vdim <= 256 && a.ld % 4 == 0 &&
-         reinterpret_cast<uintptr_t>(a.qkv) % 8 == 0;
+         reinterpret_cast<uintptr_t>(a.qkv) % 8 == 0 && far < OUT_OF_RANGE;
 }
 
 long delta_chunk_bytes(int dim, long rows, int entries) {

@@ -38,8 +38,6 @@ namespace {
 
 constexpr int MAXW = 8;             // waves per workgroup
 constexpr int MAXRANK = 64;
-constexpr int BUFFER_FLAGS = 0x00020000;   // untyped, offset-checked
-constexpr int OUT_OF_RANGE = 0x7ffffff0;   // beyond any buffer's end
 
 // place of element i (of 16) so that a lane half reads 8 in a row
 DEV_INLINE int perm16(int i) {
