@@ -52,10 +52,18 @@ struct Operands {
 template <int DT>
 struct PrepLds {
   static constexpr int DP = 32 * DT;
-  alignas(16) float b[C][DP + 4];   // summed logs, base 2
-  alignas(16) float k[C][DP + 4];   // unit keys
-  alignas(16) float l[C][C + 4];    // beta A
-  float part[4][C][C + 1];          // A, P of the channels' halves; then T, P
+  struct Rows {
+    alignas(16) float b[C][DP + 4];   // summed logs, base 2
+    alignas(16) float k[C][DP + 4];   // unit keys
+  };
+  struct Scores {
+    alignas(16) float l[C][C + 4];    // beta A
+    float part[4][C][C + 1];          // A, P of the channels' halves; T, P
+  };
+  union {
+    Rows rows;
+    Scores scores;                    // once the rows are done with
+  };
   float iq[C], beta[C];
   int direct;
 };
@@ -74,12 +82,22 @@ DEV_INLINE void put_split(const float* f, short (*dst)[WAVE][8], int lane) {
   *reinterpret_cast<short8*>(dst[1][lane]) = l;
 }
 
+// log2(1 + e^z)
+DEV_INLINE float softplus2(float z) {
+  const float x = exp2_f(-fabsf(z) * LOG2E);
+  const float l = x < 0.01f ? x * (1.f - x * (0.5f - x * (1.f / 3.f))) * LOG2E
+                            : __builtin_amdgcn_logf(1.f + x);
+  return fmaxf(z, 0.f) * LOG2E + l;
+}
+
 template <int DT>
 __global__ __launch_bounds__(PREP)
 void delta_prep_kernel(Delta<bf16_t> a, int h0,
                        Operands<DT>* __restrict__ ws) {
   constexpr int DP = 32 * DT;
   __shared__ PrepLds<DT> s;
+  auto& b = s.rows.b;
+  auto& k = s.rows.k;
   const int c = blockIdx.x, e = blockIdx.y, h = h0 + blockIdx.z;
   const Entry en = entry_of(a.seq_start, e);
   if (c * C >= en.n) return;
@@ -91,7 +109,7 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
   const int nq = a.kv_heads * a.dim;
   const int head = h / (a.heads / a.kv_heads) * a.dim;
   const bf16_t* x = a.qkv + row0 * a.ld + head;
-  const float rate = -a.rate[h] * LOG2E;
+  const float rate = -a.rate[h];
 
   if (tid == 0) s.direct = 0;
   if (tid < C)
@@ -118,7 +136,7 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
     const float inv = 1.f / sqrtf(ss + UNIT_EPS);
     if (key) {
       #pragma unroll
-      for (int j = 0; j < PER; ++j) s.k[t][at + j] = f[j] * inv;
+      for (int j = 0; j < PER; ++j) k[t][at + j] = f[j] * inv;
     } else if (tid % 4 == 0) {
       s.iq[t] = inv / sqrtf((float)a.dim);
     }
@@ -137,15 +155,15 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
     #pragma unroll
     for (int j = 0; j < N; ++j) {
       if (grp * N + j < len && d < a.dim)
-        sum += fmaxf(rate * softplus_f(z[j] + zb), -160.f);  // 0 in float
+        sum += fmaxf(rate * softplus2(z[j] + zb), -160.f);   // 0 in float
       z[j] = sum;
     }
-    s.b[grp * N + N - 1][d] = sum;
+    b[grp * N + N - 1][d] = sum;
     __syncthreads();
-    for (int p = 0; p < grp; ++p) ahead += s.b[p * N + N - 1][d];
+    for (int p = 0; p < grp; ++p) ahead += b[p * N + N - 1][d];
     __syncthreads();
     #pragma unroll
-    for (int j = 0; j < N; ++j) s.b[grp * N + j][d] = z[j] + ahead;
+    for (int j = 0; j < N; ++j) b[grp * N + j][d] = z[j] + ahead;
     if (grp == PREP / DP - 1) {
       w->end[d] = exp2_f(sum + ahead);
       if (sum + ahead < DIRECT_BELOW) s.direct = 1;
@@ -157,39 +175,34 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
   // k^: a channel per lane
   for (int it = wave; it < 2 * DT; it += PREP / WAVE) {
     const int d = 32 * (it >> 1) + lo5;
-    const float end = s.b[C - 1][d];
+    const float end = b[C - 1][d];
     float f[8];
     #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int t = ctr(it & 1, hi, j);
-      f[j] = s.k[t][d] * exp2_f(end - s.b[t][d]);
+      f[j] = k[t][d] * exp2_f(end - b[t][d]);
     }
     put_split(f, w->kt[it], lane);
   }
   // q~ and P (odd waves) or k~ and A: a token per lane, every other 16
   // channels
+  float16v acc = {};
   {
     const bool odd = wave & 1;
-    float16v acc = {};
     for (int it = wave >> 1; it < 2 * DT; it += 2) {
-      float f[8], k[8], n[8];
+      float f[8], n[8];
       #pragma unroll
       for (int g = 0; g < 8; g += 4) {
         const int d = ctr(it, hi, g);
-        float b[4];
-        ldv<4>(&s.b[lo5][d], b);
-        ldv<4>(&s.k[lo5][d], k + g);
-        float own[4] = {k[g], k[g + 1], k[g + 2], k[g + 3]};
-        if (odd) {
-          own[0] = own[1] = own[2] = own[3] = 0.f;
-          if (lo5 < len && d < a.dim) ldv<4>(x + lo5 * a.ld + d, own);
-          #pragma unroll
-          for (int j = 0; j < 4; ++j) own[j] *= s.iq[lo5];
-        }
+        float sum[4], key[4], own[4] = {};
+        ldv<4>(&b[lo5][d], sum);
+        ldv<4>(&k[lo5][d], key);
+        if (odd && lo5 < len && d < a.dim) ldv<4>(x + lo5 * a.ld + d, own);
         #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          f[g + j] = own[j] * exp2_f(b[j]);
-          n[g + j] = direct ? 0.f : k[g + j] * exp2_f(-b[j]);
+          const float y = odd ? own[j] * s.iq[lo5] : key[j];
+          f[g + j] = y * exp2_f(sum[j]);
+          n[g + j] = direct ? 0.f : key[j] * exp2_f(-sum[j]);
         }
       }
       short8 fh, fl, nh, nl;
@@ -202,28 +215,42 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
       acc = mma(fh, nl, acc);
       acc = mma(fl, nh, acc);
     }
-    #pragma unroll
-    for (int r = 0; r < 16; ++r)
-      s.part[wave][(r & 3) + 8 * (r >> 2) + 4 * hi][lo5] = acc[r];
+  }
+  constexpr int PAIRS = C * C / PREP;   // scores per thread
+  float av[PAIRS], pv[PAIRS];
+  if (direct) {
+    #pragma unroll 1
+    for (int i = 0; i < PAIRS; ++i) {
+      const int t = (tid + i * PREP) / C, j = tid % C;
+      float sa = 0.f, sp = 0.f;
+      if (j <= t && t < len) {
+        for (int d = 0; d < a.dim; ++d) {
+          const float f = k[j][d] * exp2_f(b[t][d] - b[j][d]);
+          sa += f * k[t][d];
+          sp += f * ld1(x + t * a.ld + d);
+        }
+      }
+      #pragma unroll
+      for (int n = 0; n < PAIRS; ++n)
+        if (n == i) { av[n] = sa; pv[n] = sp * s.iq[t]; }
+    }
   }
   __syncthreads();
-  for (int i = tid; i < C * C; i += PREP) {
-    const int t = i / C, k = i % C;
-    float av = s.part[0][t][k] + s.part[2][t][k];
-    float pv = s.part[1][t][k] + s.part[3][t][k];
-    if (direct) {
-      av = pv = 0.f;
-      if (k <= t && t < len) {
-        for (int d = 0; d < a.dim; ++d) {
-          const float f = s.k[k][d] * exp2_f(s.b[t][d] - s.b[k][d]);
-          av += f * s.k[t][d];
-          pv += f * ld1(x + t * a.ld + d);
-        }
-        pv *= s.iq[t];
-      }
+  auto& part = s.scores.part;
+  auto& l = s.scores.l;
+  #pragma unroll
+  for (int r = 0; r < 16; ++r)
+    part[wave][(r & 3) + 8 * (r >> 2) + 4 * hi][lo5] = acc[r];
+  __syncthreads();
+  #pragma unroll
+  for (int i = 0; i < PAIRS; ++i) {
+    const int t = (tid + i * PREP) / C, j = tid % C;
+    if (!direct) {
+      av[i] = part[0][t][j] + part[2][t][j];
+      pv[i] = part[1][t][j] + part[3][t][j];
     }
-    s.l[t][k] = k < t ? s.beta[t] * av : 0.f;
-    s.part[1][t][k] = k <= t ? pv : 0.f;
+    l[t][j] = j < t ? s.beta[t] * av[i] : 0.f;
+    part[1][t][j] = j <= t ? pv[i] : 0.f;
   }
   __syncthreads();
   if (wave == 0) {
@@ -233,24 +260,24 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
     for (int t = 0; t < C; ++t) {
       float v = t == lo5 ? 1.f : 0.f;
       #pragma unroll
-      for (int k = 0; k < t; ++k) v -= s.l[t][k] * inv[k];
+      for (int j = 0; j < t; ++j) v -= l[t][j] * inv[j];
       inv[t] = v;
     }
     if (hi == 0) {
       #pragma unroll
-      for (int t = 0; t < C; ++t) s.part[0][t][lo5] = inv[t] * s.beta[lo5];
+      for (int t = 0; t < C; ++t) part[0][t][lo5] = inv[t] * s.beta[lo5];
     }
   } else if (wave < 3) {
     float f[8];
     #pragma unroll
-    for (int j = 0; j < 8; ++j) f[j] = s.part[1][lo5][ctr(wave - 1, hi, j)];
+    for (int j = 0; j < 8; ++j) f[j] = part[1][lo5][ctr(wave - 1, hi, j)];
     put_split(f, w->p[wave - 1], lane);
   }
   __syncthreads();
   if (wave < 2) {
     float f[8];
     #pragma unroll
-    for (int j = 0; j < 8; ++j) f[j] = s.part[0][lo5][ctr(wave, hi, j)];
+    for (int j = 0; j < 8; ++j) f[j] = part[0][lo5][ctr(wave, hi, j)];
     put_split(f, w->t[wave], lane);
   }
 }
@@ -368,9 +395,10 @@ void delta_chunk_kernel(Delta<bf16_t> a, int h0,
       }
       __builtin_amdgcn_sched_barrier(0);
     }
+    unsigned g[16];
+    load16(g_in, a.g_ld, vcol, c0, g);
     #pragma unroll
     for (int r = 0; r < 16; ++r) ks[r] = -ks[r];
-    __builtin_amdgcn_sched_barrier(0);
     float16v u = {};
     #pragma unroll
     for (int y = 0; y < 2; ++y) {
@@ -410,8 +438,6 @@ void delta_chunk_kernel(Delta<bf16_t> a, int h0,
       }
       __builtin_amdgcn_sched_barrier(0);
     }
-    unsigned g[16];
-    load16(g_in, a.g_ld, vcol, c0, g);
 
     // sum of squares of each token over the wave's 32 columns: halve the set
     // of tokens a lane holds at every exchange

@@ -41,11 +41,12 @@ DEV_INLINE void st_n(T* p, int n, const float* f) {
   }
 }
 
-// Channels c .. c + n - 1, tokens [t0, t0 + run) of entry e; emit(row, y).
+// Channels c .. c + n - 1, tokens [t0, t0 + run) of entry e;
+// emit(row, y, look(row)), where look reads memory ahead of emit's writes.
 // TAPS 0: any number, inputs are read again for every tap.
-template <int VEC, int TAPS, class T, class F>
+template <int VEC, int TAPS, class T, class L, class F>
 DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
-                         int run, F emit) {
+                         int run, L look, F emit) {
   const Entry en = entry_of(a.seq_start, e);
   if (t0 >= en.n) return;
   const int t1 = min(t0 + run, en.n);
@@ -89,6 +90,9 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
       float in[N][VEC];
       #pragma unroll
       for (int i = 0; i < N; ++i) input(t + i, in[i]);
+      decltype(look(0l)) seen[N];
+      #pragma unroll
+      for (int i = 0; i < N; ++i) seen[i] = look(en.row0 + t + i);
       #pragma unroll
       for (int i = 0; i < N; ++i) {
         float y[VEC];
@@ -101,7 +105,7 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
           #pragma unroll
           for (int k = 0; k + 1 < TAPS; ++k) u[k][j] = u[k + 1][j];
         }
-        emit(en.row0 + t + i, y);
+        emit(en.row0 + t + i, y, seen[i]);
       }
     };
     int t = t0;
@@ -118,7 +122,7 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
         for (int j = 0; j < VEC; ++j)
           if (j < n) y[j] += wp[j * taps + k] * f[j];
       }
-      emit(en.row0 + t, y);
+      emit(en.row0 + t, y, look(en.row0 + t));
     }
   }
   if (t0 == 0 && state != nullptr) {
@@ -146,7 +150,8 @@ void short_conv_kernel(Conv<T> a, int run) {
   for (int j = 0; j < VEC; ++j) b[j] = 0.f;
   if (a.bias != nullptr) ld_n<VEC>(a.bias + c, VEC, b);
   convolve<VEC, TAPS>(a, blockIdx.z, c, VEC, blockIdx.y * run, run,
-                      [&](long row, float* y) {
+                      [](long) { return 0; },
+                      [&](long row, float* y, int) {
     #pragma unroll
     for (int j = 0; j < VEC; ++j) {
       y[j] += b[j];
@@ -164,25 +169,40 @@ void conv_rope_kernel(Conv<T> a, int run) {
   if (i >= heads * per) return;
   const int head = i / per, d = i % per * VEC;
   const int n = min(VEC, a.dim - d), nq = heads - a.kv;
+  const bool key = head >= nq;
+  const int pair = d / 2;
+  struct Seen {
+    int page, at;                      // of the cache
+    float turn[VEC];                   // cosine and sine per pair
+  };
   convolve<VEC, TAPS>(a, blockIdx.z, head * a.dim + d, n, blockIdx.y * run,
-                      run, [&](long row, float* y) {
-    const bool key = head >= nq;
+                      run, [&](long row) {
+    Seen f{};
+    if (key) {
+      const unsigned slot = a.slots[row], size = a.block_size;
+      f.page = slot / size;
+      f.at = slot % size;
+    }
+    const float* cs = a.rope + (row * a.half + pair) * 2;
+    #pragma unroll
+    for (int j = 0; j < VEC; j += 2) {
+      const bool there = pair + j / 2 < a.half;
+      f.turn[j] = there ? cs[j] : 1.f;
+      f.turn[j + 1] = there ? cs[j + 1] : 0.f;
+    }
+    return f;
+  }, [&](long row, float* y, const Seen& f) {
     long at = 0;
     if (key) {
-      const int slot = a.slots[row];
-      at = (((long)(slot / a.block_size) * a.kv + head - nq) * a.block_size +
-            slot % a.block_size) * a.dim + d;
+      at = (((long)f.page * a.kv + head - nq) * a.block_size + f.at) * a.dim
+           + d;
       st_n<VEC>(a.vc + at, n, y);
     }
     #pragma unroll
     for (int j = 0; j + 1 < VEC; j += 2) {
-      const int pair = (d + j) / 2;
-      if (pair < a.half) {
-        const float* cs = a.rope + (row * a.half + pair) * 2;
-        const float c = cs[0], s = cs[1], u = y[j], v = y[j + 1];
-        y[j] = u * c - v * s;
-        y[j + 1] = v * c + u * s;
-      }
+      const float c = f.turn[j], s = f.turn[j + 1], u = y[j], v = y[j + 1];
+      y[j] = u * c - v * s;
+      y[j + 1] = v * c + u * s;
     }
     if (key) st_n<VEC>(a.kc + at, n, y);
     else st_n<VEC>(a.q + row * nq * a.dim + head * a.dim + d, n, y);
