@@ -108,8 +108,11 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
         emit(en.row0 + t + i, y, seen[i]);
       }
     };
+    // tokens at once: fewer if much is looked up for each
+    constexpr int AT_ONCE = sizeof(look(0l)) > 4 ? 4 : 8;
     int t = t0;
-    for (; t + 8 <= t1; t += 8) steps(t, std::integral_constant<int, 8>{});
+    for (; t + AT_ONCE <= t1; t += AT_ONCE)
+      steps(t, std::integral_constant<int, AT_ONCE>{});
     for (; t < t1; ++t) steps(t, std::integral_constant<int, 1>{});
   } else {
     for (int t = t0; t < t1; ++t) {
@@ -168,7 +171,8 @@ void conv_rope_kernel(Conv<T> a, int run) {
   const int i = blockIdx.x * BLOCK + threadIdx.x;
   if (i >= heads * per) return;
   const int head = i / per, d = i % per * VEC;
-  const int n = min(VEC, a.dim - d), nq = heads - a.kv;
+  // whole pieces of four: launched so
+  const int n = VEC == 4 ? 4 : min(VEC, a.dim - d), nq = heads - a.kv;
   const bool key = head >= nq;
   const int pair = d / 2;
   struct Seen {

@@ -123,9 +123,7 @@ def test_loops_that_cannot_be(tmp_path, loop):
 
 def test_every_pass_has_a_cache_of_its_own(folder):
     cfg = get_config(folder("mixed")[0])
-    kv = PagedKVCache(cfg, 3, 6, dtype=torch.bfloat16, num_slots=2) \
-        if "num_slots" in PagedKVCache.__init__.__code__.co_varnames \
-        else PagedKVCache(cfg, 3, 6, dtype=torch.bfloat16)
+    kv = PagedKVCache(cfg, 1, 6, dtype=torch.bfloat16, state_slots=2)
     assert len(kv.layers) == 8
     held = [t for c in kv.layers for t in c]
     assert len({t.data_ptr() for t in held if t.numel()}) == \
