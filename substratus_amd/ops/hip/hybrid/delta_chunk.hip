@@ -82,14 +82,6 @@ DEV_INLINE void put_split(const float* f, short (*dst)[WAVE][8], int lane) {
   *reinterpret_cast<short8*>(dst[1][lane]) = l;
 }
 
-// log2(1 + e^z)
-DEV_INLINE float softplus2(float z) {
-  const float x = exp2_f(-fabsf(z) * LOG2E);
-  const float l = x < 0.01f ? x * (1.f - x * (0.5f - x * (1.f / 3.f))) * LOG2E
-                            : __builtin_amdgcn_logf(1.f + x);
-  return fmaxf(z, 0.f) * LOG2E + l;
-}
-
 template <int DT>
 __global__ __launch_bounds__(PREP)
 void delta_prep_kernel(Delta<bf16_t> a, int h0,
@@ -155,7 +147,7 @@ void delta_prep_kernel(Delta<bf16_t> a, int h0,
     #pragma unroll
     for (int j = 0; j < N; ++j) {
       if (grp * N + j < len && d < a.dim)
-        sum += fmaxf(rate * softplus2(z[j] + zb), -160.f);   // 0 in float
+        sum += fmaxf(rate * softplus2_f(z[j] + zb), -160.f);   // 0 in float
       z[j] = sum;
     }
     b[grp * N + N - 1][d] = sum;

@@ -15,6 +15,7 @@ namespace {
 constexpr int BLOCK = 256;
 constexpr int TB = 4;              // tokens loaded at once
 constexpr float LOG2E = 1.44269504088896340736f;
+constexpr float LN2 = 0.69314718055994530942f;
 
 DEV_INLINE float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 
@@ -81,6 +82,19 @@ void scan_kernel(Scan<T> a, int lanes, int tt, int nseg, int seg_len,
   const float zb = a.zb[c], d = a.d[c];
   float total = 0.f;
 
+  // the next TB tokens' values, on their way while these are computed
+  T un[TB], gn[TB];
+  float zn[TB];
+  auto load = [&](int t) {
+    #pragma unroll
+    for (int j = 0; j < TB; ++j) {
+      const long r = row0 + min(t + j, len - 1);
+      un[j] = a.u[r * a.channels + c];
+      zn[j] = a.z[r * a.channels + c];
+      if (OUT) gn[j] = a.gate[r * a.g_ld + c];
+    }
+  };
+  load(0);
   for (int b0 = 0; b0 < len; b0 += tt) {
     const int nt = min(tt, len - b0);
     __syncthreads();
@@ -97,15 +111,17 @@ void scan_kernel(Scan<T> a, int lanes, int tt, int nseg, int seg_len,
       float u[TB], z[TB], g[TB];
       #pragma unroll
       for (int j = 0; j < TB; ++j) {
-        const long r = row0 + b0 + min(t1 + j, nt - 1);
-        u[j] = ld1(a.u + r * a.channels + c);
-        z[j] = a.z[r * a.channels + c];
-        if (OUT) g[j] = ld1(a.gate + r * a.g_ld + c);
+        u[j] = ld1(&un[j]);
+        z[j] = zn[j];
+        if (OUT) g[j] = ld1(&gn[j]);
       }
+      load(b0 + t1 + TB);
       #pragma unroll
       for (int j = 0; j < TB; ++j) {
         if (t1 + j >= nt) break;
-        const float dt = softplus_f(z[j] + zb), dtu = dt * u[j];
+        const float dt = std::is_same_v<T, float>
+            ? softplus_f(z[j] + zb) : softplus2_f(z[j] + zb) * LN2;
+        const float dtu = dt * u[j];
         const float* bc = s_bc + (t1 + j) * 2 * npad + i0;
         float y = 0.f;
         #pragma unroll
@@ -125,7 +141,9 @@ void scan_kernel(Scan<T> a, int lanes, int tt, int nseg, int seg_len,
             y += __shfl_xor(y, off, WAVE);
           if (part == 0 && there)
             st1(a.out + (row0 + b0 + t1 + j) * a.out_ld + c,
-                (y + d * u[j]) * g[j] * sigmoid_f(g[j]));
+                (y + d * u[j]) * (std::is_same_v<T, float>
+                                      ? g[j] * sigmoid_f(g[j])
+                                      : fast_silu_f(g[j])));
         }
       }
     }
@@ -166,19 +184,30 @@ void scan_join_kernel(Scan<T> a, int nseg, int seg_len, float* __restrict__ ws,
 int lanes_of(int n, int np) {
   int l = 1;
   while (l * np < n) l *= 2;
-  return l;                        // n <= 512: at most 32 lanes of 16
+  return l;
 }
 
-int np_of(int n) { return n <= 4 ? 4 : n <= 8 ? 8 : 16; }
+long waves_of(int entries, int channels, int n, int np) {
+  return (long)entries * channels * lanes_of(n, np) / WAVE;
+}
+
+// Numbers of a state per thread: fewer where waves are few.
+int np_of(int entries, int channels, int n) {
+  int np = n <= 4 ? 4 : n <= 8 ? 8 : 16;
+  if (np == 16 && n <= 256 && waves_of(entries, channels, n, np) < 2048)
+    np = 8;
+  return np;                       // n <= 512: at most 32 lanes
+}
 
 }  // namespace
 
-// Segments per portion: enough threads for eight waves per SIMD, segments of
-// at least 64 tokens.
+// Segments per portion: at least two waves per SIMD.
+// (The first pass over segments costs as much as half of the scan.)
 int scan_segments(int entries, int channels, int n, int max_len) {
-  const long waves = (long)entries * channels * lanes_of(n, np_of(n)) / WAVE;
+  const long waves = waves_of(entries, channels, n,
+                              np_of(entries, channels, n));
   int k = 1;
-  while (waves * k < 4096 && max_len >= k * 2 * 64 && k < 128) k *= 2;
+  while (waves * k < 2048 && max_len >= k * 2 * 64 && k < 128) k *= 2;
   return k;
 }
 
@@ -204,7 +233,7 @@ void launch_scan(const Scan<T>& a, int entries, int max_len, int nseg,
     scan_kernel<T, NP, true><<<grid, BLOCK, lds, stream>>>(
         a, lanes, tt, nseg, seg_len, ws, ws_dt);
   };
-  switch (np_of(a.n)) {
+  switch (np_of(entries, a.channels, a.n)) {
     case 4: go(std::integral_constant<int, 4>{}); break;
     case 8: go(std::integral_constant<int, 8>{}); break;
     default: go(std::integral_constant<int, 16>{});

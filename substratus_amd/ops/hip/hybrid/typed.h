@@ -86,6 +86,22 @@ DEV_INLINE float softplus_f(float z) {
   return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
 }
 
+// log2(1 + e^z) and z sigmoid(z) in a few instructions, to 2e-6 relative
+DEV_INLINE float softplus2_f(float z) {
+  constexpr float log2e = 1.44269504088896340736f;
+  const float x = __builtin_amdgcn_exp2f(-fabsf(z) * log2e);
+  const float small = x * (1.f - x * (0.5f - x * (1.f / 3.f - x *
+                          (0.25f - x * 0.2f)))) * log2e;
+  return fmaxf(z, 0.f) * log2e +
+         (x < 0.1f ? small : __builtin_amdgcn_logf(1.f + x));
+}
+
+DEV_INLINE float fast_silu_f(float z) {
+  constexpr float log2e = 1.44269504088896340736f;
+  return z * __builtin_amdgcn_rcpf(
+      1.f + __builtin_amdgcn_exp2f(-z * log2e));
+}
+
 // One request's place in the batch, for kernels over single tokens and over
 // portions of prompts alike: rows [row0, row0 + n) of the packed activations.
 struct Entry {
