@@ -1,5 +1,6 @@
 from .config import ModelConfig, get_config, register
-from . import guronex as _guronex  # registers the architecture and its models
+from . import ditalorn as _ditalorn  # registers the architecture, its models
+from . import guronex as _guronex  # the same
 from . import kakovik as _kakovik  # the same
 from . import vurazen as _vurazen  # the same
 from .hybrid import HybridLM

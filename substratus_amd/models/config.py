@@ -37,7 +37,7 @@ class ModelConfig:
     # falcon-40b "new decoder architecture": parallel attn+MLP but with TWO
     # norms of the residual (ln_attn feeds attention, ln_mlp feeds the MLP)
     parallel_norms: bool = False
-    # opt-style: learned positional embeddings + LayerNorm + gelu
+    # opt-style: learned positional embeddings (+ LayerNorm + gelu)
     learned_pos_emb: bool = False
     activation: str = "silu"  # "silu" (gated) | "gelu"
     # models of unlike layers (models/hybrid.py): one spec per layer; the
@@ -78,7 +78,9 @@ class ModelConfig:
         h, f, L, v = self.hidden_size, self.intermediate_size, self.num_layers, self.vocab_size
         if self.layers:
             side = self.side_dim * len(self.layers)
-            return 2 * v * h + side * (v + 2 * h) \
+            tables = v * (1 if self.tie_word_embeddings else 2) \
+                + self.learned_pos_emb * self.max_position_embeddings
+            return tables * h + side * (v + 2 * h) \
                 + sum(s.params(h) for s in self.layers)
         qkv = h * (self.num_heads + 2 * self.num_kv_heads) * self.head_dim
         o = self.num_heads * self.head_dim * h

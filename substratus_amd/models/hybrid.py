@@ -24,7 +24,7 @@ from typing import Optional
 import torch
 import torch.nn as nn
 
-from ..ops import hybrid as ops
+from ..ops import hybrid as ops, linear
 from ..parallel.comm import state
 from ..parallel.tp import Linear
 from ..serve.batch import StepBatch
@@ -45,9 +45,10 @@ def _padded(rows: int) -> int:
 
 
 class AttentionMixer(nn.Module):
-    """Softmax attention over the paged cache; what AttentionSpec names is
-    there or not: whole-projection q/k norm, distance bias, chunk mask, value
-    blending, output gate."""
+    """Attention over the paged cache; what AttentionSpec names is there or
+    not: whole-projection q/k norm, distance bias or falloff, chunk mask,
+    value blending, output gate, short convolutions with query temperatures
+    and value norms, sigmoid weights instead of a softmax."""
 
     def __init__(self, spec: AttentionSpec, width: int, eps: float,
                  device=None, dtype=None):
@@ -60,8 +61,16 @@ class AttentionMixer(nn.Module):
         self.w_in = Linear(width, _padded(self.nq + self.nk + self.nv
                                           + self.ng),
                            device=device, dtype=dtype)
-        self.w_out = Linear(spec.heads * spec.vdim, width, device=device,
-                            dtype=dtype)
+        self.w_out = Linear(spec.heads * spec.vdim, width, spec.out_bias,
+                            device=device, dtype=dtype)
+        if spec.taps:
+            self.in_bias = _f32(spec.conv_rows, device=device)
+            self.conv = _f32(spec.conv_rows, spec.taps, device=device)
+        if spec.falloff:
+            self.r1 = _f32(spec.heads, device=device)
+            self.r2 = _f32(spec.heads, device=device)
+        if spec.sigmoid:
+            self.weight_bias = _f32(spec.heads, device=device)
         if spec.qk_norm:
             self.q_norm = _f32(self.nq, device=device)
             self.k_norm = _f32(self.nk, device=device)
@@ -80,10 +89,28 @@ class AttentionMixer(nn.Module):
     def forward(self, y: torch.Tensor, cache: tuple, batch: StepBatch,
                 shared: dict) -> torch.Tensor:
         s = self.spec
-        k_cache, v_cache = cache
+        k_cache, v_cache = cache[:2]
         buf = self.w_in(y)
         v_at = self.nq + self.nk
-        v_first = None
+        if s.taps:
+            q = ops.conv_qkv(buf, self.in_bias, self.conv, cache[2], k_cache,
+                             v_cache, batch, s.temp,
+                             self.eps if s.v_norm else None)
+        else:
+            q = self._prepare(buf, v_at, k_cache, v_cache, batch, shared)
+        g_at = v_at + self.nv
+        gate = buf[:, g_at:g_at + self.ng] if self.ng else None
+        a = ops.attn_ctx(
+            q, gate, k_cache, v_cache, self._bias, batch, s.scale, s.chunk,
+            falloff=(self.r1, self.r2) if s.falloff else None,
+            weight_bias=self.weight_bias if s.sigmoid else None)
+        return self.w_out(a)
+
+    def _prepare(self, buf: torch.Tensor, v_at: int, k_cache: torch.Tensor,
+                 v_cache: torch.Tensor, batch: StepBatch,
+                 shared: dict) -> torch.Tensor:
+        """Norms and blends of a projection that is not convolved."""
+        s, v_first = self.spec, None
         if s.v_mix:
             v_first = shared.get("v_first")
             if v_first is None:
@@ -94,11 +121,7 @@ class AttentionMixer(nn.Module):
                         self.k_norm if s.qk_norm else None, self.eps,
                         v_first, self.vmix if v_first is not None else None,
                         k_cache, v_cache, batch.slots)
-        g_at = v_at + self.nv
-        gate = buf[:, g_at:g_at + self.ng] if self.ng else None
-        a = ops.attn_ctx(buf[:, :self.nq], gate, k_cache, v_cache, self._bias,
-                         batch, s.scale, s.chunk)
-        return self.w_out(a)
+        return buf[:, :self.nq]
 
 
 class GLAMixer(nn.Module):
@@ -131,18 +154,27 @@ class GLAMixer(nn.Module):
 class LatentMixer(nn.Module):
     """Softmax attention over a paged cache of latents, the layer's own or an
     earlier layer's; heads expand keys and values from them, or queries and
-    outputs are moved into the latent space (ops.latent_attn)."""
+    outputs are moved into the latent space (ops.latent_attn). Queries may
+    come out of a latent of their own."""
 
     def __init__(self, spec: LatentAttentionSpec, width: int, eps: float,
                  device=None, dtype=None):
         super().__init__()
         self.spec, self.eps = spec, eps
         self.own = spec.kv_from is None
-        self.nq = spec.heads * (spec.dim + spec.rot_dim)
-        self.ng = spec.heads * spec.vdim if spec.out_gate else 0
-        self.w_in = Linear(width, _padded(self.nq + self.ng +
-                                          (spec.row if self.own else 0)),
+        nq = spec.heads * (spec.dim + spec.rot_dim)
+        self.nq = spec.q_rank or nq
+        row = spec.row if self.own else 0
+        # gates per head go last: they leave odd numbers of columns
+        self.ng = spec.heads * spec.vdim if spec.out_gate else \
+            spec.heads if spec.head_gate else 0
+        self.g_at, self.c_at = (self.nq + row, self.nq) if spec.head_gate \
+            else (self.nq, self.nq + self.ng)
+        self.w_in = Linear(width, _padded(self.nq + self.ng + row),
                            device=device, dtype=dtype)
+        if spec.q_rank:
+            self.q_norm = _f32(spec.q_rank, device=device)
+            self.w_uq = Linear(spec.q_rank, nq, device=device, dtype=dtype)
         self.w_out = Linear(spec.heads * spec.vdim, width, device=device,
                             dtype=dtype)
         # keys of all heads, then values of all heads
@@ -156,19 +188,22 @@ class LatentMixer(nn.Module):
         s = self.spec
         self._uk_t = self.w_ukv[:s.heads * s.dim].view(
             s.heads, s.dim, s.rank).transpose(1, 2).contiguous()
-        self._turns = s.rot.turns(self.w_ukv.device)
+        self._turns = s.rot.turns(self.w_ukv.device) if s.rot else \
+            torch.empty(0, dtype=torch.float64, device=self.w_ukv.device)
 
     def forward(self, y: torch.Tensor, cache: tuple, batch: StepBatch,
                 shared: dict) -> torch.Tensor:
-        buf = self.w_in(y)
-        at = self.nq + self.ng
-        ops.latent_prepare(buf, self.spec, at if self.own else -1,
+        s, buf = self.spec, self.w_in(y)
+        ops.latent_prepare(buf, s, self.c_at if self.own else -1,
                            self.c_norm if self.own else None, self.eps,
                            self._turns, batch.positions, cache[0],
-                           batch.slots)
-        gate = buf[:, self.nq:at] if self.ng else None
-        o = ops.latent_attn(buf[:, :self.nq], gate, cache[0], self.w_ukv,
-                            self._uk_t, batch, self.spec, shared)
+                           batch.slots, self.q_norm if s.q_rank else None)
+        gate = buf[:, self.g_at:self.g_at + self.ng] if self.ng else None
+        q = buf[:, :self.nq]
+        if s.q_rank:
+            q = self.w_uq(q)
+        o = ops.latent_attn(q, gate, cache[0], self.w_ukv, self._uk_t, batch,
+                            s, shared)
         return self.w_out(o)
 
 
@@ -364,13 +399,16 @@ class Experts(nn.Module):
         self.router = weight(spec.experts, width)
         if spec.bias:
             self.router_bias = _f32(spec.experts, device=device)
+        if spec.correction:
+            self.correction = _f32(spec.experts, device=device)
         # gated: rows of gate and up in turn
         self.up = weight(spec.experts, (2 if spec.glu else 1) * spec.ff, width)
         self.down = weight(spec.experts, width, spec.ff)
 
     def forward(self, y: torch.Tensor) -> ops.Picked:
         return ops.experts(y, self.router, self.up, self.down, self.spec,
-                           self.router_bias if self.spec.bias else None)
+                           self.router_bias if self.spec.bias else None,
+                           self.correction if self.spec.correction else None)
 
 
 class SideInput(nn.Module):
@@ -491,16 +529,21 @@ class HybridLM(nn.Module):
             self.side_embed = nn.Parameter(torch.empty(
                 cfg.vocab_size, cfg.side_dim * len(cfg.layers), device=device,
                 dtype=dtype))
+        if cfg.learned_pos_emb:
+            self.pos = nn.Parameter(torch.empty(
+                cfg.max_position_embeddings, cfg.hidden_size, device=device,
+                dtype=dtype))
         self.final_norm = _f32(cfg.hidden_size, device=device)
         if cfg.parallel_block:
             self.final_norm_bias = _f32(cfg.hidden_size, device=device)
-        self.head = Linear(cfg.hidden_size, cfg.vocab_size, device=device,
-                           dtype=dtype)
+        self.head = None if cfg.tie_word_embeddings else Linear(
+            cfg.hidden_size, cfg.vocab_size, device=device, dtype=dtype)
 
     @torch.no_grad()
     def init_random(self, seed: int = 0) -> None:
         """Fill every parameter (models are built on meta): matrices
-        N(0, 0.02), norms neutral, blend factors 1/2, decays near 1."""
+        N(0, 0.02), norms neutral, blend factors 1/2, decays near 1, sigmoid
+        weights small."""
         g = torch.Generator(device=self.final_norm.device).manual_seed(seed)
         neutral = 1.0 - self.cfg.norm_offset
         for name, p in self.named_parameters():
@@ -513,8 +556,10 @@ class HybridLM(nn.Module):
                 p.normal_(0.0, p.shape[1] ** -0.5, generator=g)
             elif leaf == "dt_bias":
                 p.fill_(-4.0)
-            elif leaf == "vmix":
+            elif leaf in ("vmix", "r1", "r2"):
                 p.fill_(0.5)
+            elif leaf == "weight_bias":
+                p.fill_(-4.0)
             elif leaf == "a2_bias":
                 p.fill_(2.0)
             else:
@@ -531,6 +576,10 @@ class HybridLM(nn.Module):
         for layer in self.layers:
             layer.mixer.finish_weights()
 
+    def logits(self, y: torch.Tensor) -> torch.Tensor:
+        return linear(y, self.embed.weight) if self.head is None \
+            else self.head(y)
+
     def step_ops(self, batch: StepBatch, caches: list[tuple]):
         """The forward as a generator that yields between op groups (see
         models/model.py decode_ops); returns the logits of batch.want, or of
@@ -539,8 +588,10 @@ class HybridLM(nn.Module):
             return (yield from self._parallel_ops(batch, caches))
         off, eps = self.cfg.norm_offset, self.eps
         mult = self.cfg.residual_mult
-        x, y = ops.embed_norm(batch.tokens, self.embed.weight,
-                              self.layers[0].norm1, off, eps)
+        x, y = ops.embed_norm(
+            batch.tokens, self.embed.weight, self.layers[0].norm1, off, eps,
+            self.cfg.embed_scale, self.pos if self.cfg.learned_pos_emb
+            else None, batch.positions)
         tokens = batch.tokens
         shared: dict = {}     # what a layer leaves for later layers' mixers
         for i, layer in enumerate(self.layers):
@@ -566,7 +617,7 @@ class HybridLM(nn.Module):
                     layer.side.norm
                 yield
             y = ops.stream_norm(delta, x, post, after, off, eps, scale, mult)
-        return self.head(y)
+        return self.logits(y)
 
     def _parallel_ops(self, batch: StepBatch, caches: list[tuple]):
         cfg, runs = self.cfg, self.cfg.runs()
@@ -590,7 +641,7 @@ class HybridLM(nn.Module):
             x = x[want]
         _, y = ops.add_norm(x, self.final_norm, self.final_norm_bias, self.eps,
                             dtype, rows, picked)
-        logits = self.head(y)
+        logits = self.logits(y)
         return ops.softcap(logits, cfg.logit_softcap) if cfg.logit_softcap \
             else logits
 

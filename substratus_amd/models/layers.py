@@ -49,6 +49,14 @@ class MixerSpec:
 
 
 @dataclass(frozen=True)
+class QueryTemperature:
+    """Queries at position p are multiplied by
+    1 + coef * ln(floor((p + 1) / every) + 1)."""
+    coef: float
+    every: int
+
+
+@dataclass(frozen=True)
 class AttentionSpec(MixerSpec):
     heads: int
     kv_heads: int
@@ -61,14 +69,38 @@ class AttentionSpec(MixerSpec):
     bias_max: int = 0        # distance from which the last row holds
     v_mix: bool = False      # blend in the first such layer's values
     out_gate: bool = False   # sigmoid gate per head on the output
+    taps: int = 0            # > 0: q, k and v have a bias and pass a short
+                             #   causal convolution over time
+    temp: Optional[QueryTemperature] = None   # after the convolution
+    v_norm: bool = False     # values over their root mean square, after it
+    out_bias: bool = False   # of the output projection
+    falloff: bool = False    # r1 ln(1 + r2 distance) is taken off the score
+    sigmoid: bool = False    # weights are sigmoid(score + a bias per head),
+                             #   each by itself, not a softmax
+
+    def __post_init__(self) -> None:
+        if self.taps and (self.qk_norm or self.v_mix):
+            raise ValueError("convolved projections are neither normed as a "
+                             "whole nor blended")
+        if not self.taps and (self.temp or self.v_norm):
+            raise ValueError("query temperatures and value norms follow a "
+                             "convolution")
+
+    @property
+    def conv_rows(self) -> int:
+        return (self.heads + self.kv_heads) * self.dim \
+            + self.kv_heads * self.vdim
 
     def cache(self) -> tuple:
-        return Pages(self.kv_heads, self.dim), Pages(self.kv_heads, self.vdim)
+        pages = Pages(self.kv_heads, self.dim), \
+            Pages(self.kv_heads, self.vdim)
+        return pages if not self.taps else \
+            pages + (Slots((self.taps - 1, self.conv_rows), False),)
 
     def params(self, width: int) -> int:
-        rows = (self.heads + self.kv_heads) * self.dim \
-            + self.kv_heads * self.vdim + self.heads * self.out_gate
-        return width * (rows + self.heads * self.vdim)
+        rows = self.conv_rows + self.heads * self.out_gate
+        return width * (rows + self.heads * self.vdim) \
+            + self.conv_rows * self.taps
 
 
 @dataclass(frozen=True)
@@ -114,9 +146,18 @@ class LatentAttentionSpec(MixerSpec):
     vdim: int                # value size of a head
     rank: int                # size of the latent
     scale: float
-    rot: RotarySpec
+    rot: Optional[RotarySpec]       # None: rot_dim is 0
     kv_from: Optional[int] = None   # layer whose latents it attends to
     out_gate: bool = False   # sigmoid gate per element on the output
+    head_gate: bool = False  # the same per head
+    q_rank: int = 0          # > 0: queries are projections of a normed latent
+    window: int = 0          # > 0: keys a position sees, its own included
+
+    def __post_init__(self) -> None:
+        if self.out_gate and self.head_gate:
+            raise ValueError("a gate per element or per head, not both")
+        if self.q_rank and self.rot_dim:
+            raise ValueError("queries out of a latent are not rotated")
 
     @property
     def row(self) -> int:
@@ -127,10 +168,12 @@ class LatentAttentionSpec(MixerSpec):
         return (Pages(1, self.row),) if self.kv_from is None else ()
 
     def params(self, width: int) -> int:
-        rows = self.heads * (self.dim + self.rot_dim +
-                             self.vdim * (1 + self.out_gate)) \
+        q = self.heads * (self.dim + self.rot_dim)
+        rows = self.heads * (self.vdim * (1 + self.out_gate) +
+                             self.head_gate) + (self.q_rank or q) \
             + (self.row if self.kv_from is None else 0)
-        return width * rows + self.heads * self.rank * (self.dim + self.vdim)
+        return width * rows + self.q_rank * q \
+            + self.heads * self.rank * (self.dim + self.vdim)
 
 
 @dataclass(frozen=True)
@@ -253,7 +296,9 @@ class GluSpec:
 class MoESpec:
     """Experts, of which a token uses the `top` best of the `keep` best
     groups of neighbours. Weights are softmax scores over all experts, or
-    over the chosen ones."""
+    over the chosen ones, or the sigmoid of each chosen one's score. What is
+    best goes by the scores, for the choice only with a learned correction;
+    a group's score is the sum of its `group_best` best ones."""
     experts: int
     top: int
     ff: int                  # inner size of one expert
@@ -264,8 +309,13 @@ class MoESpec:
     bias: bool = False       # of the router's scores
     shared_ff: int = 0       # an expert for every token, 0: none
     shared_glu: Optional[GluSpec] = None
+    sigmoid: bool = False
+    correction: bool = False
+    group_best: int = 1      # 1 or 2
 
     def __post_init__(self) -> None:
+        if self.sigmoid and self.over_chosen:
+            raise ValueError("sigmoid scores do not sum to anything")
         if self.experts % self.groups or not 0 < self.keep <= self.groups:
             raise ValueError(f"{self.experts} experts in {self.groups} "
                              f"groups, {self.keep} kept")

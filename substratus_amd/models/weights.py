@@ -27,6 +27,7 @@ def find_weights(model_dir: str) -> Optional[str]:
 def to_native(sd: dict, mcfg: ModelConfig) -> dict:
     """Checkpoint names of any supported layout -> the model's own."""
     from . import hf_compat as hf
+    from .ditalorn import ditalorn_to_native, is_ditalorn_state_dict
     from .guronex import guronex_to_native, is_guronex_state_dict
     from .kakovik import is_kakovik_state_dict, kakovik_to_native
     from .vurazen import is_vurazen_state_dict, vurazen_to_native
@@ -34,6 +35,7 @@ def to_native(sd: dict, mcfg: ModelConfig) -> dict:
             (hf.is_hf_llama_state_dict, hf.hf_llama_to_native),
             (hf.is_hf_falcon_state_dict, hf.hf_falcon_to_native),
             (hf.is_hf_opt_state_dict, hf.hf_opt_to_native),
+            (is_ditalorn_state_dict, ditalorn_to_native),
             (is_kakovik_state_dict, kakovik_to_native),
             (is_guronex_state_dict, guronex_to_native),
             (is_vurazen_state_dict, vurazen_to_native)):

@@ -2,12 +2,14 @@
 // single tokens and portions of prompts: one wave per (row, query head).
 //
 //   score(i, j) = f(scale * q_i . k_j) + bias[h][min(i - j, nbias - 1)]
+//                 - r1[h] ln(1 + r2[h] (i - j))
 //                 with f(s) = s, or cap * tanh(s / cap) when cap > 0
 //   visible: j <= i, and i / chunk == j / chunk when chunk > 0,
 //            and i - j < window or j < keep when window > 0
 //   out_h = softmax(score) v * sigmoid(gate_h) * mult   (gate optional)
 //
 // With a sink, the softmax's denominator has e^(sink_h) besides the keys.
+// Instead of a softmax, a key's weight may be sigmoid(score + wbias_h).
 //
 // Query head h reads key/value head h / (heads / kv_heads). 64 keys at a
 // time: lane = key for the scores, lane = column for the values. This is the
@@ -40,6 +42,8 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
   for (int c = 0; c < CMAX; ++c) acc[c] = 0.f;
   float m = -INFINITY, l = 0.f;
   if (a.sink != nullptr) { m = a.sink[h]; l = 1.f; }
+  const bool sig = a.wbias != nullptr;
+  if (sig) l = 1.f;                             // nothing to divide by
   for (int i = 0; i < part.n; ++i) {
     const int k0 = part.at(i) * WAVE, key = k0 + lane;
     float s = -INFINITY;
@@ -52,12 +56,19 @@ void attn_ctx_any_kernel(AttnCtx<T> a) {
       if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
       if (a.bias != nullptr)
         s += a.bias[(long)h * a.nbias + min(pos - key, a.nbias - 1)];
+      if (a.r1 != nullptr)
+        s -= a.r1[h] * log1pf(a.r2[h] * (float)(pos - key));
     }
-    const float mn = fmaxf(m, wave_max(s));      // finite: some key is visible
-    const float p = expf(s - mn);
-    const float keep = expf(m - mn);
-    l = l * keep + wave_sum(p);
-    m = mn;
+    float p, keep = 1.f;
+    if (sig) {
+      p = sigmoid_f(s + a.wbias[h]);             // 0 of -inf
+    } else {
+      const float mn = fmaxf(m, wave_max(s));    // finite: some key is visible
+      p = expf(s - mn);
+      keep = expf(m - mn);
+      l = l * keep + wave_sum(p);
+      m = mn;
+    }
     s_p[lane] = p;
     __syncthreads();
     #pragma unroll

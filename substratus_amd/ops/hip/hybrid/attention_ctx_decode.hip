@@ -1,6 +1,6 @@
 // Single-token attention over the paged bf16 cache with a distance bias, a
-// chunk mask, unequal key and value head sizes and a gated output (the
-// formulas are in attention_ctx.hip). HBM-bound: every K and V row is read
+// chunk mask, unequal key and value head sizes, a gated output, and softmax or
+// sigmoid weights (the formulas are in attention_ctx.hip). HBM-bound: every K and V row is read
 // once per group of GQ query heads.
 //
 // One page of 16 keys is a wave's unit of work. Scores: 4 lanes per key, each
@@ -8,8 +8,8 @@
 // columns (8 each), 64/CL rows side by side. The next page's K, V and bias
 // are in flight while the current page is computed. Queries stay bf16 and
 // scores are sums of v_dot2_f32_bf16 (two products added to a float), so K
-// needs no unpacking. Four waves take pages in turn and merge through LDS; `splits` workgroups share one long context and
-// a second kernel merges those.
+// needs no unpacking. Four waves take pages in turn and merge through LDS;
+// `splits` workgroups share one long context and a second kernel merges those.
 #include "attention_ctx.h"
 
 namespace {
@@ -26,7 +26,8 @@ DEV_INLINE float dot2(unsigned a, unsigned b, float c) {
       false);
 }
 
-template <int DCH, int CL, int GQ>
+// SIG: sigmoid weights, so partial results add up as they are
+template <int DCH, int CL, int GQ, bool SIG>
 __global__ __launch_bounds__(NW * WAVE)
 void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
                             float* __restrict__ part_o,
@@ -65,6 +66,14 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
   const float cap2 = a.cap * LOG2E;
   const float cscale = a.cap > 0.f ? 2.f * scale2 / a.cap : 0.f;
 
+  float r1[GQ], r2[GQ], wb[GQ];
+  #pragma unroll
+  for (int g = 0; g < GQ; ++g) {
+    const int h = h0 + min(g, nh - 1);
+    r1[g] = a.r1 != nullptr ? a.r1[h] : 0.f;
+    r2[g] = a.r1 != nullptr ? a.r2[h] : 0.f;
+    wb[g] = SIG ? a.wbias[h] * LOG2E : 0.f;
+  }
   uint4v kr[DCH], vr[NV];
   float br[GQ];
   auto load = [&](int pg) {
@@ -125,11 +134,18 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
     }
     const int kpos = pg * PAGE + key;
     const bool live = kpos <= pos && (kpos >= lo || kpos < a.keep);
+    const float dist = (float)(pos - kpos);
     #pragma unroll
     for (int g = 0; g < GQ; ++g) {
       s[g] += __shfl_xor(s[g], 1, WAVE);
       s[g] += __shfl_xor(s[g], 2, WAVE);
       s[g] = a.cap > 0.f ? cap2 * tanh_exp2(s[g] * cscale) : s[g] * scale2;
+      if (a.r1 != nullptr)
+        s[g] -= r1[g] * __builtin_amdgcn_logf(1.f + r2[g] * dist);
+      if constexpr (SIG) {
+        s[g] = live ? sigmoid_exp2(s[g] + bn[g] + wb[g]) : 0.f;
+        continue;
+      }
       s[g] = live ? s[g] + bn[g] : NEG;
       float mx = s[g];
       #pragma unroll
@@ -178,6 +194,20 @@ void attn_ctx_decode_kernel(AttnCtx<bf16_t> a, int splits,
 
   for (int i = threadIdx.x; i < nh * a.vdim; i += NW * WAVE) {
     const int g = i / a.vdim, c = i % a.vdim, h = h0 + g;
+    if constexpr (SIG) {
+      float o = 0.f;
+      #pragma unroll
+      for (int w = 0; w < NW; ++w) o += s_o[w][g][c];
+      if (splits == 1) {
+        float f = a.mult;
+        if (a.gate != nullptr)
+          f *= sigmoid_f(bf2f(a.gate[(long)b * a.g_ld + h]));
+        a.out[(long)b * a.out_ld + (long)h * a.vdim + c] = f2bf(o * f);
+      } else {
+        part_o[(((long)b * a.heads + h) * splits + split) * a.vdim + c] = o;
+      }
+      continue;
+    }
     float M = s_ml[0][g][0];
     #pragma unroll
     for (int w = 1; w < NW; ++w) M = fmaxf(M, s_ml[w][g][0]);
@@ -216,9 +246,11 @@ void attn_ctx_merge_kernel(AttnCtx<bf16_t> a, int splits,
   const long b = blockIdx.y, at = (b * a.heads + h) * splits;
   const int c = threadIdx.x * VEC;
   if (c >= a.vdim) return;
-  float M = NEG;
-  for (int s = 0; s < splits; ++s) M = fmaxf(M, part_ml[(at + s) * 2]);
-  float L = 0.f, o[VEC];
+  const bool sig = a.wbias != nullptr;          // sums only, no part_ml
+  float M = sig ? 0.f : NEG;
+  for (int s = 0; s < splits && !sig; ++s)
+    M = fmaxf(M, part_ml[(at + s) * 2]);
+  float L = sig ? 1.f : 0.f, o[VEC];
   if (a.sink != nullptr) {
     const float s = a.sink[h] * LOG2E;
     M = fmaxf(M, s);
@@ -228,10 +260,11 @@ void attn_ctx_merge_kernel(AttnCtx<bf16_t> a, int splits,
   for (int j = 0; j < VEC; ++j) o[j] = 0.f;
   #pragma unroll 4
   for (int s = 0; s < splits; ++s) {
-    const float f = __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
+    const float f =
+        sig ? 1.f : __builtin_amdgcn_exp2f(part_ml[(at + s) * 2] - M);
     float p[VEC];
     ldv<VEC>(part_o + (at + s) * a.vdim + c, p);
-    L += part_ml[(at + s) * 2 + 1] * f;
+    if (!sig) L += part_ml[(at + s) * 2 + 1] * f;
     #pragma unroll
     for (int j = 0; j < VEC; ++j) o[j] += p[j] * f;
   }
@@ -274,9 +307,14 @@ void launch_attn_ctx_decode(const AttnCtx<bf16_t>& a, int entries, int splits,
   const int per = a.heads / a.kv_heads, gq = pick_gq(per);
   const dim3 grid(entries, a.kv_heads, (per + gq - 1) / gq * splits);
   auto go = [&](auto dch, auto cl, auto g) {
-    attn_ctx_decode_kernel<decltype(dch)::value, decltype(cl)::value,
-                           decltype(g)::value>
-        <<<grid, dim3(NW * WAVE), 0, stream>>>(a, splits, part_o, part_ml);
+    constexpr int D = decltype(dch)::value, C = decltype(cl)::value,
+                  G = decltype(g)::value;
+    if (a.wbias != nullptr)
+      attn_ctx_decode_kernel<D, C, G, true>
+          <<<grid, dim3(NW * WAVE), 0, stream>>>(a, splits, part_o, part_ml);
+    else
+      attn_ctx_decode_kernel<D, C, G, false>
+          <<<grid, dim3(NW * WAVE), 0, stream>>>(a, splits, part_o, part_ml);
   };
   using std::integral_constant;
   auto by_g = [&](auto dch, auto cl) {

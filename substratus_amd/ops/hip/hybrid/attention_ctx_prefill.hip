@@ -1,7 +1,7 @@
 // Attention of prompt portions over the paged bf16 cache (which already holds
 // the portion's own keys and values), with a distance bias, a chunk mask,
-// unequal key and value head sizes and a gated output; the formulas are in
-// attention_ctx.hip. Rows of a portion carry their absolute positions, so a
+// unequal key and value head sizes, a gated output, and softmax or sigmoid
+// weights; the formulas are in attention_ctx.hip. Rows of a portion carry their absolute positions, so a
 // prompt can be cut anywhere.
 //
 // The structure is that of attention_v5.hip: every wave owns 32 query rows
@@ -42,8 +42,13 @@ DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
 }
 
 // KK: 16-wide steps of the key size; DC: 32-wide tiles of the value size
-// CAP: scores are capped
-template <int KK, int DC, int WAVES, bool FLAT, bool CAP>
+enum Kind {
+  PLAIN,
+  CAP,        // scores are capped
+  SIGMOID,    // weights are sigmoids: no maximum, no sum
+};
+
+template <int KK, int DC, int WAVES, bool FLAT, Kind KIND>
 __global__ __launch_bounds__(WAVES * WAVE)
 void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   constexpr int THREADS = WAVES * WAVE;
@@ -65,13 +70,14 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   if (q0_tile >= en.n) return;
   const int kvh = head / (a.heads / a.kv_heads);
   const int* bt = FLAT ? nullptr : a.block_table + (long)e * a.max_blocks;
-  const long flat0 = FLAT ? a.ctx_start[e] : 0;
   const int kd = a.dim - a.shared;               // a head's own key elements
 
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
   const int lo5 = lane & 31, hi = lane >> 5;
   const int pos0 = a.positions[en.row0];
   const int total = pos0 + en.n;                 // keys in the cache
+  const int from = FLAT ? flat_from(a.window, pos0) : 0;
+  const long flat0 = FLAT ? (long)a.ctx_start[e] - from : 0;
   const int qa0 = pos0 + q0_tile;                // first position of the tile
   const int qw0 = qa0 + wave * 32;               // first position of the wave
   const bool wave_live = qw0 < total;
@@ -107,19 +113,22 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
   int pgk[LK], pgv[LV];                          // page bases, -1: no key
   uint4 st_k[LK], st_v[LV];
   float st_b = 0.f;
+  const float wb2 = KIND == SIGMOID ? a.wbias[head] * LOG2E : 0.f;
 
   auto pages = [&](int it) {
     const int st = part.at(it);
     #pragma unroll
     for (int i = 0; i < LK; ++i) {
       const int key = st * CH + (i * THREADS + tid) / (KK * 2);
-      pgk[i] = it < part.n && key < total && key < st * CH + CH
+      pgk[i] = it < part.n && key >= from && key < total &&
+               key < st * CH + CH
           ? (FLAT ? key : bt[key / PAGE]) : -1;
     }
     #pragma unroll
     for (int i = 0; i < LV; ++i) {
       const int key = st * CH + (i * THREADS + tid) / (DC * 4);
-      pgv[i] = it < part.n && key < total && key < st * CH + CH
+      pgv[i] = it < part.n && key >= from && key < total &&
+               key < st * CH + CH
           ? (FLAT ? key : bt[key / PAGE]) : -1;
     }
   };
@@ -155,11 +164,9 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
             a.vc + (((long)pgv[i] * a.kv_heads + kvh) * PAGE +
                     (st * CH + r) % PAGE) * a.v_ld + d);
     }
-    if (a.bias != nullptr) {
-      const int n = qa0 - (st * CH + CH - 1) + tid;
-      st_b = a.bias[(long)head * a.nbias + min(max(n, 0), a.nbias - 1)] *
-             LOG2E;
-    }
+    if (a.bias != nullptr || a.r1 != nullptr)
+      st_b = distance_bias2(a, head, qa0 - (st * CH + CH - 1) + tid);
+    if constexpr (KIND == SIGMOID) st_b += wb2;
   };
   auto stage_write = [&](int buf) {
     #pragma unroll
@@ -217,8 +224,8 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
       for (int sc = 0; sc < CH / 32; ++sc)
         #pragma unroll
         for (int r = 0; r < 16; ++r)
-          sv[sc][r] = (CAP ? cap2 * tanh_exp2(sacc[sc][r] * cscale)
-                           : sacc[sc][r] * scale2) +
+          sv[sc][r] = (KIND == CAP ? cap2 * tanh_exp2(sacc[sc][r] * cscale)
+                                   : sacc[sc][r] * scale2) +
                       bw[-(sc * 32 + (r & 3) + 8 * (r >> 2))];
       // steps inside every row's range need no mask
       if (kbase < lo_last || kbase + CH - 1 > qw0 || qw0 + 31 >= total) {
@@ -233,23 +240,25 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
               sv[sc][r] = -INFINITY;
           }
       }
-      float mloc = -INFINITY;
-      #pragma unroll
-      for (int sc = 0; sc < CH / 32; ++sc)
+      if constexpr (KIND != SIGMOID) {
+        float mloc = -INFINITY;
         #pragma unroll
-        for (int r = 0; r < 16; ++r) mloc = fmaxf(mloc, sv[sc][r]);
-      mloc = fmaxf(mloc, __shfl_xor(mloc, 32, WAVE));
-      // the running maximum moves only when a score exceeds it by 2^8
-      if (!__all(mloc == -INFINITY || mloc - m <= 8.f)) {
-        const float mn = fmaxf(m, mloc);
-        const float keep = m == -INFINITY ? 0.f
-                                          : __builtin_amdgcn_exp2f(m - mn);
-        m = mn;
-        l *= keep;
-        #pragma unroll
-        for (int c = 0; c < DC; ++c)
+        for (int sc = 0; sc < CH / 32; ++sc)
           #pragma unroll
-          for (int r = 0; r < 16; ++r) o_t[c][r] *= keep;
+          for (int r = 0; r < 16; ++r) mloc = fmaxf(mloc, sv[sc][r]);
+        mloc = fmaxf(mloc, __shfl_xor(mloc, 32, WAVE));
+        // the running maximum moves only when a score exceeds it by 2^8
+        if (!__all(mloc == -INFINITY || mloc - m <= 8.f)) {
+          const float mn = fmaxf(m, mloc);
+          const float keep = m == -INFINITY ? 0.f
+                                            : __builtin_amdgcn_exp2f(m - mn);
+          m = mn;
+          l *= keep;
+          #pragma unroll
+          for (int c = 0; c < DC; ++c)
+            #pragma unroll
+            for (int r = 0; r < 16; ++r) o_t[c][r] *= keep;
+        }
       }
       float sum = 0.f;
       #pragma unroll
@@ -261,11 +270,15 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
           for (int i = 0; i < 4; ++i) {
             const float s0 = sv[sc][8 * g + 2 * i];
             const float s1 = sv[sc][8 * g + 2 * i + 1];
-            const float p0 = s0 == -INFINITY
-                ? 0.f : __builtin_amdgcn_exp2f(s0 - m);
-            const float p1 = s1 == -INFINITY
-                ? 0.f : __builtin_amdgcn_exp2f(s1 - m);
-            sum += p0 + p1;
+            float p0, p1;
+            if constexpr (KIND == SIGMOID) {
+              p0 = sigmoid_exp2(s0);
+              p1 = sigmoid_exp2(s1);
+            } else {
+              p0 = s0 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(s0 - m);
+              p1 = s1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(s1 - m);
+              sum += p0 + p1;
+            }
             wh[i] = cvt_pk_bf16(p0, p1);
             const float2 back = unpack_bf16x2(wh[i]);
             wl[i] = cvt_pk_bf16(p0 - back.x, p1 - back.y);
@@ -288,7 +301,7 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
           }
         }
       }
-      l += sum + __shfl_xor(sum, 32, WAVE);
+      if constexpr (KIND != SIGMOID) l += sum + __shfl_xor(sum, 32, WAVE);
     }
     if (it + 1 < part.n) stage_write(cur ^ 1);
     __syncthreads();
@@ -296,8 +309,8 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
 
   if (wave_live && qpos < total) {
     const long r = en.row0 + row;
-    float f = a.mult / l;
-    if (!FLAT && a.gate != nullptr)
+    float f = KIND == SIGMOID ? a.mult : a.mult / l;
+    if (!(FLAT && a.gate_each) && a.gate != nullptr)
       f *= sigmoid_f(bf2f(a.gate[r * a.g_ld + head]));
     bf16_t* op = a.out + r * a.out_ld + (long)head * a.vdim;
     #pragma unroll
@@ -309,7 +322,7 @@ void attn_ctx_prefill_kernel(AttnCtx<bf16_t> a) {
           float o[4];
           #pragma unroll
           for (int j = 0; j < 4; ++j) o[j] = o_t[c][rr * 4 + j] * f;
-          if (FLAT && a.gate != nullptr) {
+          if (FLAT && a.gate_each && a.gate != nullptr) {
             float g[4];
             ldv<4>(a.gate + r * a.g_ld + (long)head * a.vdim + d0, g);
             #pragma unroll
@@ -342,13 +355,16 @@ void launch_attn_ctx_prefill(const AttnCtx<bf16_t>& a, int entries,
     constexpr int K = decltype(kk)::value, D = decltype(dc)::value;
     const dim3 block(W * WAVE);
     if (a.ctx_start != nullptr)
-      attn_ctx_prefill_kernel<K, D, W, true, false>
+      attn_ctx_prefill_kernel<K, D, W, true, PLAIN>
+          <<<grid, block, 0, stream>>>(a);
+    else if (a.wbias != nullptr)
+      attn_ctx_prefill_kernel<K, D, W, false, SIGMOID>
           <<<grid, block, 0, stream>>>(a);
     else if (a.cap > 0.f)
-      attn_ctx_prefill_kernel<K, D, W, false, true>
+      attn_ctx_prefill_kernel<K, D, W, false, CAP>
           <<<grid, block, 0, stream>>>(a);
     else
-      attn_ctx_prefill_kernel<K, D, W, false, false>
+      attn_ctx_prefill_kernel<K, D, W, false, PLAIN>
           <<<grid, block, 0, stream>>>(a);
   };
   using std::integral_constant;

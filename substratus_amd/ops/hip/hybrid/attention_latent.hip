@@ -1,7 +1,8 @@
 // Attention in the latent space over the paged bf16 cache: all query heads
 // share one key per token, and its first `vdim` columns are the value. For
 // single tokens and portions of prompts: an entry's queries are its rows
-// times its heads, in that order, and a workgroup takes 16 * MT of them.
+// times its heads, in that order, and a workgroup takes 16 * MT of them. With
+// a window, it begins at the step with the first key that any of them sees.
 //
 // A step is 64 keys, four pages. A page is one contiguous piece of memory and
 // goes to LDS as it is (direct loads, the next step's in flight, page numbers
@@ -81,9 +82,10 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int entries, int splits,
   const int pos0 = a.positions[en.row0];
   const int last = pos0 + (min(q0 + QT, nq) - 1) / a.heads;  // of the tile
   const int pages = last / PAGE + 1;
-  const int steps = (pages + PAGES - 1) / PAGES;
-  const int st0 = (int)((long)steps * split / splits),
-            st1 = (int)((long)steps * (split + 1) / splits);
+  const int sb = first_seen(a, pos0 + q0 / a.heads) / CH;
+  const int steps = (pages + PAGES - 1) / PAGES - sb;
+  const int st0 = sb + (int)((long)steps * split / splits),
+            st1 = sb + (int)((long)steps * (split + 1) / splits);
   auto page_at = [&](int st) {
     return bt[min(st * PAGES + page, pages - 1)];
   };
@@ -115,10 +117,11 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int entries, int splits,
   const bool scoring = part < MT;
   const int mine = (scoring ? part : 0) * 16;
   short8 q[KS];
-  int qpos;
+  int qpos, qlo;                                 // first and last key seen
   {
     const int qi = min(q0 + mine + lo, nq - 1);
     qpos = pos0 + qi / a.heads;
+    qlo = first_seen(a, qpos);
     const bf16_t* qp = a.q + (long)(en.row0 + qi / a.heads) * a.q_ld +
                        (long)(qi % a.heads) * a.dim;
     #pragma unroll
@@ -170,7 +173,8 @@ void attn_latent_kernel(AttnCtx<bf16_t> a, int entries, int splits,
       float mx = NEG;
       #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        s[i] = key + i <= qpos ? (acc[0][i] + acc[1][i]) * scale2 : -INFINITY;
+        s[i] = key + i <= qpos && key + i >= qlo
+            ? (acc[0][i] + acc[1][i]) * scale2 : -INFINITY;
         mx = fmaxf(mx, s[i]);
       }
       mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));

@@ -13,13 +13,13 @@
 template <class T>
 void launch_stream_norm(T*, float*, const T*, const int*, const float*, int, const float*, const float*, long, int, float, float, float, float, hipStream_t);
 template <class T>
-void launch_latent_prepare(T*, long, int, int, int, int, int, const float*, float, const double*, int, const int*, T*, const int*, long, hipStream_t);
-void launch_latent_gather(void*, void*, const void*, int, int, int, const int*, int, const int*, int, int, hipStream_t);
+void launch_latent_prepare(T*, long, int, int, int, int, int, const float*, float, const double*, int, const int*, T*, const int*, const float*, int, long, hipStream_t);
+void launch_latent_gather(void*, void*, const void*, int, int, int, const int*, int, const int*, const int*, const int*, int, int, int, int, hipStream_t);
 int moe_max_experts();
-void launch_moe_select(int*, float*, const float*, int, int, int, int, int, int, const float*, bool, hipStream_t);
+void launch_moe_select(int*, float*, const float*, int, int, int, int, int, int, const float*, bool, bool, const float*, int, hipStream_t);
 void launch_moe_sort(int*, int*, int*, int*, const int*, int, int, int, int, hipStream_t);
 template <class T>
-void launch_embed_norm(T*, float*, const T*, const int*, const float*, long, int, int, float, float, hipStream_t);
+void launch_embed_norm(T*, float*, const T*, const int*, float, const T*, const int*, int, const float*, long, int, int, float, float, hipStream_t);
 int stream_norm_max_width(int width);
 template <class T>
 void launch_qkv_prepare(T*, long, int, int, int, const float*, const float*, float, const T*, long, const float*, T*, T*, const int*, long, int, int, hipStream_t);
@@ -70,7 +70,8 @@ void stream_norm(Tensor y, Tensor x, Tensor rows, OptTensor at,
 }
 
 void embed_norm(Tensor y, Tensor x, Tensor table, Tensor tokens,
-                OptTensor w_pre, double off, double eps) {
+                OptTensor w_pre, double off, double eps, double scale,
+                OptTensor pos, OptTensor positions) {
   const int width = table.size(1);
   const long rows = tokens.numel();
   check(x, torch::kFloat32, "x");
@@ -82,14 +83,25 @@ void embed_norm(Tensor y, Tensor x, Tensor table, Tensor tokens,
     check(*w_pre, torch::kFloat32, "w_pre");
     TORCH_CHECK(w_pre->numel() == width, "embed_norm: shapes differ");
   }
+  TORCH_CHECK(pos.has_value() == positions.has_value(),
+              "positions need their vectors");
+  if (pos) {
+    check(*positions, torch::kInt32, "positions");
+    TORCH_CHECK(positions->numel() == rows && pos->dim() == 2 &&
+                pos->size(0) > 0 && pos->size(1) == width,
+                "embed_norm: shapes differ");
+  }
   if (rows == 0) return;
   by_type(y, [&](auto tag) {
     using T = decltype(tag);
     check(y, Scalar<T>::type, "y");
     check(table, Scalar<T>::type, "table");
+    if (pos) check(*pos, Scalar<T>::type, "pos");
     launch_embed_norm<T>(ptr<T>(y), ptr<float>(x), ptr<T>(table),
-                         ptr<int>(tokens), ptr<float>(w_pre), rows, width,
-                         table.size(0), off, eps, stream());
+                         ptr<int>(tokens), scale, ptr<T>(pos),
+                         ptr<int>(positions), pos ? pos->size(0) : 0,
+                         ptr<float>(w_pre), rows, width, table.size(0), off,
+                         eps, stream());
   });
   post("embed_norm");
 }
@@ -140,7 +152,8 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
               OptTensor bias, OptTensor sink, Tensor positions,
               OptTensor seq_start, Tensor block_table, double scale,
               int64_t chunk, int64_t window, int64_t keep, double cap,
-              double mult, int64_t max_len, int64_t span, bool any) {
+              double mult, int64_t max_len, int64_t span, bool any,
+              OptTensor r1, OptTensor r2, OptTensor wbias) {
   const int kv = kc.size(1), dim = kc.size(3), vdim = vc.size(3);
   const long rows = q.size(0);
   TORCH_CHECK(q.size(1) % dim == 0, "q is not heads * dim wide");
@@ -170,6 +183,13 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     check(*sink, torch::kFloat32, "sink");
     TORCH_CHECK(sink->numel() == heads, "sink heads");
   }
+  TORCH_CHECK(r1.has_value() == r2.has_value(), "r1 needs r2");
+  for (const OptTensor* t : {&r1, &r2, &wbias})
+    if (*t) {
+      check(**t, torch::kFloat32, "numbers per head");
+      TORCH_CHECK((*t)->numel() == heads, "one number per head");
+    }
+  TORCH_CHECK(!wbias || !sink, "sigmoid weights have no sink");
   TORCH_CHECK(chunk == 0 || window == 0, "a chunk or a window, not both");
   if (rows == 0) return;
   by_type(q, [&](auto tag) {
@@ -201,6 +221,8 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
     a.max_blocks = block_table.size(1); a.block_size = kc.size(2);
     a.scale = scale;
     a.sink = ptr<float>(sink);
+    a.r1 = ptr<float>(r1); a.r2 = ptr<float>(r2);
+    a.wbias = ptr<float>(wbias);
     a.window = window; a.keep = window > 0 ? keep : 0;
     a.cap = cap; a.mult = mult;
     a.out_ld = out.stride(0);
@@ -212,8 +234,8 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
           reinterpret_cast<uintptr_t>(a.q) % 16 == 0;
       any = any || v_ld % 8 != 0;
       if (!any && aligned && kv == 1 && a.kc == a.vc && v_ld == dim && !bias &&
-          !gate && chunk == 0 && window == 0 && !sink && cap == 0 &&
-          mult == 1 && out.is_contiguous() &&
+          !gate && chunk == 0 && a.keep == 0 && !sink && !r1 && !wbias &&
+          cap == 0 && mult == 1 && out.is_contiguous() &&
           attn_latent_supported(dim, vdim, a.block_size)) {
         const int longest = seq_start ? max_len : 1;
         const int splits = attn_latent_splits(entries, longest, heads, span);
@@ -231,7 +253,7 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
                                 ptr<float>(pml), stream());
         return;
       }
-      if (!any && seq_start && aligned &&
+      if (!any && seq_start && aligned && !(wbias && cap > 0) &&
           attn_ctx_prefill_supported(dim, vdim, a.block_size)) {
         launch_attn_ctx_prefill(a, entries, max_len, stream());
         return;
@@ -260,10 +282,13 @@ void attn_ctx(Tensor out, Tensor q, OptTensor gate, Tensor kc, Tensor vc,
 
 // Portions over keys and values that lie unpaged, ctx_start[e + 1] -
 // ctx_start[e] of them per entry: kv rows [keys of all heads | values of all
-// heads], kr rows the key part that follows every head's own. gate by column.
+// heads], kr rows the key part that follows every head's own. With a window,
+// an entry's first key is the first that its rows see. gate by column or by
+// head.
 void attn_flat(Tensor out, Tensor q, OptTensor gate, Tensor kv, Tensor kr,
                Tensor positions, Tensor seq_start, Tensor ctx_start,
-               int64_t heads, int64_t vdim, double scale, int64_t max_len) {
+               int64_t heads, int64_t vdim, double scale, int64_t window,
+               int64_t max_len) {
   using T = bf16_t;
   const long rows = q.size(0), entries = seq_start.numel() - 1;
   const long dim = q.size(1) / heads, shared = kr.size(1);
@@ -288,10 +313,12 @@ void attn_flat(Tensor out, Tensor q, OptTensor gate, Tensor kv, Tensor kr,
               "attn_flat: sizes must be multiples of 8");
   if (gate) {
     check_rows(*gate, Scalar<T>::type, "gate");
-    TORCH_CHECK(gate->size(0) == rows && gate->size(1) == heads * vdim &&
-                gate->stride(0) % 4 == 0 &&
-                reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0,
-                "gate must be [rows, heads * vdim]");
+    a.gate_each = gate->size(1) == heads * vdim;
+    TORCH_CHECK(gate->size(0) == rows &&
+                (gate->size(1) == heads ||
+                 (a.gate_each && gate->stride(0) % 4 == 0 &&
+                  reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0)),
+                "gate must be [rows, heads * vdim] or [rows, heads]");
   }
   if (rows == 0) return;
   a.out = ptr<T>(out); a.q = ptr<T>(q); a.gate = ptr<T>(gate);
@@ -301,37 +328,45 @@ void attn_flat(Tensor out, Tensor q, OptTensor gate, Tensor kv, Tensor kr,
   a.q_ld = q.stride(0); a.g_ld = gate ? gate->stride(0) : 0;
   a.v_ld = kv.size(1);
   a.heads = a.kv_heads = heads; a.nbias = 1; a.block_size = 16;
-  a.scale = scale; a.mult = 1.f;
+  a.scale = scale; a.mult = 1.f; a.window = window;
   a.out_ld = out.stride(0); a.quads = vdim % 4 == 0;
   launch_attn_ctx_prefill(a, entries, max_len, stream());
   post("attn_flat");
 }
 
-// c [keys, rank] and kr [keys, rot] of whole contexts, entry by entry
+// c [keys, rank] and kr [keys, rot] of what portions see, entry by entry
 void latent_gather(Tensor c, Tensor kr, Tensor cache, Tensor block_table,
-                   Tensor ctx_start) {
+                   Tensor ctx_start, Tensor positions, Tensor seq_start,
+                   int64_t window, int64_t max_len) {
   check(block_table, torch::kInt32, "block_table");
+  check(positions, torch::kInt32, "positions");
+  check(seq_start, torch::kInt32, "seq_start");
   check(ctx_start, torch::kInt32, "ctx_start");
   check(c, cache.scalar_type(), "c");
   check(kr, cache.scalar_type(), "kr");
   check(cache, cache.scalar_type(), "cache");
   const int entries = block_table.size(0);
   TORCH_CHECK(cache.size(1) == 1 && cache.size(3) == c.size(1) + kr.size(1) &&
-              c.size(0) == kr.size(0) && ctx_start.numel() == entries + 1,
+              c.size(0) == kr.size(0) && ctx_start.numel() == entries + 1 &&
+              seq_start.numel() == entries + 1,
               "latent_gather: shapes differ");
   if (entries == 0) return;
   launch_latent_gather(c.data_ptr(), kr.data_ptr(), cache.data_ptr(),
                        cache.element_size(), c.size(1), kr.size(1),
                        ptr<int>(block_table), block_table.size(1),
-                       ptr<int>(ctx_start), entries, cache.size(2), stream());
+                       ptr<int>(ctx_start), ptr<int>(positions),
+                       ptr<int>(seq_start), window, max_len, entries,
+                       cache.size(2), stream());
   post("latent_gather");
 }
 
 // buf rows [queries | ... | latent | key part], the latter from column c_at
-// on, or nowhere (-1); cache [blocks, 1, block, rank + rot_dim]
+// on, or nowhere (-1); cache [blocks, 1, block, rank + rot_dim]. With q_norm,
+// rows begin with the latent that queries are made of.
 void latent_prepare(Tensor buf, int64_t heads, int64_t dim, int64_t rot_dim,
                     int64_t c_at, OptTensor norm, double eps, Tensor turns,
-                    Tensor positions, Tensor cache, Tensor slots) {
+                    Tensor positions, Tensor cache, Tensor slots,
+                    OptTensor q_norm) {
   const long rows = buf.size(0);
   const int half = turns.numel(), row = cache.size(3);
   const int rank = row - rot_dim;
@@ -342,6 +377,11 @@ void latent_prepare(Tensor buf, int64_t heads, int64_t dim, int64_t rot_dim,
               "one position and slot per row");
   TORCH_CHECK(2 * half <= rot_dim && half <= 4096, "too many turns");
   TORCH_CHECK(heads * (dim + rot_dim) <= buf.size(1), "buf too narrow");
+  if (q_norm) {
+    check(*q_norm, torch::kFloat32, "q_norm");
+    TORCH_CHECK(heads == 0 && q_norm->numel() <= buf.size(1),
+                "queries' latent: rows too narrow, or heads beside it");
+  }
   TORCH_CHECK(rank > 0 && cache.size(1) == 1, "cache must hold latents");
   TORCH_CHECK((c_at >= 0) == norm.has_value(), "latents need their norm");
   if (norm) {
@@ -357,7 +397,9 @@ void latent_prepare(Tensor buf, int64_t heads, int64_t dim, int64_t rot_dim,
     launch_latent_prepare<T>(ptr<T>(buf), buf.stride(0), heads, dim, rot_dim,
                              c_at, rank, ptr<float>(norm), eps,
                              ptr<double>(turns), half, ptr<int>(positions),
-                             ptr<T>(cache), ptr<int>(slots), rows, stream());
+                             ptr<T>(cache), ptr<int>(slots),
+                             ptr<float>(q_norm), q_norm ? q_norm->numel() : 0,
+                             rows, stream());
   });
   post("latent_prepare");
 }
@@ -397,8 +439,9 @@ void head_linear(Tensor out, Tensor x, Tensor w, OptTensor gate,
   TORCH_CHECK(out.dim() == 3 && out.size(0) == rows && out.size(1) == heads &&
               out.size(2) == n + tail, "out must be [rows, heads, n + tail]");
   if (gate)
-    TORCH_CHECK(gate->size(0) == rows && gate->size(1) == heads * n,
-                "gate must be [rows, heads * n]");
+    TORCH_CHECK(gate->size(0) == rows && (gate->size(1) == heads * n ||
+                                          gate->size(1) == heads),
+                "gate must be [rows, heads * n] or [rows, heads]");
   if (rows == 0) return;
   by_type(x, [&](auto tag) {
     using T = decltype(tag);
@@ -415,7 +458,9 @@ void head_linear(Tensor out, Tensor x, Tensor w, OptTensor gate,
     if (gate) {
       check_rows(*gate, Scalar<T>::type, "gate");
       a.act = Act::GATE;
-      a.gate = ptr<T>(gate); a.gate_ld = gate->stride(0); a.gate_gs = n;
+      a.gate = ptr<T>(gate); a.gate_ld = gate->stride(0);
+      a.gate_each = gate->size(1) == heads * n;
+      a.gate_gs = a.gate_each ? n : 1;
     }
     group_gemm(a, group_gemm_tile(rows, 1, std::is_same_v<T, bf16_t>, k),
                "head_linear");
@@ -486,7 +531,8 @@ Tensor linear32(Tensor x, Tensor w) {
 }
 
 void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
-                int64_t keep, OptTensor bias, bool over_chosen) {
+                int64_t keep, OptTensor bias, bool over_chosen, bool sigmoid,
+                OptTensor correction, int64_t group_best) {
   TORCH_CHECK(z.dim() == 3, "z must be [splits, rows, experts]");
   const long rows = z.size(1), experts = z.size(2), top = ids.size(1);
   check(ids, torch::kInt32, "ids");
@@ -499,13 +545,21 @@ void moe_select(Tensor ids, Tensor weights, Tensor z, int64_t groups,
     check(*bias, torch::kFloat32, "bias");
     TORCH_CHECK(bias->numel() == experts, "one bias per expert");
   }
+  if (correction) {
+    check(*correction, torch::kFloat32, "correction");
+    TORCH_CHECK(correction->numel() == experts, "one correction per expert");
+  }
+  TORCH_CHECK(group_best == 1 || group_best == 2,
+              "a group's score is its best one or two");
+  TORCH_CHECK(!(sigmoid && over_chosen), "sigmoid scores have no sum");
   TORCH_CHECK(groups > 0 && experts % groups == 0 && keep > 0 &&
               keep <= groups && top > 0 && top <= experts / groups * keep,
               "moe_select: cannot choose so many");
   if (rows == 0) return;
   launch_moe_select(ptr<int>(ids), ptr<float>(weights), ptr<float>(z),
                     z.size(0), rows, experts, top, groups, keep,
-                    ptr<float>(bias), over_chosen, stream());
+                    ptr<float>(bias), over_chosen, sigmoid,
+                    ptr<float>(correction), group_best, stream());
   post("moe_select");
 }
 
@@ -603,7 +657,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("side_gate", &side_gate);
   m.def("moe_select", &moe_select, py::arg("ids"), py::arg("weights"),
         py::arg("z"), py::arg("groups"), py::arg("keep"),
-        py::arg("bias") = py::none(), py::arg("over_chosen") = false);
+        py::arg("bias") = py::none(), py::arg("over_chosen") = false,
+        py::arg("sigmoid") = false, py::arg("correction") = py::none(),
+        py::arg("group_best") = 1);
   m.def("moe_tile", &moe_tile);
   m.def("moe_sort", &moe_sort);
   m.def("expert_linear", &expert_linear);

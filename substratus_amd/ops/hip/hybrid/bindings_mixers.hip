@@ -216,6 +216,39 @@ void conv_rope(Tensor q, Tensor x, OptTensor in_bias, Tensor weight,
   post("conv_rope");
 }
 
+void conv_qkv(Tensor q, Tensor x, OptTensor in_bias, Tensor weight,
+              Tensor state, Tensor state_slots, Tensor kc, Tensor vc,
+              Tensor positions, Tensor slots, OptTensor seq_start, double temp,
+              int64_t every, double v_eps, int64_t max_len) {
+  const long rows = x.size(0), kv = kc.size(1), dim = kc.size(3),
+             vdim = vc.size(3);
+  const int entries = check_entries(state_slots, positions, seq_start, rows);
+  check(slots, torch::kInt32, "slots");
+  TORCH_CHECK(slots.numel() == rows, "one slot per row");
+  TORCH_CHECK(kc.size(0) == vc.size(0) && kv == vc.size(1) &&
+              kc.size(2) == vc.size(2), "caches differ");
+  TORCH_CHECK(every > 0 && every < 1l << 31, "a temperature's steps");
+  TORCH_CHECK(conv_qkv_takes(vdim), "values too wide");
+  if (rows == 0) return;
+  by_type(x, [&](auto tag) {
+    using T = decltype(tag);
+    auto a = conv<T>(x, in_bias, weight, state, state_slots, positions,
+                     seq_start);
+    check(q, Scalar<T>::type, "q");
+    check(kc, Scalar<T>::type, "kc");
+    check(vc, Scalar<T>::type, "vc");
+    const long nq = a.channels - kv * (dim + vdim);
+    TORCH_CHECK(nq > 0 && nq % dim == 0 && q.size(0) == rows &&
+                q.size(1) == nq, "q must be [rows, query heads * dim]");
+    a.q = ptr<T>(q); a.kc = ptr<T>(kc); a.vc = ptr<T>(vc);
+    a.slots = ptr<int>(slots);
+    a.kv = kv; a.dim = dim; a.vdim = vdim; a.block_size = kc.size(2);
+    a.temp = temp; a.every = every; a.v_eps = v_eps;
+    launch_conv_qkv<T>(a, entries, seq_start ? max_len : 1, stream());
+  });
+  post("conv_qkv");
+}
+
 void selective_scan(Tensor out, Tensor u, Tensor gate, Tensor z, Tensor zb,
                     Tensor low, int64_t b_at, Tensor a_, Tensor d,
                     Tensor state, Tensor state_slots, Tensor positions,
@@ -426,6 +459,7 @@ void bind_mixers(pybind11::module& m) {
   m.def("rope_table", &rope_table);
   m.def("short_conv", &short_conv);
   m.def("conv_rope", &conv_rope);
+  m.def("conv_qkv", &conv_qkv);
   m.def("selective_scan", &selective_scan);
   m.def("delta", &delta);
   m.def("gla", &gla);

@@ -13,7 +13,7 @@
 enum class Act {
   NONE,
   GELU,      // exact gelu
-  GATE,      // times sigmoid(gate[row][g][n])
+  GATE,      // times sigmoid(gate[row][g][n]), or sigmoid(gate[row][g])
   SIDE,      // gelu_tanh, times table[tokens[row]][n]
   GLU,       // columns are gate and up in turn; y has half as many
 };
@@ -34,7 +34,8 @@ struct GroupGemm {
   const int* tiles;
   int max_tiles;           // bound of tiles[0]
   const T* gate;           // row r, group g, column n at
-  long gate_ld, gate_gs;   //   gate + r * gate_ld + g * gate_gs + n
+  long gate_ld, gate_gs;   //   gate + r * gate_ld + g * gate_gs + n,
+  bool gate_each;          //   or not each column: without n
   const int* tokens;
   const T* table;          // row t at table + t * t_ld
   long t_ld;
@@ -83,8 +84,16 @@ template <Act ACT, bool FAST, int N, class T, class Y>
 DEV_INLINE void group_act(const GroupGemm<T, Y>& a, int r, int g, int n,
                           float* v) {
   float f[N];
-  if constexpr (ACT == Act::GATE)
-    ldv<N>(a.gate + (long)r * a.gate_ld + (long)g * a.gate_gs + n, f);
+  if constexpr (ACT == Act::GATE) {
+    const T* p = a.gate + (long)r * a.gate_ld + (long)g * a.gate_gs;
+    if (a.gate_each) {
+      ldv<N>(p + n, f);
+    } else {
+      f[0] = ld1(p);
+      #pragma unroll
+      for (int j = 1; j < N; ++j) f[j] = f[0];
+    }
+  }
   if constexpr (ACT == Act::SIDE) {
     const int t = min(max(a.tokens[r], 0), a.vocab - 1);
     ldv<N>(a.table + (long)t * a.t_ld + n, f);

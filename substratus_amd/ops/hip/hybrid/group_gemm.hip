@@ -217,8 +217,9 @@ bool by_quads(const GroupGemm<T, Y>& a) {
     return a.n % 4 == 0 && a.y_ld % 2 == 0 && a.y_gs % 2 == 0 &&
            reinterpret_cast<uintptr_t>(a.y) % (2 * sizeof(Y)) == 0;
   return a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0 &&
-         ok(a.y, sizeof(Y)) && a.gate_ld % 4 == 0 && a.gate_gs % 4 == 0 &&
-         ok(a.gate, sizeof(T)) && a.t_ld % 4 == 0 && ok(a.table, sizeof(T));
+         ok(a.y, sizeof(Y)) &&
+         (!a.gate_each || (a.gate_ld % 4 == 0 && a.gate_gs % 4 == 0 &&
+                           ok(a.gate, sizeof(T)))) && a.t_ld % 4 == 0 && ok(a.table, sizeof(T));
 }
 
 template <class T, class Y>

@@ -3,7 +3,9 @@
 //   select   one wave per token: scores (sums of a product's shares of the
 //            inner dimension), softmax over all experts, the best groups
 //            of neighbours, the best experts of those; all in 32 bits.
-//            Or the softmax is over the chosen experts only.
+//            Or the softmax is over the chosen experts only, or every score
+//            is a sigmoid. What is best may go by scores with a correction,
+//            a group by the sum of its two best.
 //   sort     one workgroup: token rows packed by expert, and every expert's
 //            rows cut into tiles for the grouped products. The order of an
 //            expert's rows is left to chance: no row's result depends on it,
@@ -34,7 +36,9 @@ __global__ __launch_bounds__(SW * WAVE)
 void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
                        const float* __restrict__ z, int splits, int rows,
                        int experts, int top, int groups, int keep,
-                       const float* __restrict__ bias, bool over_chosen) {
+                       const float* __restrict__ bias, bool over_chosen,
+                       bool sigmoid, const float* __restrict__ correction,
+                       int group_best) {
   extern __shared__ float4 s_all[];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int pad = (experts + 3) / 4 * 4;
@@ -42,7 +46,7 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
   float* s_z = reinterpret_cast<float*>(s_all) + wave * 2 * pad;
   float* s_g = s_z + pad;                       // best score of each group
   const int size = experts / groups;
-  float v[PL];
+  float v[PL], sc[PL];                          // for the choice, as weights
   float mx = -INFINITY;
   // scores that are no numbers: weights are none either, but experts are
   for (int r = lane; r < top; r += WAVE) ids[row * top + r] = 0;
@@ -55,15 +59,18 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
       for (int s = 1; s < splits; ++s)
         v[i] += z[((long)s * rows + row) * experts + e];
       if (bias != nullptr) v[i] += bias[e];
+      if (sigmoid) v[i] = sigmoid_f(v[i]);
     }
-    if (e < pad) s_z[e] = v[i];
+    sc[i] = v[i];
     mx = fmaxf(mx, v[i]);
+    if (e < experts && correction != nullptr) v[i] += correction[e];
+    if (e < pad) s_z[e] = v[i];
   }
   mx = wave_max(mx);
   float sum = 0.f;
   #pragma unroll
   for (int i = 0; i < PL; ++i)
-    if (lane + i * WAVE < experts) sum += expf(v[i] - mx);
+    if (lane + i * WAVE < experts) sum += expf(sc[i] - mx);
   sum = wave_sum(sum);
   __syncthreads();
 
@@ -74,7 +81,15 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
       g[i] = -INFINITY;
       const int n = lane + i * WAVE;
       if (n < groups)
-        for (int e = 0; e < size; ++e) g[i] = fmaxf(g[i], s_z[n * size + e]);
+      {
+        float next = -INFINITY;
+        for (int e = 0; e < size; ++e) {
+          const float s = s_z[n * size + e];
+          next = fmaxf(next, fminf(g[i], s));
+          g[i] = fmaxf(g[i], s);
+        }
+        if (group_best > 1 && size > 1) g[i] += next;
+      }
       if (n < pad) s_g[n] = g[i];
     }
     __syncthreads();
@@ -104,14 +119,15 @@ void moe_select_kernel(int* __restrict__ ids, float* __restrict__ weights,
   for (int i = 0; i < PL; ++i) {
     const int e = lane + i * WAVE;
     r[i] = e < experts ? rank_of(s_z, experts, v[i], e) : top;
-    if (r[i] < top) chosen += expf(v[i] - mx);
+    if (r[i] < top) chosen += expf(sc[i] - mx);
   }
   if (over_chosen) sum = wave_sum(chosen);
   #pragma unroll
   for (int i = 0; i < PL; ++i) {
     if (r[i] < top) {
       ids[row * top + r[i]] = lane + i * WAVE;
-      weights[row * top + r[i]] = expf(v[i] - mx) / sum;
+      weights[row * top + r[i]] =
+          sigmoid ? sc[i] : expf(sc[i] - mx) / sum;
     }
   }
 }
@@ -170,14 +186,15 @@ int moe_max_experts() { return SORT; }
 
 void launch_moe_select(int* ids, float* weights, const float* z, int splits,
                        int rows, int experts, int top, int groups, int keep,
-                       const float* bias, bool over_chosen,
+                       const float* bias, bool over_chosen, bool sigmoid,
+                       const float* correction, int group_best,
                        hipStream_t stream) {
   auto go = [&](auto pl) {
     moe_select_kernel<decltype(pl)::value>
         <<<dim3((rows + SW - 1) / SW), dim3(SW * WAVE),
            SW * 2 * ((experts + 3) / 4 * 4) * sizeof(float), stream>>>(
             ids, weights, z, splits, rows, experts, top, groups, keep, bias,
-            over_chosen);
+            over_chosen, sigmoid, correction, group_best);
   };
   if (experts <= WAVE) go(std::integral_constant<int, 1>{});
   else if (experts <= 4 * WAVE) go(std::integral_constant<int, 4>{});

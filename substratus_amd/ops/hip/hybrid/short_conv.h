@@ -27,10 +27,18 @@ struct Conv {
   const float* rope;       // [rows, half, 2]: cosine, sine
   const int* slots;        // [rows]
   int half, kv, dim, block_size;
+  // queries, keys and values: vc [blocks, kv, block_size, vdim]
+  int vdim;
+  float temp;              // q times 1 + temp ln(floor((p + 1) / every) + 1)
+  int every;
+  float v_eps;             // values over their root mean square, < 0: not
 };
 
 template <class T>
 void launch_short_conv(const Conv<T>&, int entries, int max_len, hipStream_t);
+bool conv_qkv_takes(int vdim);
+template <class T>
+void launch_conv_qkv(const Conv<T>&, int entries, int max_len, hipStream_t);
 template <class T>
 void launch_conv_rope(const Conv<T>&, int entries, int max_len, hipStream_t);
 void launch_rope_table(float* out, const int* positions, const double* turns,

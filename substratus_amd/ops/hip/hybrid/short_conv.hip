@@ -12,6 +12,9 @@
 //   conv_rope    rows are [q | k]: y of k is the value and goes to its cache;
 //                then neighbouring elements of both turn by the row's angles,
 //                q to rows of its own, k to its cache
+//   conv_qkv     rows are [q | k | v]: q times its position's temperature to
+//                rows of its own, k to its cache, v over the root mean square
+//                of its head to its cache
 #include "short_conv.h"
 
 namespace {
@@ -41,7 +44,8 @@ DEV_INLINE void st_n(T* p, int n, const float* f) {
   }
 }
 
-// Channels c .. c + n - 1, tokens [t0, t0 + run) of entry e;
+// Channels c .. c + n - 1 (n 0: goes along, leaves no state), tokens
+// [t0, t0 + run) of entry e;
 // emit(row, y, look(row)), where look reads memory ahead of emit's writes.
 // TAPS 0: any number, inputs are read again for every tap.
 template <int VEC, int TAPS, class T, class L, class F>
@@ -128,7 +132,7 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
       emit(en.row0 + t, y, look(en.row0 + t));
     }
   }
-  if (t0 == 0 && state != nullptr) {
+  if (t0 == 0 && state != nullptr && n > 0) {
     // rows move towards the front: each is read before it is written
     for (int k = 0; k < held; ++k) {
       const int s = en.n - held + k;
@@ -213,6 +217,95 @@ void conv_rope_kernel(Conv<T> a, int run) {
   });
 }
 
+// Place of a row's key or value in the cache.
+struct Place {
+  int page, at;
+};
+
+template <class T>
+DEV_INLINE Place place_of(const Conv<T>& a, long row) {
+  const unsigned slot = a.slots[row], size = a.block_size;
+  return {(int)(slot / size), (int)(slot % size)};
+}
+
+// The first nqk workgroups have the queries and keys, VEC elements of a head
+// per thread. Every later one has BLOCK / lanes heads of values, whose threads
+// (a power of two; more than a wave: the workgroup) sum squares together.
+template <class T, int VEC, int TAPS>
+__global__ __launch_bounds__(BLOCK)
+void conv_qkv_kernel(Conv<T> a, int run, int nqk, int lanes) {
+  const int tid = threadIdx.x;
+  const int nq = (a.channels - a.kv * (a.dim + a.vdim)) / a.dim;
+  if ((int)blockIdx.x < nqk) {
+    const int per = (a.dim + VEC - 1) / VEC;
+    const int i = blockIdx.x * BLOCK + tid;
+    if (i >= (nq + a.kv) * per) return;
+    const int head = i / per, d = i % per * VEC;
+    const int n = VEC == 4 ? 4 : min(VEC, a.dim - d);
+    const bool key = head >= nq;
+    struct Seen {
+      Place to;
+      float f;
+    };
+    convolve<VEC, TAPS>(a, blockIdx.z, head * a.dim + d, n, blockIdx.y * run,
+                        run, [&](long row) {
+      Seen s{{0, 0}, 1.f};
+      if (key)
+        s.to = place_of(a, row);
+      else if (a.temp != 0.f)
+        s.f = 1.f + a.temp * log1pf((float)(
+            (unsigned)(a.positions[row] + 1) / (unsigned)a.every));
+      return s;
+    }, [&](long row, float* y, const Seen& s) {
+      if (key) {
+        st_n<VEC>(a.kc + (((long)s.to.page * a.kv + head - nq) * a.block_size +
+                          s.to.at) * a.dim + d, n, y);
+      } else {
+        #pragma unroll
+        for (int j = 0; j < VEC; ++j) y[j] *= s.f;
+        st_n<VEC>(a.q + row * nq * a.dim + head * a.dim + d, n, y);
+      }
+    });
+    return;
+  }
+  __shared__ float s_sum[2][BLOCK / WAVE];
+  int turn = 0;
+  const int i = (blockIdx.x - nqk) * BLOCK + tid;
+  const int head = i / lanes, d = i % lanes * VEC;
+  // threads past the end go along: they take part in sums
+  const bool mine = head < a.kv && d < a.vdim;
+  const int n = !mine ? 0 : VEC == 4 ? 4 : min(VEC, a.vdim - d);
+  const int c = (nq + a.kv) * a.dim + (mine ? head * a.vdim + d : 0);
+  convolve<VEC, TAPS>(a, blockIdx.z, c, n, blockIdx.y * run, run,
+                      [&](long row) { return place_of(a, row); },
+                      [&](long row, float* y, const Place& to) {
+    if (a.v_eps >= 0.f) {
+      float ss = 0.f;
+      #pragma unroll
+      for (int j = 0; j < VEC; ++j)
+        if (j < n) ss += y[j] * y[j];
+      for (int off = 1; off < min(lanes, WAVE); off <<= 1)
+        ss += __shfl_xor(ss, off, WAVE);
+      if (lanes > WAVE) {
+        // two rooms in turn: a token's sums are read before the next but one
+        // writes there
+        if (tid % WAVE == 0) s_sum[turn][tid / WAVE] = ss;
+        __syncthreads();
+        ss = 0.f;
+        #pragma unroll
+        for (int w = 0; w < BLOCK / WAVE; ++w) ss += s_sum[turn][w];
+        turn ^= 1;
+      }
+      const float f = 1.f / sqrtf(ss / (float)a.vdim + a.v_eps);
+      #pragma unroll
+      for (int j = 0; j < VEC; ++j) y[j] *= f;
+    }
+    if (mine)
+      st_n<VEC>(a.vc + (((long)to.page * a.kv + head) * a.block_size + to.at) *
+                       a.vdim + d, n, y);
+  });
+}
+
 __global__ __launch_bounds__(BLOCK)
 void rope_table_kernel(float* __restrict__ out,
                        const int* __restrict__ positions,
@@ -286,6 +379,39 @@ void launch_conv_rope(const Conv<T>& a, int entries, int max_len,
   });
 }
 
+// Threads that share a head's values, VEC elements each; more than a wave's
+// are a whole workgroup.
+static int value_lanes(int vdim, int vec) {
+  int lanes = 1;
+  while (lanes * vec < vdim) lanes *= 2;
+  return lanes > WAVE ? BLOCK : lanes;
+}
+
+bool conv_qkv_takes(int vdim) { return vdim <= 2 * BLOCK; }
+
+template <class T>
+void launch_conv_qkv(const Conv<T>& a, int entries, int max_len,
+                     hipStream_t stream) {
+  auto go = [&](auto vec, auto taps) {
+    constexpr int V = decltype(vec)::value;
+    const int units = (a.channels - a.kv * a.vdim) / a.dim *
+                      ((a.dim + V - 1) / V);
+    const int lanes = value_lanes(a.vdim, V);
+    const int nqk = (units + BLOCK - 1) / BLOCK;
+    const int nv = (a.kv * lanes + BLOCK - 1) / BLOCK;
+    const int run = run_of(a.taps, max_len,
+                           (long)(units + a.kv * lanes) * entries);
+    conv_qkv_kernel<T, V, decltype(taps)::value>
+        <<<dim3(nqk + nv, (max_len + run - 1) / run, entries), BLOCK, 0,
+           stream>>>(a, run, nqk, lanes);
+  };
+  by_taps(a.taps, [&](auto taps) {
+    if (fours(a) && a.dim % 4 == 0 && a.vdim % 4 == 0)
+      go(std::integral_constant<int, 4>{}, taps);
+    else go(std::integral_constant<int, 2>{}, taps);
+  });
+}
+
 void launch_rope_table(float* out, const int* positions, const double* turns,
                        long rows, int half, hipStream_t stream) {
   rope_table_kernel<<<dim3((rows * half + BLOCK - 1) / BLOCK), BLOCK, 0,
@@ -294,6 +420,7 @@ void launch_rope_table(float* out, const int* positions, const double* turns,
 
 #define INSTANTIATE(T)                                                       \
   template void launch_short_conv<T>(const Conv<T>&, int, int, hipStream_t); \
+  template void launch_conv_qkv<T>(const Conv<T>&, int, int, hipStream_t);   \
   template void launch_conv_rope<T>(const Conv<T>&, int, int, hipStream_t);
 INSTANTIATE(float)
 INSTANTIATE(bf16_t)

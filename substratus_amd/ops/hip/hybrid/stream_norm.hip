@@ -2,7 +2,8 @@
 //
 //   stream_norm   x += mult * rms(delta) * (off + w_post)
 //                 y  = rms(x) * (off + w_pre)
-//   embed_norm    x  = table[token];   y = rms(x) * (off + w_pre)
+//   embed_norm    x  = scale * table[token] + pos[position]
+//                 y  = rms(x) * (off + w_pre)
 //
 // Without w_pre, y is x. delta is a row per token, or the weighted sum of
 // `picks` rows of a pool (what a mixture of experts adds), formed on the way.
@@ -25,6 +26,9 @@ void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
                         int picks,
                         const T* __restrict__ table,     // [vocab, width]
                         const int* __restrict__ tokens,  // [rows]
+                        const T* __restrict__ pos, // [max_pos, width] or null
+                        const int* __restrict__ positions,   // [rows]
+                        int max_pos,
                         const float* __restrict__ w_post,
                         const float* __restrict__ w_pre, int width, int vocab,
                         float off, float eps, float out_scale,
@@ -45,6 +49,15 @@ void stream_norm_kernel(T* __restrict__ y, float* __restrict__ x,
       const int i = threadIdx.x + kk * BLOCK;
       if (i >= nvec) break;
       ldv<VEC>(src + i * VEC, xk[kk]);
+      #pragma unroll
+      for (int j = 0; j < VEC; ++j) xk[kk][j] *= mult;
+      if (pos != nullptr) {
+        const int p = min(max(positions[row], 0), max_pos - 1);
+        float f[VEC];
+        ldv<VEC>(pos + (long)p * width + i * VEC, f);
+        #pragma unroll
+        for (int j = 0; j < VEC; ++j) xk[kk][j] += f[j];
+      }
     }
   } else {
     float dk[RCAP][VEC];
@@ -135,14 +148,15 @@ int stream_norm_max_width(int width) {
 template <class T, Source SRC>
 static void launch(T* y, float* x, const T* delta, const int* at,
                    const float* wt, int picks, const T* table,
-                   const int* tokens, const float* w_post, const float* w_pre,
+                   const int* tokens, const T* pos, const int* positions,
+                   int max_pos, const float* w_post, const float* w_pre,
                    long rows, int width, int vocab, float off, float eps,
                    float out_scale, float mult, hipStream_t stream) {
   auto go = [&](auto vec, auto block) {
     constexpr int V = decltype(vec)::value, B = decltype(block)::value;
     stream_norm_kernel<T, V, B, SRC><<<dim3(rows), dim3(B), 0, stream>>>(
-        y, x, delta, at, wt, picks, table, tokens, w_post, w_pre, width,
-        vocab, off, eps, out_scale, mult);
+        y, x, delta, at, wt, picks, table, tokens, pos, positions, max_pos,
+        w_post, w_pre, width, vocab, off, eps, out_scale, mult);
   };
   using std::integral_constant;
   auto by_block = [&](auto vec) {
@@ -163,27 +177,31 @@ void launch_stream_norm(T* y, float* x, const T* delta, const int* at,
                         float eps, float out_scale, float mult,
                         hipStream_t stream) {
   if (at == nullptr)
-    launch<T, ROW>(y, x, delta, at, wt, picks, nullptr, nullptr, w_post,
-                   w_pre, rows, width, 0, off, eps, out_scale, mult, stream);
+    launch<T, ROW>(y, x, delta, at, wt, picks, nullptr, nullptr, nullptr,
+                   nullptr, 0, w_post, w_pre, rows, width, 0, off, eps,
+                   out_scale, mult, stream);
   else
-    launch<T, PICKED>(y, x, delta, at, wt, picks, nullptr, nullptr, w_post,
-                      w_pre, rows, width, 0, off, eps, out_scale, mult,
-                      stream);
+    launch<T, PICKED>(y, x, delta, at, wt, picks, nullptr, nullptr, nullptr,
+                      nullptr, 0, w_post, w_pre, rows, width, 0, off, eps,
+                      out_scale, mult, stream);
 }
 
 template <class T>
 void launch_embed_norm(T* y, float* x, const T* table, const int* tokens,
-                       const float* w_pre, long rows, int width, int vocab,
-                       float off, float eps, hipStream_t stream) {
-  launch<T, EMBED>(y, x, nullptr, nullptr, nullptr, 0, table, tokens, nullptr,
-                   w_pre, rows, width, vocab, off, eps, 1.f, 1.f, stream);
+                       float scale, const T* pos, const int* positions,
+                       int max_pos, const float* w_pre, long rows, int width,
+                       int vocab, float off, float eps, hipStream_t stream) {
+  launch<T, EMBED>(y, x, nullptr, nullptr, nullptr, 0, table, tokens, pos,
+                   positions, max_pos, nullptr, w_pre, rows, width, vocab, off,
+                   eps, 1.f, scale, stream);
 }
 
 #define INSTANTIATE(T)                                                        \
   template void launch_stream_norm<T>(T*, float*, const T*, const int*,       \
       const float*, int, const float*, const float*, long, int, float, float, \
       float, float, hipStream_t);                                             \
-  template void launch_embed_norm<T>(T*, float*, const T*, const int*,        \
-      const float*, long, int, int, float, float, hipStream_t);
+  template void launch_embed_norm<T>(T*, float*, const T*, const int*, float, \
+      const T*, const int*, int, const float*, long, int, int, float, float,  \
+      hipStream_t);
 INSTANTIATE(float)
 INSTANTIATE(bf16_t)

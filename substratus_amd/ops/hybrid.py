@@ -61,16 +61,23 @@ def stream_norm(delta: Union[torch.Tensor, Picked], x: torch.Tensor,
 
 
 def embed_norm(tokens: torch.Tensor, table: torch.Tensor,
-               w_pre: Optional[torch.Tensor], offset: float,
-               eps: float) -> tuple[torch.Tensor, torch.Tensor]:
-    """x = table[tokens] (float32) and rms(x) * (offset + w_pre), or without
-    w_pre x itself, in the table's dtype; tokens int32."""
+               w_pre: Optional[torch.Tensor], offset: float, eps: float,
+               scale: float = 1.0, pos: Optional[torch.Tensor] = None,
+               positions: Optional[torch.Tensor] = None
+               ) -> tuple[torch.Tensor, torch.Tensor]:
+    """x = scale * table[tokens] + pos[positions] (float32; without pos, the
+    former) and rms(x) * (offset + w_pre), or without w_pre x itself, in the
+    table's dtype; tokens and positions int32."""
+    if pos is None:
+        positions = None
     if not table.is_cuda:
-        return ref.embed_norm(tokens, table, w_pre, offset, eps)
+        return ref.embed_norm(tokens, table, w_pre, offset, eps, scale, pos,
+                              positions)
     shape = (tokens.shape[0], table.shape[1])
     x = torch.empty(shape, dtype=torch.float32, device=table.device)
     y = torch.empty(shape, dtype=table.dtype, device=table.device)
-    _ext().embed_norm(y, x, table, tokens, w_pre, offset, eps)
+    _ext().embed_norm(y, x, table, tokens, w_pre, offset, eps, scale, pos,
+                      positions)
     return x, y
 
 
@@ -94,8 +101,9 @@ def attn_ctx(q: torch.Tensor, gate: Optional[torch.Tensor],
              bias: Optional[torch.Tensor], batch, scale: float, chunk: int = 0,
              any_size: bool = False, window: int = 0, keep: int = 0,
              softcap: float = 0.0, sink: Optional[torch.Tensor] = None,
-             mult: float = 1.0,
-             out: Optional[torch.Tensor] = None) -> torch.Tensor:
+             mult: float = 1.0, out: Optional[torch.Tensor] = None,
+             falloff: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
+             weight_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of a batch's rows over the paged cache, which already holds
     their own keys and values.
 
@@ -105,8 +113,11 @@ def attn_ctx(q: torch.Tensor, gate: Optional[torch.Tensor],
     chunk > 0: rows see keys of their own chunk of positions only. window > 0:
     rows see that many keys up to their own, and the first `keep`. softcap > 0:
     scores are cap * tanh(score / cap) ahead of the bias. sink [heads]: a score
-    in the softmax that has no value. mult multiplies the result. any_size
-    takes the untiled kernel on the GPU."""
+    in the softmax that has no value. mult multiplies the result. falloff
+    (r1, r2), both [heads]: r1 ln(1 + r2 distance) is taken off the score.
+    weight_bias [heads]: a key's weight is sigmoid(score + weight_bias), each
+    by itself, instead of a softmax. any_size takes the untiled kernel on the
+    GPU."""
     heads = q.shape[1] // k_cache.shape[3]
     if out is None:
         out = q.new_empty(q.shape[0], heads * v_cache.shape[3])
@@ -116,25 +127,28 @@ def attn_ctx(q: torch.Tensor, gate: Optional[torch.Tensor],
     if window:
         span = min(window + keep, span)
     fn = _ext().attn_ctx if q.is_cuda else ref.attn_ctx
+    r1, r2 = falloff or (None, None)
     for rows, ents, seq_start, max_len in batch.parts():
         fn(out[rows], q[rows], None if gate is None else gate[rows], k_cache,
            v_cache, bias, sink, batch.positions[rows], seq_start,
            batch.block_table[ents], scale, chunk, window, keep, softcap, mult,
-           max_len, span, any_size)
+           max_len, span, any_size, r1, r2, weight_bias)
     return out
 
 
 def latent_prepare(buf: torch.Tensor, spec, c_at: int,
                    norm: Optional[torch.Tensor], eps: float,
                    turns: torch.Tensor, positions: torch.Tensor,
-                   cache: torch.Tensor, slots: torch.Tensor) -> None:
+                   cache: torch.Tensor, slots: torch.Tensor,
+                   q_norm: Optional[torch.Tensor] = None) -> None:
     """buf rows begin with queries, head by head [dim, rot_dim], and have
     [latent, rotated key part] from column c_at on (-1: not). Rotates the
     queries in place, writes the normed latent and the rotated key part to
-    the cache."""
+    the cache. q_norm: rows begin with the queries' latent instead, which is
+    normed in place."""
     fn = _ext().latent_prepare if buf.is_cuda else ref.latent_prepare
-    fn(buf, spec.heads, spec.dim, spec.rot_dim, c_at, norm, eps, turns,
-       positions, cache, slots)
+    fn(buf, 0 if q_norm is not None else spec.heads, spec.dim, spec.rot_dim,
+       c_at, norm, eps, turns, positions, cache, slots, q_norm)
 
 
 def head_linear(x: torch.Tensor, w: torch.Tensor,
@@ -145,8 +159,8 @@ def head_linear(x: torch.Tensor, w: torch.Tensor,
     the `tail` elements that follow in x are appended as they are.
 
     x [rows, heads, k + tail] may be a view of wider rows; w [heads, n, k];
-    gate [rows, heads * n]. Returns [rows, heads, n + tail]; out: contiguous
-    room for it."""
+    gate [rows, heads * n] or [rows, heads]. Returns [rows, heads, n + tail];
+    out: contiguous room for it."""
     shape = (x.shape[0], w.shape[0], w.shape[1] + tail)
     out = x.new_empty(shape) if out is None else out.view(shape)
     (_ext() if x.is_cuda else ref).head_linear(out, x, w, gate, tail)
@@ -164,25 +178,29 @@ def _latent_absorbed(out, q, gate, cache, w_uv, uk_t, batch, rows, ents,
     fn = _ext().attn_ctx if q.is_cuda else ref.attn_ctx
     fn(o, qa.view(n, -1), None, cache, cache[..., :spec.rank], None, None,
        batch.positions[rows], seq_start, batch.block_table[ents], spec.scale,
-       0, 0, 0, 0.0, 1.0, max_len, batch.max_context, False)
+       0, spec.window, 0, 0.0, 1.0, max_len,
+       min(spec.window or batch.max_context, batch.max_context), False, None,
+       None, None)
     head_linear(o.view(n, spec.heads, spec.rank), w_uv, gate, out=out)
 
 
 def _latent_expanded(out, q, gate, cache, w_ukv, batch, rows, ents, seq_start,
                      max_len, spec, shared) -> None:
-    """Keys and values of all heads are made for the whole contexts of the
-    batch's portions; layers on the same cache share what is read from it."""
-    held = shared.get(cache.data_ptr())
+    """Keys and values of all heads are made for all that the batch's portions
+    see; layers on the same cache share what is read from it."""
+    ctx_start, total, _ = batch.context(spec.window)
+    key = cache.data_ptr(), spec.window
+    held = shared.get(key)
     if held is None:
-        held = shared[cache.data_ptr()] = tuple(
-            q.new_empty(batch.total_context, n)
-            for n in (spec.rank, spec.rot_dim))
-        _ext().latent_gather(*held, cache, batch.block_table[ents],
-                             batch.ctx_start)
+        held = shared[key] = tuple(
+            q.new_empty(total, n) for n in (spec.rank, spec.rot_dim))
+        _ext().latent_gather(*held, cache, batch.block_table[ents], ctx_start,
+                             batch.positions[rows], seq_start, spec.window,
+                             max_len)
     c, kr = held
     _ext().attn_flat(out, q, gate, linear(c, w_ukv), kr,
-                     batch.positions[rows], seq_start, batch.ctx_start,
-                     spec.heads, spec.vdim, spec.scale, max_len)
+                     batch.positions[rows], seq_start, ctx_start, spec.heads,
+                     spec.vdim, spec.scale, spec.window, max_len)
 
 
 EXPAND_BYTES = 4 << 30      # most memory for keys and values of one layer
@@ -192,10 +210,10 @@ def _expanding_pays(batch, spec, rows: int) -> bool:
     """Fewer multiplications with keys and values made for every head than
     with queries moved into the latent space."""
     own = spec.rank * (spec.dim + spec.vdim)
-    if 2 * batch.total_context * spec.heads * (spec.dim + spec.vdim) \
-            > EXPAND_BYTES:
+    _, total, pairs = batch.context(spec.window)
+    if 2 * total * spec.heads * (spec.dim + spec.vdim) > EXPAND_BYTES:
         return False
-    return (batch.total_context - rows) * own < batch.pairs * (
+    return (total - rows) * own < pairs * (
         2 * spec.rank - spec.dim - spec.vdim)
 
 
@@ -204,7 +222,8 @@ def _flat_takes(q, gate, spec) -> bool:
     return (q.is_cuda and q.dtype == torch.bfloat16
             and not any(n % 8 for n in (spec.dim, spec.rot_dim, spec.vdim,
                                         q.stride(0), q.storage_offset()))
-            and (gate is None or gate.storage_offset() % 8 == 0)
+            and (gate is None or spec.head_gate
+                 or gate.storage_offset() % 8 == 0)
             and spec.dim + spec.rot_dim <= 256 and spec.vdim <= 256)
 
 
@@ -214,7 +233,7 @@ def latent_attn(q: torch.Tensor, gate: Optional[torch.Tensor],
                 expand: Optional[bool] = None) -> torch.Tensor:
     """Latent attention of a batch's rows over the paged cache, which already
     holds their own latents. q [rows, heads * (dim + rot_dim)] is rotated;
-    gate [rows, heads * vdim]; w_ukv has the rows that make all heads' keys,
+    gate [rows, heads * vdim], or [rows, heads]; w_ukv has the rows that make all heads' keys,
     then those that make their values; uk_t is the former as [heads, rank,
     dim]. `shared` lasts for one batch. expand: how portions are computed,
     None: as pays."""
@@ -234,14 +253,16 @@ def latent_attn(q: torch.Tensor, gate: Optional[torch.Tensor],
 
 
 def experts(y: torch.Tensor, router: torch.Tensor, up: torch.Tensor,
-            down: torch.Tensor, spec,
-            bias: Optional[torch.Tensor] = None) -> Picked:
+            down: torch.Tensor, spec, bias: Optional[torch.Tensor] = None,
+            correction: Optional[torch.Tensor] = None) -> Picked:
     """A mixture of experts: y [rows, width], router [experts, width], bias
-    [experts], up [experts, ff, width] (gated experts: twice as many rows, of
-    gate and up in turn), down [experts, width, ff]. Scores are 32-bit."""
+    and correction [experts], up [experts, ff, width] (gated experts: twice as
+    many rows, of gate and up in turn), down [experts, width, ff]. Scores are
+    32-bit; the correction is for the choice only."""
     rows = y.shape[0]
     if not y.is_cuda:
-        return Picked(*ref.experts(y, router, bias, up, down, spec))
+        return Picked(*ref.experts(y, router, bias, up, down, spec,
+                                   correction))
     ext = _ext()
     i32 = dict(dtype=torch.int32, device=y.device)
     z = ext.router_scores(y, router)
@@ -249,7 +270,8 @@ def experts(y: torch.Tensor, router: torch.Tensor, up: torch.Tensor,
     weights = torch.empty(rows, spec.top, dtype=torch.float32,
                           device=y.device)
     ext.moe_select(ids, weights, z, spec.groups, spec.keep, bias,
-                   spec.over_chosen)
+                   spec.over_chosen, spec.sigmoid, correction,
+                   spec.group_best)
     packed = rows * spec.top
     tile = ext.moe_tile(packed, spec.experts, y.dtype == torch.bfloat16,
                         y.shape[1], spec.ff)
@@ -396,6 +418,28 @@ def conv_rope(buf: torch.Tensor, in_bias: Optional[torch.Tensor],
         fn(q[rows], buf[rows], in_bias, weight, state,
            batch.state_slots[ents], rope[rows], k_cache, v_cache,
            batch.positions[rows], batch.slots[rows], seq_start, max_len)
+    return q
+
+
+def conv_qkv(buf: torch.Tensor, in_bias: Optional[torch.Tensor],
+             weight: torch.Tensor, state: torch.Tensor, k_cache: torch.Tensor,
+             v_cache: torch.Tensor, batch, temp=None,
+             v_eps: Optional[float] = None) -> torch.Tensor:
+    """buf rows are [q | k | v | ...]. in_bias is added to all, then they pass
+    a short convolution (as short_conv). q is multiplied by its position's
+    temperature (layers.QueryTemperature); each head's v is divided by its
+    root mean square with v_eps under the root (None: not); k and v go to
+    their caches. Returns q."""
+    kv = k_cache.shape[1]
+    q = buf.new_empty(buf.shape[0], weight.shape[0] - kv * (
+        k_cache.shape[3] + v_cache.shape[3]))
+    coef, every = (temp.coef, temp.every) if temp else (0.0, 1)
+    fn = (_ext() if buf.is_cuda else ref).conv_qkv
+    for rows, ents, seq_start, max_len in batch.parts():
+        fn(q[rows], buf[rows], in_bias, weight, state,
+           batch.state_slots[ents], k_cache, v_cache, batch.positions[rows],
+           batch.slots[rows], seq_start, coef, every,
+           -1.0 if v_eps is None else v_eps, max_len)
     return q
 
 

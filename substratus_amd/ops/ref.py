@@ -249,8 +249,11 @@ def stream_norm(rows, at, weights, x, w_post, w_pre, offset, eps,
     return y.to(rows.dtype, copy=True)
 
 
-def embed_norm(tokens, table, w_pre, offset, eps):
-    x = table[tokens.long()].float()
+def embed_norm(tokens, table, w_pre, offset, eps, scale=1.0, pos=None,
+               positions=None):
+    x = table[tokens.long()].float() * scale
+    if pos is not None:
+        x += pos[positions.long()].float()
     y = x if w_pre is None else _rms(x, eps) * (offset + w_pre)
     return x, y.to(table.dtype, copy=True)
 
@@ -323,6 +326,22 @@ def conv_rope(q, buf, in_bias, weight, state, state_slots, rope, k_cache,
     y[..., 1:2 * half:2] = b * cos + a * sin
     q.copy_(y[:, :-kv].reshape(q.shape).to(q.dtype))
     kv_append(y[:, -kv:], v, k_cache, v_cache, slots)
+
+
+def conv_qkv(q, buf, in_bias, weight, state, state_slots, k_cache, v_cache,
+             positions, slots, seq_start, coef, every, v_eps, max_len):
+    rows, kv = weight.shape[0], k_cache.shape[1]
+    y = torch.empty(buf.shape[0], rows, device=buf.device)
+    short_conv(y, buf[:, :rows], in_bias, weight, None, False, state,
+               state_slots, positions, seq_start, max_len)
+    yq, k, v = y.split([q.shape[1], kv * k_cache.shape[3],
+                        kv * v_cache.shape[3]], dim=1)
+    steps = torch.div(positions + 1, every, rounding_mode="floor")
+    q.copy_((yq * (1 + coef * torch.log1p(steps.float()))[:, None]).to(
+        q.dtype))
+    v = v.reshape(-1, kv, v_cache.shape[3])
+    kv_append(k.reshape(-1, kv, k_cache.shape[3]),
+              v if v_eps < 0 else _rms(v, v_eps), k_cache, v_cache, slots)
 
 
 def selective_scan(out, u, gate, z, z_bias, low, b_at, a, d, state,
@@ -416,7 +435,7 @@ def _rotate(x, turns, positions):
     half = turns.shape[0]
     t = positions.double()[:, None] * turns
     a = ((t - t.round()) * (2 * math.pi)).float()
-    a = a.view(-1, *[1] * (x.dim() - 2), half)
+    a = a.view(x.shape[0], *[1] * (x.dim() - 2), half)
     u, v = x[..., :half].clone(), x[..., half:2 * half].clone()
     x[..., :half] = u * a.cos() - v * a.sin()
     x[..., half:2 * half] = v * a.cos() + u * a.sin()
@@ -424,11 +443,16 @@ def _rotate(x, turns, positions):
 
 
 def latent_prepare(buf, heads, dim, rot_dim, c_at, norm, eps, turns,
-                   positions, cache, slots):
-    n = heads * (dim + rot_dim)
-    q = buf[:, :n].to(torch.float32, copy=True).view(-1, heads, dim + rot_dim)
-    _rotate(q[..., dim:], turns, positions)
-    buf[:, :n] = q.view(-1, n).to(buf.dtype)
+                   positions, cache, slots, q_norm=None):
+    if q_norm is not None:
+        n = q_norm.shape[0]
+        buf[:, :n] = (_rms(buf[:, :n].float(), eps) * q_norm).to(buf.dtype)
+    elif rot_dim:
+        n = heads * (dim + rot_dim)
+        q = buf[:, :n].to(torch.float32, copy=True).view(-1, heads,
+                                                         dim + rot_dim)
+        _rotate(q[..., dim:], turns, positions)
+        buf[:, :n] = q.view(-1, n).to(buf.dtype)
     if c_at < 0:
         return
     rank = norm.shape[0]
@@ -444,25 +468,32 @@ def head_linear(out, x, w, gate, tail):
     o = torch.matmul(x[..., :k].float().transpose(0, 1).contiguous(),
                      w.float().transpose(1, 2).contiguous()).transpose(0, 1)
     if gate is not None:
-        o = o * torch.sigmoid(gate.float()).view(o.shape)
+        o = o * torch.sigmoid(gate.float()).reshape(*o.shape[:2], -1)
     out[..., :w.shape[1]] = o.to(out.dtype)
     if tail:
         out[..., w.shape[1]:] = x[..., k:k + tail]
 
 
-def moe_select(z, top, groups, keep, over_chosen=False):
+def moe_select(z, top, groups, keep, over_chosen=False, sigmoid=False,
+               correction=None, group_best=1):
     """(ids [rows, top] int32, weights float32), best first, of scores z."""
-    s = torch.softmax(z, -1)
-    best = z.view(-1, groups, s.shape[1] // groups).amax(-1)
+    s = torch.sigmoid(z) if sigmoid else torch.softmax(z, -1)
+    if sigmoid:
+        z = s
+    if correction is not None:
+        z = z + correction
+    size = s.shape[1] // groups
+    best = z.view(-1, groups, size).topk(min(group_best, size), -1) \
+        .values.sum(-1)
     kept = torch.zeros_like(best, dtype=torch.bool).scatter_(
         1, best.topk(keep, 1).indices, True)
-    kept = kept.repeat_interleave(s.shape[1] // groups, 1)
+    kept = kept.repeat_interleave(size, 1)
     chosen, ids = z.masked_fill(~kept, float("-inf")).topk(top, 1)
     return ids.int(), torch.softmax(chosen, -1) if over_chosen \
         else s.gather(1, ids)
 
 
-def experts(y, router, bias, up, down, spec):
+def experts(y, router, bias, up, down, spec, correction=None):
     """(rows, at, weights) of the chosen experts' outputs, token by token.
     Gated experts' matrices have the rows of gate and up in turn."""
     f, top = y.float(), spec.top
@@ -470,7 +501,8 @@ def experts(y, router, bias, up, down, spec):
     if bias is not None:
         z = z + bias
     ids, weights = moe_select(z, top, spec.groups, spec.keep,
-                              spec.over_chosen)
+                              spec.over_chosen, spec.sigmoid, correction,
+                              spec.group_best)
     out = y.new_zeros(y.shape[0] * top, y.shape[1])
     flat = ids.reshape(-1)
     for e in flat.unique().tolist():
@@ -513,7 +545,7 @@ def _entry_rows(seq_start, rows):
 
 def attn_ctx(out, q, gate, k_cache, v_cache, bias, sink, positions, seq_start,
              block_table, scale, chunk, window, keep, cap, mult, max_len, span,
-             any_size):
+             any_size, r1=None, r2=None, weight_bias=None):
     kv, bs, dim = k_cache.shape[1:]
     vdim = v_cache.shape[3]
     for e, (a, b) in enumerate(_entry_rows(seq_start, q.shape[0])):
@@ -530,6 +562,10 @@ def attn_ctx(out, q, gate, k_cache, v_cache, bias, sink, positions, seq_start,
         if bias is not None:
             s = s + bias[:, dist.clamp(0, bias.shape[1] - 1)].view(
                 kv, -1, b - a, n)
+        if r1 is not None:
+            fall = r1[:, None, None] * torch.log1p(
+                r2[:, None, None] * dist.clamp(0))
+            s = s - fall.view(kv, -1, b - a, n)
         seen = dist >= 0
         if chunk:
             seen &= (pos // chunk)[:, None] == torch.arange(
@@ -541,7 +577,8 @@ def attn_ctx(out, q, gate, k_cache, v_cache, bias, sink, positions, seq_start,
         if sink is not None:    # a key without a value
             s = torch.cat([s, sink.view(kv, -1, 1, 1).expand(
                 kv, s.shape[1], b - a, 1)], -1)
-        p = torch.softmax(s, -1)[..., :n]
+        p = torch.softmax(s, -1)[..., :n] if weight_bias is None else \
+            torch.sigmoid(s + weight_bias.view(kv, -1, 1, 1))
         o = torch.einsum("kgij,jkd->ikgd", p, v).reshape(b - a, -1, vdim)
         if gate is not None:
             o = o * torch.sigmoid(gate[a:b].float())[:, :, None]

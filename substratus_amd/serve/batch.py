@@ -2,7 +2,7 @@
 
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Iterator, Optional
 
 import numpy as np
@@ -29,6 +29,24 @@ class StepBatch:
                                               # the portions see, summed up
     total_context: int = 0      # the last of those
     pairs: int = 0              # portions' rows times the keys they see
+    # portions' first positions and lengths, on the host
+    firsts: Optional[np.ndarray] = None
+    lengths: Optional[np.ndarray] = None
+    _windows: dict = field(default_factory=dict)
+
+    def context(self, window: int = 0) -> tuple[torch.Tensor, int, int]:
+        """ctx_start, total_context and pairs as they are where a row sees
+        `window` keys, its own included (0: all before it)."""
+        if not window:
+            return self.ctx_start, self.total_context, self.pairs
+        if window not in self._windows:
+            keys = np.minimum(self.firsts, window - 1) + self.lengths
+            starts = np.concatenate([[0], np.cumsum(keys)]).astype(np.int32)
+            seen = np.minimum(self.firsts + self.lengths, window)
+            self._windows[window] = (
+                torch.from_numpy(starts).to(self.tokens.device),
+                int(starts[-1]), int((self.lengths * seen).sum()))
+        return self._windows[window]
 
     def parts(self) -> Iterator[tuple[slice, slice, Optional[torch.Tensor],
                                       int]]:
@@ -59,7 +77,7 @@ class StepBatch:
         table = np.zeros((len(entries), maxb), np.int32)
         tokens, positions, slots = (np.empty(rows, np.int32)
                                     for _ in range(3))
-        starts, contexts, pairs = [0], [0], 0
+        starts, contexts, pairs, firsts = [0], [0], 0, []
         for at, i in enumerate(order):
             toks, first, blocks, _, _ = entries[i]
             table[at, :len(blocks)] = blocks
@@ -72,6 +90,7 @@ class StepBatch:
                 starts.append(starts[-1] + len(toks))
                 contexts.append(contexts[-1] + first + len(toks))
                 pairs += len(toks) * (first + len(toks))
+                firsts.append(first)
         state = np.array([entries[i][3] for i in order], np.int32)
         want = np.array([row_of[i] + o for i, e in enumerate(entries)
                          for o in e[4]], np.int32)
@@ -88,4 +107,5 @@ class StepBatch:
             singles, starts_t if portions else None,
             int(np.diff(starts).max()) if portions else 0,
             maxb * block_size, want.long(),
-            contexts_t if portions else None, contexts[-1], pairs)
+            contexts_t if portions else None, contexts[-1], pairs,
+            np.array(firsts, np.int64), np.diff(starts))

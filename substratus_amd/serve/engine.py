@@ -22,7 +22,7 @@ from __future__ import annotations
 
 import itertools
 import time
-from dataclasses import dataclass, field
+from dataclasses import dataclass, replace
 from typing import Optional
 
 import torch
@@ -78,8 +78,11 @@ class StepOutput:
 class Engine:
     def __init__(self, cfg: EngineConfig, device: Optional[str] = None,
                  model: Optional[CausalLM | HybridLM] = None):
-        self.cfg = cfg
         self.mcfg: ModelConfig = get_config(cfg.model)
+        if self.mcfg.learned_pos_emb:   # there are no positions after these
+            cfg = replace(cfg, max_seq_len=min(
+                cfg.max_seq_len, self.mcfg.max_position_embeddings))
+        self.cfg = cfg
         if device is None:
             device = "cuda" if torch.cuda.is_available() else "cpu"
         self.device = torch.device(device)

@@ -93,6 +93,9 @@ class TraceReplay:
             if not e["tokens"]:
                 continue
             seq.tokens.extend(e["tokens"])
+            if seq.length > self.engine.cfg.max_seq_len:
+                raise ValueError(f"request {e['id']} is longer than "
+                                 f"{self.engine.cfg.max_seq_len} tokens")
             self.engine.kv.reserve(seq, seq.length)
             work.append((seq, len(e["tokens"]), e["want"]))
         logits = self.engine.execute(work).float().cpu() if work else None
