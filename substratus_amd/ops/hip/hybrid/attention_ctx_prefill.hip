@@ -35,12 +35,6 @@ DEV_INLINE short4v tr16_read(const short* p) {
       (__attribute__((address_space(3))) short4v*)p);
 }
 
-DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
-  unsigned r;
-  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(lo), "v"(hi));
-  return r;
-}
-
 // KK: 16-wide steps of the key size; DC: 32-wide tiles of the value size
 enum Kind {
   PLAIN,

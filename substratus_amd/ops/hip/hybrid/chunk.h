@@ -19,12 +19,6 @@ constexpr int OUT_OF_RANGE = 0x7ffffff0;   // beyond any buffer's end
 
 DEV_INLINE float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 
-DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
-  unsigned r;
-  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(lo), "v"(hi));
-  return r;
-}
-
 // two floats as bf16 high parts and low parts, each pair in one word
 DEV_INLINE void split_pair(float f0, float f1, unsigned* hi, unsigned* lo) {
   *hi = cvt_pk_bf16(f0, f1);

@@ -57,6 +57,16 @@ DEV_INLINE void stv(bf16_t* p, const float* f) {
   }
 }
 
+// Two bf16 in one instruction. Not by inline assembly: the compiler does not
+// see what that reads, and leaves out the wait that the result of an
+// exponential or a reciprocal needs ahead of its first use.
+DEV_INLINE unsigned cvt_pk_bf16(float lo, float hi) {
+  typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
+  typedef __attribute__((ext_vector_type(2))) float floatx2;
+  return __builtin_bit_cast(
+      unsigned, __builtin_convertvector((floatx2){lo, hi}, bf16x2));
+}
+
 DEV_INLINE float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 
 // ln(sigmoid(z)) without overflow at either end

@@ -39,14 +39,15 @@ class StepBatch:
         `window` keys, its own included (0: all before it)."""
         if not window:
             return self.ctx_start, self.total_context, self.pairs
-        if window not in self._windows:
+        key = window, self.tokens.device
+        if key not in self._windows:
             keys = np.minimum(self.firsts, window - 1) + self.lengths
             starts = np.concatenate([[0], np.cumsum(keys)]).astype(np.int32)
             seen = np.minimum(self.firsts + self.lengths, window)
-            self._windows[window] = (
+            self._windows[key] = (
                 torch.from_numpy(starts).to(self.tokens.device),
                 int(starts[-1]), int((self.lengths * seen).sum()))
-        return self._windows[window]
+        return self._windows[key]
 
     def parts(self) -> Iterator[tuple[slice, slice, Optional[torch.Tensor],
                                       int]]:

@@ -153,6 +153,52 @@ def test_latent_attention_long(first, n, expand):
     close(got, want, BF16)
 
 
+@pytest.mark.parametrize("dtype,expand", [(F32, None), (BF16, False),
+                                          (BF16, True)])
+@pytest.mark.parametrize("shape", [(6, 32, 0, 32, 128), (3, 24, 0, 16, 40),
+                                   (16, 128, 0, 128, 512), (2, 16, 8, 24, 64)])
+@pytest.mark.parametrize("window", [1, 30, 64, 200, 1000])
+def test_windowed_latent_attention(shape, window, dtype, expand):
+    """Gates per head; a window alone, and beside a rotated key part."""
+    batch = make_batch([(0, 1), (99, 1), (301, 1), (1023, 1), (0, 2), (17, 70),
+                        (290, 33), (0, 330), (63, 2)], blocks=192)
+    h, d, r, dv, rank = shape
+    spec = LatentAttentionSpec(h, d, r, dv, rank, 1.3 * (d + r) ** -0.5, None,
+                               head_gate=True, window=window)
+    buf, cache, w = latent_inputs(spec, batch, dtype, 192, 40)
+    uk_t = w[:h * d].view(h, d, rank).transpose(1, 2).contiguous()
+    gate = rand(buf.shape[0], h + 1, seed=44, dtype=dtype)
+
+    def run(buf, cache, w, uk_t, gate, batch, expand):
+        return ops.latent_attn(buf[:, :h * (d + r)], gate[:, 1:], cache, w,
+                               uk_t, batch, spec, {}, expand)
+    want = run(buf, cache, w, uk_t, gate, batch, None)
+    got = run(*(t.cuda() for t in (buf, cache, w, uk_t, gate)),
+              on_gpu(batch), expand)
+    close(got, want, dtype)
+
+
+@pytest.mark.parametrize("z", [1, 5, 64, 65, 130, 1024])
+@pytest.mark.parametrize("rows", [1, 7])
+def test_moe_select_by_corrected_sigmoids(rows, z):
+    from substratus_amd.ops import ref
+    ext = ops._ext()
+    corr = rand(z, seed=z) - 1.5
+    for groups in (1, 2, 5, 13, 64):
+        if z % groups:
+            continue
+        keep = (groups + 1) // 2
+        for top in {1, min(6, keep * (z // groups))}:
+            s = rand(rows, z, seed=z + groups, scale=2.0)
+            ids = torch.empty(rows, top, dtype=torch.int32).cuda()
+            wt = torch.empty(rows, top).cuda()
+            ext.moe_select(ids, wt, torch.stack([s.cuda() * 0.25] * 4), groups,
+                           keep, None, False, True, corr.cuda(), 2)
+            ri, rw = ref.moe_select(s, top, groups, keep, False, True, corr, 2)
+            assert torch.equal(ids.cpu(), ri), (groups, keep, top)
+            assert torch.allclose(wt.cpu(), rw, rtol=1e-5), (groups, keep)
+
+
 @pytest.mark.parametrize("z", [1, 5, 64, 65, 130, 1024])
 @pytest.mark.parametrize("rows", [1, 7])
 def test_moe_select(rows, z):

@@ -5,7 +5,8 @@ CPU (ops/ref.py), over sizes on and off the tiles."""
 import pytest
 import torch
 
-from substratus_amd.models.layers import GluSpec, MoESpec, RotarySpec
+from substratus_amd.models.layers import (GluSpec, MoESpec, QueryTemperature,
+                                          RotarySpec)
 from substratus_amd.ops import hybrid as ops
 from test_hybrid_ops_gpu import BS, close, make_batch, on_gpu, rand
 
@@ -333,3 +334,67 @@ def test_long_contexts_shared_by_workgroups(window, keep, cap, sink):
     got = ops.attn_ctx(*cuda(q, None, kc, vc), None, on_gpu(batch), *args,
                        s.cuda() if sink else None)
     close(got, want, BF16)
+
+
+# ---- attention by sigmoids behind convolutions ------------------------------
+
+@BOTH
+@pytest.mark.parametrize("spans", [SPANS, LONG])
+@pytest.mark.parametrize("heads,kv,d,dv,taps", [
+    (4, 2, 64, 40, 4), (6, 1, 64, 80, 3), (2, 2, 9, 7, 2), (3, 3, 128, 256, 1),
+    (2, 1, 20, 300, 5), (16, 16, 128, 128, 4)])
+def test_conv_qkv(spans, heads, kv, d, dv, taps, dtype):
+    batch = make_batch(spans)
+    n, rows = batch.tokens.shape[0], (heads + kv) * d + kv * dv
+    buf = rand(n, rows + 8, seed=1, dtype=dtype)
+    bias, w = rand(rows, seed=2), rand(rows, taps, seed=3)
+    state = rand(len(spans), taps - 1, rows, seed=4, dtype=dtype)
+    caches = [torch.zeros(64, kv, BS, s, dtype=dtype) for s in (d, dv)]
+    sg, *cg = cuda(state, *caches)
+    temp = QueryTemperature(0.6, 13)
+    want = ops.conv_qkv(buf, bias, w, state, *caches, batch, temp, 1e-3)
+    got = ops.conv_qkv(*cuda(buf, bias, w), sg, *cg, on_gpu(batch), temp,
+                       1e-3)
+    close(got, want, dtype)
+    for a, b in zip(cg, caches):
+        close(a, b, dtype)
+    assert torch.equal(sg.cpu(), state)
+
+
+@BOTH
+@pytest.mark.parametrize("heads,kv,d,dv", [(4, 4, 64, 64), (6, 2, 40, 72),
+                                           (3, 1, 20, 12), (8, 1, 128, 128),
+                                           (2, 2, 192, 256)])
+@pytest.mark.parametrize("any_size", [False, True])
+@pytest.mark.parametrize("window,gated", [(0, False), (37, True)])
+def test_sigmoid_attention(heads, kv, d, dv, any_size, window, gated, dtype):
+    spans = [(0, 1), (15, 1), (899, 1), (0, 5), (30, 2), (50, 150)]
+    batch = make_batch(spans, blocks=96)
+    n = batch.tokens.shape[0]
+    q = rand(n, heads * d, seed=1, dtype=dtype, scale=2.0)
+    kc, vc = (rand(96, kv, BS, s, seed=s, dtype=dtype) for s in (d, dv))
+    gate = rand(n, heads, seed=2, dtype=dtype) if gated else None
+    r = rand(heads, seed=3).abs(), rand(heads, seed=4).abs()
+    wb = rand(heads, seed=5) - 2
+
+    def run(q, gate, kc, vc, batch, r1, r2, wb):
+        return ops.attn_ctx(q, gate, kc, vc, None, batch, d ** -0.5,
+                            any_size=any_size, window=window, mult=0.7,
+                            falloff=(r1, r2), weight_bias=wb)
+    want = run(q, gate, kc, vc, batch, *r, wb)
+    got = run(*cuda(q, gate, kc, vc), on_gpu(batch), *cuda(*r, wb))
+    close(got, want, dtype)
+
+
+@BOTH
+@pytest.mark.parametrize("any_size", [False, True])
+def test_falloff_before_a_softmax(any_size, dtype):
+    batch = make_batch([(0, 1), (700, 1), (0, 40), (90, 70)])
+    n = batch.tokens.shape[0]
+    q = rand(n, 2 * 64, seed=1, dtype=dtype, scale=2.0)
+    kc, vc = (rand(64, 1, BS, 64, seed=s, dtype=dtype) for s in (2, 3))
+    r = torch.tensor([0.3, 1.5]), torch.tensor([2.0, 0.1])
+    want = ops.attn_ctx(q, None, kc, vc, None, batch, 0.125, falloff=r)
+    got = ops.attn_ctx(*cuda(q, None, kc, vc), None, on_gpu(batch), 0.125,
+                       any_size=any_size, falloff=tuple(cuda(*r)))
+    close(got, want, dtype)
