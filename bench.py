@@ -249,10 +249,15 @@ HYBRID_PAIRS = [
                                   (16, 3072)]),
     ("vurazen-7b", "kakovik-7b", [(8, 512), (64, 512), (256, 512),
                                   (16, 3072)]),
+    ("ditalorn-1b", "guronex-1b", [(8, 512), (64, 512), (256, 512),
+                                   (16, 3072)]),
+    ("ditalorn-7b", "guronex-7b", [(8, 512), (64, 512), (256, 512),
+                                   (16, 3072)]),
 ]
 HYBRID_TINY = [("kakovik-tiny", "llama-tiny", [(2, 24)]),
                ("guronex-tiny", "llama-tiny", [(2, 24)]),
-               ("vurazen-tiny", "kakovik-tiny", [(2, 24)])]
+               ("vurazen-tiny", "kakovik-tiny", [(2, 24)]),
+               ("ditalorn-tiny", "guronex-tiny", [(2, 24)])]
 
 
 def bench_hybrid(args) -> None:

@@ -349,7 +349,7 @@ def bench_latent():
                timeit(lambda: hy._ext().attn_ctx(
                    o, qa, None, cache, cache[..., :rank], None, None,
                    sb.positions, None, sb.block_table, spec.scale, 0, 0, 0,
-                   0.0, 1.0, 1, ctx, False), 50),
+                   0.0, 1.0, 1, ctx, False, None, None, None), 50),
                b * ctx * spec.row * 2 + b * h * (spec.row + rank) * 2,
                2.0 * b * ctx * h * (spec.row + rank))
 
@@ -370,13 +370,14 @@ def bench_latent():
         report(f"  attn_flat b={b} s={s_} {h}x{d}+{r}",
                timeit(lambda: hy._ext().attn_flat(
                    o, q2, gate, kv, kr, sb.positions, sb.seq_start,
-                   sb.ctx_start, h, d, spec.scale, s_), 20),
+                   sb.ctx_start, h, d, spec.scale, 0, s_), 20),
                t * (h * (5 * d + r) + r) * 2, flops)
         cache = torch.randn(t // 16, 1, 16, spec.row, **bf)
         c = torch.empty(t, rank, **bf)
         report(f"  latent_gather keys={t}",
                timeit(lambda: hy._ext().latent_gather(
-                   c, kr, cache, sb.block_table, sb.ctx_start), 20),
+                   c, kr, cache, sb.block_table, sb.ctx_start, sb.positions,
+                   sb.seq_start, 0, s_), 20),
                t * spec.row * 4)
         del q2, gate, kv, o, cache
     for b, first, n in ((16, 2048, 16), (4, 4096, 64)):
@@ -388,7 +389,8 @@ def bench_latent():
                timeit(lambda: hy._ext().attn_ctx(
                    o, qa, None, cache, cache[..., :rank], None, None,
                    sb.positions, sb.seq_start, sb.block_table, spec.scale, 0,
-                   0, 0, 0.0, 1.0, n, first + n, False), 20),
+                   0, 0, 0.0, 1.0, n, first + n, False, None, None, None),
+                   20),
                b * (first + n) * spec.row * 2 + b * n * h * 2 * (
                    spec.row + rank),
                2.0 * b * n * (first + n / 2) * h * (spec.row + rank))
@@ -577,6 +579,199 @@ def bench_mixers():
                    it),
                max(state.numel() * 8 + t * inner * 10,
                    HBM * steps * (1 / EXP + 4 / FMA)))
+
+
+def bench_sigmoid():
+    """Kernels of sigmoid attention behind convolutions, of windowed latent
+    attention and of corrected routers beside the like kernels of Kakovik,
+    Guronex and Vurazen, at 7b sizes."""
+    from substratus_amd.models.layers import (GluSpec, LatentAttentionSpec,
+                                              MoESpec, QueryTemperature,
+                                              RotarySpec)
+    from substratus_amd.ops import hybrid as hy
+    from substratus_amd.serve.batch import StepBatch
+    torch.manual_seed(0)
+    bf = dict(device="cuda", dtype=torch.bfloat16)
+    f32, i32 = dict(device="cuda"), dict(device="cuda", dtype=torch.int32)
+    ext = hy._ext()
+
+    def batch_of(n, first, tokens):
+        need = (first + tokens + 15) // 16
+        return StepBatch.build(
+            [([1] * tokens, first, list(range(i * need, (i + 1) * need)), i,
+              []) for i in range(n)], 16, torch.device("cuda"))
+
+    w, h, d, r, rank, q_rank, win = 4096, 32, 128, 64, 512, 1536, 1024
+    old = LatentAttentionSpec(h, d, r, d, rank, (d + r) ** -0.5,
+                              RotarySpec(1e4, r), None, True)
+    new = LatentAttentionSpec(h, d, 0, d, rank, d ** -0.5, None,
+                              head_gate=True, q_rank=q_rank, window=win)
+    temp = QueryTemperature(0.1, 1024)
+    for rows in (64, 256, 16384):
+        it = 200 if rows < 1000 else 30
+        sb = batch_of(rows, 20, 1) if rows < 1000 else batch_of(8, 0, 2048)
+        n = sb.state_slots.numel()
+        table, vecs = torch.randn(32000, w, **bf), torch.randn(8192, w, **bf)
+        w32 = torch.randn(w, **f32)
+        tok = torch.randint(0, 32000, (rows,), **i32)
+        report(f"embed_norm rows={rows} w={w}",
+               timeit(lambda: hy.embed_norm(tok, table, w32, 1.0, 1e-5), it),
+               rows * w * 8)
+        report(f"  embed_norm with positions rows={rows} w={w}",
+               timeit(lambda: hy.embed_norm(tok, table, w32, 1.0, 1e-5, 64.0,
+                                            vecs, sb.positions), it),
+               rows * w * 10)
+        del table, vecs
+        x = torch.randn(rows, w, **bf)
+        pages = rows * 2 if rows < 1000 else rows // 16
+        kc = torch.zeros(pages, h, 16, d, **bf)
+        vc = torch.zeros_like(kc)
+        buf = torch.randn(rows, 3 * h * d, **bf)
+        for name, parts in (("conv_rope", 2), ("  conv_qkv", 3)):
+            ch = parts * h * d
+            cs = torch.zeros(n, 3, ch, **bf)
+            cw, cb = torch.randn(ch, 4, **f32), torch.randn(ch, **f32)
+            taps = n * 3 * ch * 4
+            if parts == 2:
+                rot = RotarySpec(1e4, d, True)
+                rope = hy.rope_table(sb, rot, rot.turns("cuda"), {})
+                dt = timeit(lambda: hy.conv_rope(buf, cb, cw, cs, rope, kc, vc,
+                                                 sb), it)
+                nbytes = rows * h * d * 2 * 5 + taps + rows * d * 4
+            else:
+                dt = timeit(lambda: hy.conv_qkv(buf, cb, cw, cs, kc, vc, sb,
+                                                temp, 1e-5), it)
+                nbytes = rows * h * d * 2 * 6 + taps
+            report(f"{name} rows={rows} {h}x{d} 4 taps", dt, nbytes)
+        del kc, vc, buf
+        pos = torch.arange(rows, **i32)
+        norm, qn = torch.ones(rank, **f32), torch.ones(q_rank, **f32)
+        buf = torch.randn(rows, h * (2 * d + r) + rank + r, **bf)
+        cache = torch.zeros((rows + 15) // 16, 1, 16, old.row, **bf)
+        turns = old.rot.turns("cuda")
+        report(f"latent_prepare rows={rows}",
+               timeit(lambda: hy.latent_prepare(
+                   buf, old, h * (2 * d + r), norm, 1e-5, turns, pos, cache,
+                   pos), it), rows * (h * r * 2 + old.row * 2) * 2)
+        buf = torch.randn(rows, q_rank + rank + h, **bf)
+        cache = torch.zeros((rows + 15) // 16, 1, 16, rank, **bf)
+        turns = torch.empty(0, dtype=torch.float64, device="cuda")
+        report(f"  latent_prepare with queries' latent rows={rows}",
+               timeit(lambda: hy.latent_prepare(
+                   buf, new, q_rank, norm, 1e-5, turns, pos, cache, pos, qn),
+                   it), rows * (q_rank + rank) * 4)
+        corr = torch.randn(32, **f32) * 0.01
+        gates = torch.randn(rows, h * d, **bf)
+        if rows < 1000:
+            uv = torch.randn(h, d, rank, **bf)
+            o3 = torch.randn(rows, h, rank, **bf)
+            for name, g in (("head_linear out", gates),
+                            ("  head_linear out, gate per head",
+                             gates[:, :h])):
+                report(f"{name} rows={rows} {h}x{rank}->{d}",
+                       timeit(lambda: hy.head_linear(o3, uv, g), it),
+                       (uv.numel() + rows * h * (d + rank) + g.numel()) * 2)
+        for name, moe, f in (
+                ("8 of 32 x 1024", MoESpec(
+                    32, 8, 1024, 8, 4, glu=GluSpec("clamped", 7.0)), 0),
+                ("8 of 32 x 1344", MoESpec(
+                    32, 8, 1344, 8, 4, GluSpec("silu"), sigmoid=True,
+                    correction=True, group_best=2), 1)):
+            z = torch.randn(1, rows, 32, **f32)
+            ids = torch.empty(rows, 8, **i32)
+            wts = torch.empty(rows, 8, **f32)
+            report(f"{'  ' * f}moe_select{' corrected' * f} rows={rows} 8/32",
+                   timeit(lambda: ext.moe_select(
+                       ids, wts, z, 8, 4, None, False, moe.sigmoid,
+                       corr if f else None, moe.group_best), it),
+                   rows * (32 + 16) * 4)
+            wu = torch.randn(32, 2 * moe.ff, w, **bf) * 0.02
+            wd = torch.randn(32, w, moe.ff, **bf) * 0.02
+            router = torch.randn(32, w, **bf) * 0.02
+            report(f"{'  ' * f}experts rows={rows} {name}",
+                   timeit(lambda: hy.experts(x, router, wu, wd, moe, None,
+                                             corr if f else None), it),
+                   (wu.numel() + wd.numel() + rows * 8 * (w + 2 * moe.ff)) * 2,
+                   6.0 * rows * 8 * moe.ff * w)
+            del wu, wd
+
+    fall = torch.full((h,), 0.5, **f32), torch.full((h,), 0.5, **f32)
+    wb, bias = torch.full((h,), -4.0, **f32), torch.randn(h, 4096, **f32)
+    for b, ctx, kv in ((8, 512, h), (64, 512, h), (256, 512, h),
+                       (64, 2048, h), (64, 2048, 8), (64, 2048, 1)):
+        nb = b * ctx // 16
+        kc = torch.randn(nb, kv, 16, d, **bf)
+        vc, q = torch.randn_like(kc), torch.randn(b, h * d, **bf)
+        sb, gate = batch_of(b, ctx - 1, 1), torch.randn(b, h, **bf)
+        what = f"single b={b} ctx={ctx} {h}/{kv}x{d}"
+        report(f"attn_ctx {what} softmax, chunk, bias",
+               timeit(lambda: hy.attn_ctx(q, gate, kc, vc, bias, sb,
+                                          d ** -0.5, 4096), 100),
+               4 * b * ctx * kv * d, 4.0 * b * ctx * h * d)
+        report(f"  attn_ctx {what} sigmoid, falloff",
+               timeit(lambda: hy.attn_ctx(
+                   q, None, kc, vc, None, sb, d ** -0.5, falloff=fall,
+                   weight_bias=wb), 100),
+               4 * b * ctx * kv * d, 4.0 * b * ctx * h * d)
+        del kc, vc
+    for b, ctx in ((8, 512), (64, 512), (256, 512), (16, 3072), (64, 4096)):
+        sb = batch_of(b, ctx - 1, 1)
+        for name, spec in (("", old), ("  ", new)):
+            row, seen = spec.row, min(spec.window or ctx, ctx)
+            cache = torch.randn(b * ctx // 16, 1, 16, row, **bf)
+            qa, o = torch.randn(b, h * row, **bf), torch.empty(b, h * rank,
+                                                               **bf)
+            report(f"{name}attn_latent single b={b} ctx={ctx} {h}x{row}"
+                   f"{' window 1024' if spec.window else ''}",
+                   timeit(lambda: ext.attn_ctx(
+                       o, qa, None, cache, cache[..., :rank], None, None,
+                       sb.positions, None, sb.block_table, spec.scale, 0,
+                       spec.window, 0, 0.0, 1.0, 1, seen, False, None, None,
+                       None), 50),
+                   b * seen * row * 2 + b * h * (row + rank) * 2,
+                   2.0 * b * seen * h * (row + rank))
+            del cache
+    for b, s_ in ((32, 512), (8, 2048), (4, 4096)):
+        t = b * s_
+        q, kc = torch.randn(t, h * d, **bf), torch.randn(t // 16, h, 16, d,
+                                                         **bf)
+        vc, sb = torch.randn_like(kc), batch_of(b, 0, s_)
+        gate = torch.randn(t, h, **bf)
+        flops = 4.0 * b * h * (s_ * (s_ + 1) / 2) * d
+        report(f"attn_ctx portions b={b} s={s_} softmax, chunk, bias",
+               timeit(lambda: hy.attn_ctx(q, gate, kc, vc, bias, sb,
+                                          d ** -0.5, 4096), 20),
+               8 * t * h * d, flops)
+        report(f"  attn_ctx portions b={b} s={s_} sigmoid, falloff",
+               timeit(lambda: hy.attn_ctx(
+                   q, None, kc, vc, None, sb, d ** -0.5, falloff=fall,
+                   weight_bias=wb), 20), 8 * t * h * d, flops)
+        del q, kc, vc
+        k = min(s_, win)
+        for name, spec in (("", old), ("  ", new)):
+            dq, r_ = d + spec.rot_dim, spec.rot_dim
+            q = torch.randn(t, h * dq, **bf)
+            kv, kr = torch.randn(t, 2 * h * d, **bf), torch.randn(t, r_, **bf)
+            o = torch.empty(t, h * d, **bf)
+            g = torch.randn(t, h * d if spec.out_gate else h, **bf)
+            pairs = k * (k + 1) / 2 + (s_ - k) * k if spec.window else \
+                s_ * (s_ + 1) / 2
+            report(f"{name}attn_flat b={b} s={s_} {h}x{d}+{r_}"
+                   f"{' window 1024' if spec.window else ''}",
+                   timeit(lambda: ext.attn_flat(
+                       o, q, g, kv, kr, sb.positions, sb.seq_start,
+                       sb.context(spec.window)[0], h, d, spec.scale,
+                       spec.window, s_), 20),
+                   (t * (h * (4 * d + r_) + r_) + g.numel()) * 2,
+                   2.0 * b * h * pairs * (2 * d + r_))
+            cache = torch.randn(t // 16, 1, 16, spec.row, **bf)
+            c = torch.empty(t, rank, **bf)
+            report(f"{name}latent_gather keys={t} of {spec.row}",
+                   timeit(lambda: ext.latent_gather(
+                       c, kr, cache, sb.block_table,
+                       sb.context(spec.window)[0], sb.positions, sb.seq_start,
+                       spec.window, s_), 20), t * spec.row * 4)
+            del q, kv, o, cache
 
 
 def bench_sample(B=64, V=32000):
@@ -814,6 +1009,8 @@ if __name__ == "__main__":
         bench_latent()
     if a.which == "mixers":
         bench_mixers()
+    if a.which == "sigmoid":
+        bench_sigmoid()
     if a.which in ("all", "norm"):
         bench_norm()
     if a.which in ("all", "sample"):

@@ -53,7 +53,7 @@ def test_bench_train_schema():
 @pytest.mark.timeout(300)
 @pytest.mark.parametrize("model,beside", [
     ("kakovik-tiny", "llama-tiny"), ("guronex-tiny", "llama-tiny"),
-    ("vurazen-tiny", "kakovik-tiny")])
+    ("vurazen-tiny", "kakovik-tiny"), ("ditalorn-tiny", "guronex-tiny")])
 def test_bench_hybrid_schema(model, beside):
     out = subprocess.run(
         [sys.executable, "bench.py", "--mode", "hybrid", "--steps", "2",

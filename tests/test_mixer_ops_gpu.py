@@ -348,7 +348,7 @@ def test_conv_qkv(spans, heads, kv, d, dv, taps, dtype):
     n, rows = batch.tokens.shape[0], (heads + kv) * d + kv * dv
     buf = rand(n, rows + 8, seed=1, dtype=dtype)
     bias, w = rand(rows, seed=2), rand(rows, taps, seed=3)
-    state = rand(len(spans), taps - 1, rows, seed=4, dtype=dtype)
+    state = conv_state(spans, taps, rows, dtype, 4)
     caches = [torch.zeros(64, kv, BS, s, dtype=dtype) for s in (d, dv)]
     sg, *cg = cuda(state, *caches)
     temp = QueryTemperature(0.6, 13)
