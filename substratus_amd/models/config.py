@@ -19,7 +19,8 @@ from .layers import LayerSpec, LoopSpec
 @dataclass
 class ModelConfig:
     name: str
-    family: str  # "llama" | "falcon" | "opt" | "kakovik" | "guronex" | "vurazen"
+    family: str  # "llama" | "falcon" | "opt" | "kakovik" | "guronex" |
+                 # "vurazen" | "ditalorn"
     hidden_size: int
     intermediate_size: int
     num_layers: int

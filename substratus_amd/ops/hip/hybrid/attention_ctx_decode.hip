@@ -1,7 +1,7 @@
 // Single-token attention over the paged bf16 cache with a distance bias, a
 // chunk mask, unequal key and value head sizes, a gated output, and softmax or
-// sigmoid weights (the formulas are in attention_ctx.hip). HBM-bound: every K and V row is read
-// once per group of GQ query heads.
+// sigmoid weights (the formulas are in attention_ctx.hip). HBM-bound: every K
+// and V row is read once per group of GQ query heads.
 //
 // One page of 16 keys is a wave's unit of work. Scores: 4 lanes per key, each
 // with every fourth 16-byte piece of the row. Values: CL lanes across the

@@ -1,8 +1,8 @@
 // Attention of prompt portions over the paged bf16 cache (which already holds
 // the portion's own keys and values), with a distance bias, a chunk mask,
 // unequal key and value head sizes, a gated output, and softmax or sigmoid
-// weights; the formulas are in attention_ctx.hip. Rows of a portion carry their absolute positions, so a
-// prompt can be cut anywhere.
+// weights; the formulas are in attention_ctx.hip. Rows of a portion carry
+// their absolute positions, so a prompt can be cut anywhere.
 //
 // The structure is that of attention_v5.hip: every wave owns 32 query rows
 // kept in registers, 64 keys per step go through LDS, S^T = K Q^T leaves a

@@ -219,7 +219,8 @@ bool by_quads(const GroupGemm<T, Y>& a) {
   return a.n % 4 == 0 && a.y_ld % 4 == 0 && a.y_gs % 4 == 0 &&
          ok(a.y, sizeof(Y)) &&
          (!a.gate_each || (a.gate_ld % 4 == 0 && a.gate_gs % 4 == 0 &&
-                           ok(a.gate, sizeof(T)))) && a.t_ld % 4 == 0 && ok(a.table, sizeof(T));
+                           ok(a.gate, sizeof(T)))) &&
+         a.t_ld % 4 == 0 && ok(a.table, sizeof(T));
 }
 
 template <class T, class Y>

@@ -47,8 +47,9 @@ DEV_INLINE void st_n(T* p, int n, const float* f) {
 // Channels c .. c + n - 1 (n 0: goes along, leaves no state), tokens
 // [t0, t0 + run) of entry e;
 // emit(row, y, look(row)), where look reads memory ahead of emit's writes.
-// TAPS 0: any number, inputs are read again for every tap.
-template <int VEC, int TAPS, class T, class L, class F>
+// TAPS 0: any number, inputs are read again for every tap. ONE: entries have
+// one token, for which fewer registers do.
+template <int VEC, int TAPS, bool ONE, class T, class L, class F>
 DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
                          int run, L look, F emit) {
   const Entry en = entry_of(a.seq_start, e);
@@ -113,10 +114,11 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
       }
     };
     // tokens at once: fewer if much is looked up for each
-    constexpr int AT_ONCE = sizeof(look(0l)) > 4 ? 4 : 8;
+    constexpr int AT_ONCE = ONE ? 1 : sizeof(look(0l)) > 4 ? 4 : 8;
     int t = t0;
-    for (; t + AT_ONCE <= t1; t += AT_ONCE)
-      steps(t, std::integral_constant<int, AT_ONCE>{});
+    if constexpr (!ONE)
+      for (; t + AT_ONCE <= t1; t += AT_ONCE)
+        steps(t, std::integral_constant<int, AT_ONCE>{});
     for (; t < t1; ++t) steps(t, std::integral_constant<int, 1>{});
   } else {
     for (int t = t0; t < t1; ++t) {
@@ -147,7 +149,7 @@ DEV_INLINE void convolve(const Conv<T>& a, int e, int c, int n, int t0,
   }
 }
 
-template <class T, int VEC, int TAPS>
+template <class T, int VEC, int TAPS, bool ONE>
 __global__ __launch_bounds__(BLOCK)
 void short_conv_kernel(Conv<T> a, int run) {
   const int c = (blockIdx.x * BLOCK + threadIdx.x) * VEC;
@@ -156,9 +158,9 @@ void short_conv_kernel(Conv<T> a, int run) {
   #pragma unroll
   for (int j = 0; j < VEC; ++j) b[j] = 0.f;
   if (a.bias != nullptr) ld_n<VEC>(a.bias + c, VEC, b);
-  convolve<VEC, TAPS>(a, blockIdx.z, c, VEC, blockIdx.y * run, run,
-                      [](long) { return 0; },
-                      [&](long row, float* y, int) {
+  convolve<VEC, TAPS, ONE>(a, blockIdx.z, c, VEC, blockIdx.y * run, run,
+                           [](long) { return 0; },
+                           [&](long row, float* y, int) {
     #pragma unroll
     for (int j = 0; j < VEC; ++j) {
       y[j] += b[j];
@@ -168,7 +170,7 @@ void short_conv_kernel(Conv<T> a, int run) {
   });
 }
 
-template <class T, int VEC, int TAPS>
+template <class T, int VEC, int TAPS, bool ONE>
 __global__ __launch_bounds__(BLOCK)
 void conv_rope_kernel(Conv<T> a, int run) {
   const int per = (a.dim + VEC - 1) / VEC, heads = a.channels / a.dim;
@@ -183,8 +185,8 @@ void conv_rope_kernel(Conv<T> a, int run) {
     int page, at;                      // of the cache
     float turn[VEC];                   // cosine and sine per pair
   };
-  convolve<VEC, TAPS>(a, blockIdx.z, head * a.dim + d, n, blockIdx.y * run,
-                      run, [&](long row) {
+  convolve<VEC, TAPS, ONE>(a, blockIdx.z, head * a.dim + d, n,
+                           blockIdx.y * run, run, [&](long row) {
     Seen f{};
     if (key) {
       const unsigned slot = a.slots[row], size = a.block_size;
@@ -231,7 +233,7 @@ DEV_INLINE Place place_of(const Conv<T>& a, long row) {
 // The first nqk workgroups have the queries and keys, VEC elements of a head
 // per thread. Every later one has BLOCK / lanes heads of values, whose threads
 // (a power of two; more than a wave: the workgroup) sum squares together.
-template <class T, int VEC, int TAPS>
+template <class T, int VEC, int TAPS, bool ONE>
 __global__ __launch_bounds__(BLOCK)
 void conv_qkv_kernel(Conv<T> a, int run, int nqk, int lanes) {
   const int tid = threadIdx.x;
@@ -247,8 +249,8 @@ void conv_qkv_kernel(Conv<T> a, int run, int nqk, int lanes) {
       Place to;
       float f;
     };
-    convolve<VEC, TAPS>(a, blockIdx.z, head * a.dim + d, n, blockIdx.y * run,
-                        run, [&](long row) {
+    convolve<VEC, TAPS, ONE>(a, blockIdx.z, head * a.dim + d, n,
+                             blockIdx.y * run, run, [&](long row) {
       Seen s{{0, 0}, 1.f};
       if (key)
         s.to = place_of(a, row);
@@ -276,9 +278,9 @@ void conv_qkv_kernel(Conv<T> a, int run, int nqk, int lanes) {
   const bool mine = head < a.kv && d < a.vdim;
   const int n = !mine ? 0 : VEC == 4 ? 4 : min(VEC, a.vdim - d);
   const int c = (nq + a.kv) * a.dim + (mine ? head * a.vdim + d : 0);
-  convolve<VEC, TAPS>(a, blockIdx.z, c, n, blockIdx.y * run, run,
-                      [&](long row) { return place_of(a, row); },
-                      [&](long row, float* y, const Place& to) {
+  convolve<VEC, TAPS, ONE>(a, blockIdx.z, c, n, blockIdx.y * run, run,
+                           [&](long row) { return place_of(a, row); },
+                           [&](long row, float* y, const Place& to) {
     if (a.v_eps >= 0.f) {
       float ss = 0.f;
       #pragma unroll
@@ -321,12 +323,16 @@ void rope_table_kernel(float* __restrict__ out,
 }
 
 template <class F>
-void by_taps(int taps, F f) {
+void by_taps(int taps, int max_len, F f) {
+  auto go = [&](auto n) {
+    if (max_len == 1) f(n, std::true_type{});
+    else f(n, std::false_type{});
+  };
   switch (taps) {
-    case 2: f(std::integral_constant<int, 2>{}); break;
-    case 3: f(std::integral_constant<int, 3>{}); break;
-    case 4: f(std::integral_constant<int, 4>{}); break;
-    default: f(std::integral_constant<int, 0>{});
+    case 2: go(std::integral_constant<int, 2>{}); break;
+    case 3: go(std::integral_constant<int, 3>{}); break;
+    case 4: go(std::integral_constant<int, 4>{}); break;
+    default: f(std::integral_constant<int, 0>{}, std::false_type{});
   }
 }
 
@@ -348,34 +354,35 @@ static int run_of(int taps, int max_len, long threads) {
 template <class T>
 void launch_short_conv(const Conv<T>& a, int entries, int max_len,
                        hipStream_t stream) {
-  auto go = [&](auto vec, auto taps) {
+  auto go = [&](auto vec, auto taps, auto one) {
     constexpr int V = decltype(vec)::value;
     const int units = (a.channels + V - 1) / V;
     const int run = run_of(a.taps, max_len, (long)units * entries);
-    short_conv_kernel<T, V, decltype(taps)::value>
+    short_conv_kernel<T, V, decltype(taps)::value, decltype(one)::value>
         <<<dim3((units + BLOCK - 1) / BLOCK, (max_len + run - 1) / run,
                 entries), BLOCK, 0, stream>>>(a, run);
   };
-  by_taps(a.taps, [&](auto taps) {
-    if (fours(a)) go(std::integral_constant<int, 4>{}, taps);
-    else go(std::integral_constant<int, 1>{}, taps);
+  by_taps(a.taps, max_len, [&](auto taps, auto one) {
+    if (fours(a)) go(std::integral_constant<int, 4>{}, taps, one);
+    else go(std::integral_constant<int, 1>{}, taps, one);
   });
 }
 
 template <class T>
 void launch_conv_rope(const Conv<T>& a, int entries, int max_len,
                       hipStream_t stream) {
-  auto go = [&](auto vec, auto taps) {
+  auto go = [&](auto vec, auto taps, auto one) {
     constexpr int V = decltype(vec)::value;
     const int units = a.channels / a.dim * ((a.dim + V - 1) / V);
     const int run = run_of(a.taps, max_len, (long)units * entries);
-    conv_rope_kernel<T, V, decltype(taps)::value>
+    conv_rope_kernel<T, V, decltype(taps)::value, decltype(one)::value>
         <<<dim3((units + BLOCK - 1) / BLOCK, (max_len + run - 1) / run,
                 entries), BLOCK, 0, stream>>>(a, run);
   };
-  by_taps(a.taps, [&](auto taps) {
-    if (fours(a) && a.dim % 4 == 0) go(std::integral_constant<int, 4>{}, taps);
-    else go(std::integral_constant<int, 2>{}, taps);
+  by_taps(a.taps, max_len, [&](auto taps, auto one) {
+    if (fours(a) && a.dim % 4 == 0)
+      go(std::integral_constant<int, 4>{}, taps, one);
+    else go(std::integral_constant<int, 2>{}, taps, one);
   });
 }
 
@@ -392,7 +399,7 @@ bool conv_qkv_takes(int vdim) { return vdim <= 2 * BLOCK; }
 template <class T>
 void launch_conv_qkv(const Conv<T>& a, int entries, int max_len,
                      hipStream_t stream) {
-  auto go = [&](auto vec, auto taps) {
+  auto go = [&](auto vec, auto taps, auto one) {
     constexpr int V = decltype(vec)::value;
     const int units = (a.channels - a.kv * a.vdim) / a.dim *
                       ((a.dim + V - 1) / V);
@@ -401,14 +408,14 @@ void launch_conv_qkv(const Conv<T>& a, int entries, int max_len,
     const int nv = (a.kv * lanes + BLOCK - 1) / BLOCK;
     const int run = run_of(a.taps, max_len,
                            (long)(units + a.kv * lanes) * entries);
-    conv_qkv_kernel<T, V, decltype(taps)::value>
+    conv_qkv_kernel<T, V, decltype(taps)::value, decltype(one)::value>
         <<<dim3(nqk + nv, (max_len + run - 1) / run, entries), BLOCK, 0,
            stream>>>(a, run, nqk, lanes);
   };
-  by_taps(a.taps, [&](auto taps) {
+  by_taps(a.taps, max_len, [&](auto taps, auto one) {
     if (fours(a) && a.dim % 4 == 0 && a.vdim % 4 == 0)
-      go(std::integral_constant<int, 4>{}, taps);
-    else go(std::integral_constant<int, 2>{}, taps);
+      go(std::integral_constant<int, 4>{}, taps, one);
+    else go(std::integral_constant<int, 2>{}, taps, one);
   });
 }
 
