@@ -261,7 +261,7 @@ def held_rows(cache, batch, e, length):
 
 @EVERY_PLACE
 @pytest.mark.parametrize("heads,kv,dim,vdim", [
-    (4, 2, 24, 40), (3, 1, 9, 7), (6, 1, 64, 80), (2, 2, 128, 128),
+    (4, 2, 24, 40), (3, 1, 9, 7), (7, 1, 56, 72), (2, 2, 128, 128),
     (5, 5, 16, 200)])
 @pytest.mark.parametrize("steep", [0.0, 1.0])
 def test_sigmoid_attention(place, heads, kv, dim, vdim, steep):

@@ -341,7 +341,7 @@ def test_long_contexts_shared_by_workgroups(window, keep, cap, sink):
 @BOTH
 @pytest.mark.parametrize("spans", [SPANS, LONG])
 @pytest.mark.parametrize("heads,kv,d,dv,taps", [
-    (4, 2, 64, 40, 4), (6, 1, 64, 80, 3), (2, 2, 9, 7, 2), (3, 3, 128, 256, 1),
+    (4, 2, 64, 40, 4), (7, 1, 56, 72, 3), (2, 2, 9, 7, 2), (3, 3, 128, 256, 1),
     (2, 1, 20, 300, 5), (16, 16, 128, 128, 4)])
 def test_conv_qkv(spans, heads, kv, d, dv, taps, dtype):
     batch = make_batch(spans)
